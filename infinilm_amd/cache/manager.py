@@ -8,7 +8,8 @@ state csrc/cache/mamba_cache.cpp:8-47 and cache_manager.py:33-68 (row 0 is the z
 from a free list).  Differences by design: pages are reserved portion by portion instead of for
 the whole prompt at admission, go straight back to the free list when a request ends or a window
 has passed them, and cache entries whose mixers keep all keys and those that keep a window form
-groups with page pools and block tables of their own.
+groups with page pools and block tables of their own (chunks of positions count like windows: the pages
+of a chunk go back once the request has moved on to the next).
 
 Prefix sharing (`prefix_caching=True`; the reference's python/infinilm/llm/prefix_cache.py and
 cache_manager.py:136-156, scheduler.py:158-164,503-523): a page all of whose tokens have been
@@ -41,6 +42,16 @@ class _Group:
     entries: List[int]
     pool: PagePool
     keep_first: int = 0          # with a window: the sequence's first positions whose pages are never given back
+    chunks: tuple = ()           # chunk sizes: a query reads from the start of its own chunk on (the earliest of these)
+
+    @property
+    def keeps_all(self) -> bool:
+        return self.window <= 0 and not self.chunks
+
+    @property
+    def span(self) -> int:
+        """The most positions before a query (and with it) that are still needed; 0: all."""
+        return self.window if self.window > 0 else (max(self.chunks) if self.chunks else 0)
 
 
 @dataclass
@@ -106,15 +117,16 @@ class CacheManager:
                 self._members.append((e, need))
         self.groups: List[_Group] = []
         self.group_of_entry: Dict[object, int] = {}
-        by_window: Dict[int, int] = {}
+        by_window: Dict[tuple, int] = {}
         for e, need in self._members:
             if isinstance(need, PagedKV):
                 kept = need.keep_first if need.window > 0 else 0
-                if (need.window, kept) not in by_window:
+                key = (need.window, kept, tuple(sorted(set(need.chunks))))
+                if key not in by_window:
                     n = (num_pages_per_group or {}).get(need.window, num_pages)
-                    by_window[(need.window, kept)] = len(self.groups)
-                    self.groups.append(_Group(need.window, [], PagePool(n), kept))
-                g = by_window[(need.window, kept)]
+                    by_window[key] = len(self.groups)
+                    self.groups.append(_Group(need.window, [], PagePool(n), kept, key[2]))
+                g = by_window[key]
                 self.groups[g].entries.append(e)
                 self.group_of_entry[e] = g
         # data plane
@@ -144,7 +156,7 @@ class CacheManager:
         self._free_slots = list(range(self.max_requests, 0, -1))
         self.requests: Dict[object, _Request] = {}
         # prefix sharing needs one group that keeps all keys, and no state beside it
-        self.prefix_caching = bool(prefix_caching) and len(self.groups) == 1 and self.groups[0].window <= 0 \
+        self.prefix_caching = bool(prefix_caching) and len(self.groups) == 1 and self.groups[0].keeps_all \
             and not self.state
         self._root_key = hashlib.blake2b(b"infinilm_amd page chain 1 " + str(self.page_size).encode(), digest_size=16).digest()
         self.prefix_hit_tokens = 0       # tokens taken over from published pages at admissions
@@ -174,7 +186,7 @@ class CacheManager:
 
     def stats(self) -> dict:
         return {"requests": len(self.requests),
-                "groups": [{"window": g.window, "keep_first": g.keep_first, "entries": len(g.entries), "pages": g.pool.num_pages,
+                "groups": [{"window": g.window, "keep_first": g.keep_first, "chunks": list(g.chunks), "entries": len(g.entries), "pages": g.pool.num_pages,
                             "free": g.pool.num_free, "idle": g.pool.num_idle, "evictions": g.pool.evictions,
                             "high_water": g.pool.high_water} for g in self.groups],
                 "state_slots_free": len(self._free_slots),
@@ -242,9 +254,12 @@ class CacheManager:
         return self.requests[req_id].length
 
     def _first_needed_page(self, group: _Group, first_query_pos: int) -> int:
-        if group.window <= 0:
+        if group.keeps_all:
             return 0
-        lo = max(0, first_query_pos - group.window + 1)
+        if group.chunks:
+            lo = min(first_query_pos - first_query_pos % size for size in group.chunks)
+        else:
+            lo = max(0, first_query_pos - group.window + 1)
         return lo // self.page_size
 
     def pages_needed(self, req_id, n_new: int) -> List[int]:
@@ -270,7 +285,7 @@ class CacheManager:
         for n, g in zip(need, self.groups):
             if n > g.pool.num_free:
                 raise OutOfPages(f"request {req_id!r}: {n} pages needed for {n_new} tokens after {r.length}, "
-                                 f"{g.pool.num_free} free of {g.pool.num_pages} (window {g.window})")
+                                 f"{g.pool.num_free} free of {g.pool.num_pages} (window {g.window}, chunks {g.chunks})")
         for n, g, table in zip(need, self.groups, r.tables):
             table.extend(g.pool.take(n))
         r.reserved = max(r.reserved, r.length + n_new)

@@ -90,12 +90,18 @@ class ModelSpec:
     # {name: shape}: tensors of the model itself that several layers read (`bind_shared` of their arrangements)
     shared_tensors: Optional[Dict[str, tuple]] = None
 
+    # copies of the residual stream that the sublayers read and write through weights of their own (arrangement
+    # "hyper_connected"); 0: one plain residual stream
+    streams: int = 0
+
     def num_cache_entries(self) -> int:
         ids = [r.cache for r in self.order if r.cache is not None] + [r.borrows for r in self.order if r.borrows is not None]
         return (max(ids) + 1) if ids else 0
 
     def validate(self) -> None:
         n = len(self.layers)
+        if self.streams and any(r.start is not None for r in self.order):
+            raise ValueError("what a run adds before it (RunStart) is for a plain residual stream")
         writers: Dict[int, int] = {}
         for i, run in enumerate(self.order):
             if not 0 <= run.layer < n:

@@ -3,7 +3,7 @@
 //
 // Contract (shared by every attention kernel here): token t belongs to request seg[t] and sits at
 // absolute position pos[t]; it sees the keys of its request at positions [lo, pos[t]] with
-// lo = max(0, pos[t] - window + 1) when window > 0, else 0.  Keys and values are read from the
+// lo = first_key(pos[t], reach) (common.h: the last positions, the token's own chunk, or all).  Keys and values are read from the
 // paged cache (keys [pages, nkv, page, d], values transposed [pages, nkv, d, page]) through block_tables[seg[t], key / page]; the step has
 // already written this step's keys there.
 //
@@ -64,14 +64,14 @@ __global__ void __launch_bounds__(64)
 attn_basic_kernel(T* __restrict__ out, float* __restrict__ ws, const T* __restrict__ q, const T* __restrict__ kc,
                   const T* __restrict__ vc, const int* __restrict__ block_tables,
                   const int* __restrict__ seg, const int* __restrict__ pos, int nh, int nkv, int d,
-                  int page, int max_blocks, int q_stride, int out_stride, float scale, int window, float softcap) {
+                  int page, int max_blocks, int q_stride, int out_stride, float scale, int reach, float softcap) {
     extern __shared__ float smem[];
     float* qs = smem;      // d
     float* ps = smem + d;  // 64
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const int kvh = h / (nh / nkv);
     const int p = pos[t];
-    const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    const int lo = first_key(p, reach);
     int c_first = lo / AB_CHUNK, c_last = p / AB_CHUNK;
     if (ws != nullptr) {
         if ((int)blockIdx.z < c_first || (int)blockIdx.z > c_last) return;   // the fold reads only the chunks the token sees
@@ -180,10 +180,10 @@ attn_basic_kernel(T* __restrict__ out, float* __restrict__ ws, const T* __restri
 template <typename T, int NA>
 __global__ void __launch_bounds__(64)
 attn_basic_fold_kernel(T* __restrict__ out, const float* __restrict__ ws, const int* __restrict__ pos, int nh, int d,
-                       int nchunks, int out_stride, int window) {
+                       int nchunks, int out_stride, int reach) {
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const int p = pos[t];
-    const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    const int lo = first_key(p, reach);
     if (p / AB_CHUNK > nchunks - 1) {
         // the caller's bound on the lengths was too small for this token: its last chunks were never computed.
         // A row of NaNs instead of a silently wrong one.
@@ -221,7 +221,7 @@ extern "C" int ilm_attn_basic_chunk() { return AB_CHUNK; }
 extern "C" int ilm_attn_basic(void* out, void* ws, int nchunks, const void* q, const void* kc, const void* vc,
                               const void* block_tables, const void* seg, const void* pos, int T_,
                               int nh, int nkv, int d, int page, int max_blocks, int q_stride,
-                              int out_stride, float scale, int window, int dtype, float softcap,
+                              int out_stride, float scale, int reach, int dtype, float softcap,
                               hipStream_t stream) {
     ILM_REQUIRE(T_ > 0 && nh > 0 && nkv > 0 && d > 0 && page > 0 && max_blocks > 0, "attn_basic: bad sizes");
     ILM_REQUIRE(nh % nkv == 0, "attn_basic: %d query heads do not divide into %d groups", nh, nkv);
@@ -237,7 +237,7 @@ extern "C" int ilm_attn_basic(void* out, void* ws, int nchunks, const void* q, c
 #define AB_LAUNCH_N(T_, VEC_, NA_)                                                                                      \
     attn_basic_kernel<T_, VEC_, NA_><<<grid, 64, shm, stream>>>(                                                        \
         (T_*)out, (float*)ws, (const T_*)q, (const T_*)kc, (const T_*)vc, (const int*)block_tables, (const int*)seg,    \
-        (const int*)pos, nh, nkv, d, page, max_blocks, q_stride, out_stride, scale, window, softcap)
+        (const int*)pos, nh, nkv, d, page, max_blocks, q_stride, out_stride, scale, reach, softcap)
     if (dtype == ILM_DTYPE_F32) {
         if (vec) { AB_LAUNCH(float, true); } else { AB_LAUNCH(float, false); }
     } else {
@@ -250,7 +250,7 @@ extern "C" int ilm_attn_basic(void* out, void* ws, int nchunks, const void* q, c
         dim3 g2(T_, nh);
 #define AB_FOLD(T_, NA_)                                                                                              \
     attn_basic_fold_kernel<T_, NA_><<<g2, 64, 0, stream>>>((T_*)out, (const float*)ws, (const int*)pos, nh, d, nchunks,   \
-                                                           out_stride, window)
+                                                           out_stride, reach)
         if (dtype == ILM_DTYPE_F32) {
             if (d <= 256) AB_FOLD(float, 4); else AB_FOLD(float, 16);
         } else {

@@ -46,7 +46,7 @@ __global__ void __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(DT <= 8
 attn_f32_kernel(float* __restrict__ out, float* __restrict__ ws, const float* __restrict__ qp, const float* __restrict__ kc,
                 const float* __restrict__ vc, const int* __restrict__ block_tables, const int* __restrict__ seg,
                 const int* __restrict__ pos, int nh, int nkv, int nsub, int page, int max_blocks, int q_stride,
-                int out_stride, float scale, int window, float softcap) {
+                int out_stride, float scale, int reach, float softcap) {
     constexpr int d = DT * 16;
     // tiles of keys (and of values) in flight: two, or one where the running result of the wave that walks all
     // chunks leaves no registers for the second (another wave of the SIMD then covers the wait)
@@ -57,7 +57,7 @@ attn_f32_kernel(float* __restrict__ out, float* __restrict__ ws, const float* __
     const int heads = (G - sub * 16 < 16) ? G - sub * 16 : 16;
     const int h = kvh * G + sub * 16 + (r < heads ? r : heads - 1);
     const int p = pos[t];
-    const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    const int lo = first_key(p, reach);
     int c_first = lo / FA_CHUNK, c_last = p / FA_CHUNK;
     if (SPLIT) {
         if ((int)blockIdx.z < c_first || (int)blockIdx.z > c_last) return;   // the fold reads only the chunks the token sees
@@ -221,10 +221,10 @@ attn_f32_kernel(float* __restrict__ out, float* __restrict__ ws, const float* __
 #define FA_FOLD_AHEAD 8
 __global__ void __launch_bounds__(256)
 attn_f32_fold_kernel(float* __restrict__ out, const float* __restrict__ ws, const int* __restrict__ pos, int nh, int d,
-                     int nchunks, int out_stride, int window) {
+                     int nchunks, int out_stride, int reach) {
     const int t = blockIdx.x, h = blockIdx.y, dim = threadIdx.x;
     const int p = pos[t];
-    const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    const int lo = first_key(p, reach);
     float* orow = out + (size_t)t * out_stride + (size_t)h * d;
     if (p / FA_CHUNK > nchunks - 1) {
         if (dim < d) orow[dim] = __int_as_float(0x7fc00000);
@@ -263,7 +263,7 @@ extern "C" int ilm_attn_f32_ws_row(int d) { return d + FA_WS_PAD; }
 // nchunks >= ceil((largest position + 1) / ilm_attn_f32_chunk()): one wave a chunk, then the fold.
 extern "C" int ilm_attn_f32(void* out, void* ws, int nchunks, const void* q, const void* kc, const void* vc,
                             const void* block_tables, const void* seg, const void* pos, int T_, int nh, int nkv, int d,
-                            int page, int max_blocks, int q_stride, int out_stride, float scale, int window, float softcap,
+                            int page, int max_blocks, int q_stride, int out_stride, float scale, int reach, float softcap,
                             hipStream_t stream) {
     ILM_REQUIRE(T_ > 0 && nh > 0 && nkv > 0 && d > 0 && page > 0 && max_blocks > 0, "attn_f32: bad sizes");
     ILM_REQUIRE(nh % nkv == 0, "attn_f32: %d query heads do not divide into %d groups", nh, nkv);
@@ -277,7 +277,7 @@ extern "C" int ilm_attn_f32(void* out, void* ws, int nchunks, const void* q, con
     ILM_REQUIRE((long long)nkv * nsub <= 65535 && nh <= 65535, "attn_f32: too many heads");
     dim3 grid(T_, nkv * nsub, ws != nullptr ? nchunks : 1);
 #define FA_ARGS (float*)out, (float*)ws, (const float*)q, (const float*)kc, (const float*)vc, (const int*)block_tables, \
-                (const int*)seg, (const int*)pos, nh, nkv, nsub, page, max_blocks, q_stride, out_stride, scale, window, softcap
+                (const int*)seg, (const int*)pos, nh, nkv, nsub, page, max_blocks, q_stride, out_stride, scale, reach, softcap
 #define FA_CASE(DT_)                                                                        \
     case DT_:                                                                               \
         if (ws != nullptr) attn_f32_kernel<DT_, true><<<grid, 64, 0, stream>>>(FA_ARGS);    \
@@ -293,7 +293,7 @@ extern "C" int ilm_attn_f32(void* out, void* ws, int nchunks, const void* q, con
     ILM_LAUNCH_CHECK("attn_f32");
     if (ws != nullptr) {
         attn_f32_fold_kernel<<<dim3(T_, nh), 64 * ((d + 63) / 64), 0, stream>>>((float*)out, (const float*)ws, (const int*)pos, nh, d, nchunks,
-                                                              out_stride, window);
+                                                              out_stride, reach);
         ILM_LAUNCH_CHECK("attn_f32_fold");
     }
     return 0;

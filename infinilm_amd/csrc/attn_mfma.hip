@@ -21,7 +21,8 @@
 // The rows of the two S tiles are assigned to keys so that each lane ends up with the
 // probabilities of 8 consecutive keys: they feed the second product without leaving registers.
 // Loads are unconditional 16-byte loads from clamped addresses, masked afterwards.
-// Needs: head size a multiple of 16 up to 128, page size a multiple of 16.
+// Needs: head size a multiple of 16 up to 128, page size a multiple of 16.  `reach` says which keys a token sees (`first_key`
+// in common.h): its last positions, its own chunk of positions, or all.
 #include "common.h"
 #include "no_alloc.h"
 #include <mutex>
@@ -42,6 +43,11 @@ __device__ __forceinline__ uint32_t pack_bf16x2(float a, float b) {
     return __builtin_bit_cast(uint32_t, __builtin_convertvector(v, bf16x2));
 }
 
+// what rounding two floats to the bfloat16 pair `hi` has left out, as a second bfloat16 pair: hi + rest holds 16 bits of each
+__device__ __forceinline__ uint32_t pack_rest(float a, float b, uint32_t hi) {
+    return pack_bf16x2(a - __uint_as_float(hi << 16), b - __uint_as_float(hi & 0xffff0000u));
+}
+
 __device__ __forceinline__ f32x4 mfma16(uint4 a, uint4 b, f32x4 c) {
     return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
 }
@@ -54,13 +60,14 @@ __device__ __forceinline__ float att_cap(float raw, float capq, float icapq) {
     return capq * (1.0f - 2.0f * __builtin_amdgcn_rcpf(e + 1.0f));
 }
 
-template <int D16>
+// WF: the softmax weights enter the second product as two bfloat16 terms each (the rounded weight and the rest)
+template <int D16, bool WF>
 __global__ void __launch_bounds__(ATT_WAVES * 64, 2)
 attn_mfma_kernel(bf16* __restrict__ out, float* __restrict__ ws_acc, float* __restrict__ ws_ml,
                  const bf16* __restrict__ q, const bf16* __restrict__ kc, const bf16* __restrict__ vc,
                  const int* __restrict__ block_tables, const int* __restrict__ seg,
                  const int* __restrict__ pos, const int* __restrict__ rows, int nh, int nkv, int page,
-                 int max_blocks, int q_stride, int out_stride, float scale_log2e, float capq, int window, int nsplit, int span) {
+                 int max_blocks, int q_stride, int out_stride, float scale_log2e, float capq, int reach, int nsplit, int span) {
     constexpr int D = D16 * 16;
     constexpr int KS = (D + 31) / 32;
     __shared__ float sm_acc[ATT_WAVES][D16][64][4];
@@ -73,7 +80,7 @@ attn_mfma_kernel(bf16* __restrict__ out, float* __restrict__ ws_acc, float* __re
     const int split = blockIdx.z;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, r = lane & 15, qg = lane >> 4;
     const int p = pos[t];
-    const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    const int lo = first_key(p, reach);
     const int hcol = hg * 16 + r;
     const bool head_ok = hcol < G;
     const int head = kvh * G + (head_ok ? hcol : G - 1);
@@ -177,11 +184,19 @@ attn_mfma_kernel(bf16* __restrict__ out, float* __restrict__ ws_acc, float* __re
             pf.y = pack_bf16x2(pe[2], pe[3]);                                                              \
             pf.z = pack_bf16x2(pe[4], pe[5]);                                                              \
             pf.w = pack_bf16x2(pe[6], pe[7]);                                                              \
+            uint4 pl;                                                                                      \
+            if (WF) {                                                                                      \
+                pl.x = pack_rest(pe[0], pe[1], pf.x);                                                      \
+                pl.y = pack_rest(pe[2], pe[3], pf.y);                                                      \
+                pl.z = pack_rest(pe[4], pe[5], pf.z);                                                      \
+                pl.w = pack_rest(pe[6], pe[7], pf.w);                                                      \
+            }                                                                                              \
             const int key0 = kb_ + qg * 8;                                                                 \
             const bool vok = key0 < kend_ && key0 + 8 > kbeg_;  /* else the loaded values are another group's */ \
             _Pragma("unroll") for (int db = 0; db < D16; ++db) {                                           \
                 _Pragma("unroll") for (int e = 0; e < 4; ++e) acc[db][e] *= corr;                          \
                 acc[db] = mfma16(vok ? VF_[db] : zero4, pf, acc[db]);                                      \
+                if (WF) acc[db] = mfma16(vok ? VF_[db] : zero4, pl, acc[db]);                              \
             }                                                                                              \
         }                                                                                                  \
     }
@@ -248,13 +263,13 @@ attn_mfma_kernel(bf16* __restrict__ out, float* __restrict__ ws_acc, float* __re
 __global__ void __launch_bounds__(64)
 attn_merge_one_wave_kernel(bf16* __restrict__ out, const float* __restrict__ ws_acc, const float* __restrict__ ws_ml,
                   const int* __restrict__ pos, const int* __restrict__ rows, int nh, int D, int out_stride,
-                  int window, int nsplit, int span) {
+                  int reach, int nsplit, int span) {
     __shared__ float wsm[64];
     const int t = rows != nullptr ? rows[blockIdx.x] : blockIdx.x;
     if (t < 0) return;   // an entry that fills up the list of a recorded step: no row (the whole workgroup leaves)
     const int h = blockIdx.y, lane = threadIdx.x;
     const int p = pos[t];
-    const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    const int lo = first_key(p, reach);
     const int s_lo = lo / span, s_hi = p / span;
     const size_t base = ((size_t)blockIdx.x * nh + h) * nsplit;
     float o[4] = {0.f, 0.f, 0.f, 0.f};  // dims lane, lane+64, ... (D <= 256)
@@ -312,7 +327,7 @@ attn_merge_one_wave_kernel(bf16* __restrict__ out, const float* __restrict__ ws_
 __global__ void __launch_bounds__(ATT_MERGE_WAVES * 64)
 attn_merge_kernel(bf16* __restrict__ out, const float* __restrict__ ws_acc, const float* __restrict__ ws_ml,
                   const int* __restrict__ pos, const int* __restrict__ rows, int nh, int D, int out_stride,
-                  int window, int nsplit, int span) {
+                  int reach, int nsplit, int span) {
     constexpr int NT = ATT_MERGE_WAVES * 64, PER = ATT_MERGE_MAX_CHUNKS / NT;
     __shared__ float wsm[ATT_MERGE_MAX_CHUNKS];
     __shared__ float red[2][ATT_MERGE_WAVES];
@@ -321,7 +336,7 @@ attn_merge_kernel(bf16* __restrict__ out, const float* __restrict__ ws_acc, cons
     if (t < 0) return;   // an entry that fills up the list of a recorded step: no row (the whole workgroup leaves)
     const int h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int p = pos[t];
-    const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    const int lo = first_key(p, reach);
     const int s_lo = lo / span, s_hi = p / span, n = s_hi - s_lo + 1;
     const size_t base = ((size_t)blockIdx.x * nh + h) * nsplit + s_lo;
     float ms[PER], ls[PER];
@@ -399,12 +414,12 @@ attn_merge_kernel(bf16* __restrict__ out, const float* __restrict__ ws_acc, cons
 
 __device__ __forceinline__ float max3(float a, float b, float c) { return fmaxf(fmaxf(a, b), c); }
 
-template <int D16, bool PAGE64>
+template <int D16, bool PAGE64, bool WF>   // WF: see attn_mfma_kernel
 __global__ void __launch_bounds__(256, 2)
 attn_tile_kernel(bf16* __restrict__ out, const bf16* __restrict__ q, const bf16* __restrict__ kc,
                  const bf16* __restrict__ vc, const int* __restrict__ block_tables, const int* __restrict__ seg,
                  const int* __restrict__ pos, const int* __restrict__ tiles, int nh, int nkv, int page,
-                 int max_blocks, int q_stride, int out_stride, float scale_log2e, float capq, int window, int pair_base) {
+                 int max_blocks, int q_stride, int out_stride, float scale_log2e, float capq, int reach, int pair_base) {
     constexpr int D = D16 * 16;
     constexpr int KS = (D + 31) / 32;
     // K rows [key][d] and V rows [d][key] in LDS, read in 16-byte pieces by 16 rows x 4 lane groups.
@@ -451,7 +466,7 @@ attn_tile_kernel(bf16* __restrict__ out, const bf16* __restrict__ q, const bf16*
     const bool head_ok = hcol < G;
     const int head = kvh * G + (head_ok ? hcol : G - 1);
     const int p_first = pos[t0], p_last = p_first + ntok - 1;
-    const int lo_first = (window > 0 && p_first - window + 1 > 0) ? p_first - window + 1 : 0;
+    const int lo_first = first_key(p_first, reach);
     const int* bt = block_tables + (size_t)seg[t0] * max_blocks;
     const uint4 zero4 = make_uint4(0u, 0u, 0u, 0u);
 
@@ -472,7 +487,7 @@ attn_tile_kernel(bf16* __restrict__ out, const bf16* __restrict__ q, const bf16*
         tok_ok[j] = i < ntok;
         tok[j] = t0 + (tok_ok[j] ? i : ntok - 1);
         pj[j] = p_first + (tok_ok[j] ? i : ntok - 1);
-        loj[j] = (window > 0 && pj[j] - window + 1 > 0) ? pj[j] - window + 1 : 0;
+        loj[j] = first_key(pj[j], reach);
         const bf16* qrow = q + (size_t)tok[j] * q_stride + (size_t)head * D;
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) {
@@ -692,18 +707,22 @@ attn_tile_kernel(bf16* __restrict__ out, const bf16* __restrict__ q, const bf16*
             }                                                                                              \
         }
         // one quarter of a sub-tile's p: token J_, key tile TAU_ -> two words of its fragment
-#define ATT_PQ(S_, J_, TAU_, LO_, HI_)                                                                     \
+#define ATT_PQ(S_, J_, TAU_, P_, A_, B_)                                                                   \
         {                                                                                                  \
             const float p0 = __builtin_amdgcn_exp2f(S_[J_][TAU_][0]);                                      \
             const float p1 = __builtin_amdgcn_exp2f(S_[J_][TAU_][1]);                                      \
             const float p2 = __builtin_amdgcn_exp2f(S_[J_][TAU_][2]);                                      \
             const float p3 = __builtin_amdgcn_exp2f(S_[J_][TAU_][3]);                                      \
-            LO_ = pack_bf16x2(p0, p1);                                                                     \
-            HI_ = pack_bf16x2(p2, p3);                                                                     \
+            pf##P_[J_].A_ = pack_bf16x2(p0, p1);                                                           \
+            pf##P_[J_].B_ = pack_bf16x2(p2, p3);                                                           \
+            if (WF) {                                                                                      \
+                pl##P_[WF ? J_ : 0].A_ = pack_rest(p0, p1, pf##P_[J_].A_);                                          \
+                pl##P_[WF ? J_ : 0].B_ = pack_rest(p2, p3, pf##P_[J_].B_);                                          \
+            }                                                                                              \
         }
         ATT_FOLLOW(s0, )
         // scores of the second sub-tile on the matrix cores, p of the first on the vector units
-        uint4 pf0[ATT_NT], pf1[ATT_NT];
+        uint4 pf0[ATT_NT], pf1[ATT_NT], pl0[WF ? ATT_NT : 1], pl1[WF ? ATT_NT : 1];
         __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) {
@@ -711,10 +730,10 @@ attn_tile_kernel(bf16* __restrict__ out, const bf16* __restrict__ q, const bf16*
             for (int tau = 0; tau < 2; ++tau)
 #pragma unroll
                 for (int j = 0; j < ATT_NT; ++j) s1[j][tau] = mfma16(kf1[tau][ks], qf[j][ks], s1[j][tau]);
-            if (ks == 0) ATT_PQ(s0, 0, 0, pf0[0].x, pf0[0].y)
-            if (ks == 1 || KS == 1) ATT_PQ(s0, 0, 1, pf0[0].z, pf0[0].w)
-            if (ks == 2 || (KS <= 2 && ks == KS - 1)) ATT_PQ(s0, 1, 0, pf0[1].x, pf0[1].y)
-            if (ks == KS - 1) ATT_PQ(s0, 1, 1, pf0[1].z, pf0[1].w)
+            if (ks == 0) ATT_PQ(s0, 0, 0, 0, x, y)
+            if (ks == 1 || KS == 1) ATT_PQ(s0, 0, 1, 0, z, w)
+            if (ks == 2 || (KS <= 2 && ks == KS - 1)) ATT_PQ(s0, 1, 0, 0, x, y)
+            if (ks == KS - 1) ATT_PQ(s0, 1, 1, 0, z, w)
             __builtin_amdgcn_sched_barrier(0);
         }
         // the next tile leaves for the registers only now: until here they held score fragments
@@ -723,12 +742,21 @@ attn_tile_kernel(bf16* __restrict__ out, const bf16* __restrict__ q, const bf16*
         // (should the reference point move now, the first sub-tile's products, made with the old one,
         // are added first, and the interleaved block below adds zeros in their place)
         ATT_FOLLOW(s1, {
-            _Pragma("unroll") for (int j = 0; j < ATT_NT; ++j) lacc[j] = mfma16(ones4, pf0[j], lacc[j]);
+            _Pragma("unroll") for (int j = 0; j < ATT_NT; ++j) {
+                lacc[j] = mfma16(ones4, pf0[j], lacc[j]);
+                if (WF) lacc[j] = mfma16(ones4, pl0[WF ? j : 0], lacc[j]);
+            }
             _Pragma("unroll") for (int db = 0; db < D16; ++db) {
                 const uint4 v = *reinterpret_cast<const uint4*>(&Vs[v_at(db * 16 + r, qg)]);
-                _Pragma("unroll") for (int j = 0; j < ATT_NT; ++j) acc[j][db] = mfma16(v, pf0[j], acc[j][db]);
+                _Pragma("unroll") for (int j = 0; j < ATT_NT; ++j) {
+                    acc[j][db] = mfma16(v, pf0[j], acc[j][db]);
+                    if (WF) acc[j][db] = mfma16(v, pl0[WF ? j : 0], acc[j][db]);
+                }
             }
-            _Pragma("unroll") for (int j = 0; j < ATT_NT; ++j) pf0[j] = zero4;
+            _Pragma("unroll") for (int j = 0; j < ATT_NT; ++j) {
+                pf0[j] = zero4;
+                if (WF) pl0[WF ? j : 0] = zero4;
+            }
         })
         constexpr int DH = (D16 + 1) / 2;   // value fragments in two halves: fewer registers live
         uint4 vf[DH];
@@ -736,7 +764,10 @@ attn_tile_kernel(bf16* __restrict__ out, const bf16* __restrict__ q, const bf16*
         for (int db = 0; db < DH; ++db) vf[db] = *reinterpret_cast<const uint4*>(&Vs[v_at(db * 16 + r, qg)]);
         __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-        for (int j = 0; j < ATT_NT; ++j) lacc[j] = mfma16(ones4, pf0[j], lacc[j]);
+        for (int j = 0; j < ATT_NT; ++j) {
+            lacc[j] = mfma16(ones4, pf0[j], lacc[j]);
+            if (WF) lacc[j] = mfma16(ones4, pl0[WF ? j : 0], lacc[j]);
+        }
 #pragma unroll
         for (int h = 0; h < 2; ++h) {
 #pragma unroll
@@ -744,12 +775,15 @@ attn_tile_kernel(bf16* __restrict__ out, const bf16* __restrict__ q, const bf16*
                 const int db = h * DH + i;
                 if (db < D16) {
 #pragma unroll
-                    for (int j = 0; j < ATT_NT; ++j) acc[j][db] = mfma16(vf[i], pf0[j], acc[j][db]);
+                    for (int j = 0; j < ATT_NT; ++j) {
+                        acc[j][db] = mfma16(vf[i], pf0[j], acc[j][db]);
+                        if (WF) acc[j][db] = mfma16(vf[i], pl0[WF ? j : 0], acc[j][db]);
+                    }
                 }
-                if (h == 0 && i == 0) ATT_PQ(s1, 0, 0, pf1[0].x, pf1[0].y)
-                if (h == 0 && i == DH - 1) ATT_PQ(s1, 0, 1, pf1[0].z, pf1[0].w)
-                if (h == 1 && i == 0) ATT_PQ(s1, 1, 0, pf1[1].x, pf1[1].y)
-                if (h == 1 && i == DH - 1) ATT_PQ(s1, 1, 1, pf1[1].z, pf1[1].w)
+                if (h == 0 && i == 0) ATT_PQ(s1, 0, 0, 1, x, y)
+                if (h == 0 && i == DH - 1) ATT_PQ(s1, 0, 1, 1, z, w)
+                if (h == 1 && i == 0) ATT_PQ(s1, 1, 0, 1, x, y)
+                if (h == 1 && i == DH - 1) ATT_PQ(s1, 1, 1, 1, z, w)
                 __builtin_amdgcn_sched_barrier(0);
             }
             // the next half: second half of this sub-tile, then the first of the other
@@ -760,7 +794,10 @@ attn_tile_kernel(bf16* __restrict__ out, const bf16* __restrict__ q, const bf16*
             }
         }
 #pragma unroll
-        for (int j = 0; j < ATT_NT; ++j) lacc[j] = mfma16(ones4, pf1[j], lacc[j]);
+        for (int j = 0; j < ATT_NT; ++j) {
+            lacc[j] = mfma16(ones4, pf1[j], lacc[j]);
+            if (WF) lacc[j] = mfma16(ones4, pl1[WF ? j : 0], lacc[j]);
+        }
 #pragma unroll
         for (int h = 0; h < 2; ++h) {
 #pragma unroll
@@ -768,7 +805,10 @@ attn_tile_kernel(bf16* __restrict__ out, const bf16* __restrict__ q, const bf16*
                 const int db = h * DH + i;
                 if (db < D16) {
 #pragma unroll
-                    for (int j = 0; j < ATT_NT; ++j) acc[j][db] = mfma16(vf[i], pf1[j], acc[j][db]);
+                    for (int j = 0; j < ATT_NT; ++j) {
+                        acc[j][db] = mfma16(vf[i], pf1[j], acc[j][db]);
+                        if (WF) acc[j][db] = mfma16(vf[i], pl1[WF ? j : 0], acc[j][db]);
+                    }
                 }
             }
             if (h == 0) {
@@ -866,7 +906,7 @@ attn_tile_kernel(bf16* __restrict__ out, const bf16* __restrict__ q, const bf16*
                         for (int e = 0; e < 4; ++e) acc[j][db][e] *= corr;
                 }
             }
-            uint4 pf[ATT_NT];
+            uint4 pf[ATT_NT], pl[WF ? ATT_NT : 1];
 #pragma unroll
             for (int j = 0; j < ATT_NT; ++j) {
                 float pe[8];
@@ -881,6 +921,13 @@ attn_tile_kernel(bf16* __restrict__ out, const bf16* __restrict__ q, const bf16*
                 pf[j].z = pack_bf16x2(pe[4], pe[5]);
                 pf[j].w = pack_bf16x2(pe[6], pe[7]);
                 lacc[j] = mfma16(ones4, pf[j], lacc[j]);
+                if (WF) {
+                    pl[WF ? j : 0].x = pack_rest(pe[0], pe[1], pf[j].x);
+                    pl[WF ? j : 0].y = pack_rest(pe[2], pe[3], pf[j].y);
+                    pl[WF ? j : 0].z = pack_rest(pe[4], pe[5], pf[j].z);
+                    pl[WF ? j : 0].w = pack_rest(pe[6], pe[7], pf[j].w);
+                    lacc[j] = mfma16(ones4, pl[WF ? j : 0], lacc[j]);
+                }
             }
             const int key0 = kbs + qg * 8;
             const bool vok = key0 <= p_last && key0 + 8 > lo_first;   // else the tile holds another group's values
@@ -889,14 +936,17 @@ attn_tile_kernel(bf16* __restrict__ out, const bf16* __restrict__ q, const bf16*
                 const uint4 v = *reinterpret_cast<const uint4*>(&Vs[v_at(db * 16 + r, sub * 4 + qg)]);
                 const uint4 vf = (PAGE64 || vok) ? v : zero4;   // PAGE64: the tile's own page, finite, times p = 0
 #pragma unroll
-                for (int j = 0; j < ATT_NT; ++j) acc[j][db] = mfma16(vf, pf[j], acc[j][db]);
+                for (int j = 0; j < ATT_NT; ++j) {
+                    acc[j][db] = mfma16(vf, pf[j], acc[j][db]);
+                    if (WF) acc[j][db] = mfma16(vf, pl[WF ? j : 0], acc[j][db]);
+                }
             }
         }
     };
     // Tiles [kb_a, kb_b) are seen whole by every token of the workgroup: from the window's edge of the
     // last token (the start without a window) to the tile before the first token's own.  Three loops
     // rather than one with a branch: each keeps its own registers.
-    const int lo_last = (window > 0 && p_last - window + 1 > 0) ? p_last - window + 1 : 0;
+    const int lo_last = first_key(p_last, reach);
     int kb_a = (lo_last + ATT_TK - 1) & ~(ATT_TK - 1);
     int kb_b = ((p_first + 1) / ATT_TK) * ATT_TK;
     if (D % 32 != 0 || kb_b < kb_a) kb_a = kb_b = kb0;
@@ -938,7 +988,7 @@ extern "C" int ilm_attn_tile_tokens() { return ATT_TT; }
 extern "C" int ilm_attn_tile(void* out, const void* q, const void* kc, const void* vc, const void* block_tables,
                              const void* seg, const void* pos, const void* tiles, int n_tiles, int nh, int nkv,
                              int d, int page, int max_blocks, int q_stride, int out_stride, float scale,
-                             int window, float softcap, hipStream_t stream) {
+                             int reach, float softcap, int float_weights, hipStream_t stream) {
     ILM_REQUIRE(n_tiles > 0 && nh > 0 && nkv > 0 && nh % nkv == 0, "attn_tile: bad sizes");
     ILM_REQUIRE(d % 16 == 0 && d >= 16 && d <= 128, "attn_tile: head size %d is not a multiple of 16 up to 128", d);
     ILM_REQUIRE(page % 16 == 0 && page > 0, "attn_tile: page size %d is not a multiple of 16", page);
@@ -953,11 +1003,14 @@ extern "C" int ilm_attn_tile(void* out, const void* q, const void* kc, const voi
     const long long n_items = (long long)n_tiles * nkv * HG;
     const int pair_base = (n_items > cus && n_items <= 2 * cus) ? cus : 0;
 #define AT_ARGS (bf16*)out, (const bf16*)q, (const bf16*)kc, (const bf16*)vc, (const int*)block_tables, (const int*)seg, \
-                (const int*)pos, (const int*)tiles, nh, nkv, page, max_blocks, q_stride, out_stride, sl2, capq, window, pair_base
+                (const int*)pos, (const int*)tiles, nh, nkv, page, max_blocks, q_stride, out_stride, sl2, capq, reach, pair_base
 #define AT_CASE(D16)                                                                   \
     case D16:                                                                          \
-        if (page % ATT_TK == 0) attn_tile_kernel<D16, true><<<grid, 256, 0, stream>>>(AT_ARGS);  \
-        else attn_tile_kernel<D16, false><<<grid, 256, 0, stream>>>(AT_ARGS);          \
+        if (float_weights) {                                                           \
+            if (page % ATT_TK == 0) attn_tile_kernel<D16, true, true><<<grid, 256, 0, stream>>>(AT_ARGS);  \
+            else attn_tile_kernel<D16, false, true><<<grid, 256, 0, stream>>>(AT_ARGS);    \
+        } else if (page % ATT_TK == 0) attn_tile_kernel<D16, true, false><<<grid, 256, 0, stream>>>(AT_ARGS);  \
+        else attn_tile_kernel<D16, false, false><<<grid, 256, 0, stream>>>(AT_ARGS);   \
         break
     switch (d / 16) {
         AT_CASE(1); AT_CASE(2); AT_CASE(3); AT_CASE(4); AT_CASE(5); AT_CASE(6); AT_CASE(7); AT_CASE(8);
@@ -975,8 +1028,8 @@ extern "C" int ilm_attn_mfma_step() { return ATT_STEP; }
 static int attn_mfma_launch(void* out, void* ws_acc, void* ws_ml, const void* q, const void* kc,
                             const void* vc, const void* block_tables, const void* seg, const void* pos,
                             const void* rows, int T_, int nh, int nkv, int d, int page, int max_blocks,
-                            int q_stride, int out_stride, float scale, int window, int nsplit, int span,
-                            float softcap, hipStream_t stream) {
+                            int q_stride, int out_stride, float scale, int reach, int nsplit, int span,
+                            float softcap, int float_weights, hipStream_t stream) {
     ILM_REQUIRE(T_ > 0 && nh > 0 && nkv > 0 && nh % nkv == 0, "attn_mfma: bad head counts nh=%d nkv=%d", nh, nkv);
     ILM_REQUIRE(d % 16 == 0 && d >= 16 && d <= 128, "attn_mfma: head size %d is not a multiple of 16 up to 128", d);
     ILM_REQUIRE(page % 16 == 0 && page > 0, "attn_mfma: page size %d is not a multiple of 16", page);
@@ -989,28 +1042,30 @@ static int attn_mfma_launch(void* out, void* ws_acc, void* ws_ml, const void* q,
     dim3 grid(T_, nkv * HG, nsplit);
     const float sl2 = scale * 1.4426950408889634f;
     const float capq = softcap > 0.f ? softcap / scale : 0.f;
+#define AM_ARGS (bf16*)out, (float*)ws_acc, (float*)ws_ml, (const bf16*)q, (const bf16*)kc, (const bf16*)vc, \
+                (const int*)block_tables, (const int*)seg, (const int*)pos, (const int*)rows, nh, nkv, page, \
+                max_blocks, q_stride, out_stride, sl2, capq, reach, nsplit, span
 #define AM_CASE(D16)                                                                                           \
     case D16:                                                                                                  \
-        attn_mfma_kernel<D16><<<grid, ATT_WAVES * 64, 0, stream>>>(                                            \
-            (bf16*)out, (float*)ws_acc, (float*)ws_ml, (const bf16*)q, (const bf16*)kc, (const bf16*)vc,      \
-            (const int*)block_tables, (const int*)seg, (const int*)pos, (const int*)rows, nh, nkv, page,      \
-            max_blocks, q_stride, out_stride, sl2, capq, window, nsplit, span);                                      \
+        if (float_weights) attn_mfma_kernel<D16, true><<<grid, ATT_WAVES * 64, 0, stream>>>(AM_ARGS);          \
+        else attn_mfma_kernel<D16, false><<<grid, ATT_WAVES * 64, 0, stream>>>(AM_ARGS);                       \
         break
     switch (d / 16) {
         AM_CASE(1); AM_CASE(2); AM_CASE(3); AM_CASE(4); AM_CASE(5); AM_CASE(6); AM_CASE(7); AM_CASE(8);
         default: ILM_REQUIRE(false, "attn_mfma: head size %d", d);
     }
 #undef AM_CASE
+#undef AM_ARGS
     ILM_LAUNCH_CHECK("attn_mfma");
     if (nsplit > 1) {
         dim3 g2(T_, nh);
         if (nsplit <= ATT_MERGE_ONE_WAVE_CHUNKS)
             attn_merge_one_wave_kernel<<<g2, 64, 0, stream>>>((bf16*)out, (const float*)ws_acc, (const float*)ws_ml, (const int*)pos,
-                                                              (const int*)rows, nh, d, out_stride, window, nsplit, span);
+                                                              (const int*)rows, nh, d, out_stride, reach, nsplit, span);
         else
             attn_merge_kernel<<<g2, ATT_MERGE_WAVES * 64, 0, stream>>>((bf16*)out, (const float*)ws_acc, (const float*)ws_ml,
                                                                        (const int*)pos, (const int*)rows, nh, d, out_stride,
-                                                                       window, nsplit, span);
+                                                                       reach, nsplit, span);
         ILM_LAUNCH_CHECK("attn_merge");
     }
     return 0;
@@ -1019,10 +1074,10 @@ static int attn_mfma_launch(void* out, void* ws_acc, void* ws_ml, const void* q,
 extern "C" int ilm_attn_mfma(void* out, void* ws_acc, void* ws_ml, const void* q, const void* kc,
                              const void* vc, const void* block_tables, const void* seg, const void* pos,
                              const void* rows, int T_, int nh, int nkv, int d, int page, int max_blocks,
-                             int q_stride, int out_stride, float scale, int window, int nsplit, int span,
-                             float softcap, hipStream_t stream) {
+                             int q_stride, int out_stride, float scale, int reach, int nsplit, int span,
+                             float softcap, int float_weights, hipStream_t stream) {
     return attn_mfma_launch(out, ws_acc, ws_ml, q, kc, vc, block_tables, seg, pos, rows, T_, nh, nkv, d, page, max_blocks,
-                            q_stride, out_stride, scale, window, nsplit, span, softcap, stream);
+                            q_stride, out_stride, scale, reach, nsplit, span, softcap, float_weights, stream);
 }
 
 // ------------------------------------------------------------------------------------------------
@@ -1065,7 +1120,7 @@ extern "C" int ilm_attn_static_init() {
 extern "C" int ilm_attn_mfma_static(void* out, const void* q, const void* kc, const void* vc,
                                     const void* block_tables, const void* seg, const void* pos, const void* rows,
                                     int T_, int nh, int nkv, int d, int page, int max_blocks, int q_stride,
-                                    int out_stride, float scale, int window, int nsplit, int span,
+                                    int out_stride, float scale, int reach, int nsplit, int span,
                                     hipStream_t stream) {
     ILM_REQUIRE(T_ > 0 && nh > 0 && d > 0 && nsplit >= 1, "attn_mfma_static: bad sizes T=%d nh=%d d=%d chunks=%d", T_, nh, d, nsplit);
     float* ws_acc = nullptr;
@@ -1082,5 +1137,5 @@ extern "C" int ilm_attn_mfma_static(void* out, const void* q, const void* kc, co
         ws_ml = base + acc_floats;   // d is a multiple of 16: 64-byte aligned
     }
     return attn_mfma_launch(out, ws_acc, ws_ml, q, kc, vc, block_tables, seg, pos, rows, T_, nh, nkv, d, page, max_blocks,
-                            q_stride, out_stride, scale, window, nsplit, span, 0.f, stream);
+                            q_stride, out_stride, scale, reach, nsplit, span, 0.f, 0, stream);
 }

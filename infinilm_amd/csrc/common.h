@@ -79,6 +79,22 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
     return t;
 }
 
+// The first key a token at position p sees.  `reach` > 0: its last `reach` positions; < 0: the positions of its own chunk, chunks
+// of -reach positions counted from the sequence's start; 0: all.  It never falls as p grows.
+__device__ __forceinline__ int first_key(int p, int reach) {
+    if (reach > 0) return p - reach + 1 > 0 ? p - reach + 1 : 0;
+    return reach < 0 ? p - p % -reach : 0;
+}
+
+// The gate's activation of a gated feed-forward
+#define ILM_GLU_SILU 0
+#define ILM_GLU_GELU_TANH 1
+// (both are g * sigmoid(z): z = g, or twice the argument of the tanh)
+__device__ __forceinline__ float glu_act(float g, int kind) {
+    const float z = kind == ILM_GLU_GELU_TANH ? 1.5957691216057308f * (g + 0.044715f * g * g * g) : g;
+    return g / (1.0f + expf(-z));
+}
+
 extern "C" const char* ilm_last_error();
 void ilm_set_error(const char* fmt, ...);
 // compute units of the current device (looked up once a process; 256 if the runtime does not say)

@@ -67,14 +67,14 @@ __device__ __forceinline__ void load8(const T* p, float* v) {
 }
 
 // ------------------------------------------------------------------------------------------
-// r += alpha * h ; x = r / sqrt(mean(r^2) + eps) * w
+// r += alpha * h ; x = r / sqrt(mean(r^2) + eps) * (w + w_offset)      (w_offset 1: weights stored around zero)
 // One block per row.  The sum of squares is reduced in an order that depends on H only, so a
 // row's result does not depend on what else is in the batch.
 // ------------------------------------------------------------------------------------------
 template <typename T, typename WT, typename HT>
 __global__ void __launch_bounds__(256)
 add_rmsnorm_kernel(T* __restrict__ x, float* __restrict__ r, const HT* __restrict__ h,
-                   const WT* __restrict__ w, int H, float alpha, float eps, int parts, size_t pstride, int frag_mg) {
+                   const WT* __restrict__ w, int H, float alpha, float eps, int parts, size_t pstride, int frag_mg, float w_offset) {
     __shared__ float red[4];
     const size_t base = (size_t)blockIdx.x * H;
     float ss = 0.f;
@@ -98,11 +98,11 @@ add_rmsnorm_kernel(T* __restrict__ x, float* __restrict__ r, const HT* __restric
         // fragment order (frag.h), H a multiple of 8; the k up to the next multiple of 32 are zeros
         const int kp = (H + 31) / 32 * 32;
         for (int j = threadIdx.x; j < kp; j += 256)
-            x[frag_x_chunk(blockIdx.x, j >> 3, frag_mg) * 8 + (j & 7)] = from_f32<T>(j < H ? r[base + j] * rstd * to_f32(w[j]) : 0.f);
+            x[frag_x_chunk(blockIdx.x, j >> 3, frag_mg) * 8 + (j & 7)] = from_f32<T>(j < H ? r[base + j] * rstd * (to_f32(w[j]) + w_offset) : 0.f);
         return;
     }
     for (int j = threadIdx.x; j < H; j += 256)
-        x[base + j] = from_f32<T>(r[base + j] * rstd * to_f32(w[j]));
+        x[base + j] = from_f32<T>(r[base + j] * rstd * (to_f32(w[j]) + w_offset));
 }
 
 // Fast form for H = 8 * 256 * NITER' (NITER' <= NITER): each thread keeps its 8 * NITER values in
@@ -111,7 +111,7 @@ add_rmsnorm_kernel(T* __restrict__ x, float* __restrict__ r, const HT* __restric
 template <typename T, typename WT, typename HT, int NITER>
 __global__ void __launch_bounds__(256)
 add_rmsnorm_vec_kernel(T* __restrict__ x, float* __restrict__ r, const HT* __restrict__ h,
-                       const WT* __restrict__ w, int H, float alpha, float eps, int parts, size_t pstride, int frag_mg) {
+                       const WT* __restrict__ w, int H, float alpha, float eps, int parts, size_t pstride, int frag_mg, float w_offset) {
     __shared__ float red[4];
     const size_t base = (size_t)blockIdx.x * H;
     float v[NITER][8];
@@ -173,7 +173,7 @@ add_rmsnorm_vec_kernel(T* __restrict__ x, float* __restrict__ r, const HT* __res
         if (j < H) {
             T o[8];
 #pragma unroll
-            for (int e = 0; e < 8; ++e) o[e] = from_f32<T>(v[it][e] * rstd * wv[it][e]);
+            for (int e = 0; e < 8; ++e) o[e] = from_f32<T>(v[it][e] * rstd * (wv[it][e] + w_offset));
             if (sizeof(T) == 2 && frag_mg > 0) {   // fragment order (frag.h): the 16-byte chunk of row blockIdx.x
                 reinterpret_cast<uint4*>(x)[frag_x_chunk(blockIdx.x, j >> 3, frag_mg)] = *reinterpret_cast<uint4*>(o);
             } else if (sizeof(T) == 2) {
@@ -201,7 +201,7 @@ add_rmsnorm_vec_kernel(T* __restrict__ x, float* __restrict__ r, const HT* __res
 template <typename WT, int PB>   // PB: slots for parts (8 or 16; slots beyond the parts load the last part again)
 __global__ void __launch_bounds__(NORM_WIDE_THREADS)
 add_rmsnorm_wide_kernel(bf16* __restrict__ x, float* __restrict__ r, const float* __restrict__ h, const WT* __restrict__ w,
-                        int H, float alpha, float eps, int parts, size_t pstride, int frag_mg) {
+                        int H, float alpha, float eps, int parts, size_t pstride, int frag_mg, float w_offset) {
     __shared__ float red[NORM_WIDE_THREADS / 64];
     const size_t base = (size_t)blockIdx.x * H;
     const int j = threadIdx.x * 4;
@@ -236,8 +236,8 @@ add_rmsnorm_wide_kernel(bf16* __restrict__ x, float* __restrict__ r, const float
     for (int i = 0; i < (int)(blockDim.x >> 6); ++i) tot += red[i];
     const float rstd = 1.0f / sqrtf(tot / (float)H + eps);
     bf16 o[4];
-    o[0] = from_f32<bf16>(v.x * rstd * wv[0]); o[1] = from_f32<bf16>(v.y * rstd * wv[1]);
-    o[2] = from_f32<bf16>(v.z * rstd * wv[2]); o[3] = from_f32<bf16>(v.w * rstd * wv[3]);
+    o[0] = from_f32<bf16>(v.x * rstd * (wv[0] + w_offset)); o[1] = from_f32<bf16>(v.y * rstd * (wv[1] + w_offset));
+    o[2] = from_f32<bf16>(v.z * rstd * (wv[2] + w_offset)); o[3] = from_f32<bf16>(v.w * rstd * (wv[3] + w_offset));
     if (frag_mg > 0) {   // fragment order (frag.h): half of the 16-byte chunk of row blockIdx.x; zeros up to the next multiple of 32 k
         const int kp = (H + 31) / 32 * 32;
         if (j < kp) {
@@ -253,7 +253,7 @@ add_rmsnorm_wide_kernel(bf16* __restrict__ x, float* __restrict__ r, const float
 // (h_dtype == ILM_DTYPE_F32, e.g. the parts of a K-split product); null: nothing to add.
 extern "C" int ilm_add_rmsnorm(void* x, void* r, const void* h, const void* w, int rows, int H,
                                float alpha, float eps, int dtype, int w_dtype, int h_dtype, int parts,
-                               long pstride, int frag_mg, hipStream_t stream) {
+                               long pstride, int frag_mg, float w_offset, hipStream_t stream) {
     // frag_mg > 0: x is bfloat16 in fragment order (frag.h) with frag_mg = ceil(rows / 16) groups of rows
     ILM_REQUIRE(rows > 0 && H > 0, "add_rmsnorm: bad sizes rows=%d H=%d", rows, H);
     ILM_REQUIRE(frag_mg == 0 || (dtype == ILM_DTYPE_BF16 && H % 8 == 0 && frag_mg == (rows + 15) / 16),
@@ -269,7 +269,7 @@ extern "C" int ilm_add_rmsnorm(void* x, void* r, const void* h, const void* w, i
     if (vec && hf && dtype == ILM_DTYPE_BF16 && parts >= 4 && parts <= NORM_WIDE_PARTS && rows <= 2 * ilm_num_cus() &&
         H <= 4 * NORM_WIDE_THREADS && (H + 31) / 32 * 32 <= 4 * NORM_WIDE_THREADS) {
         const int threads = (((H + 31) / 32 * 32 / 4) + 63) / 64 * 64;   // four columns a thread, whole waves
-#define NORM_WIDE(WT, PB) add_rmsnorm_wide_kernel<WT, PB><<<rows, threads, 0, stream>>>((bf16*)x, (float*)r, (const float*)h, (const WT*)w, H, alpha, eps, parts, (size_t)pstride, frag_mg)
+#define NORM_WIDE(WT, PB) add_rmsnorm_wide_kernel<WT, PB><<<rows, threads, 0, stream>>>((bf16*)x, (float*)r, (const float*)h, (const WT*)w, H, alpha, eps, parts, (size_t)pstride, frag_mg, w_offset)
         if (w_dtype == ILM_DTYPE_BF16) {
             if (parts <= 8) NORM_WIDE(bf16, 8); else NORM_WIDE(bf16, 16);
         } else if (w_dtype == ILM_DTYPE_F32) {
@@ -283,13 +283,13 @@ extern "C" int ilm_add_rmsnorm(void* x, void* r, const void* h, const void* w, i
 #define NORM_LAUNCH(T, WT, HT)                                                                                   \
     do {                                                                                                         \
         if (vec && niter <= 1)                                                                                   \
-            add_rmsnorm_vec_kernel<T, WT, HT, 1><<<rows, 256, 0, stream>>>((T*)x, (float*)r, (const HT*)h, (const WT*)w, H, alpha, eps, parts, (size_t)pstride, frag_mg); \
+            add_rmsnorm_vec_kernel<T, WT, HT, 1><<<rows, 256, 0, stream>>>((T*)x, (float*)r, (const HT*)h, (const WT*)w, H, alpha, eps, parts, (size_t)pstride, frag_mg, w_offset); \
         else if (vec && niter <= 2)                                                                              \
-            add_rmsnorm_vec_kernel<T, WT, HT, 2><<<rows, 256, 0, stream>>>((T*)x, (float*)r, (const HT*)h, (const WT*)w, H, alpha, eps, parts, (size_t)pstride, frag_mg); \
+            add_rmsnorm_vec_kernel<T, WT, HT, 2><<<rows, 256, 0, stream>>>((T*)x, (float*)r, (const HT*)h, (const WT*)w, H, alpha, eps, parts, (size_t)pstride, frag_mg, w_offset); \
         else if (vec)                                                                                            \
-            add_rmsnorm_vec_kernel<T, WT, HT, 4><<<rows, 256, 0, stream>>>((T*)x, (float*)r, (const HT*)h, (const WT*)w, H, alpha, eps, parts, (size_t)pstride, frag_mg); \
+            add_rmsnorm_vec_kernel<T, WT, HT, 4><<<rows, 256, 0, stream>>>((T*)x, (float*)r, (const HT*)h, (const WT*)w, H, alpha, eps, parts, (size_t)pstride, frag_mg, w_offset); \
         else                                                                                                     \
-            add_rmsnorm_kernel<T, WT, HT><<<rows, 256, 0, stream>>>((T*)x, (float*)r, (const HT*)h, (const WT*)w, H, alpha, eps, parts, (size_t)pstride, frag_mg); \
+            add_rmsnorm_kernel<T, WT, HT><<<rows, 256, 0, stream>>>((T*)x, (float*)r, (const HT*)h, (const WT*)w, H, alpha, eps, parts, (size_t)pstride, frag_mg, w_offset); \
     } while (0)
 #define NORM_CASE(T, WT)                     \
     do {                                     \
@@ -470,20 +470,20 @@ extern "C" int ilm_rope_kvwrite(void* qkv, const void* pos, const void* cosT, co
 // act[t, i] = silu(gu[t, i]) * gu[t, I + i]   (gate is the first half of the fused projection)
 // ------------------------------------------------------------------------------------------
 template <typename T>
-__global__ void swiglu_kernel(T* __restrict__ out, const T* __restrict__ gu, int I, int gu_stride) {
+__global__ void swiglu_kernel(T* __restrict__ out, const T* __restrict__ gu, int I, int gu_stride, int act) {
     const int t = blockIdx.y;
     const int i = blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= I) return;
     const float g = to_f32(gu[(size_t)t * gu_stride + i]);
     const float u = to_f32(gu[(size_t)t * gu_stride + I + i]);
-    out[(size_t)t * I + i] = from_f32<T>(g / (1.0f + expf(-g)) * u);
+    out[(size_t)t * I + i] = from_f32<T>(glu_act(g, act) * u);
 }
 
 // 8 elements a thread, 16-byte (bf16) or 32-byte (float) accesses; needs I and the row stride to be
 // multiples of 8 and 16-byte aligned rows
 template <typename T>
 __global__ void __launch_bounds__(256)
-swiglu_vec_kernel(T* __restrict__ out, const T* __restrict__ gu, int I, int gu_stride) {
+swiglu_vec_kernel(T* __restrict__ out, const T* __restrict__ gu, int I, int gu_stride, int act) {
     const int t = blockIdx.y;
     const int i = (blockIdx.x * 256 + threadIdx.x) * 8;
     if (i >= I) return;
@@ -501,7 +501,7 @@ swiglu_vec_kernel(T* __restrict__ out, const T* __restrict__ gu, int I, int gu_s
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
         const float gv = to_f32(g[e]);
-        o[e] = from_f32<T>(gv / (1.0f + expf(-gv)) * to_f32(u[e]));
+        o[e] = from_f32<T>(glu_act(gv, act) * to_f32(u[e]));
     }
     T* op = out + (size_t)t * I + i;
     if (sizeof(T) == 2) {
@@ -512,7 +512,7 @@ swiglu_vec_kernel(T* __restrict__ out, const T* __restrict__ gu, int I, int gu_s
     }
 }
 
-extern "C" int ilm_swiglu(void* out, const void* gu, int T_, int I, int gu_stride, int dtype,
+extern "C" int ilm_swiglu(void* out, const void* gu, int T_, int I, int gu_stride, int dtype, int act,
                           hipStream_t stream) {
     ILM_REQUIRE(T_ > 0 && I > 0 && gu_stride >= 2 * I, "swiglu: bad sizes T=%d I=%d stride=%d", T_, I, gu_stride);
     ILM_REQUIRE(T_ <= 65535, "swiglu: at most 65535 rows a call, got %d", T_);
@@ -520,13 +520,13 @@ extern "C" int ilm_swiglu(void* out, const void* gu, int T_, int I, int gu_strid
     dim3 grid((I + 255) / 256, T_);
     dim3 vgrid((I / 8 + 255) / 256, T_);
     if (dtype == ILM_DTYPE_F32 && vec)
-        swiglu_vec_kernel<float><<<vgrid, 256, 0, stream>>>((float*)out, (const float*)gu, I, gu_stride);
+        swiglu_vec_kernel<float><<<vgrid, 256, 0, stream>>>((float*)out, (const float*)gu, I, gu_stride, act);
     else if (dtype == ILM_DTYPE_BF16 && vec)
-        swiglu_vec_kernel<bf16><<<vgrid, 256, 0, stream>>>((bf16*)out, (const bf16*)gu, I, gu_stride);
+        swiglu_vec_kernel<bf16><<<vgrid, 256, 0, stream>>>((bf16*)out, (const bf16*)gu, I, gu_stride, act);
     else if (dtype == ILM_DTYPE_F32)
-        swiglu_kernel<float><<<grid, 256, 0, stream>>>((float*)out, (const float*)gu, I, gu_stride);
+        swiglu_kernel<float><<<grid, 256, 0, stream>>>((float*)out, (const float*)gu, I, gu_stride, act);
     else if (dtype == ILM_DTYPE_BF16)
-        swiglu_kernel<bf16><<<grid, 256, 0, stream>>>((bf16*)out, (const bf16*)gu, I, gu_stride);
+        swiglu_kernel<bf16><<<grid, 256, 0, stream>>>((bf16*)out, (const bf16*)gu, I, gu_stride, act);
     else
         ILM_REQUIRE(false, "swiglu: unknown dtype %d", dtype);
     ILM_LAUNCH_CHECK("swiglu");

@@ -259,7 +259,7 @@ template <int WAVES, int KSTEPS, int MG>
 __global__ void __launch_bounds__(WAVES * 64)
 gemm_gateup_swiglu_kernel(bf16* __restrict__ C, const bf16* __restrict__ X, const bf16* __restrict__ W,
                           const bf16* __restrict__ bias, int M, int I, int K, int lda, int ldw, int ldc, int ntiles,
-                          int ks, const float* __restrict__ SS, int ss_tiles, float eps) {
+                          int ks, const float* __restrict__ SS, int ss_tiles, float eps, int act) {
     // SS != null: X is r * w of a norm whose division is still to come (see SK_ROW_SCALE)
     static_assert(WAVES * 64 >= 128 * MG, "one reducing thread an output");
     __shared__ float part[2][MG][WAVES][64][4];
@@ -347,7 +347,7 @@ gemm_gateup_swiglu_kernel(bf16* __restrict__ C, const bf16* __restrict__ X, cons
             }
             vg = to_f32(from_f32<bf16>(vg));
             vu = to_f32(from_f32<bf16>(vu));
-            C[(size_t)m * ldc + n] = from_f32<bf16>(vg / (1.0f + expf(-vg)) * vu);
+            C[(size_t)m * ldc + n] = from_f32<bf16>(glu_act(vg, act) * vu);
         }
         buf ^= 1;  // the other buffer is free: its readers passed the barrier above one tile ago
     }
@@ -361,7 +361,7 @@ template <int WAVES, int KSTEPS, int MG>
 __global__ void __launch_bounds__(WAVES * 64)
 gemm_gateup_swiglu_pair_kernel(bf16* __restrict__ C, const bf16* __restrict__ X, const bf16* __restrict__ W,
                           const bf16* __restrict__ bias, int M, int I, int K, int lda, int ldw, int ldc, int ntiles,
-                          int ks, const float* __restrict__ SS, int ss_tiles, float eps) {
+                          int ks, const float* __restrict__ SS, int ss_tiles, float eps, int act) {
     static_assert(WAVES * 64 >= 256 * MG, "one reducing thread an output");
     __shared__ float part[2][MG][WAVES][64][4];
     __shared__ __attribute__((aligned(16))) float ssr[WAVES][32];
@@ -446,7 +446,7 @@ gemm_gateup_swiglu_pair_kernel(bf16* __restrict__ C, const bf16* __restrict__ X,
             val[hf] = to_f32(from_f32<bf16>(v));
             buf ^= 1;  // the other buffer is free: its readers passed the barrier above one tile ago
         }
-        if (writer) C[(size_t)m * ldc + n] = from_f32<bf16>(val[0] / (1.0f + expf(-val[0])) * val[1]);
+        if (writer) C[(size_t)m * ldc + n] = from_f32<bf16>(glu_act(val[0], act) * val[1]);
     }
 }
 
@@ -538,12 +538,13 @@ extern "C" int ilm_gemm_skinny(void* C, const void* X, const void* W, const void
     return 0;
 }
 
-// act [M, ldc] = silu(X Wg^T + bg) * (X Wu^T + bu) with W = [Wg; Wu] of 2 I rows (bias of 2 I entries or null).
+// out [M, ldc] = f(X Wg^T + bg) * (X Wu^T + bu) with W = [Wg; Wu] of 2 I rows (bias of 2 I entries or null) and f the gate's
+// activation `act` (glu_act in common.h: silu, or the tanh form of gelu).
 // ss != null: X is r * w of the RMS norm before the projection, not yet divided by the rows' root mean square, and
 // ss [ss_tiles][32] holds partial sums of squares of the rows of r (what ilm_gemm_tail leaves): the kernel adds them
 // up and applies 1 / sqrt(sum / K + eps) to its sums (K is also the norm's width).
 extern "C" int ilm_gemm_gateup_swiglu(void* C, int ldc, const void* X, int lda, const void* W, int ldw, const void* bias,
-                                      int M, int I, int K, const void* ss, int ss_tiles, float eps, hipStream_t stream) {
+                                      int M, int I, int K, const void* ss, int ss_tiles, float eps, int act, hipStream_t stream) {
     ILM_REQUIRE(ss == nullptr || ss_tiles > 0, "gemm_gateup_swiglu: no tiles of partial sums");
     ILM_REQUIRE(M > 0 && M <= 32 && I > 0 && K > 0, "gemm_gateup_swiglu: needs 1 <= M <= 32, got M=%d I=%d K=%d", M, I, K);
     ILM_REQUIRE(K % 8 == 0 && lda % 8 == 0 && ldw % 8 == 0 && lda >= K && ldw >= K && ldc >= I,
@@ -559,7 +560,7 @@ extern "C" int ilm_gemm_gateup_swiglu(void* C, int ldc, const void* X, int lda, 
         const int grid = ntiles < ilm_num_cus() * PER_CU ? ntiles : ilm_num_cus() * PER_CU;                         \
         KERNEL<WV, KS, MGR><<<grid, WV * 64, 0, stream>>>(                                                  \
             (bf16*)C, (const bf16*)X, (const bf16*)W, (const bf16*)bias, M, I, K, lda, ldw, ldc, ntiles,    \
-            (ksteps + WV - 1) / WV, (const float*)ss, ss_tiles, eps);                                       \
+            (ksteps + WV - 1) / WV, (const float*)ss, ss_tiles, eps, act);                                  \
     }
 #define GU_CASE(WV, KS, MGR, PER_CU)                                                       \
     {                                                                                      \

@@ -40,6 +40,7 @@ struct GtArgs {
     size_t part_stride;
     bf16* act;          // swiglu
     int ld_act;
+    int glu;            // swiglu: the gate's activation (glu_act in common.h)
 };
 
 __device__ __forceinline__ f32x4 gt_mfma(uint4 a, uint4 b, f32x4 c) {
@@ -226,7 +227,7 @@ gemm_tall_kernel(const GtArgs A) {
             for (int e = 0; e < 4; ++e) {
                 const float vg = to_f32(from_f32<bf16>(acc[g][e] + bg[e]));
                 const float vu = to_f32(from_f32<bf16>(up[e] + bu[e]));
-                o[e] = from_f32<bf16>(vg / (1.0f + expf(-vg)) * vu);
+                o[e] = from_f32<bf16>(glu_act(vg, A.glu) * vu);
             }
             bf16* dst = A.act + (size_t)m * A.ld_act + n;
             if (n + 3 < I && (A.ld_act & 3) == 0 && ((uintptr_t)A.act & 7) == 0) {
@@ -294,17 +295,17 @@ extern "C" int ilm_gemm_tall(void* C, int ldc, long c_part_stride, int kb, int c
     return 0;
 }
 
-// act [M, ld_act] = silu(X Wg^T + bg) * (X Wu^T + bu) with W = [Wg; Wu] of 2 I rows (bias of 2 I entries or null); kc: k a
+// act [M, ld_act] = f(X Wg^T + bg) * (X Wu^T + bu), f the gate's activation `glu`, with W = [Wg; Wu] of 2 I rows (bias of 2 I entries or null); kc: k a
 // chunk (64 or 128).  frag_w != 0: W is the weight in fragment order with tiles of 8 gate + 8 up rows (ldw is not used).
 extern "C" int ilm_gemm_tall_swiglu(void* act, int ld_act, const void* X, int lda, const void* W, int ldw, const void* bias,
-                                    int M, int I, int K, int kc, int frag_w, hipStream_t stream) {
+                                    int M, int I, int K, int kc, int frag_w, int glu, hipStream_t stream) {
     if (gt_check("gemm_tall_swiglu", M, I, K, kc, X, lda, W, ldw, frag_w)) return -1;
     ILM_REQUIRE(ld_act >= I, "gemm_tall_swiglu: ld_act=%d", ld_act);
     GtArgs a = {};
     a.X = (const bf16*)X; a.W = (const bf16*)W; a.bias = (const bf16*)bias; a.M = M; a.N = I; a.K = K; a.lda = lda; a.ldw = ldw;
     a.chunks = (K + kc - 1) / kc;
     a.chunks_per_part = a.chunks;
-    a.act = (bf16*)act; a.ld_act = ld_act;
+    a.act = (bf16*)act; a.ld_act = ld_act; a.glu = glu;
     gt_launch<GT_SWIGLU>(a, kc, dim3((I + GT_NT / 2 - 1) / (GT_NT / 2), 1), frag_w, stream);
     ILM_LAUNCH_CHECK("gemm_tall_swiglu");
     return 0;

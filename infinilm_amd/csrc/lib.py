@@ -20,17 +20,17 @@ _L = c_long
 
 _SIGNATURES = {
     "ilm_embed": [_P, _P, _P, _I, _I, _I, _F, _I, _P],
-    "ilm_add_rmsnorm": [_P, _P, _P, _P, _I, _I, _F, _F, _I, _I, _I, _I, _L, _I, _P],
+    "ilm_add_rmsnorm": [_P, _P, _P, _P, _I, _I, _F, _F, _I, _I, _I, _I, _L, _I, _F, _P],
     "ilm_gemm_ksplit": [_P, _I, _I, _L, _I, _P, _I, _P, _F, _I, _I, _I, _P, _I, _I, _P],
     "ilm_rope_kvwrite": [_P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P],
-    "ilm_swiglu": [_P, _P, _I, _I, _I, _I, _P],
+    "ilm_swiglu": [_P, _P, _I, _I, _I, _I, _I, _P],
     "ilm_gather_rows": [_P, _P, _P, _I, _I, _I, _P],
     "ilm_scale_rows": [_P, _I, _I, _I, _F, _P],
-    "ilm_gemm_gateup_swiglu": [_P, _I, _P, _I, _P, _I, _P, _I, _I, _I, _P, _I, _F, _P],
+    "ilm_gemm_gateup_swiglu": [_P, _I, _P, _I, _P, _I, _P, _I, _I, _I, _P, _I, _F, _I, _P],
     "ilm_gemm_tail": [_P, _I, _P, _I, _P, _P, _I, _P, _I, _P, _P, _I, _F, _I, _I, _I, _P],
     "ilm_gemm_rows64": [_P, _I, _L, _I, _P, _I, _I, _I, _I, _P, _I, _I, _P],
     "ilm_gemm_tall": [_P, _I, _L, _I, _I, _I, _P, _I, _I, _I, _I, _P, _I, _I, _P],
-    "ilm_gemm_tall_swiglu": [_P, _I, _P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _P],
+    "ilm_gemm_tall_swiglu": [_P, _I, _P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P],
     "ilm_gemm_qkv_rope": [_P, _I, _P, _I, _P, _I, _P, _I, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _P],
     "ilm_frag_pack_weight": [_P, _P, _P, _I, _I, _I, _I, _P],
     "ilm_frag_pack_rows": [_P, _P, _I, _I, _I, _P],
@@ -45,9 +45,9 @@ _SIGNATURES = {
     "ilm_gemm_basic": [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P],
     "ilm_attn_basic": [_P, _P, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _F, _P],
     "ilm_gemm_skinny": [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P],
-    "ilm_attn_mfma": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _F, _P],
+    "ilm_attn_mfma": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _F, _I, _P],
     "ilm_attn_mfma_static": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P],
-    "ilm_attn_tile": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _F, _P],
+    "ilm_attn_tile": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _F, _I, _P],
     "ilm_argmax": [_P, _P, _I, _I, _I, _P],
     "ilm_sample": [_P, _P, _P, _P, _P, _P, _I, _I, _I, _P],
     "ilm_unary": [_P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
@@ -77,11 +77,16 @@ _SIGNATURES = {
     "ilm_glu_clamp": [_P, _P, _I, _I, _I, _F, _F, _I, _P],
     "ilm_head_gemm": [_P, _P, _P, _I, _I, _I, _I, _L, _L, _L, _L, _L, _L, _L, _I, _I, _P],
     "ilm_head_gemm_mfma": [_P, _P, _P, _I, _I, _I, _I, _L, _L, _L, _L, _L, _L, _L, _P],
-    "ilm_group_norm_gate": [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _I, _I, _I, _I, _L, _P],
+    "ilm_group_norm_gate": [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _I, _I, _I, _I, _L, _F, _P],
     "ilm_causal_conv": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P],
     "ilm_ssm_steps": [_P, _P, _P, _P, _P, _I, _I, _I, _I, _P],
     "ilm_unit_qk_kvwrite": [_P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _F, _I, _I, _P],
     "ilm_weighted_sum": [_P, _P, _P, _L, _F, _F, _I, _I, _I, _P],
+    "ilm_hyper_update": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _F, _F, _F, _I, _I, _I, _I, _L, _I, _P],
+    "ilm_conv_delta_inputs": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _F, _F, _I, _I, _P],
+    "ilm_conv_norm_rope_kvwrite": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _F,
+                                   _I, _I, _I, _P],
+    "ilm_delta_step": [_P, _P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P, _P, _I, _F, _I, _I, _I, _I, _P],
     "ilm_norm_add_norm": [_P, _P, _P, _P, _P, _I, _I, _F, _F, _F, _I, _I, _I, _I, _I, _L, _P],
 }
 
@@ -122,6 +127,8 @@ def load(verbose: bool = True) -> ctypes.CDLL:
     lib.ilm_attn_headmix_mfma_ok.argtypes = [c_int, c_int, c_int, c_int]
     lib.ilm_attn_maps_mfma_ok.restype = c_int
     lib.ilm_attn_maps_mfma_ok.argtypes = [c_int, c_int, c_int, c_int, c_int, c_int]
+    lib.ilm_delta_step_norm_ok.restype = c_int
+    lib.ilm_delta_step_norm_ok.argtypes = [c_int, c_int]
     lib.ilm_attn_static_init.restype = c_int
     lib.ilm_attn_static_init.argtypes = []
     lib.ilm_attn_static_scratch_floats.restype = c_long

@@ -667,7 +667,7 @@ extern "C" int ilm_decay_scan(void* o, int o_stride, const void* q, const void* 
 // ------------------------------------------------------------------------------------------
 // RMS norm in groups with an optional gate, one wave (groups up to 512 elements) or one block a (row, group):
 //   y = x * act(gate)            (gate_before)
-//   y = y / sqrt(mean_group(y^2) + eps) * w       (w may be absent)
+//   y = y / sqrt(mean_group(y^2) + eps) * (w + w_offset)       (w may be absent)
 //   y = y * act(gate)            (otherwise)
 // Sums run over a group in an order that depends on its size only.
 // ------------------------------------------------------------------------------------------
@@ -676,7 +676,7 @@ __global__ void __launch_bounds__(256)
 group_norm_gate_kernel(void* __restrict__ out, const void* __restrict__ x, const void* __restrict__ gate,
                        const void* __restrict__ w, int rows, int n, int groups, int x_stride, int gate_stride,
                        int out_stride, float eps, int gate_act, int gate_before, int out_dt, int x_dt, int gate_dt, int w_dt,
-                       int parts, size_t pstride) {
+                       int parts, size_t pstride, float w_offset) {
     __shared__ float red[4];
     const int item = LANES == 64 ? blockIdx.x * 4 + (threadIdx.x >> 6) : blockIdx.x;
     const int lane = LANES == 64 ? (threadIdx.x & 63) : threadIdx.x;
@@ -699,7 +699,7 @@ group_norm_gate_kernel(void* __restrict__ out, const void* __restrict__ x, const
         for (int p = 1; p < parts; ++p) y += ldf(x, x_dt, p * pstride + xb + j);
         if (pre) y *= act_f(ldf(gate, gate_dt, gb + j), gate_act);
         y *= rstd;
-        if (w != nullptr) y *= ldf(w, w_dt, (size_t)g * gs + j);
+        if (w != nullptr) y *= ldf(w, w_dt, (size_t)g * gs + j) + w_offset;
         if (gate != nullptr && !gate_before) y *= act_f(ldf(gate, gate_dt, gb + j), gate_act);
         stf(out, out_dt, ob + j, y);
     }
@@ -712,7 +712,7 @@ __global__ void __launch_bounds__(256)
 group_norm_gate_vec_kernel(void* __restrict__ out, const void* __restrict__ x, const void* __restrict__ gate,
                            const void* __restrict__ w, int rows, int n, int groups, int x_stride, int gate_stride,
                            int out_stride, float eps, int gate_act, int gate_before, int out_dt, int x_dt, int gate_dt, int w_dt,
-                           int parts, size_t pstride) {
+                           int parts, size_t pstride, float w_offset) {
     __shared__ float red[4];
     const int item = LANES == 64 ? blockIdx.x * 4 + (threadIdx.x >> 6) : blockIdx.x;
     const int lane = LANES == 64 ? (threadIdx.x & 63) : threadIdx.x;
@@ -757,7 +757,7 @@ group_norm_gate_vec_kernel(void* __restrict__ out, const void* __restrict__ x, c
                 float wt[8];
                 ld8(w, w_dt, (size_t)g * gs + j, wt);
 #pragma unroll
-                for (int e = 0; e < 8; ++e) o8[e] *= wt[e];
+                for (int e = 0; e < 8; ++e) o8[e] *= wt[e] + w_offset;
             }
             if (gate != nullptr && !gate_before) {
                 float gt[8];
@@ -772,7 +772,8 @@ group_norm_gate_vec_kernel(void* __restrict__ out, const void* __restrict__ x, c
 
 extern "C" int ilm_group_norm_gate(void* out, const void* x, const void* gate, const void* w, int rows, int n, int groups,
                                    int x_stride, int gate_stride, int out_stride, float eps, int gate_act, int gate_before,
-                                   int out_dt, int x_dt, int gate_dt, int w_dt, int parts, long pstride, hipStream_t stream) {
+                                   int out_dt, int x_dt, int gate_dt, int w_dt, int parts, long pstride, float w_offset,
+                                   hipStream_t stream) {
     ILM_REQUIRE(parts >= 1, "group_norm_gate: %d parts", parts);
     ILM_REQUIRE(rows > 0 && n > 0 && groups > 0 && n % groups == 0, "group_norm_gate: %d elements do not divide into %d groups", n, groups);
     ILM_REQUIRE((long)rows * groups < (1L << 31) - 4, "group_norm_gate: too many rows");
@@ -781,7 +782,7 @@ extern "C" int ilm_group_norm_gate(void* out, const void* x, const void* gate, c
                     && (((uintptr_t)out | (uintptr_t)x | (uintptr_t)gate | (uintptr_t)w) & 15) == 0;
     if (al && gs_ <= 8192) {
 #define GN_ARGS out, x, gate, w, rows, n, groups, x_stride, gate_stride, out_stride, eps, gate_act, gate_before, out_dt, x_dt, gate_dt, \
-                w_dt, parts, (size_t)pstride
+                w_dt, parts, (size_t)pstride, w_offset
         if (gs_ <= 512) group_norm_gate_vec_kernel<64, 1><<<(rows * groups + 3) / 4, 256, 0, stream>>>(GN_ARGS);
         else if (gs_ <= 2048) group_norm_gate_vec_kernel<256, 1><<<rows * groups, 256, 0, stream>>>(GN_ARGS);
         else if (gs_ <= 4096) group_norm_gate_vec_kernel<256, 2><<<rows * groups, 256, 0, stream>>>(GN_ARGS);
@@ -792,11 +793,11 @@ extern "C" int ilm_group_norm_gate(void* out, const void* x, const void* gate, c
     }
     if (n / groups > 512) {
         group_norm_gate_kernel<256><<<rows * groups, 256, 0, stream>>>(out, x, gate, w, rows, n, groups, x_stride, gate_stride,
-                                                                       out_stride, eps, gate_act, gate_before, out_dt, x_dt, gate_dt, w_dt, parts, (size_t)pstride);
+                                                                       out_stride, eps, gate_act, gate_before, out_dt, x_dt, gate_dt, w_dt, parts, (size_t)pstride, w_offset);
     } else {
         const int blocks = (int)(((long)rows * groups + 3) / 4);
         group_norm_gate_kernel<64><<<blocks, 256, 0, stream>>>(out, x, gate, w, rows, n, groups, x_stride, gate_stride, out_stride,
-                                                               eps, gate_act, gate_before, out_dt, x_dt, gate_dt, w_dt, parts, (size_t)pstride);
+                                                               eps, gate_act, gate_before, out_dt, x_dt, gate_dt, w_dt, parts, (size_t)pstride, w_offset);
     }
     ILM_LAUNCH_CHECK("group_norm_gate");
     return 0;

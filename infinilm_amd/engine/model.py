@@ -13,10 +13,9 @@ from typing import Dict, List
 
 import torch
 
-from .. import kernels
 from ..cache.manager import Lent
 from ..config.spec import ModelSpec, PartSpec
-from ..parts import BuildContext, Param, ResidualStream, build_block
+from ..parts import BuildContext, HyperStreams, Param, ResidualStream, build_block
 from ..parts.base import join_name
 from ..parts.registry import build_embedding, build_head, build_norm
 
@@ -118,10 +117,11 @@ class CausalLM:
 
     def forward(self, batch, cache) -> torch.Tensor:
         """float32 logits [len(batch.want_rows), vocab] for the tokens of `batch`."""
-        stream = ResidualStream(self._embed(batch))
+        embedded = self._embed(batch)
+        stream = HyperStreams(embedded, self.spec.streams) if self.spec.streams else ResidualStream(embedded)
         taps = batch.taps
         if taps is not None:
-            taps["embed"] = stream.residual.clone()
+            taps["embed"] = embedded.clone()
         # the embedding's output once more for the runs that add it again (the stream itself is summed into in place)
         first = self._embed(batch) if self._keeps_embedding else None
         for i, run in enumerate(self.spec.order):
@@ -135,23 +135,10 @@ class CausalLM:
                 view = Lent(view, cache.view(run.borrows, batch, False))
             self.blocks[run.layer].forward(stream, batch, view)
             if taps is not None:
-                stream.settle()
-                taps[f"run{i}"] = (stream.residual.clone(), None if stream.pending is None else stream.pending.clone(),
-                                   stream.pending_scale)
+                taps[f"run{i}"] = stream.snapshot()
         if batch.num_wanted == 0:
             return torch.empty((0, self.spec.vocab_size), dtype=torch.float32, device=self.device)
-        if stream.more or stream.pending_gate is not None:
-            stream.settle()
         if not batch.wants_all_rows:
-            last = ResidualStream(kernels.gather_rows(stream.residual, batch.want_rows))
-            if stream.pending is not None:
-                pend = stream.pending
-                if pend.dim() == 3:   # parts of a K-split product: the rows of every part
-                    pend = torch.stack([kernels.gather_rows(p, batch.want_rows) for p in pend])
-                else:
-                    pend = kernels.gather_rows(pend, batch.want_rows)
-                last.push(pend, stream.pending_scale)
-                last.pending_norm = stream.pending_norm     # a norm still due to the branch works row by row
-            stream = last
+            stream = stream.gather(batch.want_rows)
         x = self.final_norm.forward(stream)
         return self.output_head.forward(x)

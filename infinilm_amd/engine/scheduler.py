@@ -113,11 +113,11 @@ class Scheduler:
 
     def _group_pages(self, group, n_tokens: int) -> int:
         """Pages of `group` that a request of `n_tokens` tokens holds at most at any time.  A group that keeps a
-        window gives pages back as the window passes them: a request never holds more than the window, the
-        longest portion of a step, and the page in which the window's edge lies."""
+        window (or a chunk of positions) gives pages back as the window passes them: a request never holds more than the
+        window, the longest portion of a step, and the page in which the window's edge lies."""
         pages = self._pages_for(n_tokens)
-        if group.window > 0:
-            pages = min(pages, self._pages_for(group.window + min(self.chunk_size, self.max_num_batched_tokens)) + 1
+        if group.span > 0:
+            pages = min(pages, self._pages_for(group.span + min(self.chunk_size, self.max_num_batched_tokens)) + 1
                         + self._pages_for(getattr(group, "keep_first", 0)))
         return pages
 

@@ -157,8 +157,8 @@ def embed(ids: torch.Tensor, table: torch.Tensor, scale: float) -> torch.Tensor:
 
 
 def add_rmsnorm(residual: torch.Tensor, branch: Optional[torch.Tensor], weight: torch.Tensor,
-                alpha: float, eps: float, out_dtype: torch.dtype, frag: bool = False):
-    """residual += alpha * branch (in place, float32), then its RMS norm times weight, as out_dtype.
+                alpha: float, eps: float, out_dtype: torch.dtype, frag: bool = False, weight_offset: float = 0.0):
+    """residual += alpha * branch (in place, float32), then its RMS norm times (weight + weight_offset), as out_dtype.
     `frag`: the result comes in fragment order (`FragRows`; bfloat16, at most 64 rows of a multiple of 8 elements),
     for a product that takes it so.
 
@@ -183,11 +183,11 @@ def add_rmsnorm(residual: torch.Tensor, branch: Optional[torch.Tensor], weight: 
             raise KernelError("a norm's result in fragment order is bfloat16, at most 64 rows of a multiple of 8 elements")
         out = frag_rows_empty(rows, H, residual.device)
         _run("ilm_add_rmsnorm", out.data.data_ptr(), residual.data_ptr(), _ptr(branch), weight.data_ptr(), rows, H,
-             float(alpha), float(eps), _DT[out_dtype], _dt(weight), h_dt, parts, pstride, -(-rows // 16), _stream())
+             float(alpha), float(eps), _DT[out_dtype], _dt(weight), h_dt, parts, pstride, -(-rows // 16), float(weight_offset), _stream())
         return out
     out = torch.empty((rows, H), dtype=out_dtype, device=residual.device)
     _run("ilm_add_rmsnorm", out.data_ptr(), residual.data_ptr(), _ptr(branch), weight.data_ptr(), rows, H,
-         float(alpha), float(eps), _DT[out_dtype], _dt(weight), h_dt, parts, pstride, 0, _stream())
+         float(alpha), float(eps), _DT[out_dtype], _dt(weight), h_dt, parts, pstride, 0, float(weight_offset), _stream())
     return out
 
 
@@ -250,14 +250,24 @@ def qkv_rope_gemm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor]
     return q
 
 
-def swiglu(gate_up: torch.Tensor) -> torch.Tensor:
-    """silu(gate) * up from rows [gate | up]."""
+GLU_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}    # activations of a gated feed-forward's gate (glu_act in common.h)
+
+
+def glu_code(kind: str) -> int:
+    try:
+        return GLU_ACTIVATIONS[kind]
+    except KeyError:
+        raise KernelError(f"unknown gate activation {kind!r}; known: {sorted(GLU_ACTIVATIONS)}") from None
+
+
+def swiglu(gate_up: torch.Tensor, act: str = "silu") -> torch.Tensor:
+    """act(gate) * up from rows [gate | up]; `act` "silu" or "gelu_tanh" (the tanh form of gelu)."""
     _dev(gate_up)
     T, two_i = gate_up.shape
     if two_i % 2 or gate_up.stride(1) != 1:
         raise KernelError("swiglu takes dense rows of even length")
     out = torch.empty((T, two_i // 2), dtype=gate_up.dtype, device=gate_up.device)
-    _run("ilm_swiglu", out.data_ptr(), gate_up.data_ptr(), T, two_i // 2, gate_up.stride(0), _dt(gate_up), _stream())
+    _run("ilm_swiglu", out.data_ptr(), gate_up.data_ptr(), T, two_i // 2, gate_up.stride(0), _dt(gate_up), glu_code(act), _stream())
     return out
 
 
@@ -464,18 +474,19 @@ def _gemm_tall(x: torch.Tensor, w: torch.Tensor, K: int, frag_w=None, plan: Opti
     return parts
 
 
-def gemm_tall_swiglu(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], frag_w=None, kc: int = 128) -> torch.Tensor:
-    """silu(x Wg^T + bg) * (x Wu^T + bu) for 17 to 208 rows, W = [Wg; Wu] (see gemm_tall.hip)."""
+def gemm_tall_swiglu(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], frag_w=None, kc: int = 128,
+                     act_kind: str = "silu") -> torch.Tensor:
+    """act(x Wg^T + bg) * (x Wu^T + bu) for 17 to 208 rows, W = [Wg; Wu] (see gemm_tall.hip)."""
     M, K = x.shape
     inter = w.shape[0] // 2
     act = torch.empty((M, inter), dtype=x.dtype, device=x.device)
     fw = _frag_of(frag_w) if USE_FRAG else None
     if fw is not None:
         _run("ilm_gemm_tall_swiglu", act.data_ptr(), act.stride(0), x.data_ptr(), x.stride(0), fw.data.data_ptr(), 0, _ptr(bias),
-             M, inter, K, kc, 1, _stream())
+             M, inter, K, kc, 1, glu_code(act_kind), _stream())
     else:
         _run("ilm_gemm_tall_swiglu", act.data_ptr(), act.stride(0), x.data_ptr(), x.stride(0), w.data_ptr(), w.stride(0),
-             _ptr(bias), M, inter, K, kc, 0, _stream())
+             _ptr(bias), M, inter, K, kc, 0, glu_code(act_kind), _stream())
     return act
 
 
@@ -534,8 +545,9 @@ def gateup_resident_ok(rows: int, w: torch.Tensor) -> bool:
 
 
 def gateup_swiglu_gemm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor],
-                       row_ss: Optional[torch.Tensor] = None, eps: float = 0.0, frag_w=None) -> Optional[torch.Tensor]:
-    """silu(x Wg^T + bg) * (x Wu^T + bu) for few rows in bfloat16, W = [Wg; Wu]: the fused gate/up
+                       row_ss: Optional[torch.Tensor] = None, eps: float = 0.0, frag_w=None,
+                       act: str = "silu") -> Optional[torch.Tensor]:
+    """act(x Wg^T + bg) * (x Wu^T + bu) for few rows in bfloat16, W = [Wg; Wu]: the fused gate/up
     projection with the SwiGLU in its epilogue, [M, I] (up to 32 rows with X in registers; 17 to 208 with chunks
     of X in LDS where the outputs fill the chip).  None where no kernel applies (more rows, few outputs,
     float32): the caller then runs the projection and the activation.  `row_ss`: x is what `gemm_tail` left (residual * norm weight) and row_ss its
@@ -568,10 +580,10 @@ def gateup_swiglu_gemm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Te
     if bias is not None and (bias.shape != (2 * I,) or bias.dtype != BF16 or not bias.is_contiguous()):
         raise KernelError("bias does not fit the fused gate/up projection")
     if tall:
-        return gemm_tall_swiglu(x, w, bias, frag_w)
+        return gemm_tall_swiglu(x, w, bias, frag_w, act_kind=act)
     out = torch.empty((M, I), dtype=BF16, device=x.device)
     _run("ilm_gemm_gateup_swiglu", out.data_ptr(), out.stride(0), x.data_ptr(), x.stride(0), w.data_ptr(), w.stride(0),
-         _ptr(bias), M, I, K, _ptr(row_ss), 0 if row_ss is None else row_ss.shape[0], float(eps), _stream())
+         _ptr(bias), M, I, K, _ptr(row_ss), 0 if row_ss is None else row_ss.shape[0], float(eps), glu_code(act), _stream())
     return out
 
 
@@ -678,11 +690,13 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                     seg_of_token: torch.Tensor, positions: torch.Tensor, nh: int, nkv: int, d: int,
                     scale: float, window: int = 0, max_total_len: Optional[int] = None,
                     tiles: Optional[torch.Tensor] = None, single_rows: Optional[torch.Tensor] = None,
-                    softcap: float = 0.0, float_weights: bool = False) -> torch.Tensor:
+                    softcap: float = 0.0, float_weights: bool = False, chunk: int = 0) -> torch.Tensor:
     """Attention of every token over its request's cached keys up to its own position.
     `softcap` > 0: scaled scores pass through softcap * tanh(score / softcap) before the softmax.
-    `float_weights`: the softmax weights stay float32 in the second product (the bfloat16 matrix-core kernels round them:
-    they are passed over, the plain kernel runs).
+    `window` > 0: its last `window` positions alone; `chunk` > 0: the positions of its own chunk alone (chunks of that many
+    positions, counted from the sequence's start).
+    `float_weights`: the softmax weights stay float32 up to the second product (the bfloat16 matrix-core kernels otherwise round
+    them; with it a weight enters their second product as two bfloat16 terms, the rounded weight and the rest).
 
     q: rows of T tokens in which head h lies at [h*d, (h+1)*d) (a view into the fused projection is
     fine); caches as the cache manager lays them out; block_tables [R, max_blocks]; `max_total_len`: an
@@ -694,6 +708,9 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     _i32(block_tables, "block_tables")
     _i32(seg_of_token, "seg_of_token")
     _i32(positions, "positions")
+    if window < 0 or chunk < 0 or (window > 0 and chunk > 0):
+        raise KernelError(f"a window ({window}) or a chunk ({chunk}), not both")
+    reach = -int(chunk) if chunk else int(window)     # (first_key in common.h)
     T = q.shape[0]
     if q.stride(1) != 1 or q.shape[1] < nh * d:
         raise KernelError("q rows must be dense and hold all query heads")
@@ -703,7 +720,7 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     if seg_of_token.numel() != T or positions.numel() != T or block_tables.dim() != 2:
         raise KernelError("per-token metadata does not match the number of tokens")
     out = torch.empty((T, nh * d), dtype=q.dtype, device=q.device)
-    if (q.dtype == BF16 and not FORCE_BASIC and not float_weights and d % 16 == 0 and d <= 128 and page % 16 == 0
+    if (q.dtype == BF16 and not FORCE_BASIC and d % 16 == 0 and d <= 128 and page % 16 == 0
             and q.stride(0) % 8 == 0 and max_total_len is not None):
         n_single = T
         rows = None
@@ -713,7 +730,7 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
             _run("ilm_attn_tile", out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
                  block_tables.data_ptr(), seg_of_token.data_ptr(), positions.data_ptr(), tiles.data_ptr(),
                  tiles.numel() // 2, nh, nkv, d, page, block_tables.shape[1], q.stride(0), out.stride(0), float(scale),
-                 int(window), float(softcap), _stream())
+                 reach, float(softcap), int(float_weights), _stream())
             if single_rows is None or single_rows.numel() == 0:
                 return out
             _i32(single_rows, "single_rows")
@@ -727,8 +744,8 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
             ws_ml = torch.empty((n_single * nh * nsplit * 2,), dtype=F32, device=q.device)
         _run("ilm_attn_mfma", out.data_ptr(), _ptr(ws_acc), _ptr(ws_ml), q.data_ptr(), k_cache.data_ptr(),
              v_cache.data_ptr(), block_tables.data_ptr(), seg_of_token.data_ptr(), positions.data_ptr(), _ptr(rows),
-             n_single, nh, nkv, d, page, block_tables.shape[1], q.stride(0), out.stride(0), float(scale), int(window),
-             nsplit, span, float(softcap), _stream())
+             n_single, nh, nkv, d, page, block_tables.shape[1], q.stride(0), out.stride(0), float(scale), reach,
+             nsplit, span, float(softcap), int(float_weights), _stream())
         return out
     bound = block_tables.shape[1] * page if max_total_len is None else min(int(max_total_len), block_tables.shape[1] * page)
     if (q.dtype == F32 and not FORCE_BASIC and d % 16 == 0 and d <= 256 and page % 4 == 0 and q.stride(0) % 4 == 0
@@ -742,7 +759,7 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
             ws = torch.empty((T * nh * nchunks * (d + 4),), dtype=F32, device=q.device)
         _run("ilm_attn_f32", out.data_ptr(), _ptr(ws), nchunks, q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
              block_tables.data_ptr(), seg_of_token.data_ptr(), positions.data_ptr(), T, nh, nkv, d, page,
-             block_tables.shape[1], q.stride(0), out.stride(0), float(scale), int(window), float(softcap), _stream())
+             block_tables.shape[1], q.stride(0), out.stride(0), float(scale), reach, float(softcap), _stream())
         return out
     # The plain kernel.  Few tokens over long contexts (decoding): one wave a chunk of keys and a fold of the
     # partial results, instead of one wave a head; the bits are the same (see attn_basic.hip).
@@ -752,7 +769,7 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
         ws = torch.empty((T * nh * nchunks * (d + 2),), dtype=F32, device=q.device)
     _run("ilm_attn_basic", out.data_ptr(), _ptr(ws), nchunks, q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
          block_tables.data_ptr(), seg_of_token.data_ptr(), positions.data_ptr(), T, nh, nkv, d, page, block_tables.shape[1],
-         q.stride(0), out.stride(0), float(scale), int(window), _dt(q), float(softcap), _stream())
+         q.stride(0), out.stride(0), float(scale), reach, _dt(q), float(softcap), _stream())
     return out
 
 
@@ -1146,9 +1163,9 @@ def sigmoid_root(z: torch.Tensor, tau: float, bias: Optional[torch.Tensor] = Non
 
 def group_norm_gate(x: torch.Tensor, weight: Optional[torch.Tensor], eps: float, groups: int = 1,
                     gate: Optional[torch.Tensor] = None, gate_act: str = "none", gate_before: bool = False,
-                    out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
+                    out_dtype: Optional[torch.dtype] = None, weight_offset: float = 0.0) -> torch.Tensor:
     """RMS norm of every row in `groups` equal parts (each by its own root mean square, eps inside the root), times
-    `weight` [n] if given; `gate` [T, n]: times act(gate), before the norm or after it.  Sums in float32.
+    `weight` [n] (+ `weight_offset`) if given; `gate` [T, n]: times act(gate), before the norm or after it.  Sums in float32.
     x may come as contiguous parts [P, T, n] that are summed first (a product that was split over K)."""
     _dev(x, weight, gate)
     parts, pstride = 1, 0
@@ -1170,7 +1187,7 @@ def group_norm_gate(x: torch.Tensor, weight: Optional[torch.Tensor], eps: float,
     _run("ilm_group_norm_gate", out.data_ptr(), x.data_ptr(), _ptr(gate), _ptr(weight), T, n, int(groups), x.stride(0),
          gate.stride(0) if gate is not None else 0, out.stride(0), float(eps), activation_code(gate_act), int(bool(gate_before)),
          _dt(out), _dt(x), _dt(gate) if gate is not None else 0, _dt(weight) if weight is not None else 0, parts, pstride,
-         _stream())
+         float(weight_offset), _stream())
     return out
 
 
@@ -1945,3 +1962,175 @@ def glu_clamp(gate_up: torch.Tensor, limit: float, alpha: float = 1.702) -> torc
     out = torch.empty((T, n // 2), dtype=gate_up.dtype, device=gate_up.device)
     _run("ilm_glu_clamp", out.data_ptr(), gate_up.data_ptr(), T, n // 2, gate_up.stride(0), float(limit), float(alpha), _dt(gate_up), _stream())
     return out
+
+
+# ---- a residual stream in several copies ("hyper-connections") ------------------------------------------------------------
+HYPER_MAX_STREAMS = 16       # (ilm_hyper_max_streams())
+HYPER_MAX_WIDTH = 16384      # (ilm_hyper_max_width())
+
+
+def hyper_update(streams: Optional[torch.Tensor], count: int, base: Optional[torch.Tensor] = None, branch: Optional[torch.Tensor] = None,
+                 alpha: float = 1.0, mix: Optional[torch.Tensor] = None, out_weights: Optional[torch.Tensor] = None,
+                 in_weights: Optional[torch.Tensor] = None, weight: Optional[torch.Tensor] = None, weight_offset: float = 0.0,
+                 eps: float = 0.0, out_dtype: Optional[torch.dtype] = None, write: bool = True) -> Optional[torch.Tensor]:
+    """`streams` float32 [T, count, H], or `base` [T, H] that every stream equals.  With a `branch` ([T, H], or float32 parts
+    [P, T, H] summed in order) every stream becomes sum_s mix[s, t] x_s + out_weights[t] alpha branch, all from the old ones
+    (written to `streams` if `write`); then u = sum_t in_weights[t] x_t (None: the plain sum), and its RMS norm times
+    (weight + weight_offset) as `out_dtype`, or u itself without `weight`.  out_dtype None: no result."""
+    _dev(streams, base, branch, mix, out_weights, in_weights, weight)
+    src = base if base is not None else streams
+    T, H = src.shape[0], src.shape[-1]
+    if not 1 <= count <= HYPER_MAX_STREAMS or H > HYPER_MAX_WIDTH:
+        raise KernelError(f"{count} streams of {H}: at most {HYPER_MAX_STREAMS} of {HYPER_MAX_WIDTH}")
+    for t, shape, nm in ((streams, (T, count, H), "streams"), (base, (T, H), "the common row"), (mix, (count, count), "mix"),
+                         (out_weights, (count,), "out_weights"), (in_weights, (count,), "in_weights")):
+        if t is not None and (t.dtype != F32 or tuple(t.shape) != shape or not t.is_contiguous()):
+            raise KernelError(f"{nm} must be contiguous float32 {shape}, got {tuple(t.shape)} {t.dtype}")
+    parts, pstride, y_dt = 1, 0, 0
+    if branch is not None:
+        if mix is None or out_weights is None or (write and streams is None):
+            raise KernelError("a branch joins the streams through mix and out_weights")
+        if branch.dim() == 3:
+            parts, pstride = branch.shape[0], branch.stride(0)
+        if tuple(branch.shape[-2:]) != (T, H) or not branch.is_contiguous():
+            raise KernelError(f"branch {tuple(branch.shape)} does not match streams of {(T, H)}")
+        y_dt = _dt(branch)
+    if weight is not None and (weight.shape != (H,) or not weight.is_contiguous()):
+        raise KernelError(f"norm weight has shape {tuple(weight.shape)}, expected ({H},)")
+    x = torch.empty((T, H), dtype=out_dtype, device=src.device) if out_dtype is not None else None
+    _run("ilm_hyper_update", _ptr(x), _ptr(streams), _ptr(base), _ptr(branch), _ptr(mix), _ptr(out_weights), _ptr(in_weights),
+         _ptr(weight), T, count, H, float(alpha), float(weight_offset), float(eps), _DT[out_dtype] if x is not None else 0, y_dt,
+         _dt(weight) if weight is not None else 0, parts, pstride, int(branch is not None and write), _stream())
+    return x
+
+
+# ---- mixers with short convolutions: the convolution and what follows it, in one kernel ------------------------------------
+def _conv_operands(x, weight, pool, state_in, state_out, seg_of_token, seg_offsets, segments: int, channels: int) -> int:
+    """Checks what the fused convolution kernels share; returns the taps (0: no convolution)."""
+    _dev(x, weight, pool, state_in, state_out, seg_of_token, seg_offsets)
+    _rows(x, "x")
+    T = x.shape[0]
+    _i32(seg_of_token, "seg_of_token")
+    _i32(seg_offsets, "seg_offsets")
+    if seg_of_token.numel() != T or seg_offsets.numel() < segments + 1:
+        raise KernelError("segments do not cover the tokens")
+    if weight is None:
+        return 0
+    taps = weight.shape[0]
+    if weight.dim() != 2 or weight.shape[1] != channels or not weight.is_contiguous() or weight.dtype != x.dtype or not 1 <= taps <= CONV_MAX_TAPS:
+        raise KernelError(f"convolution weight {tuple(weight.shape)} must be [taps <= {CONV_MAX_TAPS}, {channels}] of the rows' dtype")
+    if taps > 1:
+        if pool is None or pool.dtype != F32 or not pool.is_contiguous() or tuple(pool.shape[1:]) != (taps - 1, channels):
+            raise KernelError(f"the convolution's state pool must be float32 [rows, {taps - 1}, {channels}]")
+        _i32(state_in, "state_in")
+        _i32(state_out, "state_out")
+        if state_in.numel() < segments or state_out.numel() < segments:
+            raise KernelError("state rows must cover every segment")
+    return taps
+
+
+def conv_delta_inputs(x: torch.Tensor, weight: Optional[torch.Tensor], pool: Optional[torch.Tensor], state_in, state_out,
+                      seg_of_token: torch.Tensor, seg_offsets: torch.Tensor, segments: int, heads: int, groups: int, dk: int, dv: int,
+                      b_off: int, a_off: int, a_log: torch.Tensor, dt_bias: torch.Tensor, q_scale: float, unit_eps: float,
+                      max_len: Optional[int] = None):
+    """From fused rows x [q: groups dk | k: groups dk | v: heads dv | ...]: the short convolution per channel (`weight`
+    [taps, channels] as taps of whole rows, None: none) with silu; q and k of unit length per head (unit_eps beside the sum of
+    squares), q times q_scale; beta = sigmoid(x[b_off + h]), log-decay = -exp(a_log) softplus(x[a_off + h] + dt_bias).
+    float32 results (rows [q | k | v] with q and k heads filled up to the next multiple of 16, gates [T, 2 heads]).  `max_len`: a
+    bound on the segments' lengths (1: decoded tokens alone)."""
+    C = groups * 2 * dk + heads * dv
+    taps = _conv_operands(x, weight, pool, state_in, state_out, seg_of_token, seg_offsets, segments, C)
+    _dev(a_log, dt_bias)
+    T = x.shape[0]
+    if heads <= 0 or groups <= 0 or heads % groups or x.shape[1] < max(C, b_off + heads, a_off + heads):
+        raise KernelError(f"rows of {x.shape[1]} do not hold {heads} heads in {groups} groups of {dk} / {dv} and their gates")
+    for t, nm in ((a_log, "a_log"), (dt_bias, "dt_bias")):
+        if t.dtype != F32 or t.shape != (heads,) or not t.is_contiguous():
+            raise KernelError(f"{nm} must be contiguous float32 [{heads}]")
+    dkp = -(-dk // 16) * 16
+    n = 2 * groups * dkp + heads * dv
+    rows = torch.empty((T, -(-n // 4) * 4), dtype=F32, device=x.device)
+    gates = torch.empty((T, 2 * heads), dtype=F32, device=x.device)
+    _run("ilm_conv_delta_inputs", rows.data_ptr(), gates.data_ptr(), x.data_ptr(), _ptr(weight), _ptr(pool), _ptr(state_in), _ptr(state_out),
+         seg_of_token.data_ptr(), seg_offsets.data_ptr(), a_log.data_ptr(), dt_bias.data_ptr(), T, int(segments), heads, groups, dk, dkp, dv,
+         taps, x.stride(0), rows.stride(0), int(b_off), int(a_off), float(q_scale), float(unit_eps), int(max_len == 1), _dt(x), _stream())
+    return rows, gates
+
+
+def conv_norm_rope_kvwrite(x: torch.Tensor, weight: Optional[torch.Tensor], pool: Optional[torch.Tensor], state_in, state_out,
+                           seg_of_token: torch.Tensor, seg_offsets: torch.Tensor, segments: int, positions: torch.Tensor,
+                           freq: Optional[torch.Tensor], q_weight: Optional[torch.Tensor], k_weight: Optional[torch.Tensor],
+                           k_cache: torch.Tensor, v_cache: torch.Tensor, slots: Optional[torch.Tensor], heads: int, kv_heads: int, dim: int,
+                           vdim: int, rd: int, eps: float, own_kv: bool = True, max_len: Optional[int] = None) -> torch.Tensor:
+    """From fused rows x [q: heads dim | k: kv_heads dim | v: kv_heads vdim] (q alone without `own_kv`): the short convolution per
+    channel (`weight` [taps, channels], None: none), q and k each RMS-normed over all their heads together with a weight
+    (None: no norm), the first rd entries of every q and k head turned in the pairs (2i, 2i + 1) by position x freq[i]; k and v
+    go to the paged cache at `slots`.  Returns the queries as heads of the cache's size [T, heads d] in x's dtype."""
+    C = heads * dim + (kv_heads * (dim + vdim) if own_kv else 0)
+    taps = _conv_operands(x, weight, pool, state_in, state_out, seg_of_token, seg_offsets, segments, C)
+    _dev(positions, freq, q_weight, k_weight, k_cache, v_cache, slots)
+    _i32(positions, "positions")
+    T = x.shape[0]
+    if x.shape[1] < C or positions.numel() != T:
+        raise KernelError(f"rows of {x.shape[1]} do not hold {heads} + {kv_heads} heads of {dim} / {vdim}")
+    if rd and (freq is None or freq.dtype != F32 or freq.numel() != rd // 2 or not freq.is_contiguous()):
+        raise KernelError(f"frequencies must be float32 [{rd // 2}]")
+    for w, n in ((q_weight, heads * dim), (k_weight, kv_heads * dim)):
+        if w is not None and (w.shape != (n,) or not w.is_contiguous() or w.dtype != x.dtype):
+            raise KernelError(f"a query/key norm weight must be [{n}] of the rows' dtype")
+    d = k_cache.shape[3]
+    page = _check_cache(k_cache, v_cache, kv_heads, d)
+    if dim > d or vdim > d or d % 8 or k_cache.dtype != x.dtype:
+        raise KernelError(f"heads of {dim} / {vdim} ({x.dtype}) do not fit cache heads of {d} ({k_cache.dtype})")
+    write = own_kv and slots is not None
+    if write:
+        _i32(slots, "slots")
+        if slots.numel() != T:
+            raise KernelError("one slot a token")
+    q = torch.empty((T, heads * d), dtype=x.dtype, device=x.device)
+    _run("ilm_conv_norm_rope_kvwrite", q.data_ptr(), x.data_ptr(), _ptr(weight), _ptr(pool), _ptr(state_in), _ptr(state_out),
+         seg_of_token.data_ptr(), seg_offsets.data_ptr(), positions.data_ptr(), _ptr(freq), _ptr(q_weight), _ptr(k_weight),
+         k_cache.data_ptr(), v_cache.data_ptr(), _ptr(slots) if write else None, T, int(segments), heads, kv_heads, dim, vdim, d, int(rd),
+         int(bool(own_kv)), taps, x.stride(0), float(eps), page, int(max_len == 1), _dt(x), _stream())
+    return q
+
+
+# ---- the gated delta rule --------------------------------------------------------------------------------------------------
+DELTA_MAX_KEY_DIM = 512      # (ilm_delta_max_dk())
+
+
+def delta_rule(rows: torch.Tensor, gates: torch.Tensor, heads: int, groups: int, dk: int, dv: int, pool: torch.Tensor,
+               state_in: torch.Tensor, state_out: torch.Tensor, seg_offsets: torch.Tensor, segments: int, norm_weight: torch.Tensor,
+               gate: torch.Tensor, eps: float, out_dtype: torch.dtype, max_len: Optional[int] = None) -> torch.Tensor:
+    """S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q per head and token of every segment, then
+    o / sqrt(mean(o^2) + eps) * norm_weight [dv] * silu(gate) per head, [T, heads dv] as `out_dtype`.  `rows`, `gates` as
+    `conv_delta_inputs` leaves them; `gate` [T, heads dv]; `pool` [rows, heads, dv, dk] float32: segment r starts from row
+    state_in[r] and leaves its state in row state_out[r]."""
+    _dev(rows, gates, pool, state_in, state_out, seg_offsets, norm_weight, gate)
+    T = rows.shape[0]
+    dkp = -(-dk // 16) * 16
+    if (rows.dtype != F32 or gates.dtype != F32 or not rows.is_contiguous() or not gates.is_contiguous() or rows.shape[1] < 2 * groups * dkp + heads * dv
+            or tuple(gates.shape) != (T, 2 * heads)):
+        raise KernelError(f"rows {tuple(rows.shape)} / gates {tuple(gates.shape)} do not fit {heads} heads in {groups} groups of {dk} / {dv}")
+    if groups <= 0 or heads % groups or dk > DELTA_MAX_KEY_DIM:
+        raise KernelError(f"{heads} heads in {groups} groups, key size {dk} (at most {DELTA_MAX_KEY_DIM})")
+    if pool.dtype != F32 or not pool.is_contiguous() or tuple(pool.shape[1:]) != (heads, dv, dk):
+        raise KernelError(f"the state pool must be float32 [rows, {heads}, {dv}, {dk}], got {tuple(pool.shape)}")
+    for t, nm in ((state_in, "state_in"), (state_out, "state_out"), (seg_offsets, "seg_offsets")):
+        _i32(t, nm)
+    if state_in.numel() < segments or state_out.numel() < segments or seg_offsets.numel() < segments + 1:
+        raise KernelError("state rows and offsets must cover every segment")
+    _rows(gate, "gate")
+    if gate.shape != (T, heads * dv) or norm_weight.shape != (dv,) or not norm_weight.is_contiguous():
+        raise KernelError(f"gate {tuple(gate.shape)} or norm weight {tuple(norm_weight.shape)} does not fit {heads} heads of {dv}")
+    step = (rows.data_ptr(), rows.stride(0), gates.data_ptr(), pool.data_ptr(), state_in.data_ptr(), state_out.data_ptr(), seg_offsets.data_ptr(),
+            int(segments), heads, groups, dk, dkp, dv)
+    if _lib().ilm_delta_step_norm_ok(dk, dv):
+        y = torch.empty((T, heads * dv), dtype=out_dtype, device=rows.device)
+        _run("ilm_delta_step", None, y.data_ptr(), *step, 1 << 30, norm_weight.data_ptr(), gate.data_ptr(), gate.stride(0), float(eps),
+             y.stride(0), _dt(y), _dt(norm_weight), _dt(gate), _stream())
+        return y
+    o = torch.empty((T, heads * dv), dtype=F32, device=rows.device)
+    _run("ilm_delta_step", o.data_ptr(), None, *step, 1 << 30, None, None, 0, 0.0, 0, 0, 0, 0, _stream())
+    return group_norm_gate(o.view(T * heads, dv), norm_weight, eps, 1, gate=gate.reshape(T * heads, dv), gate_act="silu",
+                           out_dtype=out_dtype).view(T, heads * dv)

@@ -87,8 +87,8 @@ class LLM:
             reach = model.spec.max_positions
             if runner.cache.groups:
                 # no request holds more than the pool of the group that keeps all keys has (a group that keeps a
-                # window needs few pages however long the context: it does not bound the block table's width)
-                full = [g for g in runner.cache.groups if g.window <= 0] or runner.cache.groups
+                # window or a chunk needs few pages however long the context: it does not bound the block table's width)
+                full = [g for g in runner.cache.groups if g.keeps_all] or runner.cache.groups
                 reach = min(reach, max(g.pool.num_pages for g in full) * block_size)
             before = torch.cuda.memory_allocated()
             self.graphs_recorded_at_start = runner.record_decode_graphs(max_batch_size, reach)

@@ -37,17 +37,23 @@ class Param:
     drawn around it."""
 
     def __init__(self, tensor: torch.Tensor, keep_f32: bool = False,
-                 replace: Optional[Callable[[torch.Tensor], None]] = None, neutral: float = 0.0,
+                 replace: Optional[Callable[[torch.Tensor], None]] = None, neutral=0.0,
                  shape: Optional[tuple] = None):
         self.tensor = tensor
         self.keep_f32 = keep_f32 and replace is not None
         self._replace = replace
-        self.neutral = float(neutral)
+        self.neutral = neutral if isinstance(neutral, torch.Tensor) else float(neutral)    # (a tensor: an identity matrix)
         # the tensor's shape in a checkpoint; `tensor` may be a strided view of the same elements in another shape
         # (heads filled up with zeros to a size the kernels take)
         self.shape = tuple(shape) if shape is not None else tuple(tensor.shape)
         if shape is not None and self.keep_f32:
             raise ValueError("a parameter stored through a view cannot be replaced")
+
+    def add_neutral_(self, t: torch.Tensor) -> torch.Tensor:
+        """t (of the parameter's shape) plus the neutral value, in place."""
+        if isinstance(self.neutral, torch.Tensor):
+            return t.add_(self.neutral.to(t.device, t.dtype))
+        return t.add_(self.neutral) if self.neutral != 0.0 else t
 
     def replace(self, t: torch.Tensor) -> None:
         self._replace(t)
@@ -107,7 +113,8 @@ class ResidualStream:
         elif self.pending_gate is not None:
             x = kernels.stream_update(self.residual, self.pending, self.pending_scale, gate=self.pending_gate[0],
                                       gate_bias=self.pending_gate[1], out_dtype=out_dtype)
-        elif self.pending_norm is not None and hasattr(self.pending_norm, "weight") and getattr(self.pending_norm, "groups", 1) == 1:
+        elif self.pending_norm is not None and hasattr(self.pending_norm, "weight") and getattr(self.pending_norm, "groups", 1) == 1 \
+                and not getattr(self.pending_norm, "weight_offset", 0.0):
             x = kernels.stream_update(self.residual, self.pending, self.pending_scale, branch_weight=self.pending_norm.weight,
                                       branch_eps=self.pending_norm.eps, out_dtype=out_dtype)
         else:
@@ -115,6 +122,22 @@ class ResidualStream:
             x = kernels.stream_update(self.residual, self.pending, self.pending_scale, out_dtype=out_dtype)
         self.pending, self.pending_scale, self.pending_norm, self.pending_gate = None, 1.0, None, None
         return self.residual if x is None else x
+
+    def gather(self, rows: torch.Tensor) -> "ResidualStream":
+        """The stream of the tokens `rows` alone, with what is still due to them."""
+        from .. import kernels
+        if self.more or self.pending_gate is not None:
+            self.settle()
+        last = ResidualStream(kernels.gather_rows(self.residual, rows))
+        if self.pending is not None:
+            last.push(_gather_branch(self.pending, rows), self.pending_scale)
+            last.pending_norm = self.pending_norm     # a norm still due to the branch works row by row
+        return last
+
+    def snapshot(self) -> tuple:
+        """(the residual rows, the branch still due or None, its scale), for a dump of intermediate values."""
+        self.settle()
+        return self.residual.clone(), None if self.pending is None else self.pending.clone(), self.pending_scale
 
     def push_more(self, addend: torch.Tensor, scale: float = 1.0) -> None:
         """`addend` ([T, hidden], float32 parts [P, T, hidden], or one row [hidden] for every token) times `scale` joins
@@ -147,6 +170,65 @@ class ResidualStream:
             from .. import kernels
             more, self.more = self.more, []
             kernels.add_layernorm(self.residual, more, None, None, 0.0, torch.float32)
+
+
+def _gather_branch(branch: torch.Tensor, rows: torch.Tensor) -> torch.Tensor:
+    from .. import kernels
+    if branch.dim() == 3:   # parts of a K-split product: the rows of every part
+        return torch.stack([kernels.gather_rows(p, rows) for p in branch])
+    return kernels.gather_rows(branch, rows)
+
+
+class HyperStreams:
+    """A residual stream kept in `count` float32 copies x_1 .. x_count that start equal ("hyper-connections").  A sublayer reads
+    u = sum_s a[s] x_s, and its output y makes all copies anew: x_t <- sum_s M[s, t] x_s + b[t] y (M is indexed from, to).  The
+    model's output is their sum.  A branch pushed here stays due, together with its M and b, until the next read, whose kernel
+    does the update, the read and the norm in one pass (`kernels.hyper_update`).  `base`: the row all copies equal as long as
+    nothing has been pushed; the copies are not in memory before the first branch."""
+
+    def __init__(self, base: torch.Tensor, count: int):
+        self.base: Optional[torch.Tensor] = base
+        self.count = int(count)
+        self.streams: Optional[torch.Tensor] = None      # [T, count, hidden]
+        self.pending: Optional[torch.Tensor] = None
+        self.pending_scale, self.pending_mix, self.pending_out = 1.0, None, None
+
+    def push(self, branch: torch.Tensor, mix: torch.Tensor, out_weights: torch.Tensor, scale: float = 1.0) -> None:
+        if self.pending is not None:
+            raise RuntimeError("a branch is already pending; a norm must fold it first")
+        self.pending, self.pending_scale, self.pending_mix, self.pending_out = branch, float(scale), mix, out_weights
+
+    def read(self, norm=None, in_weights: Optional[torch.Tensor] = None, keep: bool = True) -> torch.Tensor:
+        """Folds the pending branch in and returns the copies' weighted sum (None: their plain sum), normed by `norm` (an
+        `RMSNorm`) in its dtype, or float32 as it is.  `keep` false: the new copies are not needed again and not written."""
+        from .. import kernels
+        base = self.base
+        if self.pending is not None and keep and self.streams is None:
+            self.streams = torch.empty((base.shape[0], self.count, base.shape[1]), dtype=torch.float32, device=base.device)
+        x = kernels.hyper_update(None if base is not None and not (keep and self.pending is not None) else self.streams, self.count, base=base,
+                                 branch=self.pending, alpha=self.pending_scale, mix=self.pending_mix, out_weights=self.pending_out,
+                                 in_weights=in_weights, weight=None if norm is None else norm.weight,
+                                 weight_offset=0.0 if norm is None else norm.weight_offset, eps=0.0 if norm is None else norm.eps,
+                                 out_dtype=torch.float32 if norm is None else norm.dtype, write=keep)
+        if self.pending is not None:
+            if keep:
+                self.base = None
+                self.pending, self.pending_scale, self.pending_mix, self.pending_out = None, 1.0, None, None
+        return x
+
+    def gather(self, rows: torch.Tensor) -> "HyperStreams":
+        """The copies of the tokens `rows` alone, with the branch still due to them."""
+        from .. import kernels
+        last = HyperStreams(None if self.base is None else kernels.gather_rows(self.base, rows), self.count)
+        if self.base is None:
+            T, n, H = self.streams.shape
+            last.streams = kernels.gather_rows(self.streams.view(T, n * H), rows).view(rows.numel(), n, H)
+        if self.pending is not None:
+            last.push(_gather_branch(self.pending, rows), self.pending_mix, self.pending_out, self.pending_scale)
+        return last
+
+    def snapshot(self) -> tuple:
+        return self.read(None, keep=False), None, 1.0
 
 
 @dataclass

@@ -10,8 +10,9 @@ from typing import Dict
 
 import torch
 
+from .. import kernels
 from ..config.spec import LayerSpec
-from .base import BuildContext, DeferredNorm, Param, ResidualStream, join_name
+from .base import BuildContext, DeferredNorm, HyperStreams, Param, Part, ResidualStream, join_name
 from .registry import ARRANGEMENTS, build_feed_forward, build_mixer, build_norm, register_arrangement
 
 
@@ -266,6 +267,73 @@ class BranchNormBlock:
         if self.ffn is not None:
             y = self.ffn.forward(stream.rows(self.dtype), batch)
             stream.push_normed(y, self.norm2, self.residual_scale)
+
+
+@register_arrangement("hyper_connected")
+class HyperConnectedBlock:
+    """Pre-norm sublayers around a residual stream of several copies (`HyperStreams`): the sublayer reads
+    norm(sum_s a[s] x_s), and its output y makes the copies anew, x_t <- sum_s M[s, t] x_s + b[t] y.  `connect1`, `connect2`:
+    PartSpec("hyper_connection", {"streams": n, "names": (a, b, M)}), the sublayers' own a, b [n] and M [n, n] (indexed from, to),
+    float32.  A layer may have no feed-forward (then no `norm2`, no `connect2`)."""
+
+    def __init__(self, spec: LayerSpec, ctx: BuildContext):
+        from .norm import RMSNorm
+        self.spec = spec
+        self.slots = tuple(s for s in ("norm1", "connect1", "mixer", "norm2", "connect2", "ffn") if s in spec.parts)
+        if not {"norm1", "connect1", "mixer"} <= set(self.slots) or len({"norm2", "connect2", "ffn"} & set(self.slots)) not in (0, 3):
+            raise ValueError(f"layer {spec.prefix}: a layer of several streams has norm1, connect1, mixer and, with a feed-forward, norm2 and connect2")
+        self.norm1 = build_norm(spec.parts["norm1"], ctx)
+        self.connect1 = HyperConnection(ctx=ctx, **spec.parts["connect1"].params)
+        self.mixer = build_mixer(spec.parts["mixer"], ctx)
+        self.ffn = self.norm2 = self.connect2 = None
+        if "ffn" in self.slots:
+            self.norm2 = build_norm(spec.parts["norm2"], ctx)
+            self.connect2 = HyperConnection(ctx=ctx, **spec.parts["connect2"].params)
+            self.ffn = build_feed_forward(spec.parts["ffn"], ctx)
+        for norm in (self.norm1, self.norm2):
+            if norm is not None and not isinstance(norm, RMSNorm):
+                raise ValueError(f"layer {spec.prefix}: several streams are read through an RMS norm over the whole row")
+        self.residual_scale = float(spec.residual_scale)
+
+    def named_parameters(self) -> Dict[str, Param]:
+        out: Dict[str, Param] = {}
+        for slot in self.slots:
+            for name, p in getattr(self, slot).named_parameters().items():
+                out[join_name(self.spec.prefix, self.spec.names[slot], name)] = p
+        return out
+
+    def cache_need(self):
+        return self.mixer.cache_need()
+
+    @property
+    def records_mixed_steps(self) -> bool:
+        return bool(getattr(self.mixer, "records_mixed_steps", False)
+                    and (self.ffn is None or getattr(self.ffn, "records_mixed_steps", False)))
+
+    def forward(self, stream: HyperStreams, batch, cache_view) -> None:
+        y = self.mixer.forward(stream.read(self.norm1, self.connect1.read), batch, cache_view)
+        stream.push(y, self.connect1.mix, self.connect1.write, self.residual_scale)
+        if self.ffn is not None:
+            y = self.ffn.forward(stream.read(self.norm2, self.connect2.read), batch)
+            stream.push(y, self.connect2.mix, self.connect2.write, self.residual_scale)
+
+
+class HyperConnection(Part):
+    """A sublayer's weights into and out of the copies of the residual stream: `read` a [n], `write` b [n], `mix` M [n, n]
+    (from, to), float32 whatever the activations' dtype."""
+
+    def __init__(self, streams: int, ctx: BuildContext, names=("in", "out", "mix")):
+        n = int(streams)
+        if not 1 <= n <= kernels.HYPER_MAX_STREAMS:
+            raise ValueError(f"{streams} streams: 1 to {kernels.HYPER_MAX_STREAMS}")
+        self.names = tuple(names)
+        self.read, self.write = (torch.empty((n,), dtype=torch.float32, device=ctx.device) for _ in range(2))
+        self.mix = torch.empty((n, n), dtype=torch.float32, device=ctx.device)
+
+    def named_parameters(self) -> Dict[str, Param]:
+        n = self.read.numel()
+        return {self.names[0]: Param(self.read, neutral=1.0 / n), self.names[1]: Param(self.write, neutral=1.0),
+                self.names[2]: Param(self.mix, neutral=torch.eye(n))}
 
 
 def build_block(spec: LayerSpec, ctx: BuildContext):

@@ -1,4 +1,4 @@
-"""SwiGLU feed-forward: down(silu(gate x) * up x).
+"""Gated feed-forward: down(act(gate x) * up x), act silu (SwiGLU) or the tanh form of gelu.
 
 Reference: csrc/layers/mlp/mlp.cpp:7-38; gate and up are the two halves (gate first) of one fused
 projection: csrc/layers/linear/fused_linear.cpp:152-158,177-180.
@@ -20,7 +20,9 @@ class SwiGLU(FeedForward):
     records_mixed_steps = True
 
     def __init__(self, hidden_size: int, intermediate_size: int, bias: bool, ctx: BuildContext,
-                 names=("gate_proj", "up_proj", "down_proj"), suffix: str = "weight"):
+                 names=("gate_proj", "up_proj", "down_proj"), suffix: str = "weight", activation: str = "silu"):
+        kernels.glu_code(activation)
+        self.activation = activation
         self.gate_up = FusedLinear(hidden_size, [intermediate_size, intermediate_size], [names[0], names[1]],
                                    bias, ctx, suffix=suffix)
         self.down = Linear(intermediate_size, hidden_size, names[2], bias, ctx, suffix=suffix)
@@ -35,18 +37,27 @@ class SwiGLU(FeedForward):
 
     def forward(self, x, batch) -> torch.Tensor:
         if isinstance(x, DeferredNorm):   # the norm's division happens in the gate/up kernel's epilogue
-            act = kernels.gateup_swiglu_gemm(x.x, self.gate_up.weight, self.gate_up.bias, row_ss=x.sumsq, eps=x.eps)
+            act = kernels.gateup_swiglu_gemm(x.x, self.gate_up.weight, self.gate_up.bias, row_ss=x.sumsq, eps=x.eps,
+                                             act=self.activation)
             return self.down.forward(act, allow_parts=True)
         frag = (lambda: self.gate_up.frag_weight("gate_up8")) if kernels.frag_weight_ok(self.gate_up.weight) else None
-        act = kernels.gateup_swiglu_gemm(x, self.gate_up.weight, self.gate_up.bias, frag_w=frag)   # few rows: activation in the epilogue
+        act = kernels.gateup_swiglu_gemm(x, self.gate_up.weight, self.gate_up.bias, frag_w=frag, act=self.activation)   # few rows: activation in the epilogue
         if act is not None:
             return self.down.forward(act, allow_parts=True)
         gu = self.gate_up.forward(x)
-        if self.down.bias is None:
+        if self.down.bias is None and self.activation == "silu":
             fused = kernels.swiglu_gemm(gu, self.down.weight)   # few rows: activation inside the product
             if fused is not None:
                 return fused
-        return self.down.forward(kernels.swiglu(gu), allow_parts=True)
+        return self.down.forward(kernels.swiglu(gu, self.activation), allow_parts=True)
+
+
+@register_feed_forward("gated_mlp")
+class GatedMLP(SwiGLU):
+    """The same with the gate's activation named (`activation`: "silu" or "gelu_tanh")."""
+
+    def __init__(self, hidden_size: int, intermediate_size: int, activation: str, bias: bool, ctx: BuildContext, **names):
+        super().__init__(hidden_size, intermediate_size, bias, ctx, activation=activation, **names)
 
 
 @register_feed_forward("activation_mlp")

@@ -12,7 +12,7 @@ from typing import Dict
 import torch
 
 from .. import kernels
-from .base import BuildContext, Norm, NormTail, Param, ResidualStream
+from .base import BuildContext, HyperStreams, Norm, NormTail, Param, ResidualStream
 from .registry import register_norm
 
 
@@ -20,9 +20,11 @@ from .registry import register_norm
 class RMSNorm(Norm):
     takes_frag_request = True
 
-    def __init__(self, size: int, eps: float, ctx: BuildContext, param_name: str = "weight"):
+    def __init__(self, size: int, eps: float, ctx: BuildContext, param_name: str = "weight", weight_offset: float = 0.0):
         self.size = int(size)
         self.eps = float(eps)
+        # rows are multiplied by weight + weight_offset (1: a checkpoint's weights lie around zero); added in float32
+        self.weight_offset = float(weight_offset)
         self.dtype = ctx.dtype
         self.param_name = param_name    # "": the weight lies under the norm's own name in a checkpoint
         self.weight = torch.empty((self.size,), dtype=ctx.dtype, device=ctx.device)
@@ -31,14 +33,16 @@ class RMSNorm(Norm):
         self.weight = t
 
     def named_parameters(self) -> Dict[str, Param]:
-        return {self.param_name: Param(self.weight, keep_f32=True, replace=self._set_weight, neutral=1.0)}
+        return {self.param_name: Param(self.weight, keep_f32=True, replace=self._set_weight, neutral=1.0 - self.weight_offset)}
 
     def apply(self, x: torch.Tensor, out_dtype: torch.dtype = torch.float32) -> torch.Tensor:
         """The norm of rows that are not the residual stream (a branch's output normed before it is added): sums in
         float32, the result in `out_dtype`."""
-        return kernels.group_norm_gate(x, self.weight, self.eps, 1, out_dtype=out_dtype)
+        return kernels.group_norm_gate(x, self.weight, self.eps, 1, out_dtype=out_dtype, weight_offset=self.weight_offset)
 
     def tail(self, stream: ResidualStream, scale: float, rows: int):
+        if self.weight_offset:
+            return None
         stream.settle()
         if stream.pending is not None or self.dtype != torch.bfloat16 or rows > kernels.TAIL_MAX_ROWS:
             return None
@@ -46,10 +50,12 @@ class RMSNorm(Norm):
 
     def forward(self, stream: ResidualStream, frag: bool = False):
         """`frag`: the consumer takes its rows in fragment order (`kernels.FragRows`)."""
+        if isinstance(stream, HyperStreams):
+            return stream.read(self)
         if stream.more:
             stream.settle()
         post = stream.pending_norm
-        if post is not None and not frag and isinstance(post, RMSNorm):
+        if post is not None and not frag and isinstance(post, RMSNorm) and not (post.weight_offset or self.weight_offset):
             # the branch's own norm, the sum and this norm in one kernel
             x = kernels.norm_add_norm(stream.residual, stream.pending, post.weight, post.eps, stream.pending_scale, self.weight,
                                       self.eps, self.dtype)
@@ -57,7 +63,7 @@ class RMSNorm(Norm):
             return x
         stream.settle()
         x = kernels.add_rmsnorm(stream.residual, stream.pending, self.weight, stream.pending_scale, self.eps,
-                                self.dtype, frag=frag)
+                                self.dtype, frag=frag, weight_offset=self.weight_offset)
         stream.pending = None
         stream.pending_scale = 1.0
         return x
@@ -88,7 +94,7 @@ class GroupRMSNorm(Norm):
         if stream.more:
             stream.settle()
         post = stream.pending_norm
-        if post is not None and not (isinstance(post, RMSNorm) and post.weight.dtype == self.weight.dtype):
+        if post is not None and not (isinstance(post, RMSNorm) and post.weight.dtype == self.weight.dtype and not post.weight_offset):
             stream.settle()      # a branch norm of another kind: applied by itself
             post = None
         gate, bias = stream.pending_gate if stream.pending_gate is not None else (None, None)

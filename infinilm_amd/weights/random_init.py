@@ -38,8 +38,8 @@ def random_state_dict(config: dict, seed: int, std: float = 0.02, norm_init: str
             continue
         g = torch.Generator().manual_seed((int(seed) * 1000003 + i) & 0x7fffffffffff)
         t = torch.randn(tuple(p.shape), generator=g, dtype=torch.float32) * std
-        if norm_init == "one_plus" and p.neutral != 0.0:
-            t = t + p.neutral
+        if norm_init == "one_plus":
+            t = p.add_neutral_(t)
         out[name] = t.to(store).contiguous()
     return out
 
@@ -81,5 +81,5 @@ def fill_random_(model, seed: int, std: float = 0.02, norm_init: str = "one_plus
             for a in range(0, flat.numel(), step):
                 b = min(flat.numel(), a + step)
                 flat[a:b] = (torch.randn((b - a,), generator=g, device=t.device, dtype=torch.float32) * std).to(t.dtype)
-        if norm_init == "one_plus" and p.neutral != 0.0:
-            t.add_(p.neutral)
+        if norm_init == "one_plus":
+            p.add_neutral_(t)
