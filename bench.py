@@ -54,8 +54,8 @@ def main() -> int:
                     help="instead of the default workload: prefill and decode throughput of another design (--design) beside MiniCPM4 "
                          "at equal layer sizes (random weights), with the time and the roofline share of every kernel")
     ap.add_argument("--design-shapes", default="1024,4096", help="widths to compare with --designs")
-    ap.add_argument("--design", default="kekevik", choices=["kekevik", "pugavik", "patadra", "bebuzen"],
-                    help="the design that --designs puts beside MiniCPM4")
+    ap.add_argument("--design", default="kekevik", choices=["kekevik", "pugavik", "patadra", "bebuzen", "moputar"],
+                    help="the design that --designs puts beside MiniCPM4 (moputar: beside Kekevik too, whose recurrence is the closest to its)")
     args = ap.parse_args()
     if args.gpus != 1 or int(os.environ.get("WORLD_SIZE", "1")) != 1:
         print("bench.py measures one GPU: this engine has no multi-GPU path (N>1 is not run)")
@@ -94,7 +94,7 @@ def compare_designs(args) -> dict:
     from infinilm_amd.sampling import Sampler, SamplingParams
     from infinilm_amd.weights import fill_random_
     sys.path.insert(0, os.path.join(ROOT, "examples"))
-    from shapes import bebuzen_shape, kekevik_shape, patadra_shape, pugavik_shape
+    from shapes import bebuzen_shape, kekevik_shape, moputar_shape, patadra_shape, pugavik_shape
 
     layers = 8 if args.layers == 32 else args.layers
     T, ctx, ps = args.prefill_tokens, min(args.context, 2048), args.page_size
@@ -112,7 +112,10 @@ def compare_designs(args) -> dict:
                          "rms_norm_eps": 1e-6, "tie_word_embeddings": True},
             design: patadra_shape(width, heads, d, layers, V) if design == "patadra" else
             bebuzen_shape(width, heads, d, kv, layers, V) if design == "bebuzen" else
+            moputar_shape(width, heads, d, kv, layers, V) if design == "moputar" else
             (kekevik_shape if design == "kekevik" else pugavik_shape)(width, heads, d, kv, layers, V, 6 * width)}
+        if design == "moputar":
+            cfgs["kekevik"] = kekevik_shape(width, heads, d, kv, layers, V, 6 * width)
         rec = {}
         for name, cfg in cfgs.items():
             model = build_model(cfg, "bfloat16", "cuda:0")
@@ -233,17 +236,34 @@ def compare_designs(args) -> dict:
                         if us(rep_p, "ilm_stream_update"):
                             share["stream_update prefill (stream read + written, branch read, rows written / HBM peak)"] = round(
                                 T * Hs * (4 + 4 + 2 + 2) / us(rep_p, "ilm_stream_update") / HBM_PEAK, 4)
+                    if name == "moputar":
+                        chunk, n = 1024, cfg["streams"]
+                        seen, pairs = (ctx - 1) % chunk + 1, sum(i % chunk + 1 for i in range(T))
+                        C = 2 * (max(heads // 2, 1)) * d + heads * d       # convolved channels of a delta layer
+                        Ca = heads * d + 2 * kv * d                        # ... of an attention layer with keys and values of its own
+                        share["attention decode (own chunk's cache read / HBM peak)"] = round(64 * seen * kvb / us(rep_d, "ilm_attn_mfma") / HBM_PEAK, 4)
+                        share["attention prefill (4 d flops a visible key and head / bf16 matrix peak)"] = round(
+                            4.0 * d * pairs * heads / us(rep_p, "ilm_attn_tile") / FLOP_PEAK["bf16"], 4)
+                        share["delta_step decode (state read + written / HBM peak)"] = round(64 * 2 * state / us(rep_d, "ilm_delta_step") / HBM_PEAK, 4)
+                        share["delta_chunks prefill (6 dk dv flops a token and head / float32 vector peak)"] = round(
+                            6.0 * T * heads * d * d / us(rep_p, "ilm_delta_chunks") / FLOP_PEAK["fp32"], 4)
+                        share["hyper_update prefill (streams read + written, branch read, rows written / HBM peak)"] = round(
+                            T * Hs * (4 * n + 4 * n + 2 + 2) / us(rep_p, "ilm_hyper_update") / HBM_PEAK, 4)
+                        share["conv_delta_inputs prefill (rows read, float rows written / HBM peak)"] = round(
+                            T * C * (2 + 4) / us(rep_p, "ilm_conv_delta_inputs") / HBM_PEAK, 4)
+                        share["conv_norm_rope_kvwrite prefill (rows read and written, mean of both layer kinds / HBM peak)"] = round(
+                            T * (Ca + heads * d) / 2 * (2 + 2) / us(rep_p, "ilm_conv_norm_rope_kvwrite") / HBM_PEAK, 4)
                     if name == "minicpm4" and us(rep_p, "library_gemm"):
                         flops = 2.0 * T * Hs * ((heads + 2 * kv) * d + heads * d + 3 * cfg["intermediate_size"]) * layers
                         share["library products prefill, all of a step (flops / bf16 matrix peak)"] = round(
                             flops / (rep_p["library_gemm"]["total_ms"] * 1e-3 / 2) / FLOP_PEAK["bf16"], 4)
-                    if name not in ("pugavik", "patadra", "bebuzen") and us(rep_d, "ilm_decay_scan"):
+                    if name not in ("pugavik", "patadra", "bebuzen", "moputar") and us(rep_d, "ilm_decay_scan"):
                         share["decay_scan decode (state read + written / HBM peak)"] = round(64 * 2 * state / us(rep_d, "ilm_decay_scan") / HBM_PEAK, 4)
                         share["decay_scan prefill (4 dk dv flops a token and head / float32 vector peak)"] = round(
                             4.0 * T * heads * d * d / us(rep_p, "ilm_decay_scan") / FLOP_PEAK["fp32"], 4)
-                    if name not in ("pugavik", "patadra", "bebuzen") and us(rep_d, "ilm_attn_mfma"):
+                    if name not in ("pugavik", "patadra", "bebuzen", "moputar") and us(rep_d, "ilm_attn_mfma"):
                         share["attention decode (cache read / HBM peak)"] = round(64 * ctx * kvb / us(rep_d, "ilm_attn_mfma") / HBM_PEAK, 4)
-                    if name not in ("pugavik", "patadra", "bebuzen") and us(rep_p, "ilm_attn_tile"):
+                    if name not in ("pugavik", "patadra", "bebuzen", "moputar") and us(rep_p, "ilm_attn_tile"):
                         share["attention prefill (4 d flops a visible key and head / bf16 matrix peak)"] = round(
                             4.0 * T * T / 2 * heads * d / us(rep_p, "ilm_attn_tile") / FLOP_PEAK["bf16"], 4)
                     if name == "pugavik":

@@ -137,3 +137,20 @@ def bebuzen_shape(width: int, heads: int, head_dim: int, kv_heads: int, layers: 
         else:
             out.append({"type": "attention", "mixer": dict(diff, kv_from=i - 2), "mlp": dict(moe)})
     return {"architecture": "Bebuzen", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "residual_mult": 0.5, "layers": out}
+
+
+def moputar_shape(width: int, heads: int, head_dim: int, kv_heads: int, layers: int, vocab: int, chunk: int = 1024, streams: int = 4) -> dict:
+    """A Moputar configuration with the layer sizes of a transformer of this width: three layer kinds in turn (a gated delta rule
+    with half as many query/key heads as value heads; an attention inside chunks of positions; an attention that reads that layer's
+    keys and values), convolutions of four taps, half of every attention head turned, `streams` residual streams, a
+    gelu-gated feed-forward of 4 x width in every layer."""
+    att = {"heads": heads, "kv_heads": kv_heads, "dim": head_dim, "vdim": head_dim, "scale": head_dim ** -0.5, "conv": 4,
+           "rot": {"base": 500000.0, "dims": head_dim // 2}, "mask": {"size": chunk}}
+    delta = {"heads": heads, "kv_heads": max(heads // 2, 1), "dim": head_dim, "vdim": head_dim, "conv": 4}
+    mlp = {"kind": "dense", "ff": 4 * width}
+    out = []
+    for i in range(layers):
+        kind, mixer = ("delta", delta) if i % 3 == 0 else ("attention", att if i % 3 == 1 else dict(att, kv_from=i - 1))
+        out.append({"type": kind, "mixer": dict(mixer), "mlp": dict(mlp)})
+    return {"architecture": "Moputar", "vocab": vocab, "width": width, "streams": streams, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-5},
+            "layers": out}

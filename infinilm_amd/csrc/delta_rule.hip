@@ -12,7 +12,21 @@
 //       read-out after the write is S^T q + u (k . q)), and k . q are folded over the lanes of a column together.  Where a block
 //       holds all columns of its head it can end with the head's output norm, weight and gate:
 //       y = o / sqrt(mean(o^2) + eps) * w * silu(gate), in the activations' dtype.
+//
+//   ilm_delta_chunks   long segments (portions of prompts), in chunks of DC = 64 tokens on the float matrix instruction
+//       (v_mfma_f32_16x16x4_f32: IEEE float products and sums).  With L_t the sum of the log-decays of a chunk's tokens up to t,
+//       S_0 the state at its start, and A[t, i] = beta_t exp(L_t - L_i) k_t . k_i for i < t (0 elsewhere), the corrections u of
+//       a chunk solve  (I + A) U = diag(beta) (V - diag(exp L) K S_0), so that
+//           U  = V' - W S_0,     V' = (I + A)^-1 diag(beta) V,     W = (I + A)^-1 diag(beta exp L) K
+//           o_t = exp(L_t) S_0^T q_t + sum_{i <= t} exp(L_t - L_i) (k_i . q_t) u_i
+//           S   = exp(L_end) S_0 + sum_i exp(L_end - L_i) k_i u_i^T.
+//       Two kernels: the first makes V', W, the weights of the second sum and the decayed keys of every chunk, all chunks and
+//       heads side by side; the second walks a segment's chunks in order with 16 value columns of a head's state a block.
+//       Differences of L are taken in double, so that a token's decay keeps its float precision however much has been
+//       forgotten before it.  Chunk p of segment r has the workspace slot floor(first row of r / DC) + r + p.
 #include "common.h"
+
+typedef __attribute__((ext_vector_type(4))) float f32x4;
 
 #define DS_NK 8
 
@@ -188,5 +202,348 @@ extern "C" int ilm_delta_step(void* o, void* y, const void* rows, int row_stride
     else delta_step_kernel<256, 1, false><<<dim3((dv + VT - 1) / VT, H, R), 256, 0, stream>>>(DS_ARGS);
 #undef DS_ARGS
     ILM_LAUNCH_CHECK("delta_step");
+    return 0;
+}
+
+// ---- long segments in chunks ----------------------------------------------------------------------------------------------
+#define DC 64
+#define DC_MAX_DK 128
+#define DC_EL (DC + 4)       // exp(L_t) of a chunk's tokens, then exp(L_end)
+
+__device__ __forceinline__ f32x4 dc_mfma(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+// D += A[16 x 16] B[16 x 16]: lane (r, q) brings A[r][4q .. 4q + 3] and holds B and D as rows 4q .. 4q + 3 of column r
+__device__ __forceinline__ f32x4 dc_mma(const float4& a, const f32x4& b, f32x4 c) {
+    c = dc_mfma(a.x, b[0], c);
+    c = dc_mfma(a.y, b[1], c);
+    c = dc_mfma(a.z, b[2], c);
+    return dc_mfma(a.w, b[3], c);
+}
+// D += A[16 x 16] B^T: both sides as rows, lane (r, q) brings A[r][4q ..] and B[r][4q ..]
+__device__ __forceinline__ f32x4 dc_mmt(const float4& a, const float4& b, f32x4 c) {
+    c = dc_mfma(a.x, b.x, c);
+    c = dc_mfma(a.y, b.y, c);
+    c = dc_mfma(a.z, b.z, c);
+    return dc_mfma(a.w, b.w, c);
+}
+
+// the segment whose slots hold slot s (-1: none), its chunk p
+__device__ __forceinline__ int dc_find(const int* __restrict__ seg_offsets, int R, int s, int& p) {
+    int lo = 0, hi = R - 1;     // the last segment whose first slot is <= s
+    while (lo < hi) {
+        const int mid = (lo + hi + 1) >> 1;
+        if (seg_offsets[mid] / DC + mid <= s) lo = mid; else hi = mid - 1;
+    }
+    p = s - (seg_offsets[lo] / DC + lo);
+    return (p >= 0 && p * DC < seg_offsets[lo + 1] - seg_offsets[lo]) ? lo : -1;
+}
+
+#define DC_XT 4      // column tiles of [V | K] a wave solves together
+
+// KT: key entries / 16
+template <int KT>
+__global__ void __launch_bounds__(256)
+delta_chunk_prepare_kernel(float* __restrict__ ws_v, float* __restrict__ ws_w, float* __restrict__ ws_k, float* __restrict__ ws_p,
+                           float* __restrict__ ws_e, const float* __restrict__ rows, int row_stride, const float* __restrict__ gates,
+                           const int* __restrict__ seg_offsets, int R, int H, int G, int dv, int dvp, int min_len) {
+    constexpr int DK = KT * 16, KS = DK + 4, AS = DC + 4, TS = 20;
+    __shared__ __attribute__((aligned(16))) float Ks[DC * KS];
+    __shared__ __attribute__((aligned(16))) float An[DC * AS];          // -A
+    __shared__ __attribute__((aligned(16))) float Ti[4 * 16 * TS];      // inverses of the diagonal blocks of I + A
+    __shared__ double Ls[DC];
+    __shared__ float bs[DC];
+    const int h = blockIdx.x, slot = blockIdx.y;
+    int p;
+    const int seg = dc_find(seg_offsets, R, slot, p);
+    if (seg < 0) return;
+    const int len = seg_offsets[seg + 1] - seg_offsets[seg];
+    if (len < min_len) return;                         // (the step kernel's)
+    const int t0 = seg_offsets[seg] + p * DC, n = min(DC, len - p * DC);
+    const int tid = threadIdx.x, lane = tid & 63, r = lane & 15, q = lane >> 4;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int g = h / (H / G);
+    const float* qrow = rows + (size_t)t0 * row_stride + (size_t)g * DK;
+    const float* krow = qrow + (size_t)G * DK;
+    const float* vrow = rows + (size_t)t0 * row_stride + (size_t)2 * G * DK + (size_t)h * dv;
+    const size_t sh = (size_t)slot * H + h;
+    for (int i = tid; i < DC * (DK / 4); i += 256) {
+        const int t = i / (DK / 4), c = (i % (DK / 4)) * 4;
+        const float4 v = *reinterpret_cast<const float4*>(krow + (size_t)(t < n ? t : n - 1) * row_stride + c);
+        *reinterpret_cast<float4*>(&Ks[t * KS + c]) = t < n ? v : make_float4(0.f, 0.f, 0.f, 0.f);
+    }
+    if (wave == 0) {
+        const float* gt = gates + (size_t)(t0 + (lane < n ? lane : n - 1)) * 2 * H + h;
+        double L = lane < n ? (double)gt[H] : 0.0;
+#pragma unroll
+        for (int off = 1; off < 64; off <<= 1) {
+            const double up = __shfl_up(L, off, 64);
+            if (lane >= off) L += up;
+        }
+        Ls[lane] = L;
+        bs[lane] = lane < n ? gt[0] : 0.f;
+        ws_e[sh * DC_EL + lane] = expf((float)L);
+        if (lane == 63) ws_e[sh * DC_EL + DC] = expf((float)L);
+    }
+    __syncthreads();
+    // ---- k_t . k_i and q_t . k_i by tiles of 16 x 16 at and below the diagonal
+    for (int tile = wave; tile < 10; tile += 4) {
+        const int rt = tile < 1 ? 0 : (tile < 3 ? 1 : (tile < 6 ? 2 : 3)), ct = tile - rt * (rt + 1) / 2;
+        f32x4 kk = f32x4{0.f, 0.f, 0.f, 0.f}, qk = kk;
+        const int tq = 16 * rt + r < n ? 16 * rt + r : n - 1;
+#pragma unroll
+        for (int j = 0; j < KT; ++j) {
+            const float4 qa = *reinterpret_cast<const float4*>(qrow + (size_t)tq * row_stride + 16 * j + 4 * q);
+            const float4 ka = *reinterpret_cast<const float4*>(&Ks[(16 * rt + r) * KS + 16 * j + 4 * q]);
+            const float4 kb = *reinterpret_cast<const float4*>(&Ks[(16 * ct + r) * KS + 16 * j + 4 * q]);
+            kk = dc_mmt(ka, kb, kk);
+            qk = dc_mmt(qa, kb, qk);
+        }
+        const int i = 16 * ct + r;
+        const double Li = Ls[i];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int t = 16 * rt + 4 * q + e;
+            const float dec = expf(i <= t ? (float)(Ls[t] - Li) : 0.f);
+            An[t * AS + i] = i < t ? -bs[t] * dec * kk[e] : 0.f;
+            ws_p[(sh * DC + t) * DC + i] = (i <= t && t < n) ? dec * qk[e] : 0.f;
+        }
+    }
+    __syncthreads();
+    if (wave == 0) {      // column r of the inverse of diagonal block q, by substitution
+        float x[16];
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            float v = i == r ? 1.0f : 0.f;
+#pragma unroll
+            for (int j = 0; j < i; ++j) v = fmaf(An[(16 * q + i) * AS + 16 * q + j], x[j], v);
+            x[i] = v;
+        }
+#pragma unroll
+        for (int i = 0; i < 16; ++i) Ti[(q * 16 + i) * TS + r] = x[i];
+    } else {              // the decayed keys, transposed
+        const float f = expf((float)(Ls[DC - 1] - Ls[lane]));
+        for (int i = wave - 1; i < DK; i += 3) ws_k[(sh * DK + i) * DC + lane] = f * Ks[lane * KS + i];
+    }
+    __syncthreads();
+    // ---- (I + A) X = [beta V | beta exp(L) K], DC_XT column tiles of 16 a wave, the rows' blocks one after the other
+    const int nv = dvp / 16, nt = nv + KT;
+    for (int c0 = wave * DC_XT; c0 < nt; c0 += 4 * DC_XT) {
+        f32x4 X[4][DC_XT];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            f32x4 acc[DC_XT];
+#pragma unroll
+            for (int c = 0; c < DC_XT; ++c) {
+                const int ct = c0 + c;                 // wave-uniform
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    const int t = 16 * i + 4 * q + e;
+                    float v = 0.f;
+                    if (ct < nv) {
+                        const int col = 16 * ct + r;
+                        v = vrow[(size_t)(t < n ? t : n - 1) * row_stride + (col < dv ? col : dv - 1)];
+                        v = col < dv ? v * bs[t] : 0.f;
+                    } else if (ct < nt) {
+                        v = bs[t] * expf((float)Ls[t]) * Ks[t * KS + 16 * (ct - nv) + r];
+                    }
+                    acc[c][e] = v;
+                }
+            }
+#pragma unroll
+            for (int j = 0; j < i; ++j) {
+                const float4 a = *reinterpret_cast<const float4*>(&An[(16 * i + r) * AS + 16 * j + 4 * q]);
+#pragma unroll
+                for (int c = 0; c < DC_XT; ++c) acc[c] = dc_mma(a, X[j][c], acc[c]);
+            }
+            const float4 d = *reinterpret_cast<const float4*>(&Ti[(i * 16 + r) * TS + 4 * q]);
+#pragma unroll
+            for (int c = 0; c < DC_XT; ++c) X[i][c] = dc_mma(d, acc[c], f32x4{0.f, 0.f, 0.f, 0.f});
+        }
+#pragma unroll
+        for (int c = 0; c < DC_XT; ++c) {
+            const int ct = c0 + c;
+            if (ct >= nt) break;
+            float* dst = ct < nv ? ws_v + sh * DC * dvp + 16 * ct + r : ws_w + sh * DC * DK + 16 * (ct - nv) + r;
+            const int ld = ct < nv ? dvp : DK;
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) dst[(size_t)(16 * i + 4 * q + e) * ld] = X[i][c][e];
+        }
+    }
+}
+
+// What a wave reads of a chunk: its 16 rows of W, q and the sums' weights, its tiles of the decayed keys, its corner of V'
+template <int KT>
+struct dc_operands {
+    static constexpr int MT = (KT + 3) / 4;
+    float4 w[KT], q[KT], p[4], k[MT][4], e;
+    f32x4 v;
+    float end;
+};
+
+template <int KT>
+__device__ __forceinline__ void dc_load(dc_operands<KT>& o, const float* ws_v, const float* ws_w, const float* ws_k, const float* ws_p,
+                                        const float* ws_e, const float* qhead, int row_stride, size_t sh, int t0, int n, int dvp, int col0,
+                                        int wave, int r, int q) {
+    constexpr int DK = KT * 16;
+    const int row = 16 * wave + r, tq = row < n ? row : n - 1;
+#pragma unroll
+    for (int j = 0; j < KT; ++j) {
+        o.w[j] = *reinterpret_cast<const float4*>(ws_w + (sh * DC + row) * DK + 16 * j + 4 * q);
+        o.q[j] = *reinterpret_cast<const float4*>(qhead + (size_t)(t0 + tq) * row_stride + 16 * j + 4 * q);
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        // (blocks above the diagonal are not in memory: the diagonal's own is read in their place and not used)
+        o.p[j] = *reinterpret_cast<const float4*>(ws_p + (sh * DC + row) * DC + 16 * (j <= wave ? j : wave) + 4 * q);
+#pragma unroll
+        for (int m = 0; m < dc_operands<KT>::MT; ++m) {
+            const int mt = wave + 4 * m < KT ? wave + 4 * m : KT - 1;
+            o.k[m][j] = *reinterpret_cast<const float4*>(ws_k + (sh * DK + 16 * mt + r) * DC + 16 * j + 4 * q);
+        }
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o.v[e] = ws_v[(sh * DC + 16 * wave + 4 * q + e) * dvp + col0 + r];
+    o.e = *reinterpret_cast<const float4*>(ws_e + sh * DC_EL + 16 * wave + 4 * q);
+    o.end = ws_e[sh * DC_EL + DC];
+}
+
+template <int KT>
+__global__ void __launch_bounds__(256, 1)
+delta_chunk_walk_kernel(float* __restrict__ out, const float* __restrict__ ws_v, const float* __restrict__ ws_w, const float* __restrict__ ws_k,
+                        const float* __restrict__ ws_p, const float* __restrict__ ws_e, const float* __restrict__ rows, int row_stride,
+                        float* __restrict__ pool, const int* __restrict__ state_in, const int* __restrict__ state_out,
+                        const int* __restrict__ seg_offsets, int H, int G, int dk, int dv, int dvp, int min_len) {
+    constexpr int DK = KT * 16, MT = dc_operands<KT>::MT;
+    __shared__ f32x4 Us[4][64];
+    __shared__ f32x4 Ss[KT][64];
+    // blocks go to the eight dies in turn; with this numbering the column blocks of a head share a die, whose cache then holds
+    // the operands that they all read
+    const int nb = dvp / 16, items = nb * H, per = (items + 7) / 8;
+    const int item = (int)(blockIdx.x & 7) * per + (int)(blockIdx.x >> 3);
+    if ((int)(blockIdx.x >> 3) >= per || item >= items) return;
+    const int h = item / nb, col0 = (item % nb) * 16, seg = blockIdx.y;
+    const int s0 = seg_offsets[seg], len = seg_offsets[seg + 1] - s0;
+    if (len <= 0 || len < min_len) return;
+    const int chunks = (len + DC - 1) / DC, slot0 = s0 / DC + seg;
+    const int lane = threadIdx.x & 63, r = lane & 15, q = lane >> 4;
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const float* qhead = rows + (size_t)(h / (H / G)) * DK;
+    const bool col_ok = col0 + r < dv, v4 = dk % 4 == 0;
+    // state tile m: entries 16 m + 4 q + e of column col0 + r; every wave holds all of them
+    f32x4 S[KT];
+    {
+        const float* src = pool + (((size_t)state_in[seg] * H + h) * dv + (col_ok ? col0 + r : 0)) * dk;
+#pragma unroll
+        for (int m = 0; m < KT; ++m) {
+            const int k0 = 16 * m + 4 * q;
+            if (v4) {
+                const float4 t = *reinterpret_cast<const float4*>(src + (k0 < dk ? k0 : 0));
+                const bool ok = col_ok && k0 < dk;
+                S[m] = f32x4{ok ? t.x : 0.f, ok ? t.y : 0.f, ok ? t.z : 0.f, ok ? t.w : 0.f};
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) S[m][e] = (col_ok && k0 + e < dk) ? src[k0 + e] : 0.f;
+            }
+        }
+    }
+    dc_operands<KT> cur, nxt;
+    dc_load<KT>(nxt, ws_v, ws_w, ws_k, ws_p, ws_e, qhead, row_stride, (size_t)slot0 * H + h, s0, min(DC, len), dvp, col0, wave, r, q);
+    for (int c = 0; c < chunks; ++c) {
+        cur = nxt;
+        const int t0 = s0 + c * DC, n = min(DC, len - c * DC);
+        if (c + 1 < chunks)
+            dc_load<KT>(nxt, ws_v, ws_w, ws_k, ws_p, ws_e, qhead, row_stride, (size_t)(slot0 + c + 1) * H + h, t0 + DC, min(DC, len - (c + 1) * DC),
+                        dvp, col0, wave, r, q);
+        f32x4 ws = f32x4{0.f, 0.f, 0.f, 0.f}, qs = ws;
+#pragma unroll
+        for (int m = 0; m < KT; ++m) {
+            ws = dc_mma(cur.w[m], S[m], ws);
+            qs = dc_mma(cur.q[m], S[m], qs);
+        }
+        Us[wave][lane] = cur.v - ws;
+        __syncthreads();
+        f32x4 U[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) U[j] = Us[j][lane];
+#pragma unroll
+        for (int m = 0; m < MT; ++m)
+            if (wave + 4 * m < KT) {                    // wave-uniform
+                f32x4 s;
+#pragma unroll
+                for (int mm = 0; mm < KT; ++mm)
+                    if (mm == wave + 4 * m) s = S[mm];
+                s = s * cur.end;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) s = dc_mma(cur.k[m][j], U[j], s);
+                Ss[wave + 4 * m][lane] = s;
+            }
+        f32x4 o = f32x4{qs[0] * cur.e.x, qs[1] * cur.e.y, qs[2] * cur.e.z, qs[3] * cur.e.w};
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+            if (j <= wave) o = dc_mma(cur.p[j], U[j], o);
+        if (col_ok) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int t = 16 * wave + 4 * q + e;
+                if (t < n) out[((size_t)(t0 + t) * H + h) * dv + col0 + r] = o[e];
+            }
+        }
+        __syncthreads();
+#pragma unroll
+        for (int m = 0; m < KT; ++m) S[m] = Ss[m][lane];
+    }
+    if (!col_ok) return;
+    float* dst = pool + (((size_t)state_out[seg] * H + h) * dv + col0 + r) * dk;
+#pragma unroll
+    for (int m = 0; m < KT; ++m)
+        if ((m & 3) == wave) {
+            const int k0 = 16 * m + 4 * q;
+            if (v4) {
+                if (k0 < dk) *reinterpret_cast<float4*>(dst + k0) = make_float4(S[m][0], S[m][1], S[m][2], S[m][3]);
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (k0 + e < dk) dst[k0 + e] = S[m][e];
+            }
+        }
+}
+
+extern "C" int ilm_delta_chunk() { return DC; }
+extern "C" int ilm_delta_chunk_max_dk() { return DC_MAX_DK; }
+// floats of workspace a (slot, head) takes
+extern "C" int ilm_delta_chunk_ws(int dkp, int dvp) { return DC * dvp + 2 * DC * dkp + DC * DC + DC_EL; }
+
+// Segments of at least min_len tokens; the others are passed over.  ws: (T / DC + R) * H * ilm_delta_chunk_ws floats.
+extern "C" int ilm_delta_chunks(void* o, const void* rows, int row_stride, const void* gates, void* pool, const void* state_in,
+                                const void* state_out, const void* seg_offsets, int R, int H, int G, int dk, int dkp, int dv, int T_, int min_len,
+                                void* ws, hipStream_t stream) {
+    ILM_REQUIRE(T_ > 0 && R > 0 && R <= 65535 && H > 0 && G > 0 && H % G == 0 && dk > 0 && dv > 0, "delta_chunks: bad sizes");
+    ILM_REQUIRE(dk <= DC_MAX_DK && dkp == (dk + 15) / 16 * 16, "delta_chunks: keys of %d in %d, at most %d", dk, dkp, DC_MAX_DK);
+    ILM_REQUIRE(row_stride % 4 == 0 && (((uintptr_t)rows | (uintptr_t)pool | (uintptr_t)ws) & 15) == 0, "delta_chunks: rows must be 16-byte aligned");
+    const int slots = T_ / DC + R, dvp = (dv + 15) / 16 * 16;
+    ILM_REQUIRE(slots <= 65535 && ws != nullptr, "delta_chunks: %d chunks in a step, at most 65535", slots);
+    const size_t sh = (size_t)slots * H;
+    float* ws_v = (float*)ws;
+    float* ws_w = ws_v + sh * DC * dvp;
+    float* ws_k = ws_w + sh * DC * dkp;
+    float* ws_p = ws_k + sh * DC * dkp;
+    float* ws_e = ws_p + sh * DC * DC;
+    const dim3 ga(H, slots), gb(8 * ((dvp / 16 * H + 7) / 8), R);
+#define DC_CASE(KT_)                                                                                                                  \
+    case KT_:                                                                                                                         \
+        delta_chunk_prepare_kernel<KT_><<<ga, 256, 0, stream>>>(ws_v, ws_w, ws_k, ws_p, ws_e, (const float*)rows, row_stride,          \
+                                                                (const float*)gates, (const int*)seg_offsets, R, H, G, dv, dvp, min_len); \
+        ILM_LAUNCH_CHECK("delta_chunks (prepare)");                                                                                   \
+        delta_chunk_walk_kernel<KT_><<<gb, 256, 0, stream>>>((float*)o, ws_v, ws_w, ws_k, ws_p, ws_e, (const float*)rows, row_stride,  \
+                                                             (float*)pool, (const int*)state_in, (const int*)state_out,                \
+                                                             (const int*)seg_offsets, H, G, dk, dv, dvp, min_len);                     \
+        break
+    switch (dkp / 16) {
+        DC_CASE(1); DC_CASE(2); DC_CASE(3); DC_CASE(4); DC_CASE(5); DC_CASE(6); DC_CASE(7); DC_CASE(8);
+        default: ILM_REQUIRE(false, "delta_chunks: keys of %d", dk);
+    }
+#undef DC_CASE
+    ILM_LAUNCH_CHECK("delta_chunks (walk)");
     return 0;
 }

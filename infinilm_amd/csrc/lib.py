@@ -77,7 +77,7 @@ _SIGNATURES = {
     "ilm_glu_clamp": [_P, _P, _I, _I, _I, _F, _F, _I, _P],
     "ilm_head_gemm": [_P, _P, _P, _I, _I, _I, _I, _L, _L, _L, _L, _L, _L, _L, _I, _I, _P],
     "ilm_head_gemm_mfma": [_P, _P, _P, _I, _I, _I, _I, _L, _L, _L, _L, _L, _L, _L, _P],
-    "ilm_group_norm_gate": [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _I, _I, _I, _I, _L, _F, _P],
+    "ilm_group_norm_gate": [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _I, _I, _I, _I, _L, _F, _I, _P],
     "ilm_causal_conv": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P],
     "ilm_ssm_steps": [_P, _P, _P, _P, _P, _I, _I, _I, _I, _P],
     "ilm_unit_qk_kvwrite": [_P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _F, _I, _I, _P],
@@ -87,6 +87,7 @@ _SIGNATURES = {
     "ilm_conv_norm_rope_kvwrite": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _F,
                                    _I, _I, _I, _P],
     "ilm_delta_step": [_P, _P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P, _P, _I, _F, _I, _I, _I, _I, _P],
+    "ilm_delta_chunks": [_P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P, _P],
     "ilm_norm_add_norm": [_P, _P, _P, _P, _P, _I, _I, _F, _F, _F, _I, _I, _I, _I, _I, _L, _P],
 }
 
@@ -129,6 +130,8 @@ def load(verbose: bool = True) -> ctypes.CDLL:
     lib.ilm_attn_maps_mfma_ok.argtypes = [c_int, c_int, c_int, c_int, c_int, c_int]
     lib.ilm_delta_step_norm_ok.restype = c_int
     lib.ilm_delta_step_norm_ok.argtypes = [c_int, c_int]
+    lib.ilm_delta_chunk_ws.restype = c_int
+    lib.ilm_delta_chunk_ws.argtypes = [c_int, c_int]
     lib.ilm_attn_static_init.restype = c_int
     lib.ilm_attn_static_init.argtypes = []
     lib.ilm_attn_static_scratch_floats.restype = c_long

@@ -667,7 +667,7 @@ extern "C" int ilm_decay_scan(void* o, int o_stride, const void* q, const void* 
 // ------------------------------------------------------------------------------------------
 // RMS norm in groups with an optional gate, one wave (groups up to 512 elements) or one block a (row, group):
 //   y = x * act(gate)            (gate_before)
-//   y = y / sqrt(mean_group(y^2) + eps) * (w + w_offset)       (w may be absent)
+//   y = y / sqrt(mean_group(y^2) + eps) * (w + w_offset)       (w may be absent; w_gstride 0: one weight of a group's size for all groups)
 //   y = y * act(gate)            (otherwise)
 // Sums run over a group in an order that depends on its size only.
 // ------------------------------------------------------------------------------------------
@@ -676,7 +676,7 @@ __global__ void __launch_bounds__(256)
 group_norm_gate_kernel(void* __restrict__ out, const void* __restrict__ x, const void* __restrict__ gate,
                        const void* __restrict__ w, int rows, int n, int groups, int x_stride, int gate_stride,
                        int out_stride, float eps, int gate_act, int gate_before, int out_dt, int x_dt, int gate_dt, int w_dt,
-                       int parts, size_t pstride, float w_offset) {
+                       int parts, size_t pstride, float w_offset, int w_gstride) {
     __shared__ float red[4];
     const int item = LANES == 64 ? blockIdx.x * 4 + (threadIdx.x >> 6) : blockIdx.x;
     const int lane = LANES == 64 ? (threadIdx.x & 63) : threadIdx.x;
@@ -699,24 +699,24 @@ group_norm_gate_kernel(void* __restrict__ out, const void* __restrict__ x, const
         for (int p = 1; p < parts; ++p) y += ldf(x, x_dt, p * pstride + xb + j);
         if (pre) y *= act_f(ldf(gate, gate_dt, gb + j), gate_act);
         y *= rstd;
-        if (w != nullptr) y *= ldf(w, w_dt, (size_t)g * gs + j) + w_offset;
+        if (w != nullptr) y *= ldf(w, w_dt, (size_t)g * w_gstride + j) + w_offset;
         if (gate != nullptr && !gate_before) y *= act_f(ldf(gate, gate_dt, gb + j), gate_act);
         stf(out, out_dt, ob + j, y);
     }
 }
 
 // The same with eight elements a thread and the group in registers between the sum and the stores: groups in multiples
-// of 8 up to 8 * LANES * NITER elements, rows 16 bytes aligned.
+// of 8 up to 8 * LANES * NITER elements, rows 16 bytes aligned.  Groups of up to 128 elements take 16 lanes each.
 template <int LANES, int NITER>
 __global__ void __launch_bounds__(256)
 group_norm_gate_vec_kernel(void* __restrict__ out, const void* __restrict__ x, const void* __restrict__ gate,
                            const void* __restrict__ w, int rows, int n, int groups, int x_stride, int gate_stride,
                            int out_stride, float eps, int gate_act, int gate_before, int out_dt, int x_dt, int gate_dt, int w_dt,
-                           int parts, size_t pstride, float w_offset) {
+                           int parts, size_t pstride, float w_offset, int w_gstride) {
     __shared__ float red[4];
-    const int item = LANES == 64 ? blockIdx.x * 4 + (threadIdx.x >> 6) : blockIdx.x;
-    const int lane = LANES == 64 ? (threadIdx.x & 63) : threadIdx.x;
-    if (item >= rows * groups) return;
+    const int item = LANES < 256 ? (int)(blockIdx.x * (256 / LANES) + threadIdx.x / LANES) : (int)blockIdx.x;
+    const int lane = threadIdx.x % LANES;
+    if (item >= rows * groups) return;      // (whole waves, or whole groups of the 16 lanes that fold together)
     const int t = item / groups, g = item % groups, gs = n / groups;
     const size_t xb = (size_t)t * x_stride + (size_t)g * gs, gb = (size_t)t * gate_stride + (size_t)g * gs;
     const size_t ob = (size_t)t * out_stride + (size_t)g * gs;
@@ -744,7 +744,12 @@ group_norm_gate_vec_kernel(void* __restrict__ out, const void* __restrict__ x, c
             for (int e = 0; e < 8; ++e) ss = fmaf(v[it][e], v[it][e], ss);
         }
     }
-    ss = LANES == 64 ? wave_sum(ss) : block_sum<4>(ss, red);
+    if constexpr (LANES == 16) {
+#pragma unroll
+        for (int off = 1; off < 16; off <<= 1) ss += __shfl_xor(ss, off, 64);
+    } else {
+        ss = LANES == 64 ? wave_sum(ss) : block_sum<4>(ss, red);
+    }
     const float rstd = 1.0f / sqrtf(ss / (float)gs + eps);
 #pragma unroll
     for (int it = 0; it < NITER; ++it) {
@@ -755,7 +760,7 @@ group_norm_gate_vec_kernel(void* __restrict__ out, const void* __restrict__ x, c
             for (int e = 0; e < 8; ++e) o8[e] = v[it][e] * rstd;
             if (w != nullptr) {
                 float wt[8];
-                ld8(w, w_dt, (size_t)g * gs + j, wt);
+                ld8(w, w_dt, (size_t)g * w_gstride + j, wt);
 #pragma unroll
                 for (int e = 0; e < 8; ++e) o8[e] *= wt[e] + w_offset;
             }
@@ -773,7 +778,7 @@ group_norm_gate_vec_kernel(void* __restrict__ out, const void* __restrict__ x, c
 extern "C" int ilm_group_norm_gate(void* out, const void* x, const void* gate, const void* w, int rows, int n, int groups,
                                    int x_stride, int gate_stride, int out_stride, float eps, int gate_act, int gate_before,
                                    int out_dt, int x_dt, int gate_dt, int w_dt, int parts, long pstride, float w_offset,
-                                   hipStream_t stream) {
+                                   int w_gstride, hipStream_t stream) {
     ILM_REQUIRE(parts >= 1, "group_norm_gate: %d parts", parts);
     ILM_REQUIRE(rows > 0 && n > 0 && groups > 0 && n % groups == 0, "group_norm_gate: %d elements do not divide into %d groups", n, groups);
     ILM_REQUIRE((long)rows * groups < (1L << 31) - 4, "group_norm_gate: too many rows");
@@ -782,8 +787,9 @@ extern "C" int ilm_group_norm_gate(void* out, const void* x, const void* gate, c
                     && (((uintptr_t)out | (uintptr_t)x | (uintptr_t)gate | (uintptr_t)w) & 15) == 0;
     if (al && gs_ <= 8192) {
 #define GN_ARGS out, x, gate, w, rows, n, groups, x_stride, gate_stride, out_stride, eps, gate_act, gate_before, out_dt, x_dt, gate_dt, \
-                w_dt, parts, (size_t)pstride, w_offset
-        if (gs_ <= 512) group_norm_gate_vec_kernel<64, 1><<<(rows * groups + 3) / 4, 256, 0, stream>>>(GN_ARGS);
+                w_dt, parts, (size_t)pstride, w_offset, w_gstride
+        if (gs_ <= 128) group_norm_gate_vec_kernel<16, 1><<<(unsigned)(((long)rows * groups + 15) / 16), 256, 0, stream>>>(GN_ARGS);
+        else if (gs_ <= 512) group_norm_gate_vec_kernel<64, 1><<<(rows * groups + 3) / 4, 256, 0, stream>>>(GN_ARGS);
         else if (gs_ <= 2048) group_norm_gate_vec_kernel<256, 1><<<rows * groups, 256, 0, stream>>>(GN_ARGS);
         else if (gs_ <= 4096) group_norm_gate_vec_kernel<256, 2><<<rows * groups, 256, 0, stream>>>(GN_ARGS);
         else group_norm_gate_vec_kernel<256, 4><<<rows * groups, 256, 0, stream>>>(GN_ARGS);
@@ -793,11 +799,11 @@ extern "C" int ilm_group_norm_gate(void* out, const void* x, const void* gate, c
     }
     if (n / groups > 512) {
         group_norm_gate_kernel<256><<<rows * groups, 256, 0, stream>>>(out, x, gate, w, rows, n, groups, x_stride, gate_stride,
-                                                                       out_stride, eps, gate_act, gate_before, out_dt, x_dt, gate_dt, w_dt, parts, (size_t)pstride, w_offset);
+                                                                       out_stride, eps, gate_act, gate_before, out_dt, x_dt, gate_dt, w_dt, parts, (size_t)pstride, w_offset, w_gstride);
     } else {
         const int blocks = (int)(((long)rows * groups + 3) / 4);
         group_norm_gate_kernel<64><<<blocks, 256, 0, stream>>>(out, x, gate, w, rows, n, groups, x_stride, gate_stride, out_stride,
-                                                               eps, gate_act, gate_before, out_dt, x_dt, gate_dt, w_dt, parts, (size_t)pstride, w_offset);
+                                                               eps, gate_act, gate_before, out_dt, x_dt, gate_dt, w_dt, parts, (size_t)pstride, w_offset, w_gstride);
     }
     ILM_LAUNCH_CHECK("group_norm_gate");
     return 0;

@@ -1165,7 +1165,7 @@ def group_norm_gate(x: torch.Tensor, weight: Optional[torch.Tensor], eps: float,
                     gate: Optional[torch.Tensor] = None, gate_act: str = "none", gate_before: bool = False,
                     out_dtype: Optional[torch.dtype] = None, weight_offset: float = 0.0) -> torch.Tensor:
     """RMS norm of every row in `groups` equal parts (each by its own root mean square, eps inside the root), times
-    `weight` [n] (+ `weight_offset`) if given; `gate` [T, n]: times act(gate), before the norm or after it.  Sums in float32.
+    `weight` [n] (or one [n / groups] for all parts; + `weight_offset`) if given; `gate` [T, n]: times act(gate), before the norm or after it.  Sums in float32.
     x may come as contiguous parts [P, T, n] that are summed first (a product that was split over K)."""
     _dev(x, weight, gate)
     parts, pstride = 1, 0
@@ -1177,8 +1177,8 @@ def group_norm_gate(x: torch.Tensor, weight: Optional[torch.Tensor], eps: float,
     T, n = x.shape
     if groups <= 0 or n % groups:
         raise KernelError(f"rows of {n} do not divide into {groups} groups")
-    if weight is not None and (weight.shape != (n,) or not weight.is_contiguous()):
-        raise KernelError(f"norm weight has shape {tuple(weight.shape)}, expected ({n},)")
+    if weight is not None and (weight.shape not in ((n,), (n // groups,)) or not weight.is_contiguous()):
+        raise KernelError(f"norm weight has shape {tuple(weight.shape)}, expected ({n},) or ({n // groups},)")
     if gate is not None:
         _rows(gate, "gate")
         if gate.shape != (T, n):
@@ -1187,7 +1187,7 @@ def group_norm_gate(x: torch.Tensor, weight: Optional[torch.Tensor], eps: float,
     _run("ilm_group_norm_gate", out.data_ptr(), x.data_ptr(), _ptr(gate), _ptr(weight), T, n, int(groups), x.stride(0),
          gate.stride(0) if gate is not None else 0, out.stride(0), float(eps), activation_code(gate_act), int(bool(gate_before)),
          _dt(out), _dt(x), _dt(gate) if gate is not None else 0, _dt(weight) if weight is not None else 0, parts, pstride,
-         float(weight_offset), _stream())
+         float(weight_offset), n // groups if weight is not None and weight.shape[0] == n else 0, _stream())
     return out
 
 
@@ -2097,6 +2097,9 @@ def conv_norm_rope_kvwrite(x: torch.Tensor, weight: Optional[torch.Tensor], pool
 
 # ---- the gated delta rule --------------------------------------------------------------------------------------------------
 DELTA_MAX_KEY_DIM = 512      # (ilm_delta_max_dk())
+DELTA_CHUNK = 64             # tokens a chunk of a long segment (ilm_delta_chunk())
+DELTA_CHUNK_MAX_KEY_DIM = 128    # (ilm_delta_chunk_max_dk())
+DELTA_CHUNK_FROM = int(os.environ.get("INFINILM_AMD_DELTA_CHUNK_FROM", "32"))   # segments from this length on go in chunks (0: never)
 
 
 def delta_rule(rows: torch.Tensor, gates: torch.Tensor, heads: int, groups: int, dk: int, dv: int, pool: torch.Tensor,
@@ -2104,7 +2107,9 @@ def delta_rule(rows: torch.Tensor, gates: torch.Tensor, heads: int, groups: int,
                gate: torch.Tensor, eps: float, out_dtype: torch.dtype, max_len: Optional[int] = None) -> torch.Tensor:
     """S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q per head and token of every segment, then
     o / sqrt(mean(o^2) + eps) * norm_weight [dv] * silu(gate) per head, [T, heads dv] as `out_dtype`.  `rows`, `gates` as
-    `conv_delta_inputs` leaves them; `gate` [T, heads dv]; `pool` [rows, heads, dv, dk] float32: segment r starts from row
+    `conv_delta_inputs` leaves them; `gate` [T, heads dv]; `max_len`: a bound on the segments' lengths known on the host: from
+    DELTA_CHUNK_FROM tokens on, segments go in chunks on the float matrix instruction (the result differs from the token-by-token
+    form by rounding); `pool` [rows, heads, dv, dk] float32: segment r starts from row
     state_in[r] and leaves its state in row state_out[r]."""
     _dev(rows, gates, pool, state_in, state_out, seg_offsets, norm_weight, gate)
     T = rows.shape[0]
@@ -2125,12 +2130,17 @@ def delta_rule(rows: torch.Tensor, gates: torch.Tensor, heads: int, groups: int,
         raise KernelError(f"gate {tuple(gate.shape)} or norm weight {tuple(norm_weight.shape)} does not fit {heads} heads of {dv}")
     step = (rows.data_ptr(), rows.stride(0), gates.data_ptr(), pool.data_ptr(), state_in.data_ptr(), state_out.data_ptr(), seg_offsets.data_ptr(),
             int(segments), heads, groups, dk, dkp, dv)
-    if _lib().ilm_delta_step_norm_ok(dk, dv):
+    slots = T // DELTA_CHUNK + int(segments)
+    chunked = DELTA_CHUNK_FROM > 0 and max_len is not None and max_len >= DELTA_CHUNK_FROM and dk <= DELTA_CHUNK_MAX_KEY_DIM and slots <= 65535
+    if not chunked and _lib().ilm_delta_step_norm_ok(dk, dv):
         y = torch.empty((T, heads * dv), dtype=out_dtype, device=rows.device)
         _run("ilm_delta_step", None, y.data_ptr(), *step, 1 << 30, norm_weight.data_ptr(), gate.data_ptr(), gate.stride(0), float(eps),
              y.stride(0), _dt(y), _dt(norm_weight), _dt(gate), _stream())
         return y
     o = torch.empty((T, heads * dv), dtype=F32, device=rows.device)
-    _run("ilm_delta_step", o.data_ptr(), None, *step, 1 << 30, None, None, 0, 0.0, 0, 0, 0, 0, _stream())
-    return group_norm_gate(o.view(T * heads, dv), norm_weight, eps, 1, gate=gate.reshape(T * heads, dv), gate_act="silu",
-                           out_dtype=out_dtype).view(T, heads * dv)
+    if chunked:
+        ws = torch.empty((slots * heads * _lib().ilm_delta_chunk_ws(dkp, -(-dv // 16) * 16),), dtype=F32, device=rows.device)
+        _run("ilm_delta_chunks", o.data_ptr(), *step, T, DELTA_CHUNK_FROM, ws.data_ptr(), _stream())
+    if not chunked or segments > 1:
+        _run("ilm_delta_step", o.data_ptr(), None, *step, DELTA_CHUNK_FROM - 1 if chunked else 1 << 30, None, None, 0, 0.0, 0, 0, 0, 0, _stream())
+    return group_norm_gate(o, norm_weight, eps, heads, gate=gate, gate_act="silu", out_dtype=out_dtype)

@@ -165,7 +165,7 @@ def forward(cfg: dict, W: Dict[str, torch.Tensor], tokens: List[int], return_lay
 def _forward(cfg, W, tokens, return_layers):
     W = {k: v.to(F64) for k, v in W.items()}
     eps = float(cfg["norm"]["eps"])
-    x = W["embed"][torch.tensor(tokens)] * float(cfg["embedding"]["scale"])
+    x = W["embed"][torch.tensor(tokens)] * float(cfg.get("embedding", {}).get("scale", 1.0))
     X = x[None].repeat(int(cfg["streams"]), 1, 1)
     pos = torch.arange(len(tokens))
     kvs, layers = {}, []
@@ -223,4 +223,74 @@ def tensor_shapes(cfg: dict) -> Dict[str, tuple]:
             out.update({f"l{i}.mlp.gate": (ff, Wd), f"l{i}.mlp.up": (ff, Wd), f"l{i}.mlp.down": (Wd, ff)})
     out["final.norm"] = (Wd,)
     out["head"] = (int(cfg["vocab"]), Wd)
+    return out
+
+
+# ---- configurations and weights for tests --------------------------------------------------------------------------------
+def config_a():
+    """Odd sizes, three streams, a reader with wider chunks (and other taps) than its writer."""
+    att = {"heads": 4, "kv_heads": 2, "dim": 12, "vdim": 20, "scale": 0.35, "conv": 3, "rot": {"base": 100.0, "dims": 6}}
+    return {"architecture": "Moputar", "vocab": 97, "width": 60, "streams": 3, "embedding": {"scale": 2.5}, "norm": {"eps": 1e-5}, "layers": [
+        {"type": "attention", "mixer": dict(att, mask={"size": 20}), "mlp": {"kind": "dense", "ff": 44}},
+        {"type": "delta", "mixer": {"heads": 6, "kv_heads": 2, "dim": 10, "vdim": 14, "conv": 2}, "mlp": None},
+        {"type": "attention", "mixer": dict(att, mask={"size": 33}, kv_from=0, conv=2), "mlp": None},
+        {"type": "delta", "mixer": {"heads": 2, "kv_heads": 2, "dim": 24, "vdim": 8, "conv": 5}, "mlp": {"kind": "dense", "ff": 30}}]}
+
+
+def config_b():
+    """One stream, no embedding scale, layers without convolution, mask or rotation, one head, a writer that keeps all keys for
+    itself and a reader with chunks."""
+    att = {"heads": 3, "kv_heads": 3, "dim": 16, "vdim": 8, "scale": 0.3}
+    return {"architecture": "Moputar", "vocab": 130, "width": 96, "streams": 1, "norm": {"eps": 1e-6}, "layers": [
+        {"type": "delta", "mixer": {"heads": 1, "kv_heads": 1, "dim": 7, "vdim": 9, "conv": 1}, "mlp": {"kind": "dense", "ff": 72}},
+        {"type": "attention", "mixer": dict(att), "mlp": None},
+        {"type": "attention", "mixer": dict(att, mask={"size": 50}, kv_from=1), "mlp": {"kind": "dense", "ff": 40}},
+        {"type": "attention", "mixer": {"heads": 2, "kv_heads": 1, "dim": 48, "vdim": 48, "scale": 0.2, "rot": {"base": 10000.0, "dims": 48},
+                                        "conv": 4}, "mlp": None},
+        {"type": "delta", "mixer": {"heads": 3, "kv_heads": 1, "dim": 40, "vdim": 20, "conv": 8}, "mlp": None}]}
+
+
+def config_c():
+    """Sizes the matrix-core kernels take, six streams."""
+    att = {"heads": 8, "kv_heads": 2, "dim": 64, "vdim": 64, "scale": 0.15, "conv": 4, "rot": {"base": 5000.0, "dims": 32}}
+    return {"architecture": "Moputar", "vocab": 200, "width": 128, "streams": 6, "embedding": {"scale": 8.0}, "norm": {"eps": 1e-5}, "layers": [
+        {"type": "delta", "mixer": {"heads": 4, "kv_heads": 2, "dim": 64, "vdim": 32, "conv": 4}, "mlp": {"kind": "dense", "ff": 256}},
+        {"type": "attention", "mixer": dict(att, mask={"size": 96}), "mlp": {"kind": "dense", "ff": 128}},
+        {"type": "attention", "mixer": dict(att, mask={"size": 40}, kv_from=1), "mlp": None},
+        {"type": "delta", "mixer": {"heads": 2, "kv_heads": 1, "dim": 128, "vdim": 128, "conv": 3}, "mlp": None}]}
+
+
+CONFIGS = {"A": config_a, "B": config_b, "C": config_c}
+
+
+def random_weights(cfg: dict, seed: int) -> Dict[str, torch.Tensor]:
+    """float32 tensors of a size that keeps every mechanism at work: streams that differ, decays spread over (0, 1)."""
+    g = torch.Generator().manual_seed(seed)
+    out, n = {}, int(cfg["streams"])
+    for name, shape in tensor_shapes(cfg).items():
+        leaf = name.split(".")[-1]
+        r = torch.randn(shape, generator=g)
+        if leaf in ("norm1", "norm2") or name == "final.norm":
+            t = 0.2 * r
+        elif leaf == "norm":
+            t = 1.0 + 0.3 * r
+        elif leaf == "in":
+            t = 1.0 / n + 0.2 * r
+        elif leaf == "out":
+            t = 1.0 + 0.3 * r
+        elif leaf == "mix" and ".hc" in name:
+            t = 0.9 * torch.eye(n) + 0.3 * r / math.sqrt(n)
+        elif leaf == "A_log":
+            t = torch.log(0.05 + 1.5 * torch.rand(shape, generator=g))
+        elif leaf == "dt_bias":
+            t = -2.5 + r
+        elif leaf == "conv":
+            t = 0.6 * r
+        elif name == "embed":
+            t = r / float(cfg.get("embedding", {}).get("scale", 1.0))
+        elif len(shape) == 2:
+            t = r * (1.3 / math.sqrt(shape[1]))
+        else:
+            t = r
+        out[name] = t
     return out
