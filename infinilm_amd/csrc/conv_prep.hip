@@ -50,12 +50,16 @@ __device__ __forceinline__ void cp_store(T* p, const float (&v)[VEC]) {
     }
 }
 
+// x * sigmoid(x) on the hardware's exponential and reciprocal (each within an ulp)
+__device__ __forceinline__ float cp_silu(float x) { return x * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * x)); }
+
 // Blocks go to the eight dies in turn: with this numbering a die takes a run of consecutive tokens, whose convolutions read
 // the same rows.  A grid of cp_blocks(T) blocks; block numbers beyond the last token give -1.
 __device__ __forceinline__ int cp_token(int T_) {
     const int per = (T_ + 7) / 8, t = (int)(blockIdx.x & 7) * per + (int)(blockIdx.x >> 3);
     return (int)(blockIdx.x >> 3) < per && t < T_ ? t : -1;
 }
+
 static inline unsigned cp_blocks(int T_) { return 8u * (unsigned)((T_ + 7) / 8); }
 
 // What a block needs to know of its token's request
@@ -162,10 +166,9 @@ conv_delta_inputs_kernel(float* __restrict__ out, float* __restrict__ gates, con
         float y[VEC];
         cp_conv<VEC, T>(y, x, x_stride, w, t, c, C, taps, p);
 #pragma unroll
-        for (int e = 0; e < VEC; ++e) y[e] = y[e] / (1.0f + expf(-y[e]));
+        for (int e = 0; e < VEC; ++e) y[e] = cp_silu(y[e]);
         if (c < nqk) {
-#pragma unroll
-            for (int e = 0; e < VEC; ++e) qk[c + e] = y[e];
+            cp_store<VEC, float>(qk + c, y);
         } else {
             cp_store<VEC, float>(orow + 2 * G * dkp + (c - nqk), y);
         }
@@ -183,6 +186,82 @@ conv_delta_inputs_kernel(float* __restrict__ out, float* __restrict__ gates, con
         for (int e = lane; e < dk; e += 64) ss = fmaf(qk[u * dk + e], qk[u * dk + e], ss);
         const float f = (u < G ? q_scale : 1.0f) / sqrtf(wave_sum(ss) + unit_eps);
         for (int e = lane; e < dkp; e += 64) orow[u * dkp + e] = e < dk ? qk[u * dk + e] * f : 0.f;
+    }
+}
+
+// The same without LDS where a head is a power of two of pieces of 8 entries (keys of 16 to 512), convolutions of 1 to 4 taps: a
+// thread keeps the taps of its 8 channels and walks TB consecutive tokens, whose rows are all on their way from the start; a
+// head's sum of squares is folded over its lanes.
+template <typename T, int TB, int TAPS>
+__global__ void __launch_bounds__(256)
+conv_delta_inputs_fast_kernel(float* __restrict__ out, float* __restrict__ gates, const T* __restrict__ x, const T* __restrict__ w,
+                              float* __restrict__ pool, const int* __restrict__ state_in, const int* __restrict__ state_out,
+                              const int* __restrict__ seg, const int* __restrict__ seg_offsets, const float* __restrict__ a_log,
+                              const float* __restrict__ dt_bias, int T_, int H, int G, int dk, int dv, int x_stride, int out_stride,
+                              int b_off, int a_off, float q_scale, float unit_eps) {
+    const int grp = cp_token((T_ + TB - 1) / TB);
+    if (grp < 0) return;
+    const int tb = grp * TB;
+    const int nqk = 2 * G * dk, C = nqk + H * dv, lanes = dk >> 3;
+    if (blockIdx.y == 0)
+        for (int i = threadIdx.x; i < TB * H; i += 256) {
+            const int t = tb + i / H, h = i % H;
+            if (t >= T_) break;
+            const float b = to_f32(x[(size_t)t * x_stride + b_off + h]);
+            const float z = to_f32(x[(size_t)t * x_stride + a_off + h]) + dt_bias[h];
+            const float sp = z > 20.0f ? z : log1pf(expf(z));
+            gates[(size_t)t * 2 * H + h] = 1.0f / (1.0f + expf(-b));
+            gates[(size_t)t * 2 * H + H + h] = -expf(a_log[h]) * sp;
+        }
+    const int c = (blockIdx.y * 256 + threadIdx.x) * 8;
+    if (c >= C) return;                     // (values' lanes: no head's sum misses them)
+    float own[TB][8], wv[TAPS][8];
+#pragma unroll
+    for (int i = 0; i < TB; ++i) cp_load<8, T>(x + (size_t)(tb + i < T_ ? tb + i : T_ - 1) * x_stride + c, own[i]);
+#pragma unroll
+    for (int i = 0; i < TAPS; ++i) cp_load<8, T>(w + (size_t)i * C + c, wv[i]);
+    float win[TAPS > 1 ? TAPS - 1 : 1][8];
+#pragma unroll
+    for (int i = 0; i < TB; ++i) {
+        const int t = tb + i;
+        if (t >= T_) return;
+        const cp_place p = cp_find(t, seg, seg_offsets, state_in, state_out, pool, TAPS, C);
+        if constexpr (TAPS > 1) {
+            if (i == 0 || p.j == 0) {
+#pragma unroll
+                for (int m = 0; m < TAPS - 1; ++m) {
+                    const int back = TAPS - 1 - m;
+                    if (back <= p.j) cp_load<8, T>(x + (size_t)(t - back) * x_stride + c, win[m]);
+                    else cp_load<8, float>(p.in + (size_t)(TAPS - 1 - (back - p.j)) * C + c, win[m]);
+                }
+            }
+        }
+        float y[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            y[e] = 0.f;
+#pragma unroll
+            for (int m = 0; m < TAPS - 1; ++m) y[e] = fmaf(wv[m][e], win[m][e], y[e]);
+            y[e] = cp_silu(fmaf(wv[TAPS - 1][e], own[i][e], y[e]));
+        }
+        if (c < nqk) {                      // (the lanes of a head agree)
+            float ss = 0.f;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) ss = fmaf(y[e], y[e], ss);
+            for (int off = 1; off < lanes; off <<= 1) ss += __shfl_xor(ss, off, 64);
+            const float f = (c < G * dk ? q_scale : 1.0f) / sqrtf(ss + unit_eps);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) y[e] *= f;
+        }
+        cp_store<8, float>(out + (size_t)t * out_stride + c, y);
+        if constexpr (TAPS > 1) {
+#pragma unroll
+            for (int m = 0; m < TAPS - 1; ++m) {
+#pragma unroll
+                for (int e = 0; e < 8; ++e) win[m][e] = m + 1 < TAPS - 1 ? win[m + 1 < TAPS - 1 ? m + 1 : 0][e] : own[i][e];
+                if (p.only) cp_store<8, float>(p.out + (size_t)m * C + c, win[m]);
+            }
+        }
     }
 }
 
@@ -204,6 +283,28 @@ extern "C" int ilm_conv_delta_inputs(void* out, void* gates, const void* x, cons
     const bool vec = dk % 4 == 0 && (G * dk) % 4 == 0 && nqk % 8 == 0 && C % 8 == 0 && x_stride % 8 == 0 && out_stride % 4 == 0 && (2 * G * dkp) % 4 == 0
                      && (((uintptr_t)x | (uintptr_t)w | (uintptr_t)pool | (uintptr_t)out) & 15) == 0;
     const bool wide = T_ <= 2 * ilm_num_cus();
+    const bool fast = vec && dk == dkp && (dk & (dk - 1)) == 0 && dk >= 16 && dk <= 512 && dv % 8 == 0 && taps >= 1 && taps <= 4;
+    if (fast) {
+        const int TB = T_ >= 8 * 64 ? 8 : 1;
+        const dim3 grid(cp_blocks((T_ + TB - 1) / TB), (C / 8 + 255) / 256);
+#define CF_ARGS(T__) (float*)out, (float*)gates, (const T__*)x, (const T__*)w, (float*)pool, (const int*)state_in, (const int*)state_out, \
+                     (const int*)seg, (const int*)seg_offsets, (const float*)a_log, (const float*)dt_bias, T_, H, G, dk, dv, x_stride,  \
+                     out_stride, b_off, a_off, q_scale, unit_eps
+#define CF_TAPS(T__, TAPS_)                                                                                                          \
+    case TAPS_:                                                                                                                      \
+        if (TB == 8) conv_delta_inputs_fast_kernel<T__, 8, TAPS_><<<grid, 256, 0, stream>>>(CF_ARGS(T__));                           \
+        else conv_delta_inputs_fast_kernel<T__, 1, TAPS_><<<grid, 256, 0, stream>>>(CF_ARGS(T__));                                   \
+        break
+        if (dtype == ILM_DTYPE_F32) {
+            switch (taps) { CF_TAPS(float, 1); CF_TAPS(float, 2); CF_TAPS(float, 3); CF_TAPS(float, 4); }
+        } else if (dtype == ILM_DTYPE_BF16) {
+            switch (taps) { CF_TAPS(bf16, 1); CF_TAPS(bf16, 2); CF_TAPS(bf16, 3); CF_TAPS(bf16, 4); }
+        } else {
+            ILM_REQUIRE(false, "conv_delta_inputs: unknown dtype %d", dtype);
+        }
+#undef CF_TAPS
+#undef CF_ARGS
+    } else {
 #define CD_ARGS(T__) (float*)out, (float*)gates, (const T__*)x, (const T__*)w, (float*)pool, (const int*)state_in, (const int*)state_out, \
                      (const int*)seg, (const int*)seg_offsets, (const float*)a_log, (const float*)dt_bias, T_, H, G, dk, dkp, dv, taps,  \
                      x_stride, out_stride, b_off, a_off, q_scale, unit_eps
@@ -213,11 +314,12 @@ extern "C" int ilm_conv_delta_inputs(void* out, void* gates, const void* x, cons
         else if (vec) conv_delta_inputs_kernel<8, T__, 256><<<cp_blocks(T_), 256, nqk * 4, stream>>>(CD_ARGS(T__));                 \
         else conv_delta_inputs_kernel<1, T__, 256><<<cp_blocks(T_), 256, nqk * 4, stream>>>(CD_ARGS(T__));                          \
     } while (0)
-    if (dtype == ILM_DTYPE_F32) CD_LAUNCH(float);
-    else if (dtype == ILM_DTYPE_BF16) CD_LAUNCH(bf16);
-    else ILM_REQUIRE(false, "conv_delta_inputs: unknown dtype %d", dtype);
+        if (dtype == ILM_DTYPE_F32) CD_LAUNCH(float);
+        else if (dtype == ILM_DTYPE_BF16) CD_LAUNCH(bf16);
+        else ILM_REQUIRE(false, "conv_delta_inputs: unknown dtype %d", dtype);
 #undef CD_LAUNCH
 #undef CD_ARGS
+    }
     ILM_LAUNCH_CHECK("conv_delta_inputs");
     if (taps > 1 && !singles)
         return dtype == ILM_DTYPE_F32 ? cp_state<float>(x, pool, state_in, state_out, seg_offsets, R, C, taps, x_stride, stream)
@@ -249,11 +351,9 @@ conv_norm_rope_kvwrite_kernel(T* __restrict__ q_out, const T* __restrict__ x, co
         float y[VEC];
         cp_conv<VEC, T>(y, x, x_stride, w, t, c, C, taps, p);
         float s = 0.f;
+        cp_store<VEC, float>(sm + c, y);
 #pragma unroll
-        for (int e = 0; e < VEC; ++e) {
-            sm[c + e] = y[e];
-            s = fmaf(y[e], y[e], s);
-        }
+        for (int e = 0; e < VEC; ++e) s = fmaf(y[e], y[e], s);
         if (c < Cq) sq += s;
         else if (c < Cq + Ck) sk += s;
     }
@@ -282,8 +382,14 @@ conv_norm_rope_kvwrite_kernel(T* __restrict__ q_out, const T* __restrict__ x, co
         const T* wn = is_q ? wq : wk;
         const float f = is_q ? rq : rk;
         float v[8];
+        if constexpr (VEC == 8) {        // (a piece lies inside its head whole, or beyond it whole)
+            cp_load<8, float>(sm + (e0 < dim ? src : 0), v);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) v[e] = e0 + e < dim ? sm[src + e] * f : 0.f;
+            for (int e = 0; e < 8; ++e) v[e] = e0 < dim ? v[e] * f : 0.f;
+        } else {
+#pragma unroll
+            for (int e = 0; e < 8; ++e) v[e] = e0 + e < dim ? sm[src + e] * f : 0.f;
+        }
         if (wn != nullptr) {
             if constexpr (VEC == 8) {
                 if (e0 < dim) {

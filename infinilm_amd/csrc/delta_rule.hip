@@ -7,8 +7,8 @@
 // query/key head h / (H / G)) and [beta: H | log g: H].  A request's state passes from step to step through a row of a pool,
 // [H, dv, dk] (the key index fastest).
 //
-//   ilm_delta_step     token by token, a block a (request, head, columns).  A thread keeps DS_NK consecutive state entries
-//       of VC value columns in registers; the two sums a token needs, S^T k and S^T q (both from the decayed state: the
+//   ilm_delta_step     token by token, a block a (request, head, columns).  A thread keeps DS_NK state entries (two pieces of
+//       four, KP pieces apart, so that the lanes of a column read whole lines) of VC value columns in registers; the two sums a token needs, S^T k and S^T q (both from the decayed state: the
 //       read-out after the write is S^T q + u (k . q)), and k . q are folded over the lanes of a column together.  Where a block
 //       holds all columns of its head it can end with the head's output norm, weight and gate:
 //       y = o / sqrt(mean(o^2) + eps) * w * silu(gate), in the activations' dtype.
@@ -23,7 +23,8 @@
 //       Two kernels: the first makes V', W, the weights of the second sum and the decayed keys of every chunk, all chunks and
 //       heads side by side; the second walks a segment's chunks in order with 16 value columns of a head's state a block.
 //       Differences of L are taken in double, so that a token's decay keeps its float precision however much has been
-//       forgotten before it.  Chunk p of segment r has the workspace slot floor(first row of r / DC) + r + p.
+//       forgotten before it.  What passes from the first to the second lies in memory as the matrix instruction takes it (tiles of
+//       16 x 16, a lane's 16 bytes after another's), so that a wave reads it in whole kilobytes.  Chunk p of segment r has the workspace slot floor(first row of r / DC) + r + p.
 #include "common.h"
 
 typedef __attribute__((ext_vector_type(4))) float f32x4;
@@ -41,39 +42,41 @@ delta_step_kernel(float* __restrict__ o, void* __restrict__ y, const float* __re
     const int h = blockIdx.y, r = blockIdx.z;
     const int t0 = seg_offsets[r], t1 = seg_offsets[r + 1];
     if (t0 >= t1 || t1 - t0 > max_len) return;       // (longer segments are another kernel's)
-    const int kp = threadIdx.x % KP, c0 = (blockIdx.x * (THREADS / KP) + threadIdx.x / KP) * VC, k0 = kp * DS_NK;
+    const int kp = threadIdx.x % KP, c0 = (blockIdx.x * (THREADS / KP) + threadIdx.x / KP) * VC;
     const size_t hs = (size_t)dk * dv;
     const float* src = pool + ((size_t)state_in[r] * H + h) * hs;
     const bool v4 = dk % 4 == 0;
+    // the thread's entries 4 p .. 4 p + 3 are k = kof[p] .. kof[p] + 3
+    const int kof[2] = {4 * kp, 4 * (KP + kp)};
     float S[VC][DS_NK];
 #pragma unroll
     for (int c = 0; c < VC; ++c) {
 #pragma unroll
-        for (int i = 0; i < DS_NK; i += 4) {
-            const bool ok = c0 + c < dv && k0 + i < dk;
-            const float* p = src + (size_t)(c0 + c) * dk + k0 + i;
+        for (int p = 0; p < 2; ++p) {
+            const bool ok = c0 + c < dv && kof[p] < dk;
+            const float* at = src + (size_t)(c0 + c) * dk + kof[p];
             if (v4) {
-                const float4 t = ok ? *reinterpret_cast<const float4*>(p) : make_float4(0.f, 0.f, 0.f, 0.f);
-                S[c][i] = t.x; S[c][i + 1] = t.y; S[c][i + 2] = t.z; S[c][i + 3] = t.w;
+                const float4 t = ok ? *reinterpret_cast<const float4*>(at) : make_float4(0.f, 0.f, 0.f, 0.f);
+                S[c][4 * p] = t.x; S[c][4 * p + 1] = t.y; S[c][4 * p + 2] = t.z; S[c][4 * p + 3] = t.w;
             } else {
 #pragma unroll
-                for (int e = 0; e < 4; ++e) S[c][i + e] = (ok && k0 + i + e < dk) ? p[e] : 0.f;
+                for (int e = 0; e < 4; ++e) S[c][4 * p + e] = (ok && kof[p] + e < dk) ? at[e] : 0.f;
             }
         }
     }
     const int g = h / (H / G);
-    const bool kin = k0 < dkp;                          // (dkp is a multiple of 8: a thread's entries all lie inside, or none does)
-    const float* qp = rows + (size_t)g * dkp + (kin ? k0 : 0);
+    const float* qp = rows + (size_t)g * dkp;           // (dkp is a multiple of 4: a piece lies inside it whole, or beyond it whole)
     const float* kq = qp + (size_t)G * dkp;
     const float* vp = rows + (size_t)2 * G * dkp + (size_t)h * dv;
     for (int t = t0; t < t1; ++t) {
         float q[DS_NK], k[DS_NK], v[VC];
 #pragma unroll
-        for (int i = 0; i < DS_NK; i += 4) {
-            const float4 a = *reinterpret_cast<const float4*>(qp + (size_t)t * row_stride + i);
-            const float4 b = *reinterpret_cast<const float4*>(kq + (size_t)t * row_stride + i);
-            q[i] = kin ? a.x : 0.f; q[i + 1] = kin ? a.y : 0.f; q[i + 2] = kin ? a.z : 0.f; q[i + 3] = kin ? a.w : 0.f;
-            k[i] = kin ? b.x : 0.f; k[i + 1] = kin ? b.y : 0.f; k[i + 2] = kin ? b.z : 0.f; k[i + 3] = kin ? b.w : 0.f;
+        for (int p = 0; p < 2; ++p) {
+            const bool in = kof[p] < dkp;
+            const float4 a = *reinterpret_cast<const float4*>(qp + (size_t)t * row_stride + (in ? kof[p] : 0));
+            const float4 b = *reinterpret_cast<const float4*>(kq + (size_t)t * row_stride + (in ? kof[p] : 0));
+            q[4 * p] = in ? a.x : 0.f; q[4 * p + 1] = in ? a.y : 0.f; q[4 * p + 2] = in ? a.z : 0.f; q[4 * p + 3] = in ? a.w : 0.f;
+            k[4 * p] = in ? b.x : 0.f; k[4 * p + 1] = in ? b.y : 0.f; k[4 * p + 2] = in ? b.z : 0.f; k[4 * p + 3] = in ? b.w : 0.f;
         }
 #pragma unroll
         for (int c = 0; c < VC; ++c) v[c] = vp[(size_t)t * row_stride + (c0 + c < dv ? c0 + c : 0)];
@@ -137,14 +140,14 @@ delta_step_kernel(float* __restrict__ o, void* __restrict__ y, const float* __re
     for (int c = 0; c < VC; ++c)
         if (c0 + c < dv) {
 #pragma unroll
-            for (int i = 0; i < DS_NK; i += 4) {
-                float* p = dst + (size_t)(c0 + c) * dk + k0 + i;
+            for (int p = 0; p < 2; ++p) {
+                float* at = dst + (size_t)(c0 + c) * dk + kof[p];
                 if (v4) {
-                    if (k0 + i < dk) *reinterpret_cast<float4*>(p) = make_float4(S[c][i], S[c][i + 1], S[c][i + 2], S[c][i + 3]);
+                    if (kof[p] < dk) *reinterpret_cast<float4*>(at) = make_float4(S[c][4 * p], S[c][4 * p + 1], S[c][4 * p + 2], S[c][4 * p + 3]);
                 } else {
 #pragma unroll
                     for (int e = 0; e < 4; ++e)
-                        if (k0 + i + e < dk) p[e] = S[c][i + e];
+                        if (kof[p] + e < dk) at[e] = S[c][4 * p + e];
                 }
             }
         }
@@ -242,15 +245,16 @@ __device__ __forceinline__ int dc_find(const int* __restrict__ seg_offsets, int 
 // KT: key entries / 16
 template <int KT>
 __global__ void __launch_bounds__(256)
-delta_chunk_prepare_kernel(float* __restrict__ ws_v, float* __restrict__ ws_w, float* __restrict__ ws_k, float* __restrict__ ws_p,
-                           float* __restrict__ ws_e, const float* __restrict__ rows, int row_stride, const float* __restrict__ gates,
+delta_chunk_prepare_kernel(float4* __restrict__ ws_v, float4* __restrict__ ws_w, float4* __restrict__ ws_q, float4* __restrict__ ws_k,
+                           float4* __restrict__ ws_p, float* __restrict__ ws_e, const float* __restrict__ rows, int row_stride, const float* __restrict__ gates,
                            const int* __restrict__ seg_offsets, int R, int H, int G, int dv, int dvp, int min_len) {
     constexpr int DK = KT * 16, KS = DK + 4, AS = DC + 4, TS = 20;
     __shared__ __attribute__((aligned(16))) float Ks[DC * KS];
     __shared__ __attribute__((aligned(16))) float An[DC * AS];          // -A
     __shared__ __attribute__((aligned(16))) float Ti[4 * 16 * TS];      // inverses of the diagonal blocks of I + A
+    __shared__ __attribute__((aligned(16))) float Tp[4 * 16 * TS];      // a wave's tile on its way into fragment order
     __shared__ double Ls[DC];
-    __shared__ float bs[DC];
+    __shared__ float bs[DC], fs[DC];                                    // beta; exp(L_end - L)
     const int h = blockIdx.x, slot = blockIdx.y;
     int p;
     const int seg = dc_find(seg_offsets, R, slot, p);
@@ -280,6 +284,7 @@ delta_chunk_prepare_kernel(float* __restrict__ ws_v, float* __restrict__ ws_w, f
         }
         Ls[lane] = L;
         bs[lane] = lane < n ? gt[0] : 0.f;
+        fs[lane] = expf((float)(__shfl(L, 63, 64) - L));
         ws_e[sh * DC_EL + lane] = expf((float)L);
         if (lane == 63) ws_e[sh * DC_EL + DC] = expf((float)L);
     }
@@ -287,7 +292,7 @@ delta_chunk_prepare_kernel(float* __restrict__ ws_v, float* __restrict__ ws_w, f
     // ---- k_t . k_i and q_t . k_i by tiles of 16 x 16 at and below the diagonal
     for (int tile = wave; tile < 10; tile += 4) {
         const int rt = tile < 1 ? 0 : (tile < 3 ? 1 : (tile < 6 ? 2 : 3)), ct = tile - rt * (rt + 1) / 2;
-        f32x4 kk = f32x4{0.f, 0.f, 0.f, 0.f}, qk = kk;
+        f32x4 kk = f32x4{0.f, 0.f, 0.f, 0.f}, kq = kk;      // k_t . k_i as [t, i]; k_i . q_t as [i, t]
         const int tq = 16 * rt + r < n ? 16 * rt + r : n - 1;
 #pragma unroll
         for (int j = 0; j < KT; ++j) {
@@ -295,17 +300,19 @@ delta_chunk_prepare_kernel(float* __restrict__ ws_v, float* __restrict__ ws_w, f
             const float4 ka = *reinterpret_cast<const float4*>(&Ks[(16 * rt + r) * KS + 16 * j + 4 * q]);
             const float4 kb = *reinterpret_cast<const float4*>(&Ks[(16 * ct + r) * KS + 16 * j + 4 * q]);
             kk = dc_mmt(ka, kb, kk);
-            qk = dc_mmt(qa, kb, qk);
+            kq = dc_mmt(kb, qa, kq);
+            if (ct == rt) ws_q[((sh * 4 + rt) * KT + j) * 64 + lane] = qa;
         }
-        const int i = 16 * ct + r;
-        const double Li = Ls[i];
+        const double Li = Ls[16 * ct + r], Lt = Ls[16 * rt + r];
+        float4 pw;
+        float* pe = reinterpret_cast<float*>(&pw);
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-            const int t = 16 * rt + 4 * q + e;
-            const float dec = expf(i <= t ? (float)(Ls[t] - Li) : 0.f);
-            An[t * AS + i] = i < t ? -bs[t] * dec * kk[e] : 0.f;
-            ws_p[(sh * DC + t) * DC + i] = (i <= t && t < n) ? dec * qk[e] : 0.f;
+            const int t = 16 * rt + 4 * q + e, i = 16 * ct + 4 * q + e;
+            An[t * AS + 16 * ct + r] = 16 * ct + r < t ? -bs[t] * expf((float)(Ls[t] - Li)) * kk[e] : 0.f;
+            pe[e] = i <= 16 * rt + r ? expf((float)(Lt - Ls[i])) * kq[e] : 0.f;
         }
+        ws_p[((sh * 4 + rt) * 4 + ct) * 64 + lane] = pw;
     }
     __syncthreads();
     if (wave == 0) {      // column r of the inverse of diagonal block q, by substitution
@@ -319,9 +326,15 @@ delta_chunk_prepare_kernel(float* __restrict__ ws_v, float* __restrict__ ws_w, f
         }
 #pragma unroll
         for (int i = 0; i < 16; ++i) Ti[(q * 16 + i) * TS + r] = x[i];
-    } else {              // the decayed keys, transposed
-        const float f = expf((float)(Ls[DC - 1] - Ls[lane]));
-        for (int i = wave - 1; i < DK; i += 3) ws_k[(sh * DK + i) * DC + lane] = f * Ks[lane * KS + i];
+    } else {              // the decayed keys, transposed: tile (m, j) holds keys' entries 16 m .. by tokens 16 j ..
+        for (int i = wave - 1; i < KT * 4; i += 3) {
+            const int m = i >> 2, j = i & 3;
+            float4 v;
+            float* ve = reinterpret_cast<float*>(&v);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) ve[e] = fs[16 * j + 4 * q + e] * Ks[(16 * j + 4 * q + e) * KS + 16 * m + r];
+            ws_k[((sh * KT + m) * 4 + j) * 64 + lane] = v;
+        }
     }
     __syncthreads();
     // ---- (I + A) X = [beta V | beta exp(L) K], DC_XT column tiles of 16 a wave, the rows' blocks one after the other
@@ -362,12 +375,19 @@ delta_chunk_prepare_kernel(float* __restrict__ ws_v, float* __restrict__ ws_w, f
         for (int c = 0; c < DC_XT; ++c) {
             const int ct = c0 + c;
             if (ct >= nt) break;
-            float* dst = ct < nv ? ws_v + sh * DC * dvp + 16 * ct + r : ws_w + sh * DC * DK + 16 * (ct - nv) + r;
-            const int ld = ct < nv ? dvp : DK;
 #pragma unroll
-            for (int i = 0; i < 4; ++i)
+            for (int i = 0; i < 4; ++i) {
+                if (ct < nv) {       // V' as the walk's results lie: rows 4 q .. 4 q + 3 of column r
+                    ws_v[((sh * 4 + i) * nv + ct) * 64 + lane] = make_float4(X[i][c][0], X[i][c][1], X[i][c][2], X[i][c][3]);
+                } else {             // W as an operand: row r, entries 4 q .. 4 q + 3
+                    float* tp = Tp + wave * 16 * TS;
 #pragma unroll
-                for (int e = 0; e < 4; ++e) dst[(size_t)(16 * i + 4 * q + e) * ld] = X[i][c][e];
+                    for (int e = 0; e < 4; ++e) tp[(4 * q + e) * TS + r] = X[i][c][e];
+                    __builtin_amdgcn_wave_barrier();
+                    ws_w[((sh * 4 + i) * KT + ct - nv) * 64 + lane] = *reinterpret_cast<const float4*>(&tp[r * TS + 4 * q]);
+                    __builtin_amdgcn_wave_barrier();
+                }
+            }
         }
     }
 }
@@ -382,39 +402,34 @@ struct dc_operands {
 };
 
 template <int KT>
-__device__ __forceinline__ void dc_load(dc_operands<KT>& o, const float* ws_v, const float* ws_w, const float* ws_k, const float* ws_p,
-                                        const float* ws_e, const float* qhead, int row_stride, size_t sh, int t0, int n, int dvp, int col0,
-                                        int wave, int r, int q) {
-    constexpr int DK = KT * 16;
-    const int row = 16 * wave + r, tq = row < n ? row : n - 1;
+__device__ __forceinline__ void dc_load(dc_operands<KT>& o, const float4* ws_v, const float4* ws_w, const float4* ws_q, const float4* ws_k,
+                                        const float4* ws_p, const float* ws_e, size_t sh, int nv, int blk, int wave, int lane) {
+    // (every piece is 64 consecutive 16-byte entries, one a lane)
 #pragma unroll
     for (int j = 0; j < KT; ++j) {
-        o.w[j] = *reinterpret_cast<const float4*>(ws_w + (sh * DC + row) * DK + 16 * j + 4 * q);
-        o.q[j] = *reinterpret_cast<const float4*>(qhead + (size_t)(t0 + tq) * row_stride + 16 * j + 4 * q);
+        o.w[j] = ws_w[((sh * 4 + wave) * KT + j) * 64 + lane];
+        o.q[j] = ws_q[((sh * 4 + wave) * KT + j) * 64 + lane];
     }
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
         // (blocks above the diagonal are not in memory: the diagonal's own is read in their place and not used)
-        o.p[j] = *reinterpret_cast<const float4*>(ws_p + (sh * DC + row) * DC + 16 * (j <= wave ? j : wave) + 4 * q);
+        o.p[j] = ws_p[((sh * 4 + wave) * 4 + (j <= wave ? j : wave)) * 64 + lane];
 #pragma unroll
-        for (int m = 0; m < dc_operands<KT>::MT; ++m) {
-            const int mt = wave + 4 * m < KT ? wave + 4 * m : KT - 1;
-            o.k[m][j] = *reinterpret_cast<const float4*>(ws_k + (sh * DK + 16 * mt + r) * DC + 16 * j + 4 * q);
-        }
+        for (int m = 0; m < dc_operands<KT>::MT; ++m) o.k[m][j] = ws_k[((sh * KT + (wave + 4 * m < KT ? wave + 4 * m : KT - 1)) * 4 + j) * 64 + lane];
     }
-#pragma unroll
-    for (int e = 0; e < 4; ++e) o.v[e] = ws_v[(sh * DC + 16 * wave + 4 * q + e) * dvp + col0 + r];
-    o.e = *reinterpret_cast<const float4*>(ws_e + sh * DC_EL + 16 * wave + 4 * q);
+    const float4 v = ws_v[((sh * 4 + wave) * nv + blk) * 64 + lane];
+    o.v = f32x4{v.x, v.y, v.z, v.w};
+    o.e = *reinterpret_cast<const float4*>(ws_e + sh * DC_EL + 16 * wave + 4 * (lane >> 4));
     o.end = ws_e[sh * DC_EL + DC];
 }
 
 template <int KT>
 __global__ void __launch_bounds__(256, 1)
-delta_chunk_walk_kernel(float* __restrict__ out, const float* __restrict__ ws_v, const float* __restrict__ ws_w, const float* __restrict__ ws_k,
-                        const float* __restrict__ ws_p, const float* __restrict__ ws_e, const float* __restrict__ rows, int row_stride,
+delta_chunk_walk_kernel(float* __restrict__ out, const float4* __restrict__ ws_v, const float4* __restrict__ ws_w, const float4* __restrict__ ws_q,
+                        const float4* __restrict__ ws_k, const float4* __restrict__ ws_p, const float* __restrict__ ws_e,
                         float* __restrict__ pool, const int* __restrict__ state_in, const int* __restrict__ state_out,
-                        const int* __restrict__ seg_offsets, int H, int G, int dk, int dv, int dvp, int min_len) {
-    constexpr int DK = KT * 16, MT = dc_operands<KT>::MT;
+                        const int* __restrict__ seg_offsets, int H, int dk, int dv, int dvp, int min_len) {
+    constexpr int MT = dc_operands<KT>::MT;
     __shared__ f32x4 Us[4][64];
     __shared__ f32x4 Ss[KT][64];
     // blocks go to the eight dies in turn; with this numbering the column blocks of a head share a die, whose cache then holds
@@ -428,7 +443,6 @@ delta_chunk_walk_kernel(float* __restrict__ out, const float* __restrict__ ws_v,
     const int chunks = (len + DC - 1) / DC, slot0 = s0 / DC + seg;
     const int lane = threadIdx.x & 63, r = lane & 15, q = lane >> 4;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-    const float* qhead = rows + (size_t)(h / (H / G)) * DK;
     const bool col_ok = col0 + r < dv, v4 = dk % 4 == 0;
     // state tile m: entries 16 m + 4 q + e of column col0 + r; every wave holds all of them
     f32x4 S[KT];
@@ -448,13 +462,12 @@ delta_chunk_walk_kernel(float* __restrict__ out, const float* __restrict__ ws_v,
         }
     }
     dc_operands<KT> cur, nxt;
-    dc_load<KT>(nxt, ws_v, ws_w, ws_k, ws_p, ws_e, qhead, row_stride, (size_t)slot0 * H + h, s0, min(DC, len), dvp, col0, wave, r, q);
+    dc_load<KT>(nxt, ws_v, ws_w, ws_q, ws_k, ws_p, ws_e, (size_t)slot0 * H + h, nb, item % nb, wave, lane);
     for (int c = 0; c < chunks; ++c) {
         cur = nxt;
         const int t0 = s0 + c * DC, n = min(DC, len - c * DC);
         if (c + 1 < chunks)
-            dc_load<KT>(nxt, ws_v, ws_w, ws_k, ws_p, ws_e, qhead, row_stride, (size_t)(slot0 + c + 1) * H + h, t0 + DC, min(DC, len - (c + 1) * DC),
-                        dvp, col0, wave, r, q);
+            dc_load<KT>(nxt, ws_v, ws_w, ws_q, ws_k, ws_p, ws_e, (size_t)(slot0 + c + 1) * H + h, nb, item % nb, wave, lane);
         f32x4 ws = f32x4{0.f, 0.f, 0.f, 0.f}, qs = ws;
 #pragma unroll
         for (int m = 0; m < KT; ++m) {
@@ -512,7 +525,7 @@ delta_chunk_walk_kernel(float* __restrict__ out, const float* __restrict__ ws_v,
 extern "C" int ilm_delta_chunk() { return DC; }
 extern "C" int ilm_delta_chunk_max_dk() { return DC_MAX_DK; }
 // floats of workspace a (slot, head) takes
-extern "C" int ilm_delta_chunk_ws(int dkp, int dvp) { return DC * dvp + 2 * DC * dkp + DC * DC + DC_EL; }
+extern "C" int ilm_delta_chunk_ws(int dkp, int dvp) { return DC * dvp + 3 * DC * dkp + DC * DC + DC_EL; }
 
 // Segments of at least min_len tokens; the others are passed over.  ws: (T / DC + R) * H * ilm_delta_chunk_ws floats.
 extern "C" int ilm_delta_chunks(void* o, const void* rows, int row_stride, const void* gates, void* pool, const void* state_in,
@@ -524,20 +537,21 @@ extern "C" int ilm_delta_chunks(void* o, const void* rows, int row_stride, const
     const int slots = T_ / DC + R, dvp = (dv + 15) / 16 * 16;
     ILM_REQUIRE(slots <= 65535 && ws != nullptr, "delta_chunks: %d chunks in a step, at most 65535", slots);
     const size_t sh = (size_t)slots * H;
-    float* ws_v = (float*)ws;
-    float* ws_w = ws_v + sh * DC * dvp;
-    float* ws_k = ws_w + sh * DC * dkp;
-    float* ws_p = ws_k + sh * DC * dkp;
-    float* ws_e = ws_p + sh * DC * DC;
+    float4* ws_v = (float4*)ws;
+    float4* ws_w = ws_v + sh * (DC / 4) * dvp;
+    float4* ws_q = ws_w + sh * (DC / 4) * dkp;
+    float4* ws_k = ws_q + sh * (DC / 4) * dkp;
+    float4* ws_p = ws_k + sh * (DC / 4) * dkp;
+    float* ws_e = (float*)(ws_p + sh * (DC / 4) * DC);
     const dim3 ga(H, slots), gb(8 * ((dvp / 16 * H + 7) / 8), R);
 #define DC_CASE(KT_)                                                                                                                  \
     case KT_:                                                                                                                         \
-        delta_chunk_prepare_kernel<KT_><<<ga, 256, 0, stream>>>(ws_v, ws_w, ws_k, ws_p, ws_e, (const float*)rows, row_stride,          \
+        delta_chunk_prepare_kernel<KT_><<<ga, 256, 0, stream>>>(ws_v, ws_w, ws_q, ws_k, ws_p, ws_e, (const float*)rows, row_stride,    \
                                                                 (const float*)gates, (const int*)seg_offsets, R, H, G, dv, dvp, min_len); \
         ILM_LAUNCH_CHECK("delta_chunks (prepare)");                                                                                   \
-        delta_chunk_walk_kernel<KT_><<<gb, 256, 0, stream>>>((float*)o, ws_v, ws_w, ws_k, ws_p, ws_e, (const float*)rows, row_stride,  \
-                                                             (float*)pool, (const int*)state_in, (const int*)state_out,                \
-                                                             (const int*)seg_offsets, H, G, dk, dv, dvp, min_len);                     \
+        delta_chunk_walk_kernel<KT_><<<gb, 256, 0, stream>>>((float*)o, ws_v, ws_w, ws_q, ws_k, ws_p, ws_e, (float*)pool,              \
+                                                             (const int*)state_in, (const int*)state_out, (const int*)seg_offsets, H,  \
+                                                             dk, dv, dvp, min_len);                                                    \
         break
     switch (dkp / 16) {
         DC_CASE(1); DC_CASE(2); DC_CASE(3); DC_CASE(4); DC_CASE(5); DC_CASE(6); DC_CASE(7); DC_CASE(8);
