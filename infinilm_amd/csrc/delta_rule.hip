@@ -240,11 +240,12 @@ __device__ __forceinline__ int dc_find(const int* __restrict__ seg_offsets, int 
     return (p >= 0 && p * DC < seg_offsets[lo + 1] - seg_offsets[lo]) ? lo : -1;
 }
 
-#define DC_XT 4      // column tiles of [V | K] a wave solves together
+#define DC_PW 8      // waves of the first kernel's blocks
+#define DC_XT 2      // column tiles of [V | K] a wave solves together
 
 // KT: key entries / 16
 template <int KT>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(DC_PW * 64, 4)
 delta_chunk_prepare_kernel(float4* __restrict__ ws_v, float4* __restrict__ ws_w, float4* __restrict__ ws_q, float4* __restrict__ ws_k,
                            float4* __restrict__ ws_p, float* __restrict__ ws_e, const float* __restrict__ rows, int row_stride, const float* __restrict__ gates,
                            const int* __restrict__ seg_offsets, int R, int H, int G, int dv, int dvp, int min_len) {
@@ -252,9 +253,9 @@ delta_chunk_prepare_kernel(float4* __restrict__ ws_v, float4* __restrict__ ws_w,
     __shared__ __attribute__((aligned(16))) float Ks[DC * KS];
     __shared__ __attribute__((aligned(16))) float An[DC * AS];          // -A
     __shared__ __attribute__((aligned(16))) float Ti[4 * 16 * TS];      // inverses of the diagonal blocks of I + A
-    __shared__ __attribute__((aligned(16))) float Tp[4 * 16 * TS];      // a wave's tile on its way into fragment order
+    __shared__ __attribute__((aligned(16))) float Tp[DC_PW * 16 * TS];      // a wave's tile on its way into fragment order
     __shared__ double Ls[DC];
-    __shared__ float bs[DC], fs[DC];                                    // beta; exp(L_end - L)
+    __shared__ float bs[DC], fs[DC], es[DC];                            // beta; exp(L_end - L); beta exp(L)
     const int h = blockIdx.x, slot = blockIdx.y;
     int p;
     const int seg = dc_find(seg_offsets, R, slot, p);
@@ -269,11 +270,29 @@ delta_chunk_prepare_kernel(float4* __restrict__ ws_v, float4* __restrict__ ws_w,
     const float* krow = qrow + (size_t)G * DK;
     const float* vrow = rows + (size_t)t0 * row_stride + (size_t)2 * G * DK + (size_t)h * dv;
     const size_t sh = (size_t)slot * H + h;
-    for (int i = tid; i < DC * (DK / 4); i += 256) {
+    // the values of the wave's first column tiles, on their way from the start
+    const int nv = dvp / 16, nt = nv + KT;
+    float rv[4][DC_XT][4];
+    auto load_values = [&](int c0) {
+#pragma unroll
+        for (int c = 0; c < DC_XT; ++c) {
+            if (c0 + c >= nv) continue;                // wave-uniform
+            const int col = 16 * (c0 + c) + r;
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    const int t = 16 * i + 4 * q + e;
+                    rv[i][c][e] = vrow[(size_t)(t < n ? t : n - 1) * row_stride + (col < dv ? col : dv - 1)];
+                }
+        }
+    };
+    for (int i = tid; i < DC * (DK / 4); i += DC_PW * 64) {
         const int t = i / (DK / 4), c = (i % (DK / 4)) * 4;
         const float4 v = *reinterpret_cast<const float4*>(krow + (size_t)(t < n ? t : n - 1) * row_stride + c);
         *reinterpret_cast<float4*>(&Ks[t * KS + c]) = t < n ? v : make_float4(0.f, 0.f, 0.f, 0.f);
     }
+    load_values(wave * DC_XT);
     if (wave == 0) {
         const float* gt = gates + (size_t)(t0 + (lane < n ? lane : n - 1)) * 2 * H + h;
         double L = lane < n ? (double)gt[H] : 0.0;
@@ -285,34 +304,47 @@ delta_chunk_prepare_kernel(float4* __restrict__ ws_v, float4* __restrict__ ws_w,
         Ls[lane] = L;
         bs[lane] = lane < n ? gt[0] : 0.f;
         fs[lane] = expf((float)(__shfl(L, 63, 64) - L));
-        ws_e[sh * DC_EL + lane] = expf((float)L);
-        if (lane == 63) ws_e[sh * DC_EL + DC] = expf((float)L);
+        const float eL = expf((float)L);
+        es[lane] = bs[lane] * eL;
+        ws_e[sh * DC_EL + lane] = eL;
+        if (lane == 63) ws_e[sh * DC_EL + DC] = eL;
     }
     __syncthreads();
     // ---- k_t . k_i and q_t . k_i by tiles of 16 x 16 at and below the diagonal
-    for (int tile = wave; tile < 10; tile += 4) {
-        const int rt = tile < 1 ? 0 : (tile < 3 ? 1 : (tile < 6 ? 2 : 3)), ct = tile - rt * (rt + 1) / 2;
-        f32x4 kk = f32x4{0.f, 0.f, 0.f, 0.f}, kq = kk;      // k_t . k_i as [t, i]; k_i . q_t as [i, t]
-        const int tq = 16 * rt + r < n ? 16 * rt + r : n - 1;
+    for (int task = wave; task < 20; task += DC_PW) {
+        const int tile = task >> 1, rt = tile < 1 ? 0 : (tile < 3 ? 1 : (tile < 6 ? 2 : 3)), ct = tile - rt * (rt + 1) / 2;
+        f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (task & 1) {      // k_i . q_t as [i, t]
+            const int tq = 16 * rt + r < n ? 16 * rt + r : n - 1;
+            float4 qa[KT];
 #pragma unroll
-        for (int j = 0; j < KT; ++j) {
-            const float4 qa = *reinterpret_cast<const float4*>(qrow + (size_t)tq * row_stride + 16 * j + 4 * q);
-            const float4 ka = *reinterpret_cast<const float4*>(&Ks[(16 * rt + r) * KS + 16 * j + 4 * q]);
-            const float4 kb = *reinterpret_cast<const float4*>(&Ks[(16 * ct + r) * KS + 16 * j + 4 * q]);
-            kk = dc_mmt(ka, kb, kk);
-            kq = dc_mmt(kb, qa, kq);
-            if (ct == rt) ws_q[((sh * 4 + rt) * KT + j) * 64 + lane] = qa;
-        }
-        const double Li = Ls[16 * ct + r], Lt = Ls[16 * rt + r];
-        float4 pw;
-        float* pe = reinterpret_cast<float*>(&pw);
+            for (int j = 0; j < KT; ++j) qa[j] = *reinterpret_cast<const float4*>(qrow + (size_t)tq * row_stride + 16 * j + 4 * q);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const int t = 16 * rt + 4 * q + e, i = 16 * ct + 4 * q + e;
-            An[t * AS + 16 * ct + r] = 16 * ct + r < t ? -bs[t] * expf((float)(Ls[t] - Li)) * kk[e] : 0.f;
-            pe[e] = i <= 16 * rt + r ? expf((float)(Lt - Ls[i])) * kq[e] : 0.f;
+            for (int j = 0; j < KT; ++j) {
+                acc = dc_mmt(*reinterpret_cast<const float4*>(&Ks[(16 * ct + r) * KS + 16 * j + 4 * q]), qa[j], acc);
+                if (ct == rt) ws_q[((sh * 4 + rt) * KT + j) * 64 + lane] = qa[j];
+            }
+            const double Lt = Ls[16 * rt + r];
+            float4 pw;
+            float* pe = reinterpret_cast<float*>(&pw);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int i = 16 * ct + 4 * q + e;
+                pe[e] = i <= 16 * rt + r ? expf((float)(Lt - Ls[i])) * acc[e] : 0.f;
+            }
+            ws_p[((sh * 4 + rt) * 4 + ct) * 64 + lane] = pw;
+        } else {             // k_t . k_i as [t, i]
+#pragma unroll
+            for (int j = 0; j < KT; ++j)
+                acc = dc_mmt(*reinterpret_cast<const float4*>(&Ks[(16 * rt + r) * KS + 16 * j + 4 * q]),
+                             *reinterpret_cast<const float4*>(&Ks[(16 * ct + r) * KS + 16 * j + 4 * q]), acc);
+            const double Li = Ls[16 * ct + r];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int t = 16 * rt + 4 * q + e;
+                An[t * AS + 16 * ct + r] = 16 * ct + r < t ? -bs[t] * expf((float)(Ls[t] - Li)) * acc[e] : 0.f;
+            }
         }
-        ws_p[((sh * 4 + rt) * 4 + ct) * 64 + lane] = pw;
     }
     __syncthreads();
     if (wave == 0) {      // column r of the inverse of diagonal block q, by substitution
@@ -321,13 +353,19 @@ delta_chunk_prepare_kernel(float4* __restrict__ ws_v, float4* __restrict__ ws_w,
         for (int i = 0; i < 16; ++i) {
             float v = i == r ? 1.0f : 0.f;
 #pragma unroll
-            for (int j = 0; j < i; ++j) v = fmaf(An[(16 * q + i) * AS + 16 * q + j], x[j], v);
+            for (int j = 0; j < i; j += 4) {
+                const float4 a = *reinterpret_cast<const float4*>(&An[(16 * q + i) * AS + 16 * q + j]);
+                v = fmaf(a.x, x[j], v);
+                if (j + 1 < i) v = fmaf(a.y, x[j + 1], v);
+                if (j + 2 < i) v = fmaf(a.z, x[j + 2], v);
+                if (j + 3 < i) v = fmaf(a.w, x[j + 3], v);
+            }
             x[i] = v;
         }
 #pragma unroll
         for (int i = 0; i < 16; ++i) Ti[(q * 16 + i) * TS + r] = x[i];
     } else {              // the decayed keys, transposed: tile (m, j) holds keys' entries 16 m .. by tokens 16 j ..
-        for (int i = wave - 1; i < KT * 4; i += 3) {
+        for (int i = wave - 1; i < KT * 4; i += DC_PW - 1) {
             const int m = i >> 2, j = i & 3;
             float4 v;
             float* ve = reinterpret_cast<float*>(&v);
@@ -338,8 +376,7 @@ delta_chunk_prepare_kernel(float4* __restrict__ ws_v, float4* __restrict__ ws_w,
     }
     __syncthreads();
     // ---- (I + A) X = [beta V | beta exp(L) K], DC_XT column tiles of 16 a wave, the rows' blocks one after the other
-    const int nv = dvp / 16, nt = nv + KT;
-    for (int c0 = wave * DC_XT; c0 < nt; c0 += 4 * DC_XT) {
+    for (int c0 = wave * DC_XT; c0 < nt; c0 += DC_PW * DC_XT) {
         f32x4 X[4][DC_XT];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
@@ -351,13 +388,8 @@ delta_chunk_prepare_kernel(float4* __restrict__ ws_v, float4* __restrict__ ws_w,
                 for (int e = 0; e < 4; ++e) {
                     const int t = 16 * i + 4 * q + e;
                     float v = 0.f;
-                    if (ct < nv) {
-                        const int col = 16 * ct + r;
-                        v = vrow[(size_t)(t < n ? t : n - 1) * row_stride + (col < dv ? col : dv - 1)];
-                        v = col < dv ? v * bs[t] : 0.f;
-                    } else if (ct < nt) {
-                        v = bs[t] * expf((float)Ls[t]) * Ks[t * KS + 16 * (ct - nv) + r];
-                    }
+                    if (ct < nv) v = 16 * ct + r < dv ? rv[i][c][e] * bs[t] : 0.f;
+                    else if (ct < nt) v = es[t] * Ks[t * KS + 16 * (ct - nv) + r];
                     acc[c][e] = v;
                 }
             }
@@ -371,6 +403,7 @@ delta_chunk_prepare_kernel(float4* __restrict__ ws_v, float4* __restrict__ ws_w,
 #pragma unroll
             for (int c = 0; c < DC_XT; ++c) X[i][c] = dc_mma(d, acc[c], f32x4{0.f, 0.f, 0.f, 0.f});
         }
+        load_values(c0 + DC_PW * DC_XT);
 #pragma unroll
         for (int c = 0; c < DC_XT; ++c) {
             const int ct = c0 + c;
@@ -392,44 +425,29 @@ delta_chunk_prepare_kernel(float4* __restrict__ ws_v, float4* __restrict__ ws_w,
     }
 }
 
-// What a wave reads of a chunk: its 16 rows of W, q and the sums' weights, its tiles of the decayed keys, its corner of V'
+// The walk: eight waves a block.  Waves 0 to 3 form a chunk's corrections, U = V' - W S_0, 16 rows each; waves 4 to 7 its outputs,
+// exp(L) (Q S_0) + P U; every wave makes one tile of 16 entries of the next state.  What a wave reads of a chunk:
 template <int KT>
 struct dc_operands {
-    static constexpr int MT = (KT + 3) / 4;
-    float4 w[KT], q[KT], p[4], k[MT][4], e;
-    f32x4 v;
-    float end;
+    float4 a[KT];       // its 16 rows of W, or of q
+    float4 k[4];        // its tile of the decayed keys
+    float4 p[4];        // outputs: the second sum's weights; corrections: V' (the first of them)
+    float4 e;           // outputs: exp(L) of the lane's four rows
+    float end;          // exp(L_end)
+};
+
+struct dc_source {
+    const float4 *a, *k, *p;
+    const float *e, *end;
 };
 
 template <int KT>
-__device__ __forceinline__ void dc_load(dc_operands<KT>& o, const float4* ws_v, const float4* ws_w, const float4* ws_q, const float4* ws_k,
-                                        const float4* ws_p, const float* ws_e, size_t sh, int nv, int blk, int wave, int lane) {
-    // (every piece is 64 consecutive 16-byte entries, one a lane)
-#pragma unroll
-    for (int j = 0; j < KT; ++j) {
-        o.w[j] = ws_w[((sh * 4 + wave) * KT + j) * 64 + lane];
-        o.q[j] = ws_q[((sh * 4 + wave) * KT + j) * 64 + lane];
-    }
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-        // (blocks above the diagonal are not in memory: the diagonal's own is read in their place and not used)
-        o.p[j] = ws_p[((sh * 4 + wave) * 4 + (j <= wave ? j : wave)) * 64 + lane];
-#pragma unroll
-        for (int m = 0; m < dc_operands<KT>::MT; ++m) o.k[m][j] = ws_k[((sh * KT + (wave + 4 * m < KT ? wave + 4 * m : KT - 1)) * 4 + j) * 64 + lane];
-    }
-    const float4 v = ws_v[((sh * 4 + wave) * nv + blk) * 64 + lane];
-    o.v = f32x4{v.x, v.y, v.z, v.w};
-    o.e = *reinterpret_cast<const float4*>(ws_e + sh * DC_EL + 16 * wave + 4 * (lane >> 4));
-    o.end = ws_e[sh * DC_EL + DC];
-}
-
-template <int KT>
-__global__ void __launch_bounds__(256, 1)
+__global__ void __launch_bounds__(512, 2)
 delta_chunk_walk_kernel(float* __restrict__ out, const float4* __restrict__ ws_v, const float4* __restrict__ ws_w, const float4* __restrict__ ws_q,
                         const float4* __restrict__ ws_k, const float4* __restrict__ ws_p, const float* __restrict__ ws_e,
                         float* __restrict__ pool, const int* __restrict__ state_in, const int* __restrict__ state_out,
                         const int* __restrict__ seg_offsets, int H, int dk, int dv, int dvp, int min_len) {
-    constexpr int MT = dc_operands<KT>::MT;
+    static_assert(KT <= 8, "a wave makes one tile of the state");
     __shared__ f32x4 Us[4][64];
     __shared__ f32x4 Ss[KT][64];
     // blocks go to the eight dies in turn; with this numbering the column blocks of a head share a die, whose cache then holds
@@ -437,89 +455,112 @@ delta_chunk_walk_kernel(float* __restrict__ out, const float4* __restrict__ ws_v
     const int nb = dvp / 16, items = nb * H, per = (items + 7) / 8;
     const int item = (int)(blockIdx.x & 7) * per + (int)(blockIdx.x >> 3);
     if ((int)(blockIdx.x >> 3) >= per || item >= items) return;
-    const int h = item / nb, col0 = (item % nb) * 16, seg = blockIdx.y;
+    const int h = item / nb, blk = item % nb, col0 = blk * 16, seg = blockIdx.y;
     const int s0 = seg_offsets[seg], len = seg_offsets[seg + 1] - s0;
     if (len <= 0 || len < min_len) return;
-    const int chunks = (len + DC - 1) / DC, slot0 = s0 / DC + seg;
+    const int chunks = (len + DC - 1) / DC;
     const int lane = threadIdx.x & 63, r = lane & 15, q = lane >> 4;
-    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), wr = wave & 3;      // wr: its tile of 16 rows
+    const bool outputs = wave >= 4, makes = wave < KT;
     const bool col_ok = col0 + r < dv, v4 = dk % 4 == 0;
-    // state tile m: entries 16 m + 4 q + e of column col0 + r; every wave holds all of them
-    f32x4 S[KT];
+    // state tile m: entries 16 m + 4 q + e of column col0 + r
+    const float* src = pool + (((size_t)state_in[seg] * H + h) * dv + (col_ok ? col0 + r : 0)) * dk;
+    auto state_tile = [&](int m) -> f32x4 {
+        const int k0 = 16 * m + 4 * q;
+        f32x4 s = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (v4) {
+            const float4 t = *reinterpret_cast<const float4*>(src + (k0 < dk ? k0 : 0));
+            if (col_ok && k0 < dk) s = f32x4{t.x, t.y, t.z, t.w};
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                if (col_ok && k0 + e < dk) s[e] = src[k0 + e];
+        }
+        return s;
+    };
+    f32x4 S[KT], own = state_tile(makes ? wave : 0);      // every wave holds the whole state, and the tile it makes once more
+#pragma unroll
+    for (int m = 0; m < KT; ++m) S[m] = state_tile(m);
+    // (every piece is 64 consecutive 16-byte entries, one a lane; a chunk's pieces lie H heads after the last chunk's)
+    dc_source at;
     {
-        const float* src = pool + (((size_t)state_in[seg] * H + h) * dv + (col_ok ? col0 + r : 0)) * dk;
-#pragma unroll
-        for (int m = 0; m < KT; ++m) {
-            const int k0 = 16 * m + 4 * q;
-            if (v4) {
-                const float4 t = *reinterpret_cast<const float4*>(src + (k0 < dk ? k0 : 0));
-                const bool ok = col_ok && k0 < dk;
-                S[m] = f32x4{ok ? t.x : 0.f, ok ? t.y : 0.f, ok ? t.z : 0.f, ok ? t.w : 0.f};
-            } else {
-#pragma unroll
-                for (int e = 0; e < 4; ++e) S[m][e] = (col_ok && k0 + e < dk) ? src[k0 + e] : 0.f;
-            }
-        }
+        const size_t sh = (size_t)(s0 / DC + seg) * H + h;
+        at.a = (outputs ? ws_q : ws_w) + (sh * 4 + wr) * KT * 64 + lane;
+        at.k = ws_k + (sh * KT + (makes ? wave : 0)) * 4 * 64 + lane;
+        at.p = outputs ? ws_p + (sh * 4 + wr) * 4 * 64 + lane : ws_v + ((sh * 4 + wr) * nb + blk) * 64 + lane;
+        at.e = ws_e + sh * DC_EL + 16 * wr + 4 * q;
+        at.end = ws_e + sh * DC_EL + DC;
     }
-    dc_operands<KT> cur, nxt;
-    dc_load<KT>(nxt, ws_v, ws_w, ws_q, ws_k, ws_p, ws_e, (size_t)slot0 * H + h, nb, item % nb, wave, lane);
-    for (int c = 0; c < chunks; ++c) {
-        cur = nxt;
-        const int t0 = s0 + c * DC, n = min(DC, len - c * DC);
-        if (c + 1 < chunks)
-            dc_load<KT>(nxt, ws_v, ws_w, ws_q, ws_k, ws_p, ws_e, (size_t)(slot0 + c + 1) * H + h, nb, item % nb, wave, lane);
-        f32x4 ws = f32x4{0.f, 0.f, 0.f, 0.f}, qs = ws;
+    const size_t step_a = (size_t)H * 4 * KT * 64, step_p = (size_t)H * 4 * (outputs ? 4 : nb) * 64, step_e = (size_t)H * DC_EL;
+    auto load = [&](dc_operands<KT>& o) {
+#pragma unroll
+        for (int j = 0; j < KT; ++j) o.a[j] = at.a[j * 64];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) o.k[j] = at.k[j * 64];
+        o.p[0] = at.p[0];
+        if (outputs) {
+            // (blocks above the diagonal are not in memory: the diagonal's own is read in their place and not used)
+#pragma unroll
+            for (int j = 1; j < 4; ++j) o.p[j] = at.p[(j <= wr ? j : wr) * 64];
+            o.e = *reinterpret_cast<const float4*>(at.e);
+        }
+        o.end = *at.end;
+        at.a += step_a;
+        at.k += step_a;
+        at.p += step_p;
+        at.e += step_e;
+        at.end += step_e;
+    };
+    auto chunk = [&](int c, dc_operands<KT>& cur, dc_operands<KT>& nxt) {
+        if (c + 1 < chunks) load(nxt);
+        f32x4 x0 = f32x4{0.f, 0.f, 0.f, 0.f}, x1 = x0;
 #pragma unroll
         for (int m = 0; m < KT; ++m) {
-            ws = dc_mma(cur.w[m], S[m], ws);
-            qs = dc_mma(cur.q[m], S[m], qs);
+            if (m & 1) x1 = dc_mma(cur.a[m], S[m], x1);
+            else x0 = dc_mma(cur.a[m], S[m], x0);
         }
-        Us[wave][lane] = cur.v - ws;
+        x0 = x0 + x1;
+        if (!outputs) Us[wr][lane] = f32x4{cur.p[0].x, cur.p[0].y, cur.p[0].z, cur.p[0].w} - x0;
         __syncthreads();
         f32x4 U[4];
 #pragma unroll
         for (int j = 0; j < 4; ++j) U[j] = Us[j][lane];
+        if (makes) {
+            own = own * cur.end;
 #pragma unroll
-        for (int m = 0; m < MT; ++m)
-            if (wave + 4 * m < KT) {                    // wave-uniform
-                f32x4 s;
-#pragma unroll
-                for (int mm = 0; mm < KT; ++mm)
-                    if (mm == wave + 4 * m) s = S[mm];
-                s = s * cur.end;
-#pragma unroll
-                for (int j = 0; j < 4; ++j) s = dc_mma(cur.k[m][j], U[j], s);
-                Ss[wave + 4 * m][lane] = s;
-            }
-        f32x4 o = f32x4{qs[0] * cur.e.x, qs[1] * cur.e.y, qs[2] * cur.e.z, qs[3] * cur.e.w};
-#pragma unroll
-        for (int j = 0; j < 4; ++j)
-            if (j <= wave) o = dc_mma(cur.p[j], U[j], o);
-        if (col_ok) {
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const int t = 16 * wave + 4 * q + e;
-                if (t < n) out[((size_t)(t0 + t) * H + h) * dv + col0 + r] = o[e];
-            }
+            for (int j = 0; j < 4; ++j) own = dc_mma(cur.k[j], U[j], own);
+            Ss[wave][lane] = own;
         }
         __syncthreads();
 #pragma unroll
         for (int m = 0; m < KT; ++m) S[m] = Ss[m][lane];
-    }
-    if (!col_ok) return;
-    float* dst = pool + (((size_t)state_out[seg] * H + h) * dv + col0 + r) * dk;
+        if (outputs) {       // (off the path from state to state)
+            f32x4 o = f32x4{x0[0] * cur.e.x, x0[1] * cur.e.y, x0[2] * cur.e.z, x0[3] * cur.e.w};
 #pragma unroll
-    for (int m = 0; m < KT; ++m)
-        if ((m & 3) == wave) {
-            const int k0 = 16 * m + 4 * q;
-            if (v4) {
-                if (k0 < dk) *reinterpret_cast<float4*>(dst + k0) = make_float4(S[m][0], S[m][1], S[m][2], S[m][3]);
-            } else {
+            for (int j = 0; j < 4; ++j)
+                if (j <= wr) o = dc_mma(cur.p[j], U[j], o);
+            const int t0 = c * DC + 16 * wr + 4 * q;
 #pragma unroll
-                for (int e = 0; e < 4; ++e)
-                    if (k0 + e < dk) dst[k0 + e] = S[m][e];
-            }
+            for (int e = 0; e < 4; ++e)
+                if (col_ok && t0 + e < len) out[((size_t)(s0 + t0 + e) * H + h) * dv + col0 + r] = o[e];
         }
+    };
+    dc_operands<KT> A, B;
+    load(A);
+    for (int c = 0; c < chunks; c += 2) {
+        chunk(c, A, B);
+        if (c + 1 < chunks) chunk(c + 1, B, A);
+    }
+    if (!col_ok || !makes) return;
+    float* dst = pool + (((size_t)state_out[seg] * H + h) * dv + col0 + r) * dk;
+    const int k0 = 16 * wave + 4 * q;
+    if (v4) {
+        if (k0 < dk) *reinterpret_cast<float4*>(dst + k0) = make_float4(own[0], own[1], own[2], own[3]);
+    } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+            if (k0 + e < dk) dst[k0 + e] = own[e];
+    }
 }
 
 extern "C" int ilm_delta_chunk() { return DC; }
@@ -546,10 +587,10 @@ extern "C" int ilm_delta_chunks(void* o, const void* rows, int row_stride, const
     const dim3 ga(H, slots), gb(8 * ((dvp / 16 * H + 7) / 8), R);
 #define DC_CASE(KT_)                                                                                                                  \
     case KT_:                                                                                                                         \
-        delta_chunk_prepare_kernel<KT_><<<ga, 256, 0, stream>>>(ws_v, ws_w, ws_q, ws_k, ws_p, ws_e, (const float*)rows, row_stride,    \
+        delta_chunk_prepare_kernel<KT_><<<ga, DC_PW * 64, 0, stream>>>(ws_v, ws_w, ws_q, ws_k, ws_p, ws_e, (const float*)rows, row_stride,    \
                                                                 (const float*)gates, (const int*)seg_offsets, R, H, G, dv, dvp, min_len); \
         ILM_LAUNCH_CHECK("delta_chunks (prepare)");                                                                                   \
-        delta_chunk_walk_kernel<KT_><<<gb, 256, 0, stream>>>((float*)o, ws_v, ws_w, ws_q, ws_k, ws_p, ws_e, (float*)pool,              \
+        delta_chunk_walk_kernel<KT_><<<gb, 512, 0, stream>>>((float*)o, ws_v, ws_w, ws_q, ws_k, ws_p, ws_e, (float*)pool,              \
                                                              (const int*)state_in, (const int*)state_out, (const int*)seg_offsets, H,  \
                                                              dk, dv, dvp, min_len);                                                    \
         break
