@@ -81,7 +81,7 @@ __device__ __forceinline__ cp_place cp_find(int t, const int* seg, const int* se
 }
 
 // y of channels c .. c + VEC - 1, and the shift of the state row where the token is its segment's only one
-template <int VEC, typename T>
+template <int VEC, typename T, int MT>     // MT: the most taps
 __device__ __forceinline__ void cp_conv(float (&y)[VEC], const T* x, int x_stride, const T* w, int t, int c, int C, int taps,
                                         const cp_place& p) {
     float own[VEC];
@@ -91,9 +91,9 @@ __device__ __forceinline__ void cp_conv(float (&y)[VEC], const T* x, int x_strid
         for (int e = 0; e < VEC; ++e) y[e] = own[e];
         return;
     }
-    float xv[CP_MAX_TAPS][VEC];
+    float xv[MT][VEC];
 #pragma unroll
-    for (int i = 0; i < CP_MAX_TAPS - 1; ++i)
+    for (int i = 0; i < MT - 1; ++i)
         if (i < taps - 1) {
             const int back = taps - 1 - i;
             if (back <= p.j) cp_load<VEC, T>(x + (size_t)(t - back) * x_stride + c, xv[i]);
@@ -102,17 +102,17 @@ __device__ __forceinline__ void cp_conv(float (&y)[VEC], const T* x, int x_strid
 #pragma unroll
     for (int e = 0; e < VEC; ++e) y[e] = 0.f;
 #pragma unroll
-    for (int i = 0; i < CP_MAX_TAPS; ++i)
+    for (int i = 0; i < MT; ++i)
         if (i < taps) {
             float wv[VEC];
             cp_load<VEC, T>(w + (size_t)i * C + c, wv);
 #pragma unroll
-            for (int e = 0; e < VEC; ++e) y[e] = fmaf(wv[e], i == taps - 1 ? own[e] : xv[i < CP_MAX_TAPS - 1 ? i : 0][e], y[e]);
+            for (int e = 0; e < VEC; ++e) y[e] = fmaf(wv[e], i == taps - 1 ? own[e] : xv[i < MT - 1 ? i : 0][e], y[e]);
         }
     if (p.only && taps > 1) {
 #pragma unroll
-        for (int i = 0; i < CP_MAX_TAPS - 1; ++i)
-            if (i < taps - 1) cp_store<VEC, float>(p.out + (size_t)i * C + c, i == taps - 2 ? own : xv[i + 1 < CP_MAX_TAPS ? i + 1 : 0]);
+        for (int i = 0; i < MT - 1; ++i)
+            if (i < taps - 1) cp_store<VEC, float>(p.out + (size_t)i * C + c, i == taps - 2 ? own : xv[i + 1 < MT ? i + 1 : 0]);
     }
 }
 
@@ -164,7 +164,7 @@ conv_delta_inputs_kernel(float* __restrict__ out, float* __restrict__ gates, con
     float* orow = out + (size_t)t * out_stride;
     for (int c = tid * VEC; c < C; c += THREADS * VEC) {
         float y[VEC];
-        cp_conv<VEC, T>(y, x, x_stride, w, t, c, C, taps, p);
+        cp_conv<VEC, T, CP_MAX_TAPS>(y, x, x_stride, w, t, c, C, taps, p);
 #pragma unroll
         for (int e = 0; e < VEC; ++e) y[e] = cp_silu(y[e]);
         if (c < nqk) {
@@ -329,8 +329,8 @@ extern "C" int ilm_conv_delta_inputs(void* out, void* gates, const void* x, cons
 
 // ------------------------------------------------------------------------------------------
 // LDS floats: rows y [C] | cosines, sines [rd / 2 each]
-template <int VEC, typename T, int THREADS>
-__global__ void __launch_bounds__(THREADS)
+template <int VEC, typename T, int THREADS, int MT>
+__global__ void __launch_bounds__(THREADS, MT <= 4 && VEC == 8 ? 8 : 1)     // (up to 4 taps: 64 registers, as many waves as a unit holds)
 conv_norm_rope_kvwrite_kernel(T* __restrict__ q_out, const T* __restrict__ x, const T* __restrict__ w, float* __restrict__ pool,
                               const int* __restrict__ state_in, const int* __restrict__ state_out, const int* __restrict__ seg,
                               const int* __restrict__ seg_offsets, const int* __restrict__ pos, const float* __restrict__ freq,
@@ -338,7 +338,7 @@ conv_norm_rope_kvwrite_kernel(T* __restrict__ q_out, const T* __restrict__ x, co
                               const int* __restrict__ slots, int T_, int H, int G, int dim, int vdim, int d, int rd, int own_kv, int taps,
                               int x_stride, float eps, int page) {
     extern __shared__ __attribute__((aligned(16))) float sm[];
-    __shared__ float red[THREADS / 64];
+    __shared__ float red[2 * (THREADS / 64)];
     const int t = cp_token(T_);
     if (t < 0) return;
     const int tid = threadIdx.x;
@@ -349,7 +349,7 @@ conv_norm_rope_kvwrite_kernel(T* __restrict__ q_out, const T* __restrict__ x, co
     float sq = 0.f, sk = 0.f;
     for (int c = tid * VEC; c < C; c += THREADS * VEC) {
         float y[VEC];
-        cp_conv<VEC, T>(y, x, x_stride, w, t, c, C, taps, p);
+        cp_conv<VEC, T, MT>(y, x, x_stride, w, t, c, C, taps, p);
         float s = 0.f;
         cp_store<VEC, float>(sm + c, y);
 #pragma unroll
@@ -364,13 +364,22 @@ conv_norm_rope_kvwrite_kernel(T* __restrict__ q_out, const T* __restrict__ x, co
         cs[i] = cn;
         cs[half + i] = sn;
     }
-    float rq = 1.0f, rk = 1.0f;
-    sq = block_sum<THREADS / 64>(sq, red);      // (its barriers also publish sm and cs)
-    if (wq != nullptr) rq = 1.0f / sqrtf(sq / (float)Cq + eps);
-    if (own_kv) {
-        sk = block_sum<THREADS / 64>(sk, red);
-        if (wk != nullptr) rk = 1.0f / sqrtf(sk / (float)Ck + eps);
+    // both sums over the block's waves (the barrier also publishes sm and cs)
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    if ((tid & 63) == 0) {
+        red[tid >> 6] = sq;
+        red[THREADS / 64 + (tid >> 6)] = sk;
     }
+    __syncthreads();
+    sq = sk = 0.f;
+#pragma unroll
+    for (int i = 0; i < THREADS / 64; ++i) {
+        sq += red[i];
+        sk += red[THREADS / 64 + i];
+    }
+    const float rq = wq != nullptr ? 1.0f / sqrtf(sq / (float)Cq + eps) : 1.0f;
+    const float rk = wk != nullptr && own_kv ? 1.0f / sqrtf(sk / (float)Ck + eps) : 1.0f;
     const int slot = (own_kv && slots != nullptr) ? slots[t] : -1;
     const int pg = slot >= 0 ? slot / page : 0, off = slot >= 0 ? slot % page : 0;
     // pieces of 8 entries of q and k heads (of d entries in what is written; d is a multiple of 8)
@@ -442,16 +451,22 @@ extern "C" int ilm_conv_norm_rope_kvwrite(void* q_out, const void* x, const void
 #define CN_ARGS(T__) (T__*)q_out, (const T__*)x, (const T__*)w, (float*)pool, (const int*)state_in, (const int*)state_out,            \
                      (const int*)seg, (const int*)seg_offsets, (const int*)pos, (const float*)freq, (const T__*)wq, (const T__*)wk,    \
                      (T__*)kc, (T__*)vc, (const int*)slots, T_, H, G, dim, vdim, d, rd, own_kv, taps, x_stride, eps, page
-#define CN_LAUNCH(T__)                                                                                                              \
+#define CN_LAUNCH_T(T__, MT_)                                                                                                       \
     do {                                                                                                                            \
-        if (vec && wide) conv_norm_rope_kvwrite_kernel<8, T__, 1024><<<cp_blocks(T_), 1024, shm, stream>>>(CN_ARGS(T__));           \
-        else if (vec) conv_norm_rope_kvwrite_kernel<8, T__, 256><<<cp_blocks(T_), 256, shm, stream>>>(CN_ARGS(T__));                \
-        else conv_norm_rope_kvwrite_kernel<1, T__, 256><<<cp_blocks(T_), 256, shm, stream>>>(CN_ARGS(T__));                         \
+        if (vec && wide) conv_norm_rope_kvwrite_kernel<8, T__, 1024, MT_><<<cp_blocks(T_), 1024, shm, stream>>>(CN_ARGS(T__));      \
+        else if (vec) conv_norm_rope_kvwrite_kernel<8, T__, 256, MT_><<<cp_blocks(T_), 256, shm, stream>>>(CN_ARGS(T__));           \
+        else conv_norm_rope_kvwrite_kernel<1, T__, 256, MT_><<<cp_blocks(T_), 256, shm, stream>>>(CN_ARGS(T__));                    \
+    } while (0)
+#define CN_LAUNCH(T__)                                       \
+    do {                                                     \
+        if (taps <= 4) CN_LAUNCH_T(T__, 4);                  \
+        else CN_LAUNCH_T(T__, CP_MAX_TAPS);                  \
     } while (0)
     if (dtype == ILM_DTYPE_F32) CN_LAUNCH(float);
     else if (dtype == ILM_DTYPE_BF16) CN_LAUNCH(bf16);
     else ILM_REQUIRE(false, "conv_norm_rope_kvwrite: unknown dtype %d", dtype);
 #undef CN_LAUNCH
+#undef CN_LAUNCH_T
 #undef CN_ARGS
     ILM_LAUNCH_CHECK("conv_norm_rope_kvwrite");
     if (taps > 1 && !singles)
