@@ -83,7 +83,7 @@ def main() -> int:
 
 
 def compare_designs(args) -> dict:
-    """Kekevik beside MiniCPM4 at equal width, layers, heads, head size and feed-forward parameters: prefill of
+    """`--design` (and with moputar Kekevik too) beside MiniCPM4 at equal width, layers, heads, head size and feed-forward parameters: prefill of
     `--prefill-tokens` tokens in one step, decode at batch 8 and 64 over `--context` tokens (recorded steps), and for
     every kernel entry point its calls, its time a call in eager steps and, where one bound names it, the share of that
     bound it reaches: bytes it must move over the HBM peak, or floating-point work over the vector float32 peak."""

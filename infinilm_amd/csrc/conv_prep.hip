@@ -4,7 +4,7 @@
 //                                                         first token of this step comes from its state row, zeros at first)
 // and what follows it token by token:
 //
-//   ilm_conv_delta_inputs   rows [q: G dk | k: G dk | v: H dv | ...], y through silu; q and k made unit vectors per head,
+//   ilm_conv_delta_inputs   rows [q: G dk | k: G dk | v: H dv | ...], y through silu; every q and k head divided by its length,
 //       x / sqrt(sum(x^2) + unit_eps), q times q_scale; and from the rows' columns b and a [H each] the step's
 //       beta = sigmoid(b) and log-decay = -exp(A_log) softplus(a + dt_bias).  Float results: rows [q | k | v] whose q and k heads
 //       are filled up with zeros to dkp entries, and [T, 2 H] (beta | log-decay).

@@ -1,16 +1,18 @@
 // The gated delta rule: a linear attention whose state forgets by a decay per head and step and is corrected by the
 // difference between a token's value and what the state already holds under the token's key.  Per head, all in float:
 //
-//   S <- g S;   u = beta (v - S^T k);   S <- S + k u^T;   o = S^T q            S [dk, dv], zero at a sequence's start
+//   D_t = g_t S_{t-1},   u_t = beta_t (v_t - k_t D_t),   S_t = D_t + outer(k_t, u_t),   o_t = q_t S_t
+//
+// with the vectors of token t as rows; S [dk, dv] is zero before a sequence's start.
 //
 // Inputs are float rows [q: G dkp | k: G dkp | v: H dv] (query and key heads filled up with zeros to dkp entries; head h reads
 // query/key head h / (H / G)) and [beta: H | log g: H].  A request's state passes from step to step through a row of a pool,
 // [H, dv, dk] (the key index fastest).
 //
 //   ilm_delta_step     token by token, a block a (request, head, columns).  A thread keeps DS_NK state entries (two pieces of
-//       four, KP pieces apart, so that the lanes of a column read whole lines) of VC value columns in registers; the two sums a token needs, S^T k and S^T q (both from the decayed state: the
-//       read-out after the write is S^T q + u (k . q)), and k . q are folded over the lanes of a column together.  Where a block
-//       holds all columns of its head it can end with the head's output norm, weight and gate:
+//       four, KP pieces apart, so that the lanes of a column read whole lines) of VC value columns in registers; the two sums a
+//       token needs, k D and q D (the read-out after the write is q D + (k . q) u), and k . q are folded over the lanes of a
+//       column together.  Where a block holds all columns of its head it can end with the head's output norm, weight and gate:
 //       y = o / sqrt(mean(o^2) + eps) * w * silu(gate), in the activations' dtype.
 //
 //   ilm_delta_chunks   long segments (portions of prompts), in chunks of DC = 64 tokens on the float matrix instruction
@@ -24,7 +26,8 @@
 //       heads side by side; the second walks a segment's chunks in order with 16 value columns of a head's state a block.
 //       Differences of L are taken in double, so that a token's decay keeps its float precision however much has been
 //       forgotten before it.  What passes from the first to the second lies in memory as the matrix instruction takes it (tiles of
-//       16 x 16, a lane's 16 bytes after another's), so that a wave reads it in whole kilobytes.  Chunk p of segment r has the workspace slot floor(first row of r / DC) + r + p.
+//       16 x 16, a lane's 16 bytes after another's), so that a wave reads it in whole kilobytes.
+//       Chunk p of segment r has the workspace slot floor(first row of r / DC) + r + p.
 #include "common.h"
 
 typedef __attribute__((ext_vector_type(4))) float f32x4;

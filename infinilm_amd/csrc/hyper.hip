@@ -1,8 +1,8 @@
 // A residual stream kept in several copies that the sublayers read and write through small weights ("hyper-connections").
 //
 //   ilm_hyper_update    rows X [T, n, H] float.  With a branch y (rows, or float parts of a K-split product that are summed
-//       first) all streams are first made anew from the old ones, X'_t = sum_s M[s, t] X_s + b[t] alpha y; then the next
-//       sublayer's input is read, u = sum_t a[t] X'_t (a absent: the plain sum), and normed:
+//       first) a token's streams are first made anew, X' = M^T X + outer(b, alpha y) (M[s, t]: from stream s to t); then the next
+//       sublayer's input is read, u = a X' (a absent: the plain sum), and normed:
 //       x = u / sqrt(mean(u^2) + eps) * (w + w_offset); without w, x is u itself.  `base` [T, H]: every old stream is this one
 //       row (the start, before any branch has made the streams differ).  X' is written to X if asked for.
 //

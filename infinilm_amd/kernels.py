@@ -1974,8 +1974,8 @@ def hyper_update(streams: Optional[torch.Tensor], count: int, base: Optional[tor
                  in_weights: Optional[torch.Tensor] = None, weight: Optional[torch.Tensor] = None, weight_offset: float = 0.0,
                  eps: float = 0.0, out_dtype: Optional[torch.dtype] = None, write: bool = True) -> Optional[torch.Tensor]:
     """`streams` float32 [T, count, H], or `base` [T, H] that every stream equals.  With a `branch` ([T, H], or float32 parts
-    [P, T, H] summed in order) every stream becomes sum_s mix[s, t] x_s + out_weights[t] alpha branch, all from the old ones
-    (written to `streams` if `write`); then u = sum_t in_weights[t] x_t (None: the plain sum), and its RMS norm times
+    [P, T, H] summed in order) a row's streams X [count, H] become mix^T X + outer(out_weights, alpha branch)
+    (written to `streams` if `write`); then u = in_weights X (None: the plain sum), and its RMS norm times
     (weight + weight_offset) as `out_dtype`, or u itself without `weight`.  out_dtype None: no result."""
     _dev(streams, base, branch, mix, out_weights, in_weights, weight)
     src = base if base is not None else streams
@@ -2105,7 +2105,7 @@ DELTA_CHUNK_FROM = int(os.environ.get("INFINILM_AMD_DELTA_CHUNK_FROM", "32"))   
 def delta_rule(rows: torch.Tensor, gates: torch.Tensor, heads: int, groups: int, dk: int, dv: int, pool: torch.Tensor,
                state_in: torch.Tensor, state_out: torch.Tensor, seg_offsets: torch.Tensor, segments: int, norm_weight: torch.Tensor,
                gate: torch.Tensor, eps: float, out_dtype: torch.dtype, max_len: Optional[int] = None) -> torch.Tensor:
-    """S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q per head and token of every segment, then
+    """D = g S; u = beta (v - k D); S = D + outer(k, u); o = q S (row vectors) per head and token of every segment, then
     o / sqrt(mean(o^2) + eps) * norm_weight [dv] * silu(gate) per head, [T, heads dv] as `out_dtype`.  `rows`, `gates` as
     `conv_delta_inputs` leaves them; `gate` [T, heads dv]; `max_len`: a bound on the segments' lengths known on the host: from
     DELTA_CHUNK_FROM tokens on, segments go in chunks on the float matrix instruction (the result differs from the token-by-token

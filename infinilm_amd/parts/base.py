@@ -180,8 +180,8 @@ def _gather_branch(branch: torch.Tensor, rows: torch.Tensor) -> torch.Tensor:
 
 
 class HyperStreams:
-    """A residual stream kept in `count` float32 copies x_1 .. x_count that start equal ("hyper-connections").  A sublayer reads
-    u = sum_s a[s] x_s, and its output y makes all copies anew: x_t <- sum_s M[s, t] x_s + b[t] y (M is indexed from, to).  The
+    """A residual stream kept in `count` float32 copies, a token's rows X [count, width], that start equal ("hyper-connections").  A sublayer reads
+    u = a X, and its output y makes all copies anew: X' = M^T X + outer(b, y) (M[s, t]: from copy s to copy t).  The
     model's output is their sum.  A branch pushed here stays due, together with its M and b, until the next read, whose kernel
     does the update, the read and the norm in one pass (`kernels.hyper_update`).  `base`: the row all copies equal as long as
     nothing has been pushed; the copies are not in memory before the first branch."""

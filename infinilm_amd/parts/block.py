@@ -272,8 +272,8 @@ class BranchNormBlock:
 @register_arrangement("hyper_connected")
 class HyperConnectedBlock:
     """Pre-norm sublayers around a residual stream of several copies (`HyperStreams`): the sublayer reads
-    norm(sum_s a[s] x_s), and its output y makes the copies anew, x_t <- sum_s M[s, t] x_s + b[t] y.  `connect1`, `connect2`:
-    PartSpec("hyper_connection", {"streams": n, "names": (a, b, M)}), the sublayers' own a, b [n] and M [n, n] (indexed from, to),
+    norm(a X) of a token's copies X [n, width], and its output y makes them anew, X' = M^T X + outer(b, y).  `connect1`, `connect2`:
+    PartSpec("hyper_connection", {"streams": n, "names": (a, b, M)}), the sublayers' own a, b [n] and M [n, n] (M[s, t]: from copy s to t),
     float32.  A layer may have no feed-forward (then no `norm2`, no `connect2`)."""
 
     def __init__(self, spec: LayerSpec, ctx: BuildContext):

@@ -1,6 +1,6 @@
 """Grouped-query attention with short convolutions, norms over whole rows and masks by chunks.
 
-  q = W_q h [heads x dim],  k = W_k h [kv_heads x dim],  v = W_v h [kv_heads x vdim]
+  projections without bias: heads query heads and kv_heads key heads of dim entries, kv_heads value heads of vdim entries
   a short causal convolution per channel of q, k and v right after the projection (`conv_taps` inputs, the last the token's
         own, zeros before a sequence's start; no bias; 0: none), whose last conv_taps - 1 inputs are state of the request
   q and k RMS-normed over all rows of all heads at once, with weights of that size (`row_norm`)

@@ -1,15 +1,18 @@
 """The gated delta rule: a linear attention whose state forgets by a decay computed from the input and is corrected by what
 it already holds under a token's key.
 
-  q = W_q h, k = W_k h  [kv_heads x dim],  v = W_v h  [heads x vdim]         (head h reads query/key head h // (heads / kv_heads))
+  projections without bias: kv_heads query and key heads of dim entries, heads value heads of vdim entries (consecutive
+        value heads share a query/key head)
   a short causal convolution per channel of q, k and v (`conv_taps` inputs, the last the token's own, zeros before a
         sequence's start; no bias), then silu
-  q and k made unit vectors per head, x / sqrt(sum(x^2) + unit_eps); q times dim^(-1/2)
-  beta = sigmoid(W_b h),  g = exp(-exp(A_log) softplus(W_a h + dt_bias))       one each per head
-  S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q                  per head, S [dim, vdim] starts at zero
-  o / sqrt(mean(o^2) + eps) * norm [vdim] * silu(W_g h)  per head, then W_o.
+  every query and key head divided by its length (the root of its sum of squares + unit_eps), queries by sqrt(dim) too
+  per value head a strength beta_t in (0, 1), sigmoid of its projection, and a decay g_t: log g_t = -exp(A_log)
+        softplus(projection + dt_bias)
+  per value head a matrix M [dim, vdim], zero before a sequence's start; with the vectors of token t as rows
+        D_t = g_t M_{t-1},   c_t = beta_t (v_t - k_t D_t),   M_t = D_t + outer(k_t, c_t),   y_t = q_t M_t
+  y_t divided by its root mean square, times norm [vdim] and silu of a gate's projection, per head; then the output product.
 
-Two states a request, float32 rows of the cache manager's pools: the convolution's last conv_taps - 1 inputs, and S as
+Two states a request, float32 rows of the cache manager's pools: the convolution's last conv_taps - 1 inputs, and M as
 [heads, vdim, dim].  Everything between the projections is float32 whatever the activations' dtype.
 """
 from __future__ import annotations

@@ -36,7 +36,7 @@ def silu(x):
 
 
 def short_conv(u: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """u [T, C], w [C, taps]: y_t = sum_j w[:, j] u_(t - taps + 1 + j), zeros before the start."""
+    """u [T, C], w [C, taps]: the last tap takes a token's own row, the one before it the row before; nothing precedes the first."""
     T, C = u.shape
     taps = w.shape[1]
     pad = torch.cat([torch.zeros((taps - 1, C), dtype=u.dtype), u], 0)

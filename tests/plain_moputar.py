@@ -4,7 +4,7 @@ Nothing here is shared with the engine: the functions take a dict of tensors by 
 config.json, and follow the design's equations directly.  The residual stream is `streams` rows a token, all equal to
 the scaled embedding at the start; a sublayer f with its own vectors a, b [streams] and matrix M [streams, streams] does
 
-    u = sum_s a[s] x_s;   y = f(rms(u) * (1 + w));   x_t <- sum_s M[s, t] x_s + b[t] y         (all t from the old rows)
+    u = a X;   y = f(rms(u) * (1 + w));   X' = M^T X + outer(b, y)         (X [streams, width], one token's rows)
 
 with two mixers (a gated delta rule with short convolutions; a softmax attention inside chunks of positions, with short
 convolutions, one norm over all of q and one over all of k, rotated pairs, which may read another layer's keys and
@@ -40,7 +40,7 @@ def gelu_tanh(x):
 
 
 def short_conv(u: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
-    """u [T, C], w [C, taps]: y_t = sum_j w[:, j] u_(t - taps + 1 + j), zeros before the start."""
+    """u [T, C], w [C, taps]: the last tap takes a token's own row, the one before it the row before; nothing precedes the first."""
     T, C = u.shape
     taps = w.shape[1]
     pad = torch.cat([torch.zeros((taps - 1, C), dtype=u.dtype), u], 0)
@@ -141,7 +141,7 @@ def feed_forward(W, p: str, h):
 
 
 def read_streams(X, a):
-    """X [streams, T, width] -> sum_s a[s] X_s."""
+    """X [streams, T, width] -> the rows' sum with weights a."""
     return (a[:, None, None] * X).sum(0)
 
 

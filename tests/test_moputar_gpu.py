@@ -59,7 +59,7 @@ def _segments(lens):
 
 
 # ---- the kernels alone ------------------------------------------------------------------------------------------------
-@pytest.mark.parametrize("n,H,T,parts,ydt,out", [(4, 320, 5, 1, "bfloat16", "bfloat16"), (1, 52, 3, 1, "float32", "float32"), (3, 61, 7, 3, "float32", "float32"),
+@pytest.mark.parametrize("n,H,T,parts,ydt,out", [(4, 352, 5, 1, "bfloat16", "bfloat16"), (1, 52, 3, 1, "float32", "float32"), (3, 61, 7, 3, "float32", "float32"),
                                                  (6, 4096, 33, 4, "float32", "bfloat16"), (2, 2304, 9, 16, "float32", "bfloat16"),
                                                  (16, 40, 4, 1, "bfloat16", "bfloat16"), (4, 4096, 1100, 1, "bfloat16", "bfloat16"), (11, 64, 2, 2, "float32", "float32")])
 def test_hyper_update(K, n, H, T, parts, ydt, out):
@@ -221,7 +221,7 @@ def test_conv_delta_inputs(K, H, G, dk, dv, taps, dtype):
 
 
 @pytest.mark.parametrize("dtype", [F32, BF])
-@pytest.mark.parametrize("H,G,dim,vdim,rd,taps,own", [(4, 2, 12, 20, 6, 3, True), (8, 2, 64, 32, 16, 4, True), (4, 4, 16, 16, 16, 2, False), (3, 1, 7, 9, 0, 0, True),
+@pytest.mark.parametrize("H,G,dim,vdim,rd,taps,own", [(4, 2, 12, 20, 6, 3, True), (6, 2, 64, 48, 24, 4, True), (4, 4, 16, 16, 16, 2, False), (3, 1, 7, 9, 0, 0, True),
                                                       (6, 3, 32, 48, 2, 1, True), (2, 1, 128, 128, 128, 8, True), (8, 1, 24, 16, 8, 5, False)])
 def test_conv_norm_rope_kvwrite(K, H, G, dim, vdim, rd, taps, own, dtype):
     g = torch.Generator().manual_seed(H * dim + taps)
@@ -322,7 +322,7 @@ def test_delta_rule_chunks_and_steps_agree(K):
     _close(res[0][1], res[1][1], 1e-5, "state")
 
 
-@pytest.mark.parametrize("dtype,nh,nkv,d,page", [("bfloat16", 8, 2, 64, 64), ("bfloat16", 4, 2, 128, 64), ("bfloat16", 6, 3, 48, 16), ("bfloat16", 20, 1, 32, 32), ("float32", 8, 2, 64, 64),
+@pytest.mark.parametrize("dtype,nh,nkv,d,page", [("bfloat16", 8, 4, 64, 64), ("bfloat16", 4, 2, 128, 64), ("bfloat16", 6, 3, 48, 16), ("bfloat16", 20, 1, 32, 32), ("float32", 6, 2, 64, 64),
                                                  ("float32", 4, 2, 128, 16), ("float32", 3, 3, 12, 4), ("bfloat16", 2, 2, 24, 8), ("bfloat16", 4, 1, 128, 16)])
 @pytest.mark.parametrize("chunk", [1, 7, 40, 64, 100, 256])
 def test_attention_by_chunks(K, dtype, nh, nkv, d, page, chunk):
@@ -398,7 +398,7 @@ def _one_layer(kind, mixer, mlp=None, streams=2):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("dim,vdim,page,chunk", [(16, 16, 16, 48), (64, 32, 64, 64), (12, 20, 4, 33), (64, 64, 64, 100)])
+@pytest.mark.parametrize("dim,vdim,page,chunk", [(16, 16, 16, 48), (64, 48, 64, 128), (12, 20, 4, 33), (64, 64, 64, 100)])
 def test_a_key_at_a_chunks_edge(dim, vdim, page, chunk, dtype, tmp_path):
     """A token whose key outweighs all others for every query (its own embedding row makes it so), once next to every chunk edge and
     page border near 200, one position inside and outside: in a prompt, in portions and for decoded tokens."""
