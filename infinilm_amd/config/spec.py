@@ -31,9 +31,11 @@ class LayerSpec:
 class RunStart:
     """What is added to the residual stream right before a run (a pass over a stretch of layers that opens with it):
     `embedding` times the embedding's output as it was before the first layer (0: nothing), and row `vector_row` of the
-    model's tensor `ModelSpec.run_vectors` (None: no row)."""
+    model's tensor `ModelSpec.run_vectors` (None: no row).  `project_embedding`: then the stream x becomes W [x; x0], x0 the embedding's
+    output, W the model's matrix `ModelSpec.run_projection`."""
     embedding: float = 0.0
     vector_row: Optional[int] = None
+    project_embedding: bool = False
 
 
 @dataclass(frozen=True)
@@ -87,6 +89,8 @@ class ModelSpec:
     position_axes: int = 1
     # (name, rows): a tensor [rows, hidden] of vectors that runs add to the residual stream (`RunStart.vector_row`)
     run_vectors: Optional[tuple] = None
+    # name of the matrix [hidden, 2 hidden] by which a run makes the residual stream anew (`RunStart.project_embedding`)
+    run_projection: Optional[str] = None
     # {name: shape}: tensors of the model itself that several layers read (`bind_shared` of their arrangements)
     shared_tensors: Optional[Dict[str, tuple]] = None
 
@@ -115,6 +119,8 @@ class ModelSpec:
             if row is not None and (self.run_vectors is None or not 0 <= row < self.run_vectors[1]):
                 raise ValueError(f"order[{i}] adds row {row} of the run vectors, of which there are "
                                  f"{self.run_vectors[1] if self.run_vectors else 0}")
+            if run.start is not None and run.start.project_embedding and self.run_projection is None:
+                raise ValueError(f"order[{i}] projects the stream, but the model names no matrix for it")
         for i, run in enumerate(self.order):
             if run.cache is not None and not run.writes_cache:
                 if run.cache not in writers or writers[run.cache] > i:

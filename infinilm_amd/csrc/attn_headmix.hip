@@ -4,7 +4,9 @@
 //   ilm_qkv_norm_rope_kvwrite   per head of the fused projection rows [T, (nh + 2 nkv) d]: an RMS norm over the first
 //       dn entries of every q and k head with a weight shared by the heads (or none), a turn of the entry pairs
 //       (2i, 2i + 1), i < rd / 2, by the angle pos * freq[i], every value head divided by its root mean square
-//       over its first dv entries (or not); q and k are rewritten in place, k and v go to the paged cache.
+//       over its first dv entries (or not); q and k are rewritten in place, k and v go to the paged cache.  Options: the pairs are
+//       (i, i + rd / 2) (`half`); cosine and sine times a magnitude; rows [T, (nh + nkv) d] whose key heads, as projected, are
+//       the values too (`v_from_k`).
 //   ilm_attn_headmix            raw_g(j) = scale q_g . k_kv(g),j;  s_h(j) = sum_g M[h, g] raw_g(j);  over the keys j
 //       the token sees (its last `window` positions and the sequence's first `keep_first`, or all): p_h(j) = exp(s_h(j)) / (sum_j' exp(s_h(j')) + exp(sink_h));
 //       o_h = sum_j p_h(j) v_kv(h),j.  M and sink may be absent (identity, no term).
@@ -32,11 +34,11 @@ __global__ void __launch_bounds__(256)
 qkv_norm_rope_kvwrite_kernel(T* __restrict__ qkv, const int* __restrict__ pos, const float* __restrict__ freq,
                              const TW* __restrict__ wq, const TW* __restrict__ wk, T* __restrict__ kc, T* __restrict__ vc,
                              const int* __restrict__ slots, int nh, int nkv, int d, int dn, int dv, int rd, int v_norm,
-                             float eps, int page, int stride) {
+                             float eps, int page, int stride, int half, float mag, int v_from_k) {
     extern __shared__ float smem[];
     const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int head = blockIdx.y * 4 + wave;
-    const bool active = head < nh + 2 * nkv;      // (waves beyond the last head go along to the barriers and do nothing)
+    const bool active = head < nh + (v_from_k ? nkv : 2 * nkv);      // (waves beyond the last head go along to the barriers and do nothing)
     float* x = smem + wave * d;
     T* src = qkv + (size_t)t * stride + (size_t)(active ? head : 0) * d;
     const bool is_q = head < nh, is_k = !is_q && head < nh + nkv;
@@ -60,14 +62,21 @@ qkv_norm_rope_kvwrite_kernel(T* __restrict__ qkv, const int* __restrict__ pos, c
         for (int i = lane; i < rd / 2; i += 64) {
             float sn, cs;
             sincosf(p * freq[i], &sn, &cs);
-            const float u = x[2 * i], v = x[2 * i + 1];
-            x[2 * i] = u * cs - v * sn;
-            x[2 * i + 1] = v * cs + u * sn;
+            sn *= mag;
+            cs *= mag;
+            const int iu = half ? i : 2 * i, iv = half ? i + rd / 2 : 2 * i + 1;
+            const float u = x[iu], v = x[iv];
+            x[iu] = u * cs - v * sn;
+            x[iv] = v * cs + u * sn;
         }
     }
     __syncthreads();
     if (!active) return;
     const int slot = (slots != nullptr && !is_q) ? slots[t] : -1;
+    if (v_from_k && slot >= 0) {      // (the projected key is still in its place)
+        T* dst = vc + ((size_t)(slot / page) * nkv + (head - nh)) * d * page + slot % page;
+        for (int e = lane; e < d; e += 64) dst[(size_t)e * page] = e < dv ? src[e] : from_f32<T>(0.f);
+    }
     if (is_q || is_k)
         for (int e = lane; e < d; e += 64) src[e] = from_f32<T>(x[e]);
     if (slot >= 0) {
@@ -82,22 +91,140 @@ qkv_norm_rope_kvwrite_kernel(T* __restrict__ qkv, const int* __restrict__ pos, c
     }
 }
 
+// The same with pairs (i, i + rd / 2), eight entries of either side a thread: d, dn and rd multiples of 16, everything 16 bytes aligned,
+// values as they are.  One block a token; its cosines and sines pass through LDS.  Keys go to the cache alone.
+template <typename T>
+__device__ __forceinline__ void hm_load8(const T* p, float* v) { hm_load4(p, v); hm_load4(p + 4, v + 4); }
+__device__ __forceinline__ void hm_store8(float* p, const float* v) {
+    *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+    *reinterpret_cast<float4*>(p + 4) = make_float4(v[4], v[5], v[6], v[7]);
+}
+__device__ __forceinline__ void hm_store8(bf16* p, const float* v) {
+    uint32_t w[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) w[i] = (uint32_t)from_f32<bf16>(v[2 * i]).bits | ((uint32_t)from_f32<bf16>(v[2 * i + 1]).bits << 16);
+    *reinterpret_cast<uint4*>(p) = make_uint4(w[0], w[1], w[2], w[3]);
+}
+
+template <typename T, typename TW>
+__global__ void __launch_bounds__(256)
+qk_half_rope_kvwrite_kernel(T* __restrict__ qkv, const int* __restrict__ pos, const float* __restrict__ freq, const TW* __restrict__ wq,
+                            const TW* __restrict__ wk, T* __restrict__ kc, T* __restrict__ vc, const int* __restrict__ slots, int nh, int nkv,
+                            int d, int dn, int rd, float eps, int page, int stride, float mag, int v_from_k, int GS) {
+    extern __shared__ float smem[];      // cosines [rd / 2], sines [rd / 2]
+    // blocks go to the eight dies in turn: with this numbering a die takes a run of consecutive tokens, whose values lie beside one
+    // another in the cache
+    const int per = (int)gridDim.x >> 3;
+    const int t = (int)blockIdx.x < per * 8 ? (int)(blockIdx.x & 7) * per + (int)(blockIdx.x >> 3) : (int)blockIdx.x;
+    const int nr = rd / 2;
+    const float p = (float)pos[t];
+    for (int i = threadIdx.x; i < nr; i += 256) {
+        float sn, cs;
+        sincosf(p * freq[i], &sn, &cs);
+        smem[i] = cs * mag;
+        smem[nr + i] = sn * mag;
+    }
+    __syncthreads();
+    const int slot = slots != nullptr ? slots[t] : -1;
+    const int pg = slot >= 0 ? slot / page : 0, off = slot >= 0 ? slot % page : 0;
+    T* row = qkv + (size_t)t * stride;
+    const int qk_items = (nh + nkv) * GS, v_items = v_from_k || slot < 0 ? 0 : nkv * (d / 8);
+    for (int it = threadIdx.x; it < qk_items; it += 256) {
+        const int head = it / GS, l = it % GS;
+        const bool in = l < d / 16, turned = l < rd / 16;
+        const int e0 = !in ? 0 : (turned ? 8 * l : rd + 16 * (l - rd / 16)), e1 = !in ? 0 : (turned ? nr + 8 * l : e0 + 8);
+        T* src = row + (size_t)head * d;
+        float a[8], b[8];
+        hm_load8(src + e0, a);
+        hm_load8(src + e1, b);
+        const bool is_k = head >= nh;
+        if (is_k && v_from_k && slot >= 0 && in) {
+            T* dst = vc + ((size_t)pg * nkv + (head - nh)) * d * page + off;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                dst[(size_t)(e0 + e) * page] = from_f32<T>(a[e]);
+                dst[(size_t)(e1 + e) * page] = from_f32<T>(b[e]);
+            }
+        }
+        const TW* w = is_k ? wk : wq;
+        if (w != nullptr) {
+            float ss = 0.f;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) ss = fmaf(a[e], a[e], fmaf(b[e], b[e], ss));
+            if (!in) ss = 0.f;
+            for (int o = 1; o < GS; o <<= 1) ss += __shfl_xor(ss, o, 64);
+            const float rstd = 1.0f / sqrtf(ss / (float)dn + eps);
+            if (in && e0 < dn) {
+                float w0[8], w1[8];
+                hm_load8(w + e0, w0);
+                hm_load8(w + e1, w1);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) {
+                    a[e] = a[e] * rstd * w0[e];
+                    b[e] = b[e] * rstd * w1[e];
+                }
+            }
+        }
+        if (!in) continue;
+        if (turned) {
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                const float cs = smem[8 * l + e], sn = smem[nr + 8 * l + e], u = a[e], v = b[e];
+                a[e] = u * cs - v * sn;
+                b[e] = v * cs + u * sn;
+            }
+        }
+        T* dst = src;
+        if (is_k) {
+            if (slot < 0) continue;
+            dst = kc + (((size_t)pg * nkv + (head - nh)) * page + off) * d;
+        }
+        hm_store8(dst + e0, a);
+        hm_store8(dst + e1, b);
+    }
+    for (int it = threadIdx.x; it < v_items; it += 256) {
+        const int kv = it / (d / 8), e0 = it % (d / 8) * 8;
+        const T* src = row + (size_t)(nh + nkv + kv) * d + e0;
+        T* dst = vc + (((size_t)pg * nkv + kv) * d + e0) * page + off;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) dst[(size_t)e * page] = src[e];
+    }
+}
+
 extern "C" int ilm_qkv_norm_rope_kvwrite(void* qkv, const void* pos, const void* freq, const void* wq, const void* wk,
                                          void* kc, void* vc, const void* slots, int T_, int nh, int nkv, int d, int dn, int dv,
                                          int rd, int v_norm, float eps, int page, int stride, int dtype, int w_dt,
-                                         hipStream_t stream) {
+                                         int half, float mag, int v_from_k, hipStream_t stream) {
     ILM_REQUIRE(T_ > 0 && nh > 0 && nkv > 0 && d > 0 && page > 0, "qkv_norm_rope_kvwrite: bad sizes");
     ILM_REQUIRE(dn > 0 && dn <= d && dv > 0 && dv <= d, "qkv_norm_rope_kvwrite: %d / %d entries that count in heads of %d", dn, dv, d);
     ILM_REQUIRE(rd >= 0 && rd % 2 == 0 && rd <= dn && (rd == 0 || freq != nullptr), "qkv_norm_rope_kvwrite: %d turned entries", rd);
     ILM_REQUIRE((wq == nullptr) == (wk == nullptr), "qkv_norm_rope_kvwrite: a norm weight for q and k, or for neither");
     ILM_REQUIRE(d <= 4096 && T_ <= 0x7fffffff / 1, "qkv_norm_rope_kvwrite: head size %d", d);
     ILM_REQUIRE(slots == nullptr || (kc != nullptr && vc != nullptr), "qkv_norm_rope_kvwrite: slots without a cache");
+    ILM_REQUIRE(!(v_from_k && v_norm), "qkv_norm_rope_kvwrite: values are the projected keys or normed, not both");
+    ILM_REQUIRE(stride >= (nh + (v_from_k ? nkv : 2 * nkv)) * d, "qkv_norm_rope_kvwrite: rows of %d are too short", stride);
+    if (half && !v_norm && d % 16 == 0 && dn % 16 == 0 && rd % 16 == 0 && d <= 1024 && stride % 8 == 0 && (dv == d || !v_from_k)
+        && (((uintptr_t)qkv | (uintptr_t)kc | (uintptr_t)wq | (uintptr_t)wk) & 15) == 0 && (dtype == ILM_DTYPE_F32 || dtype == ILM_DTYPE_BF16)) {
+        int GS = 1;
+        while (GS * 16 < d) GS <<= 1;
+#define QH_LAUNCH(T__, TW__)                                                                                              \
+    qk_half_rope_kvwrite_kernel<T__, TW__><<<T_, 256, (size_t)rd * sizeof(float), stream>>>(                               \
+        (T__*)qkv, (const int*)pos, (const float*)freq, (const TW__*)wq, (const TW__*)wk, (T__*)kc, (T__*)vc,              \
+        (const int*)slots, nh, nkv, d, dn, rd, eps, page, stride, mag, v_from_k, GS)
+        if (dtype == ILM_DTYPE_F32 && w_dt == ILM_DTYPE_F32) QH_LAUNCH(float, float);
+        else if (dtype == ILM_DTYPE_BF16 && w_dt == ILM_DTYPE_BF16) QH_LAUNCH(bf16, bf16);
+        else if (dtype == ILM_DTYPE_BF16 && w_dt == ILM_DTYPE_F32) QH_LAUNCH(bf16, float);
+        else ILM_REQUIRE(false, "qkv_norm_rope_kvwrite: dtypes %d / %d", dtype, w_dt);
+#undef QH_LAUNCH
+        ILM_LAUNCH_CHECK("qkv_norm_rope_kvwrite (halves)");
+        return 0;
+    }
     dim3 grid(T_, (nh + 2 * nkv + 3) / 4);
     const size_t shm = (size_t)4 * d * sizeof(float);
 #define QN_LAUNCH(T__, TW__)                                                                                              \
     qkv_norm_rope_kvwrite_kernel<T__, TW__><<<grid, 256, shm, stream>>>(                                                  \
         (T__*)qkv, (const int*)pos, (const float*)freq, (const TW__*)wq, (const TW__*)wk, (T__*)kc, (T__*)vc,              \
-        (const int*)slots, nh, nkv, d, dn, dv, rd, v_norm, eps, page, stride)
+        (const int*)slots, nh, nkv, d, dn, dv, rd, v_norm, eps, page, stride, half, mag, v_from_k)
     if (dtype == ILM_DTYPE_F32 && w_dt == ILM_DTYPE_F32) QN_LAUNCH(float, float);
     else if (dtype == ILM_DTYPE_BF16 && w_dt == ILM_DTYPE_BF16) QN_LAUNCH(bf16, bf16);
     else if (dtype == ILM_DTYPE_BF16 && w_dt == ILM_DTYPE_F32) QN_LAUNCH(bf16, float);
@@ -282,5 +409,49 @@ extern "C" int ilm_attn_headmix(void* out, const void* q, const void* kc, const 
     }
 #undef HM_LAUNCH
     ILM_LAUNCH_CHECK("attn_headmix");
+    return 0;
+}
+
+// ------------------------------------------------------------------------------------------
+// o[t, h, :] *= sigmoid(g[t, h]): one number a head and token
+// ------------------------------------------------------------------------------------------
+template <typename T, bool VEC>
+__global__ void __launch_bounds__(256)
+head_gate_kernel(T* __restrict__ o, const T* __restrict__ g, int nh, int d, int o_stride, int g_stride) {
+    constexpr int N = VEC ? 8 : 1;
+    const int t = blockIdx.y, j = (blockIdx.x * 256 + threadIdx.x) * N;
+    if (j >= nh * d) return;
+    const float w = 1.0f / (1.0f + expf(-to_f32(g[(size_t)t * g_stride + j / d])));
+    T* p = o + (size_t)t * o_stride + j;
+    if constexpr (VEC) {
+        float v[8];
+        hm_load8(p, v);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] *= w;
+        hm_store8(p, v);
+    } else {
+        p[0] = from_f32<T>(to_f32(p[0]) * w);
+    }
+}
+
+extern "C" int ilm_head_gate(void* o, const void* g, int T_, int nh, int d, int o_stride, int g_stride, int dtype, hipStream_t stream) {
+    ILM_REQUIRE(T_ > 0 && nh > 0 && d > 0 && o_stride >= nh * d && g_stride >= nh, "head_gate: bad sizes");
+    ILM_REQUIRE(dtype == ILM_DTYPE_F32 || dtype == ILM_DTYPE_BF16, "head_gate: unknown dtype %d", dtype);
+    const bool vec = d % 8 == 0 && o_stride % 8 == 0 && ((uintptr_t)o & 15) == 0;
+    const int per = vec ? 2048 : 256;
+    const size_t es = dtype == ILM_DTYPE_F32 ? 4 : 2;
+    for (int t0 = 0; t0 < T_; t0 += 65535) {
+        const dim3 grid((nh * d + per - 1) / per, T_ - t0 < 65535 ? T_ - t0 : 65535);
+        void* op = (char*)o + (size_t)t0 * o_stride * es;
+        const void* gp = (const char*)g + (size_t)t0 * g_stride * es;
+        if (dtype == ILM_DTYPE_F32) {
+            if (vec) head_gate_kernel<float, true><<<grid, 256, 0, stream>>>((float*)op, (const float*)gp, nh, d, o_stride, g_stride);
+            else head_gate_kernel<float, false><<<grid, 256, 0, stream>>>((float*)op, (const float*)gp, nh, d, o_stride, g_stride);
+        } else {
+            if (vec) head_gate_kernel<bf16, true><<<grid, 256, 0, stream>>>((bf16*)op, (const bf16*)gp, nh, d, o_stride, g_stride);
+            else head_gate_kernel<bf16, false><<<grid, 256, 0, stream>>>((bf16*)op, (const bf16*)gp, nh, d, o_stride, g_stride);
+        }
+    }
+    ILM_LAUNCH_CHECK("head_gate");
     return 0;
 }

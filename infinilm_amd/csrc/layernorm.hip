@@ -5,6 +5,10 @@
 // over K (summed in order), or one row [H] that is added to every row (row stride 0).  Without w the kernel
 // only sums.  One block a row; the row stays in LDS between the three passes (sum, deviations, result), so the
 // variance is the mean of the squared deviations from the mean, not a difference of sums.
+//
+// ilm_add_rows does the same sum and then, in place of the norm, element by element
+//   x = tanh(alpha r) * w + b       (a "dynamic tanh", alpha one number in memory), or
+//   x = [r | r0]                    (the row beside a row of another tensor, for a product over both).
 #include "common.h"
 
 #define LN_MAX_ADD 4
@@ -103,7 +107,82 @@ add_layernorm_kernel(TO* __restrict__ x, float* __restrict__ r, LnAddends a, con
     }
 }
 
+// MODE 0: tanh(alpha r) w + b; 1: [r | r0] (rows of 2 H).  VEC as above.
+template <typename TO, typename TW, int MODE, bool VEC>
+__global__ void __launch_bounds__(256)
+add_rows_kernel(TO* __restrict__ x, float* __restrict__ r, LnAddends a, const float* __restrict__ alpha, const TW* __restrict__ w,
+                const TW* __restrict__ b, const float* __restrict__ r0, int H) {
+    constexpr int N = VEC ? 4 : 1;
+    const int t = blockIdx.y, j = (blockIdx.x * 256 + threadIdx.x) * N;
+    if (j >= H) return;
+    float* rr = r + (size_t)t * H + j;
+    float v[N];
+    if (VEC) {
+        const float4 q = *reinterpret_cast<const float4*>(rr);
+        v[0] = q.x; v[1 % N] = q.y; v[2 % N] = q.z; v[3 % N] = q.w;
+    } else {
+        v[0] = rr[0];
+    }
+    for (int i = 0; i < a.n; ++i) {
+        float u[N] = {};
+        for (int p = 0; p < a.parts[i]; ++p) {
+            const size_t at = (size_t)p * a.pstride[i] + (size_t)t * a.rstride[i] + j;
+            if (VEC) {
+                const float4 q = ln_load4(a.p[i], a.dt[i], at);
+                u[0] += q.x; u[1 % N] += q.y; u[2 % N] += q.z; u[3 % N] += q.w;
+            } else {
+                u[0] += ln_load(a.p[i], a.dt[i], at);
+            }
+        }
+#pragma unroll
+        for (int e = 0; e < N; ++e) v[e] = fmaf(a.scale[i], u[e], v[e]);
+    }
+    if (a.n > 0) {
+        if (VEC) *reinterpret_cast<float4*>(rr) = make_float4(v[0], v[1 % N], v[2 % N], v[3 % N]);
+        else rr[0] = v[0];
+    }
+    if (MODE == 0) {
+        const float al = *alpha;
+        float y[N];
+        if (VEC) {
+            const float4 ww = ln_get4(w + j), bb = b != nullptr ? ln_get4(b + j) : make_float4(0.f, 0.f, 0.f, 0.f);
+            y[0] = tanhf(al * v[0]) * ww.x + bb.x;
+            y[1 % N] = tanhf(al * v[1 % N]) * ww.y + bb.y;
+            y[2 % N] = tanhf(al * v[2 % N]) * ww.z + bb.z;
+            y[3 % N] = tanhf(al * v[3 % N]) * ww.w + bb.w;
+            ln_put4(x + (size_t)t * H + j, make_float4(y[0], y[1 % N], y[2 % N], y[3 % N]));
+        } else {
+            x[(size_t)t * H + j] = from_f32<TO>(tanhf(al * v[0]) * to_f32(w[j]) + (b != nullptr ? to_f32(b[j]) : 0.f));
+        }
+    } else {
+        TO* xr = x + (size_t)t * 2 * H + j;
+        const float* o = r0 + (size_t)t * H + j;
+        if (VEC) {
+            ln_put4(xr, make_float4(v[0], v[1 % N], v[2 % N], v[3 % N]));
+            ln_put4(xr + H, *reinterpret_cast<const float4*>(o));
+        } else {
+            xr[0] = from_f32<TO>(v[0]);
+            xr[H] = from_f32<TO>(o[0]);
+        }
+    }
+}
+
 #define LN_WIDE_ROWS 512
+
+// the addends' arguments of an entry point as one LnAddends `a`
+#define LN_FILL(what)                                                                                                        \
+    const void* ps[4] = {p0, p1, p2, p3};                                                                                   \
+    const int dts[4] = {dt0, dt1, dt2, dt3}, parts[4] = {parts0, parts1, parts2, parts3};                                   \
+    const long pss[4] = {ps0, ps1, ps2, ps3}, rss[4] = {rs0, rs1, rs2, rs3};                                                \
+    const float scs[4] = {sc0, sc1, sc2, sc3};                                                                              \
+    a.n = n_add;                                                                                                            \
+    for (int i = 0; i < LN_MAX_ADD; ++i) {                                                                                  \
+        a.p[i] = ps[i]; a.dt[i] = dts[i]; a.parts[i] = parts[i]; a.pstride[i] = pss[i]; a.rstride[i] = rss[i]; a.scale[i] = scs[i];\
+        if (i < n_add) {                                                                                                    \
+            ILM_REQUIRE(ps[i] != nullptr && parts[i] >= 1, what ": addend %d is empty", i);                                 \
+            ILM_REQUIRE(dts[i] == ILM_DTYPE_F32 || dts[i] == ILM_DTYPE_BF16, what ": addend %d has unknown dtype %d", i, dts[i]);\
+        }                                                                                                                   \
+    }
 
 extern "C" int ilm_add_layernorm_max_addends() { return LN_MAX_ADD; }
 
@@ -117,18 +196,7 @@ extern "C" int ilm_add_layernorm(void* x, void* r, const void* w, const void* b,
     ILM_REQUIRE(rows > 0 && H > 0 && H <= 16384, "add_layernorm: bad sizes rows=%d H=%d", rows, H);
     ILM_REQUIRE(n_add >= 0 && n_add <= LN_MAX_ADD, "add_layernorm: %d addends, at most %d", n_add, LN_MAX_ADD);
     LnAddends a;
-    const void* ps[4] = {p0, p1, p2, p3};
-    const int dts[4] = {dt0, dt1, dt2, dt3}, parts[4] = {parts0, parts1, parts2, parts3};
-    const long pss[4] = {ps0, ps1, ps2, ps3}, rss[4] = {rs0, rs1, rs2, rs3};
-    const float scs[4] = {sc0, sc1, sc2, sc3};
-    a.n = n_add;
-    for (int i = 0; i < LN_MAX_ADD; ++i) {
-        a.p[i] = ps[i]; a.dt[i] = dts[i]; a.parts[i] = parts[i]; a.pstride[i] = pss[i]; a.rstride[i] = rss[i]; a.scale[i] = scs[i];
-        if (i < n_add) {
-            ILM_REQUIRE(ps[i] != nullptr && parts[i] >= 1, "add_layernorm: addend %d is empty", i);
-            ILM_REQUIRE(dts[i] == ILM_DTYPE_F32 || dts[i] == ILM_DTYPE_BF16, "add_layernorm: addend %d has unknown dtype %d", i, dts[i]);
-        }
-    }
+    LN_FILL("add_layernorm")
     const size_t shm = (size_t)H * sizeof(float);
     bool vec = H % 4 == 0 && ((uintptr_t)r & 15) == 0 && ((uintptr_t)x & 15) == 0 && ((uintptr_t)w & 15) == 0 && ((uintptr_t)b & 15) == 0;
     for (int i = 0; i < n_add; ++i)
@@ -150,5 +218,50 @@ extern "C" int ilm_add_layernorm(void* x, void* r, const void* w, const void* b,
 #undef LN_LAUNCH
 #undef LN_LAUNCH_NV
     ILM_LAUNCH_CHECK("add_layernorm");
+    return 0;
+}
+
+// mode 0: x [rows, H] = tanh(alpha r) w + b (b may be null); 1: x [rows, 2 H] = [r | r0], r0 float [rows, H]
+extern "C" int ilm_add_rows(void* x, void* r, const void* alpha, const void* w, const void* b, const void* r0, int mode, int rows, int H, int out_dt,
+                            int w_dt, int n_add,
+                            const void* p0, int dt0, int parts0, long ps0, long rs0, float sc0,
+                            const void* p1, int dt1, int parts1, long ps1, long rs1, float sc1,
+                            const void* p2, int dt2, int parts2, long ps2, long rs2, float sc2,
+                            const void* p3, int dt3, int parts3, long ps3, long rs3, float sc3, hipStream_t stream) {
+    ILM_REQUIRE(rows > 0 && H > 0, "add_rows: bad sizes rows=%d H=%d", rows, H);
+    ILM_REQUIRE(n_add >= 0 && n_add <= LN_MAX_ADD, "add_rows: %d addends, at most %d", n_add, LN_MAX_ADD);
+    ILM_REQUIRE(mode == 0 ? (alpha != nullptr && w != nullptr) : (mode == 1 && r0 != nullptr), "add_rows: mode %d lacks its operands", mode);
+    LnAddends a;
+    LN_FILL("add_rows")
+    bool vec = H % 4 == 0 && (((uintptr_t)r | (uintptr_t)x | (uintptr_t)w | (uintptr_t)b | (uintptr_t)r0) & 15) == 0;
+    for (int i = 0; i < n_add; ++i) vec = vec && ((uintptr_t)ps[i] & 15) == 0 && pss[i] % 4 == 0 && rss[i] % 4 == 0;
+    const int per = vec ? 1024 : 256;
+#define AR_ONE(TO_, TW_, M_, V_, T0_, N_)                                                                                                 \
+    {                                                                                                                                    \
+        LnAddends c = a;                                                                                                                 \
+        for (int i = 0; i < n_add; ++i)                                                                                                  \
+            c.p[i] = (const char*)a.p[i] + (size_t)(T0_) * a.rstride[i] * (a.dt[i] == ILM_DTYPE_F32 ? 4 : 2);                             \
+        add_rows_kernel<TO_, TW_, M_, V_><<<dim3((H + per - 1) / per, N_), 256, 0, stream>>>(                                             \
+            (TO_*)x + (size_t)(T0_) * H * (M_ + 1), (float*)r + (size_t)(T0_) * H, c, (const float*)alpha, (const TW_*)w, (const TW_*)b,   \
+            r0 != nullptr ? (const float*)r0 + (size_t)(T0_) * H : nullptr, H);                                                           \
+    }
+#define AR_LAUNCH(TO_, TW_, M_)                                                                                                           \
+    for (int t0 = 0; t0 < rows; t0 += 65535) {                                                                                            \
+        const int n = rows - t0 < 65535 ? rows - t0 : 65535;                                                                              \
+        if (vec) AR_ONE(TO_, TW_, M_, true, t0, n) else AR_ONE(TO_, TW_, M_, false, t0, n)                                                 \
+    }
+    if (mode == 1) {
+        if (out_dt == ILM_DTYPE_F32) { AR_LAUNCH(float, float, 1) }
+        else if (out_dt == ILM_DTYPE_BF16) { AR_LAUNCH(bf16, float, 1) }
+        else ILM_REQUIRE(false, "add_rows: unknown dtype %d", out_dt);
+    }
+    else if (out_dt == ILM_DTYPE_F32 && w_dt == ILM_DTYPE_F32) { AR_LAUNCH(float, float, 0) }
+    else if (out_dt == ILM_DTYPE_BF16 && w_dt == ILM_DTYPE_BF16) { AR_LAUNCH(bf16, bf16, 0) }
+    else if (out_dt == ILM_DTYPE_BF16 && w_dt == ILM_DTYPE_F32) { AR_LAUNCH(bf16, float, 0) }
+    else if (out_dt == ILM_DTYPE_F32 && w_dt == ILM_DTYPE_BF16) { AR_LAUNCH(float, bf16, 0) }
+    else ILM_REQUIRE(false, "add_rows: unknown dtypes %d / %d", out_dt, w_dt);
+#undef AR_LAUNCH
+#undef AR_ONE
+    ILM_LAUNCH_CHECK("add_rows");
     return 0;
 }

@@ -55,7 +55,9 @@ _SIGNATURES = {
     "ilm_decay_scan": [_P, _I, _P, _P, _I, _I, _P, _I, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _P, _P, _I, _P],
     "ilm_sigmoid_root": [_P, _P, _P, _I, _I, _I, _I, _F, _I, _I, _P],
     "ilm_add_layernorm": [_P, _P, _P, _P, _I, _I, _F, _I, _I, _I] + [_P, _I, _I, _L, _L, _F] * 4 + [_P],
-    "ilm_qkv_norm_rope_kvwrite": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _I, _P],
+    "ilm_add_rows": [_P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I] + [_P, _I, _I, _L, _L, _F] * 4 + [_P],
+    "ilm_qkv_norm_rope_kvwrite": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _I, _I, _F, _I, _P],
+    "ilm_head_gate": [_P, _P, _I, _I, _I, _I, _I, _I, _P],
     "ilm_attn_headmix": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P],
     "ilm_headmix_queries": [_P, _P, _P, _I, _I, _I, _I, _I, _P],
     "ilm_attn_headmix_mfma": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _F, _I, _P, _I, _I, _P, _I, _I, _P],
@@ -65,9 +67,10 @@ _SIGNATURES = {
     "ilm_embed_gate": [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
     "ilm_softcap": [_P, _L, _F, _P],
     "ilm_moe_route": [_P, _P, _P, _I, _I, _I, _I, _I, _F, _P],
+    "ilm_moe_route_groups": [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _P],
     "ilm_moe_sort": [_P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _P],
     "ilm_moe_gemm": [_P, _I, _P, _I, _P, _I, _P, _P, _L, _I, _P, _P, _I, _I, _I, _I, _F, _F, _I, _I, _I, _I, _I, _P],
-    "ilm_moe_combine": [_P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _P, _I, _P],
+    "ilm_moe_combine": [_P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _P, _P, _I, _I, _P],
     "ilm_maps_norm_rope_kvwrite": [_P, _P, _I, _I, _I, _I, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _I, _I, _P],
     "ilm_attn_maps_mfma": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P, _P, _P, _P, _P, _F, _F, _F, _I, _P],
     "ilm_maps_combine": [_P, _P, _I, _I, _I, _I, _I, _P, _P, _P, _P, _F, _F, _F, _I, _I, _P],
@@ -88,6 +91,8 @@ _SIGNATURES = {
                                    _I, _I, _I, _P],
     "ilm_delta_step": [_P, _P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P, _P, _I, _F, _I, _I, _I, _I, _P],
     "ilm_delta_chunks": [_P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P, _P],
+    "ilm_mlstm_step": [_P, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _F, _F, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P, _I, _F, _I, _I, _P],
+    "ilm_mlstm_chunks": [_P, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _F, _F, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P, _I, _F, _I, _I, _P, _P],
     "ilm_norm_add_norm": [_P, _P, _P, _P, _P, _I, _I, _F, _F, _F, _I, _I, _I, _I, _I, _L, _P],
 }
 
@@ -130,6 +135,9 @@ def load(verbose: bool = True) -> ctypes.CDLL:
     lib.ilm_attn_maps_mfma_ok.argtypes = [c_int, c_int, c_int, c_int, c_int, c_int]
     lib.ilm_delta_step_norm_ok.restype = c_int
     lib.ilm_delta_step_norm_ok.argtypes = [c_int, c_int]
+    for name in ("ilm_mlstm_step_norm_ok", "ilm_mlstm_chunk_ws"):
+        getattr(lib, name).restype = c_int
+        getattr(lib, name).argtypes = [c_int, c_int]
     lib.ilm_delta_chunk_ws.restype = c_int
     lib.ilm_delta_chunk_ws.argtypes = [c_int, c_int]
     lib.ilm_attn_static_init.restype = c_int

@@ -2,18 +2,24 @@
 //
 //   ilm_moe_route     per token: the `top` largest of E router logits (ties to the lower index), their indices and as weights
 //                     a scale times sigmoid(logit) or the logit's softmax over all E experts; one wave a token, all float32.
+//   ilm_moe_route_groups  the same with softmax scores s, where the choice goes by s + correction, the experts form equal groups of
+//                     neighbours of which only the `keep` with the largest member may be chosen from, and a chosen expert's weight is a
+//                     scale times s divided by the sum of the chosen scores.
 //   ilm_moe_sort      the (token, slot) pairs of a step ordered by expert: offsets per expert, the pair at every sorted
 //                     place and the place of every pair, and the list of row tiles (expert, first place, rows) that the
 //                     products below walk.  One block; the order inside an expert is whatever the atomics give, which no
-//                     row's result depends on.
+//                     row's result depends on.  Pairs whose index is E or more ("identity" experts, whose result is the token's
+//                     row itself) are left out; their place is -1.
 //   ilm_moe_gemm      for every tile of rows of one expert e: out[place] = f(W_e x[place]) with
 //                       GLU form    x = weight(pair) * h[token of the pair], W_e = [gate rows | up rows],
-//                                   g = min(gate, limit), u = clamp(up, -limit, limit), out = g sigmoid(alpha g) (u + 1)
+//                                   g = min(gate, limit), u = clamp(up, -limit, limit), out = g sigmoid(alpha g) (u + 1),
+//                                   or silu(gate) up; without the pairs' weights x is h itself
 //                       plain form  x = rows in sorted order (or, with the list of pairs, the pairs' token rows), out = W_e x
 //                                   or the square of relu(W_e x)
 //                     bfloat16 on v_mfma_f32_16x16x32_bf16 (tiles of 64 rows x 64 outputs, operands through LDS in steps of
 //                     64 k, the next step's loads in flight), float32 and odd sizes by FMA in ascending k.
-//   ilm_moe_combine   y[t] = sum over the token's slots of (weight of the pair *) out[place of (t, slot)] (+ shared[t] * sigmoid(sg[t])).
+//   ilm_moe_combine   (identity pairs take the token's row for out[place])
+//                     y[t] = sum over the token's slots of (weight of the pair *) out[place of (t, slot)] (+ shared[t] * sigmoid(sg[t])).
 //   ilm_glu_clamp     the experts' activation on fused [gate | up] rows of a dense product.
 #include "common.h"
 
@@ -93,6 +99,98 @@ extern "C" int ilm_moe_route(void* ids, void* wts, const void* z, int T_, int E,
     return 0;
 }
 
+// One wave a token.  The choice scores lie in LDS while the groups are compared; the pairs' scores without the correction are taken
+// from the logits again.
+__global__ void __launch_bounds__(256)
+moe_route_groups_kernel(int* __restrict__ ids, float* __restrict__ wts, const float* __restrict__ z, const void* __restrict__ corr, int c_dt,
+                        int T_, int E, int top, int z_stride, int groups, int keep, float wscale) {
+    __shared__ float cs[4][MOE_MAX_E];
+    __shared__ float gs[4][MOE_MAX_E];
+    const int w = threadIdx.x >> 6, t = blockIdx.x * 4 + w, lane = threadIdx.x & 63;
+    const bool live = t < T_;
+    const float* row = z + (size_t)(live ? t : 0) * z_stride;
+    float zmax = -INFINITY, zsum = 0.f;
+    for (int e = lane; e < E; e += 64) zmax = fmaxf(zmax, row[e]);
+    zmax = wave_max(zmax);
+    for (int e = lane; e < E; e += 64) zsum += expf(row[e] - zmax);
+    zsum = wave_sum(zsum);
+    for (int e = lane; e < E; e += 64) {
+        const float c = corr == nullptr ? 0.f : (c_dt == ILM_DTYPE_F32 ? ((const float*)corr)[e] : to_f32(((const bf16*)corr)[e]));
+        cs[w][e] = expf(row[e] - zmax) / zsum + c;
+    }
+    __syncthreads();
+    // the largest of `n` values, ties to the lower index, taken out of the list; every lane gets the index
+    auto take = [&](float* v, int n, int fallback) {
+        float best = -INFINITY;
+        int bi = 0x7fffffff;
+        for (int i = lane; i < n; i += 64)
+            if (v[i] > best || (v[i] == best && i < bi)) { best = v[i]; bi = i; }
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) {
+            const float ov = __shfl_xor(best, o, 64);
+            const int oi = __shfl_xor(bi, o, 64);
+            if (ov > best || (ov == best && oi < bi)) { best = ov; bi = oi; }
+        }
+        if (bi >= n) bi = fallback;        // nothing compared larger (a row of NaNs): any valid index
+        return bi;
+    };
+    if (groups > 1 && keep < groups) {
+        const int size = E / groups;
+        for (int g = lane; g < groups; g += 64) {
+            float b = -INFINITY;
+            for (int i = 0; i < size; ++i) b = fmaxf(b, cs[w][g * size + i]);
+            gs[w][g] = b;
+        }
+        __syncthreads();
+        unsigned long long kept[MOE_MAX_E / 64] = {};
+        for (int k = 0; k < keep; ++k) {
+            const int g = take(gs[w], groups, k);
+#pragma unroll
+            for (int i = 0; i < MOE_MAX_E / 64; ++i)
+                if ((g >> 6) == i) kept[i] |= 1ull << (g & 63);
+            __syncthreads();
+            if (lane == 0) gs[w][g] = -INFINITY;
+            __syncthreads();
+        }
+        for (int e = lane; e < E; e += 64) {
+            const int g = e / size;
+            bool in = false;
+#pragma unroll
+            for (int i = 0; i < MOE_MAX_E / 64; ++i)
+                if ((g >> 6) == i) in = (kept[i] >> (g & 63)) & 1ull;
+            if (!in) cs[w][e] = -INFINITY;
+        }
+        __syncthreads();
+    }
+    float sum = 0.f;
+    for (int s = 0; s < top; ++s) {
+        const int e = take(cs[w], E, s);
+        const float sc = expf(row[e] - zmax) / zsum;
+        sum += sc;
+        if (live && lane == 0) {
+            ids[(size_t)t * top + s] = e;
+            wts[(size_t)t * top + s] = sc;
+        }
+        __syncthreads();
+        if (lane == 0) cs[w][e] = -INFINITY;
+        __syncthreads();
+    }
+    if (live && lane == 0)
+        for (int s = 0; s < top; ++s) wts[(size_t)t * top + s] = wts[(size_t)t * top + s] / (sum + 1e-20f) * wscale;
+}
+
+extern "C" int ilm_moe_route_groups(void* ids, void* wts, const void* z, const void* corr, int c_dt, int T_, int E, int top, int z_stride, int groups,
+                                    int keep, float wscale, hipStream_t stream) {
+    ILM_REQUIRE(T_ > 0 && E > 0 && E <= MOE_MAX_E && top > 0 && top <= E, "moe_route_groups: %d tokens, %d experts (at most %d), top %d", T_, E,
+                MOE_MAX_E, top);
+    ILM_REQUIRE(groups > 0 && E % groups == 0 && keep > 0 && keep <= groups && top <= keep * (E / groups),
+                "moe_route_groups: %d of %d groups of %d experts, top %d", keep, groups, E, top);
+    moe_route_groups_kernel<<<(T_ + 3) / 4, 256, 0, stream>>>((int*)ids, (float*)wts, (const float*)z, corr, c_dt, T_, E, top, z_stride, groups,
+                                                              keep, wscale);
+    ILM_LAUNCH_CHECK("moe_route_groups");
+    return 0;
+}
+
 // ---- ordering by expert --------------------------------------------------------------------------------------------
 __global__ void __launch_bounds__(1024)
 moe_sort_kernel(int* __restrict__ offsets, int* __restrict__ perm, int* __restrict__ inv, int* __restrict__ tiles, int* __restrict__ n_tiles,
@@ -134,6 +232,8 @@ moe_sort_kernel(int* __restrict__ offsets, int* __restrict__ perm, int* __restri
             const int at = atomicAdd(&cur[e], 1);
             perm[at] = p;
             inv[p] = at;
+        } else {
+            inv[p] = -1;
         }
     }
 }
@@ -152,7 +252,11 @@ extern "C" int ilm_moe_sort(void* offsets, void* perm, void* inv, void* tiles, v
 }
 
 // ---- the experts' products -----------------------------------------------------------------------------------------
-__device__ __forceinline__ float moe_glu(float g, float u, float limit, float alpha) {
+#define MOE_ACT_NONE 0
+#define MOE_ACT_RELU2 1     // plain form
+#define MOE_ACT_SILU 2      // GLU form: silu(gate) up, no limits
+__device__ __forceinline__ float moe_glu(float g, float u, float limit, float alpha, int act) {
+    if (act == MOE_ACT_SILU) return g * moe_sigmoid(g) * u;
     g = fminf(g, limit);
     u = fminf(fmaxf(u, -limit), limit);
     return g * moe_sigmoid(alpha * g) * (u + 1.0f);
@@ -222,7 +326,7 @@ moe_gemm_mfma_kernel(bf16* __restrict__ out, int ld_out, const bf16* __restrict_
                 /* the pair's score on the rows as they are loaded: with few rows an expert this kernel streams W, and */  \
                 /* measured against the score on the float sums (as the many-rows kernel has it) it is the faster one */   \
                 /* here (192 against 235 us for 64 tokens x 2 of 16 experts at width 4,096) */                             \
-                if (GLU) v = moe_scale8(v, src_w[lr + 32 * i]);                                                            \
+                if (GLU && pair_w != nullptr) v = moe_scale8(v, src_w[lr + 32 * i]);                                                            \
             }                                                                                                              \
             XR[i] = v;                                                                                                     \
         }                                                                                                                  \
@@ -296,8 +400,8 @@ moe_gemm_mfma_kernel(bf16* __restrict__ out, int ld_out, const bf16* __restrict_
                 const int n = n0 + hb * MOE_TN + wave * 16 + q * 4 + i;
                 if (n < N) {
                     float v = acc[hb][g][i];
-                    if (GLU) v = moe_glu(v, acc[WR - 1][g][i], limit, alpha);
-                    else if (act == 1) { v = fmaxf(v, 0.f); v *= v; }
+                    if (GLU) v = moe_glu(v, acc[WR - 1][g][i], limit, alpha, act);
+                    else if (act == MOE_ACT_RELU2) { v = fmaxf(v, 0.f); v *= v; }
                     orow[n] = from_f32<bf16>(v);
                 }
             }
@@ -455,8 +559,8 @@ moe_gemm_mfma128_kernel(bf16* __restrict__ out, int ld_out, const bf16* __restri
             for (int i = 0; i < 4; ++i) {
                 if (nb + i < N) {
                     float v = acc[f][g][i];
-                    if (GLU) v = moe_glu(sw * v, sw * acc[f + 2][g][i], limit, alpha);
-                    else if (act == 1) { v = fmaxf(v, 0.f); v *= v; }
+                    if (GLU) v = moe_glu(sw * v, sw * acc[f + 2][g][i], limit, alpha, act);
+                    else if (act == MOE_ACT_RELU2) { v = fmaxf(v, 0.f); v *= v; }
                     orow[nb + i] = from_f32<bf16>(v);
                 }
             }
@@ -545,8 +649,8 @@ moe_gemm_plain_kernel(T* __restrict__ out, int ld_out, const T* __restrict__ X, 
             const int n = n0 + tx + 16 * b;
             if (n < N) {
                 float v = acc[0][a][b];
-                if (GLU) v = moe_glu(v, acc[WR - 1][a][b], limit, alpha);
-                else if (act == 1) { v = fmaxf(v, 0.f); v *= v; }
+                if (GLU) v = moe_glu(v, acc[WR - 1][a][b], limit, alpha, act);
+                else if (act == MOE_ACT_RELU2) { v = fmaxf(v, 0.f); v *= v; }
                 out[(size_t)(place0 + m) * ld_out + n] = from_f32<T>(v);
             }
         }
@@ -556,7 +660,8 @@ moe_gemm_plain_kernel(T* __restrict__ out, int ld_out, const T* __restrict__ X, 
 extern "C" int ilm_moe_gemm(void* out, int ld_out, const void* X, int ldx, const void* perm, int top, const void* pair_w, const void* W,
                             long w_expert, int ldw, const void* tiles, const void* n_tiles, int max_tiles, int N, int K, int glu,
                             float limit, float alpha, int act, int dtype, int force_plain, int tile_rows, int wide_mode, hipStream_t stream) {
-    ILM_REQUIRE(act == 0 || (act == 1 && !glu), "moe_gemm: activation %d (0: none, 1: the square of relu, in the plain form)", act);
+    ILM_REQUIRE(act == MOE_ACT_NONE || act == (glu ? MOE_ACT_SILU : MOE_ACT_RELU2), "moe_gemm: activation %d (0: none, 1: the square of relu, in the plain form, "
+                "2: silu, in the GLU form)", act);
     ILM_REQUIRE(tile_rows == MOE_TM || tile_rows == MOE_BM, "moe_gemm: tiles of %d rows (%d or %d)", tile_rows, MOE_TM, MOE_BM);
     ILM_REQUIRE(max_tiles > 0 && max_tiles <= 65535 && N > 0 && K > 0 && top > 0, "moe_gemm: bad sizes (tiles %d, N %d, K %d)", max_tiles, N, K);
     ILM_REQUIRE(ld_out >= N && ldx >= K && ldw >= K, "moe_gemm: rows shorter than their products");
@@ -600,34 +705,64 @@ extern "C" int ilm_moe_gemm(void* out, int ld_out, const void* X, int ldx, const
 }
 
 // ---- the sum over a token's experts --------------------------------------------------------------------------------
-template <typename T>
-__global__ void moe_combine_kernel(T* __restrict__ y, const T* __restrict__ pair_out, const int* __restrict__ inv, int top,
-                                   const T* __restrict__ shared, const float* __restrict__ sg, int sg_stride, int H, int ld_pair,
-                                   const float* __restrict__ pair_w) {
+__device__ __forceinline__ void moe_get(const float* p, float (&v)[1]) { v[0] = *p; }
+__device__ __forceinline__ void moe_get(const bf16* p, float (&v)[1]) { v[0] = to_f32(*p); }
+__device__ __forceinline__ void moe_get(const float* p, float (&v)[4]) {
+    const float4 a = *reinterpret_cast<const float4*>(p);
+    v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
+}
+__device__ __forceinline__ void moe_get(const bf16* p, float (&v)[4]) {
+    const uint2 a = *reinterpret_cast<const uint2*>(p);
+    v[0] = __uint_as_float(a.x << 16); v[1] = __uint_as_float(a.x & 0xffff0000u);
+    v[2] = __uint_as_float(a.y << 16); v[3] = __uint_as_float(a.y & 0xffff0000u);
+}
+__device__ __forceinline__ void moe_put(float* p, const float (&v)[1]) { *p = v[0]; }
+__device__ __forceinline__ void moe_put(bf16* p, const float (&v)[1]) { *p = from_f32<bf16>(v[0]); }
+__device__ __forceinline__ void moe_put(float* p, const float (&v)[4]) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
+__device__ __forceinline__ void moe_put(bf16* p, const float (&v)[4]) {
+    *reinterpret_cast<uint2*>(p) = make_uint2((uint32_t)from_f32<bf16>(v[0]).bits | ((uint32_t)from_f32<bf16>(v[1]).bits << 16),
+                                              (uint32_t)from_f32<bf16>(v[2]).bits | ((uint32_t)from_f32<bf16>(v[3]).bits << 16));
+}
+
+template <typename T, int N>
+__global__ void __launch_bounds__(256)
+moe_combine_kernel(T* __restrict__ y, const T* __restrict__ pair_out, const int* __restrict__ inv, int top,
+                   const T* __restrict__ shared, const float* __restrict__ sg, int sg_stride, int H, int ld_pair,
+                   const float* __restrict__ pair_w, const T* __restrict__ x, int x_stride) {
     const int t = blockIdx.x;
     const float gate = sg != nullptr ? moe_sigmoid(sg[(size_t)t * sg_stride]) : 1.0f;
-    for (int j = threadIdx.x; j < H; j += blockDim.x) {
-        float v = 0.f;
+    for (int j = threadIdx.x * N; j < H; j += 256 * N) {
+        float v[N] = {}, o[N];
         for (int s = 0; s < top; ++s) {
-            const float o = to_f32(pair_out[(size_t)inv[(size_t)t * top + s] * ld_pair + j]);
-            v = pair_w != nullptr ? fmaf(pair_w[(size_t)t * top + s], o, v) : v + o;
+            const int at = inv[(size_t)t * top + s];
+            if (at < 0 && x == nullptr) continue;
+            moe_get(at < 0 ? x + (size_t)t * x_stride + j : pair_out + (size_t)at * ld_pair + j, o);
+            const float w = pair_w != nullptr ? pair_w[(size_t)t * top + s] : 1.0f;
+#pragma unroll
+            for (int e = 0; e < N; ++e) v[e] = fmaf(w, o[e], v[e]);
         }
-        if (shared != nullptr) v = fmaf(to_f32(shared[(size_t)t * H + j]), gate, v);
-        y[(size_t)t * H + j] = from_f32<T>(v);
+        if (shared != nullptr) {
+            moe_get(shared + (size_t)t * H + j, o);
+#pragma unroll
+            for (int e = 0; e < N; ++e) v[e] = fmaf(o[e], gate, v[e]);
+        }
+        moe_put(y + (size_t)t * H + j, v);
     }
 }
 
+// x: the tokens' rows for pairs without a place (identity experts), or null
 extern "C" int ilm_moe_combine(void* y, const void* pair_out, const void* inv, int top, const void* shared, const void* sg, int sg_stride,
-                               int T_, int H, int ld_pair, const void* pair_w, int dtype, hipStream_t stream) {
-    ILM_REQUIRE(T_ > 0 && H > 0 && top > 0 && ld_pair >= H, "moe_combine: bad sizes");
-    if (dtype == ILM_DTYPE_F32)
-        moe_combine_kernel<float><<<T_, 256, 0, stream>>>((float*)y, (const float*)pair_out, (const int*)inv, top, (const float*)shared,
-                                                          (const float*)sg, sg_stride, H, ld_pair, (const float*)pair_w);
-    else if (dtype == ILM_DTYPE_BF16)
-        moe_combine_kernel<bf16><<<T_, 256, 0, stream>>>((bf16*)y, (const bf16*)pair_out, (const int*)inv, top, (const bf16*)shared,
-                                                         (const float*)sg, sg_stride, H, ld_pair, (const float*)pair_w);
-    else
-        ILM_REQUIRE(false, "moe_combine: unknown dtype %d", dtype);
+                               int T_, int H, int ld_pair, const void* pair_w, const void* x, int x_stride, int dtype, hipStream_t stream) {
+    ILM_REQUIRE(T_ > 0 && H > 0 && top > 0 && ld_pair >= H && (x == nullptr || x_stride >= H), "moe_combine: bad sizes");
+    const bool vec = H % 4 == 0 && ld_pair % 4 == 0 && x_stride % 4 == 0
+                     && (((uintptr_t)y | (uintptr_t)pair_out | (uintptr_t)shared | (uintptr_t)x) & 15) == 0;
+#define MC_LAUNCH(T__, N__)                                                                                                            \
+    moe_combine_kernel<T__, N__><<<T_, 256, 0, stream>>>((T__*)y, (const T__*)pair_out, (const int*)inv, top, (const T__*)shared,        \
+                                                         (const float*)sg, sg_stride, H, ld_pair, (const float*)pair_w, (const T__*)x, x_stride)
+    if (dtype == ILM_DTYPE_F32) { if (vec) MC_LAUNCH(float, 4); else MC_LAUNCH(float, 1); }
+    else if (dtype == ILM_DTYPE_BF16) { if (vec) MC_LAUNCH(bf16, 4); else MC_LAUNCH(bf16, 1); }
+    else ILM_REQUIRE(false, "moe_combine: unknown dtype %d", dtype);
+#undef MC_LAUNCH
     ILM_LAUNCH_CHECK("moe_combine");
     return 0;
 }
@@ -640,7 +775,7 @@ __global__ void glu_clamp_kernel(T* __restrict__ out, const T* __restrict__ gu, 
     const long t = i / I;
     const int j = (int)(i % I);
     const T* row = gu + (size_t)t * gu_stride;
-    out[(size_t)t * I + j] = from_f32<T>(moe_glu(to_f32(row[j]), to_f32(row[I + j]), limit, alpha));
+    out[(size_t)t * I + j] = from_f32<T>(moe_glu(to_f32(row[j]), to_f32(row[I + j]), limit, alpha, MOE_ACT_NONE));
 }
 
 extern "C" int ilm_glu_clamp(void* out, const void* gu, int T_, int I, int gu_stride, float limit, float alpha, int dtype, hipStream_t stream) {

@@ -17,6 +17,7 @@ from ..cache.manager import Lent
 from ..config.spec import ModelSpec, PartSpec
 from ..parts import BuildContext, HyperStreams, Param, ResidualStream, build_block
 from ..parts.base import join_name
+from ..parts.linear import Linear
 from ..parts.registry import build_embedding, build_head, build_norm
 
 
@@ -38,6 +39,9 @@ class CausalLM:
         self.run_vectors = None
         if spec.run_vectors is not None:
             self.run_vectors = torch.empty((int(spec.run_vectors[1]), spec.hidden_size), dtype=dtype, device=self.device)
+        self.run_projection = None
+        if spec.run_projection is not None:
+            self.run_projection = Linear(2 * spec.hidden_size, spec.hidden_size, spec.run_projection, False, ctx, suffix="")
         # tensors of the model that several layers read (a table of which every layer takes its own columns): made here, loaded
         # under their own names, handed to every block that asks for them
         self.shared_tensors = {name: torch.empty(tuple(shape), dtype=dtype, device=self.device)
@@ -45,7 +49,7 @@ class CausalLM:
         for b in self.blocks:
             if hasattr(b, "bind_shared"):
                 b.bind_shared(self.shared_tensors)
-        self._keeps_embedding = any(r.start is not None and r.start.embedding != 0.0 for r in spec.order)
+        self._keeps_embedding = any(r.start is not None and (r.start.embedding != 0.0 or r.start.project_embedding) for r in spec.order)
         # cache entry -> what its writer's mixer needs
         self.cache_needs: List = [None] * spec.num_cache_entries()
         for run in spec.order:
@@ -89,6 +93,8 @@ class CausalLM:
             out[join_name(self.spec.final_norm_name, name)] = p
         if self.run_vectors is not None:
             out[self.spec.run_vectors[0]] = Param(self.run_vectors)
+        if self.run_projection is not None:
+            out.update(self.run_projection.named_parameters())
         for name, t in self.shared_tensors.items():
             out[name] = Param(t)
         if not self.spec.head.always_tied:
@@ -130,6 +136,8 @@ class CausalLM:
                     stream.push_more(first, run.start.embedding)
                 if run.start.vector_row is not None:
                     stream.push_more(self.run_vectors[run.start.vector_row], 1.0)
+                if run.start.project_embedding:
+                    stream.project_beside(first, self.run_projection, self.dtype)
             view = cache.view(run.cache, batch, run.writes_cache) if run.cache is not None else None
             if run.borrows is not None:
                 view = Lent(view, cache.view(run.borrows, batch, False))

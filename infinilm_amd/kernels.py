@@ -1298,23 +1298,17 @@ def norm_add_norm(residual: torch.Tensor, branch: torch.Tensor, branch_weight: t
 LN_MAX_ADDENDS = 4   # (ilm_add_layernorm_max_addends())
 
 
-def add_layernorm(residual: torch.Tensor, addends, weight: Optional[torch.Tensor], bias: Optional[torch.Tensor], eps: float,
-                  out_dtype: torch.dtype) -> Optional[torch.Tensor]:
-    """residual += sum of scale * addend (in place, float32) over `addends` = [(tensor, scale), ...], then its layer norm
-    (x - mean) / sqrt(mean of squared deviations + eps) * weight + bias as out_dtype.  An addend is [rows, H] (float32 or
-    bfloat16), contiguous float32 parts [P, rows, H] that are summed in order, or one row [H] added to every row.
-    Without `weight` only the sum is done and None returned.  More addends than the kernel takes are summed by a call
-    of their own first."""
-    _dev(residual, weight, bias)
-    rows, H = residual.shape
-    if residual.dtype != F32 or not residual.is_contiguous():
-        raise KernelError("the residual stream is a contiguous float32 tensor")
+def _fold_extra(residual: torch.Tensor, addends) -> list:
+    """The addends a kernel takes in one call; more than that are summed into the stream by calls of their own first."""
     addends = list(addends)
     while len(addends) > LN_MAX_ADDENDS:
-        add_layernorm(residual, addends[:LN_MAX_ADDENDS], None, None, eps, out_dtype)
+        add_layernorm(residual, addends[:LN_MAX_ADDENDS], None, None, 0.0, F32)
         addends = addends[LN_MAX_ADDENDS:]
-    if weight is None and not addends:
-        return None
+    return addends
+
+
+def _addend_args(residual: torch.Tensor, addends) -> list:
+    rows, H = residual.shape
     flat = []
     for t, scale in addends:
         _dev(t)
@@ -1327,6 +1321,24 @@ def add_layernorm(residual: torch.Tensor, addends, weight: Optional[torch.Tensor
             raise KernelError(f"an addend of shape {tuple(t.shape)} does not fit the residual stream {tuple(residual.shape)}")
         flat += [t.data_ptr(), _dt(t), parts, pstride, rstride, float(scale)]
     flat += [None, 0, 0, 0, 0, 0.0] * (LN_MAX_ADDENDS - len(addends))
+    return flat
+
+
+def add_layernorm(residual: torch.Tensor, addends, weight: Optional[torch.Tensor], bias: Optional[torch.Tensor], eps: float,
+                  out_dtype: torch.dtype) -> Optional[torch.Tensor]:
+    """residual += sum of scale * addend (in place, float32) over `addends` = [(tensor, scale), ...], then its layer norm
+    (x - mean) / sqrt(mean of squared deviations + eps) * weight + bias as out_dtype.  An addend is [rows, H] (float32 or
+    bfloat16), contiguous float32 parts [P, rows, H] that are summed in order, or one row [H] added to every row.
+    Without `weight` only the sum is done and None returned.  More addends than the kernel takes are summed by a call
+    of their own first."""
+    _dev(residual, weight, bias)
+    rows, H = residual.shape
+    if residual.dtype != F32 or not residual.is_contiguous():
+        raise KernelError("the residual stream is a contiguous float32 tensor")
+    addends = _fold_extra(residual, addends)
+    if weight is None and not addends:
+        return None
+    flat = _addend_args(residual, addends)
     out = None
     if weight is not None:
         if weight.shape != (H,) or not weight.is_contiguous() or (bias is not None and (bias.shape != (H,) or bias.dtype != weight.dtype
@@ -1335,6 +1347,41 @@ def add_layernorm(residual: torch.Tensor, addends, weight: Optional[torch.Tensor
         out = torch.empty((rows, H), dtype=out_dtype, device=residual.device)
     _run("ilm_add_layernorm", _ptr(out), residual.data_ptr(), _ptr(weight), _ptr(bias), rows, H, float(eps), _DT[out_dtype],
          _dt(weight) if weight is not None else 0, len(addends), *flat, _stream())
+    return out
+
+
+def add_dynamic_tanh(residual: torch.Tensor, addends, alpha: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor],
+                     out_dtype: torch.dtype) -> torch.Tensor:
+    """residual += sum of scale * addend (in place, float32; `addends` as for `add_layernorm`), then tanh(alpha * residual) * weight +
+    bias as out_dtype; alpha: one float32 number on the device."""
+    _dev(residual, alpha, weight, bias)
+    rows, H = residual.shape
+    if residual.dtype != F32 or not residual.is_contiguous():
+        raise KernelError("the residual stream is a contiguous float32 tensor")
+    if alpha.dtype != F32 or alpha.numel() != 1:
+        raise KernelError("alpha is one float32 number")
+    if weight.shape != (H,) or not weight.is_contiguous() or (bias is not None and (bias.shape != (H,) or bias.dtype != weight.dtype
+                                                                                     or not bias.is_contiguous())):
+        raise KernelError(f"weight and bias must be [{H}] of one dtype")
+    addends = _fold_extra(residual, addends)
+    out = torch.empty((rows, H), dtype=out_dtype, device=residual.device)
+    _run("ilm_add_rows", out.data_ptr(), residual.data_ptr(), alpha.data_ptr(), weight.data_ptr(), _ptr(bias), None, 0, rows, H, _DT[out_dtype],
+         _dt(weight), len(addends), *_addend_args(residual, addends), _stream(), label="ilm_add_rows (dynamic tanh)")
+    return out
+
+
+def add_beside(residual: torch.Tensor, addends, other: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+    """residual += sum of scale * addend (in place, float32), then the rows [residual | other] as out_dtype, [rows, 2 H]; other:
+    float32 [rows, H]."""
+    _dev(residual, other)
+    rows, H = residual.shape
+    for t in (residual, other):
+        if t.dtype != F32 or not t.is_contiguous() or tuple(t.shape) != (rows, H):
+            raise KernelError("the residual stream and the rows beside it are contiguous float32 tensors of one shape")
+    addends = _fold_extra(residual, addends)
+    out = torch.empty((rows, 2 * H), dtype=out_dtype, device=residual.device)
+    _run("ilm_add_rows", out.data_ptr(), residual.data_ptr(), None, None, None, other.data_ptr(), 1, rows, H, _DT[out_dtype], 0, len(addends),
+         *_addend_args(residual, addends), _stream(), label="ilm_add_rows (beside)")
     return out
 
 
@@ -1350,17 +1397,19 @@ USE_HEADMIX_MFMA = os.environ.get("INFINILM_AMD_HEADMIX_MFMA", "1") == "1"   # 0
 def qkv_norm_rope_kvwrite(qkv: torch.Tensor, positions: torch.Tensor, freq: Optional[torch.Tensor], q_weight: Optional[torch.Tensor],
                           k_weight: Optional[torch.Tensor], k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor],
                           slots: Optional[torch.Tensor], nh: int, nkv: int, d: int, dn: int, dv: int, rd: int, v_norm: bool,
-                          eps: float) -> None:
+                          eps: float, half: bool = False, magnitude: float = 1.0, values_are_keys: bool = False) -> None:
     """In the fused projection rows [T, (nh + 2 nkv) d]: every q and k head RMS-normed over its first `dn` entries times
     `q_weight` / `k_weight` [dn] (None: no norm), then its entry pairs (2i, 2i + 1), i < rd / 2, turned by position x
     freq[i]; every v head divided by its root mean square over its first `dv` entries (`v_norm`); k and v written to the
-    paged cache at `slots` (None: no write).  Entries of a head beyond those that count become zeros."""
+    paged cache at `slots` (None: no write).  Entries of a head beyond those that count become zeros.  `half`: the pairs are
+    (i, i + rd / 2); `magnitude`: cosine and sine times it; `values_are_keys`: rows [T, (nh + nkv) d], whose key heads as
+    projected (before norm and turn) are the values too.  Only the queries' place in the rows is sure to hold the result."""
     _dev(qkv, positions, freq, q_weight, k_weight, k_cache, v_cache, slots)
     _rows(qkv, "qkv")
     _i32(positions, "positions")
     T = qkv.shape[0]
-    if qkv.shape[1] != (nh + 2 * nkv) * d or positions.numel() != T:
-        raise KernelError(f"rows of {qkv.shape[1]} do not hold {nh} + 2 x {nkv} heads of {d}")
+    if qkv.shape[1] != (nh + (1 if values_are_keys else 2) * nkv) * d or positions.numel() != T:
+        raise KernelError(f"rows of {qkv.shape[1]} do not hold {nh} + {1 if values_are_keys else 2} x {nkv} heads of {d}")
     if rd and (freq is None or freq.dtype != F32 or freq.numel() != rd // 2 or not freq.is_contiguous()):
         raise KernelError(f"frequencies must be float32 [{rd // 2}]")
     for w in (q_weight, k_weight):
@@ -1375,7 +1424,18 @@ def qkv_norm_rope_kvwrite(qkv: torch.Tensor, positions: torch.Tensor, freq: Opti
     _run("ilm_qkv_norm_rope_kvwrite", qkv.data_ptr(), positions.data_ptr(), _ptr(freq), _ptr(q_weight), _ptr(k_weight),
          _ptr(k_cache) if slots is not None else None, _ptr(v_cache) if slots is not None else None, _ptr(slots), T, nh, nkv, d,
          int(dn), int(dv), int(rd), int(bool(v_norm)), float(eps), page, qkv.stride(0), _dt(qkv),
-         _dt(q_weight) if q_weight is not None else _dt(qkv), _stream())
+         _dt(q_weight) if q_weight is not None else _dt(qkv), int(bool(half)), float(magnitude), int(bool(values_are_keys)), _stream())
+
+
+def head_gate_(o: torch.Tensor, gate: torch.Tensor, heads: int, d: int) -> torch.Tensor:
+    """o[t, h d + e] *= sigmoid(gate[t, h]) in place; o [T, heads d], gate [T, heads] (a view into wider rows is fine), of one dtype."""
+    _dev(o, gate)
+    _rows(o, "o")
+    _rows(gate, "gate")
+    if o.shape[1] != heads * d or tuple(gate.shape) != (o.shape[0], heads) or o.dtype != gate.dtype:
+        raise KernelError(f"gate {tuple(gate.shape)} does not fit {heads} heads of {d} in rows {tuple(o.shape)}")
+    _run("ilm_head_gate", o.data_ptr(), gate.data_ptr(), o.shape[0], int(heads), int(d), o.stride(0), gate.stride(0), _dt(o), _stream())
+    return o
 
 
 def headmix_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor,
@@ -1873,14 +1933,25 @@ class ExpertPlan:
 
 
 def moe_route(logits: torch.Tensor, experts: int, top: int, big_tiles_ok: bool = False, softmax: bool = False,
-              weight_scale: float = 1.0) -> ExpertPlan:
+              weight_scale: float = 1.0, identity: int = 0, correction: Optional[torch.Tensor] = None, groups: int = 1, keep: int = 1,
+              normalise: bool = False) -> ExpertPlan:
     """From float32 router logits [T, >= experts] (the first `experts` entries of a row count): the `top` experts of every token
     with weight_scale x sigmoid(logit) (or, `softmax`, weight_scale x the logit's softmax over all experts) as their weights, and
     the pairs ordered by expert for `moe_gemm`.  `big_tiles_ok`: the products that
-    follow are bfloat16 with every K a multiple of 8, so a step of many pairs an expert may be cut into tiles of 128 rows."""
-    _dev(logits)
-    if logits.dtype != F32 or logits.dim() != 2 or logits.stride(1) != 1 or logits.shape[1] < experts:
+    follow are bfloat16 with every K a multiple of 8, so a step of many pairs an expert may be cut into tiles of 128 rows.
+    `identity`: so many experts more, the last entries, have no matrices: their result is the token's row itself, and their pairs
+    have no place in the order.  `normalise` (softmax alone): the weights are divided by their sum over the chosen experts;
+    `correction` float32 [experts + identity] is added to the scores for the choice alone; of `groups` equal groups of
+    neighbours only the `keep` with the largest corrected score may be chosen from."""
+    _dev(logits, correction)
+    total = experts + int(identity)
+    if logits.dtype != F32 or logits.dim() != 2 or logits.stride(1) != 1 or logits.shape[1] < total:
         raise KernelError("router logits are float32 rows that hold every expert")
+    grouped = normalise or correction is not None or groups > 1
+    if grouped and not (softmax and normalise):
+        raise KernelError("a choice by groups or with a correction goes with softmax scores divided by their sum")
+    if correction is not None and (correction.dtype != F32 or tuple(correction.shape) != (total,) or not correction.is_contiguous()):
+        raise KernelError(f"the choice's correction must be contiguous float32 [{total}]")
     T = logits.shape[0]
     P = T * top
     plan = ExpertPlan()
@@ -1888,8 +1959,12 @@ def moe_route(logits: torch.Tensor, experts: int, top: int, big_tiles_ok: bool =
     plan.top, plan.pairs = int(top), P
     plan.ids = torch.empty((T, top), dtype=torch.int32, device=dev)
     plan.weights = torch.empty((T, top), dtype=F32, device=dev)
-    _run("ilm_moe_route", plan.ids.data_ptr(), plan.weights.data_ptr(), logits.data_ptr(), T, int(experts), int(top), logits.stride(0),
-         int(bool(softmax)), float(weight_scale), _stream())
+    if grouped:
+        _run("ilm_moe_route_groups", plan.ids.data_ptr(), plan.weights.data_ptr(), logits.data_ptr(), _ptr(correction), 0, T, total, int(top),
+             logits.stride(0), int(groups), int(keep), float(weight_scale), _stream())
+    else:
+        _run("ilm_moe_route", plan.ids.data_ptr(), plan.weights.data_ptr(), logits.data_ptr(), T, total, int(top), logits.stride(0),
+             int(bool(softmax)), float(weight_scale), _stream())
     plan.tile_rows = MOE_BIG_TILE_ROWS if big_tiles_ok and not MOE_FORCE_PLAIN and P >= MOE_BIG_MIN_ROWS * experts else MOE_TILE_ROWS
     plan.max_tiles = min(P, P // plan.tile_rows + min(experts, P))
     book = torch.empty((experts + 1 + 2 * P + 3 * plan.max_tiles + 1,), dtype=torch.int32, device=dev)
@@ -1904,8 +1979,8 @@ def moe_route(logits: torch.Tensor, experts: int, top: int, big_tiles_ok: bool =
 
 
 def moe_gemm(x: torch.Tensor, w: torch.Tensor, plan: ExpertPlan, glu: bool, limit: float = 0.0, alpha: float = 1.702,
-             gather: bool = False, act: str = "none") -> torch.Tensor:
-    """The experts' products over the ordered pairs.  `glu`: x [T, K] are the tokens' rows, w [E, 2 I, K] holds every expert's
+             gather: bool = False, act: str = "none", weighted: bool = True) -> torch.Tensor:
+    """The experts' products over the ordered pairs.  `glu` (`act` "silu": silu(gate) * up instead; `weighted` false: the rows as they are): x [T, K] are the tokens' rows, w [E, 2 I, K] holds every expert's
     gate rows and then its up rows; a pair's row is its token's row times the pair's weight, and the result [pairs, I] is
     min(gate, limit) * sigmoid(alpha * min(gate, limit)) * (clamp(up, -limit, limit) + 1) in sorted order.  Otherwise x [pairs, K] are rows
     in sorted order (`gather`: the tokens' rows [T, K], from which every pair takes its token's, unweighted) and w [E, N, K]: the
@@ -1918,22 +1993,23 @@ def moe_gemm(x: torch.Tensor, w: torch.Tensor, plan: ExpertPlan, glu: bool, limi
     N = Nw // 2 if glu else Nw
     if not glu and not gather and x.shape[0] != plan.pairs:
         raise KernelError("rows in sorted order: one a pair")
-    if act not in ("none", "relu2") or (glu and act != "none"):
-        raise KernelError(f"the experts' plain product takes no activation or relu2, got {act!r}")
+    if act not in (("none", "silu") if glu else ("none", "relu2")):
+        raise KernelError(f"the experts' plain product takes no activation or relu2, the gated one none or silu, got {act!r}")
     out = torch.empty((plan.pairs, N), dtype=x.dtype, device=x.device)
     _run("ilm_moe_gemm", out.data_ptr(), N, x.data_ptr(), x.stride(0), plan.perm.data_ptr() if (glu or gather) else None, plan.top,
-         plan.weights.data_ptr() if glu else None,
+         plan.weights.data_ptr() if glu and weighted else None,
          w.data_ptr(), Nw * K, K, plan.tiles.data_ptr(), plan.n_tiles.data_ptr(), plan.max_tiles, N, K, int(bool(glu)), float(limit),
-         float(alpha), 1 if act == "relu2" else 0, _dt(x), int(MOE_FORCE_PLAIN), plan.tile_rows, int(MOE_WIDE) | (2 if MOE_PLAIN_PAIR else 0), _stream(), label="ilm_moe_gemm (gate/up)" if glu else ("ilm_moe_gemm (up)" if gather else "ilm_moe_gemm (down)"))
+         float(alpha), {"none": 0, "relu2": 1, "silu": 2}[act], _dt(x), int(MOE_FORCE_PLAIN), plan.tile_rows, int(MOE_WIDE) | (2 if MOE_PLAIN_PAIR else 0), _stream(), label="ilm_moe_gemm (gate/up)" if glu else ("ilm_moe_gemm (up)" if gather else "ilm_moe_gemm (down)"))
     return out
 
 
 def moe_combine(pair_out: torch.Tensor, plan: ExpertPlan, shared: Optional[torch.Tensor] = None,
-                shared_gate: Optional[torch.Tensor] = None, weighted: bool = False) -> torch.Tensor:
+                shared_gate: Optional[torch.Tensor] = None, weighted: bool = False,
+                identity_rows: Optional[torch.Tensor] = None) -> torch.Tensor:
     """y[t] = sum over the token's slots of pair_out[place of (t, slot)] (`weighted`: times the pair's weight of the plan, in
     float32) + shared[t] * sigmoid(shared_gate[t]); `shared_gate` is a float32 column (one number a token, any stride; None: the
-    shared rows are added as they are)."""
-    _dev(pair_out, shared, shared_gate)
+    shared rows are added as they are).  `identity_rows` [T, H]: what a pair of an identity expert contributes, its token's row."""
+    _dev(pair_out, shared, shared_gate, identity_rows)
     _rows(pair_out, "pair_out")
     P, H = pair_out.shape
     T = P // plan.top
@@ -1947,10 +2023,15 @@ def moe_combine(pair_out: torch.Tensor, plan: ExpertPlan, shared: Optional[torch
             if shared_gate.dtype != F32 or shared_gate.shape[0] != T:
                 raise KernelError("the shared expert's gate is one float32 number a token")
             sg_stride = shared_gate.stride(0)
+    if identity_rows is not None:
+        _rows(identity_rows, "identity_rows")
+        if tuple(identity_rows.shape) != (T, H) or identity_rows.dtype != pair_out.dtype:
+            raise KernelError("the identity experts' rows must match the tokens'")
     out = torch.empty((T, H), dtype=pair_out.dtype, device=pair_out.device)
     _run("ilm_moe_combine", out.data_ptr(), pair_out.data_ptr(), plan.inv.data_ptr(), plan.top, _ptr(shared),
          _ptr(shared_gate) if shared is not None else None, sg_stride, T, H, pair_out.stride(0),
-         plan.weights.data_ptr() if weighted else None, _dt(pair_out), _stream())
+         plan.weights.data_ptr() if weighted else None, _ptr(identity_rows), identity_rows.stride(0) if identity_rows is not None else 0,
+         _dt(pair_out), _stream())
     return out
 
 
@@ -2144,3 +2225,72 @@ def delta_rule(rows: torch.Tensor, gates: torch.Tensor, heads: int, groups: int,
     if not chunked or segments > 1:
         _run("ilm_delta_step", o.data_ptr(), None, *step, DELTA_CHUNK_FROM - 1 if chunked else 1 << 30, None, None, 0, 0.0, 0, 0, 0, 0, _stream())
     return group_norm_gate(o, norm_weight, eps, heads, gate=gate, gate_act="silu", out_dtype=out_dtype)
+
+
+# ---- matrix memories with exponential gates (mLSTM) --------------------------------------------------------------------------
+MLSTM_MAX_KEY_DIM = 512          # (ilm_mlstm_max_dk())
+MLSTM_CHUNK = 64                 # tokens a chunk of a long segment (ilm_mlstm_chunk())
+MLSTM_CHUNK_MAX_KEY_DIM = 256    # (ilm_mlstm_chunk_max_dk())
+MLSTM_CHUNK_COLS = 128           # columns of v a workgroup of the chunked form holds (ilm_mlstm_chunk_cols())
+MLSTM_CHUNK_FROM = int(os.environ.get("INFINILM_AMD_MLSTM_CHUNK_FROM", "32"))   # segments from this length on go in chunks (0: never)
+MLSTM_PIECE = int(os.environ.get("INFINILM_AMD_MLSTM_PIECE", "0"))              # tokens a piece (0: as `mlstm_piece` picks)
+MLSTM_MAX_PIECE = 1024
+
+
+def mlstm_piece(tokens: int, heads: int, dv: int, cus: int) -> int:
+    """Tokens a piece of a long segment: as long as the pieces of all heads still give every compute unit one."""
+    blocks = heads * -(-dv // MLSTM_CHUNK_COLS)
+    return MLSTM_CHUNK * max(1, min(MLSTM_MAX_PIECE // MLSTM_CHUNK, tokens * blocks // (MLSTM_CHUNK * cus)))
+
+
+def mlstm(rows: torch.Tensor, bias_i: torch.Tensor, bias_f: torch.Tensor, i_off: int, f_off: int, g_off: int, heads: int, dk: int, dv: int,
+          cap: float, pool: torch.Tensor, pool_m: torch.Tensor, state_in: torch.Tensor, state_out: torch.Tensor, seg_offsets: torch.Tensor,
+          segments: int, norm_weight: torch.Tensor, eps: float, out_dtype: torch.dtype, max_len: Optional[int] = None) -> torch.Tensor:
+    """Per head and token of every segment, from the fused projection's rows [q: heads dk | k: heads dk | v: heads dv | ...] with the raw
+    input and forget gates [heads] at columns i_off, f_off and the output gate [heads dv] at g_off:
+      li = cap tanh((raw_i + bias_i) / cap), lf = log sigmoid(cap tanh((raw_f + bias_f) / cap)), m' = max(lf + m, li)
+      S = exp(lf + m - m') S + exp(li - m') outer(k, v), n likewise with k, o = q S / (max(|n . q|, exp(-m')) + 1e-6), q / sqrt(dk)
+      y = o / sqrt(mean(o^2) + eps) * norm_weight [heads dv] * sigmoid(gate), per head, [T, heads dv] as `out_dtype`.
+    `pool` [rows, heads, dv + 1, dk] (row dv: n) and `pool_m` [rows, heads], float32: segment r starts from row state_in[r] and leaves
+    its state in row state_out[r].  `max_len`: a bound on the segments' lengths known on the host: from MLSTM_CHUNK_FROM tokens on,
+    segments go in pieces and chunks on the matrix cores (the result differs from the token-by-token form by rounding)."""
+    _dev(rows, bias_i, bias_f, pool, pool_m, state_in, state_out, seg_offsets, norm_weight)
+    _rows(rows, "rows")
+    T = rows.shape[0]
+    H = int(heads)
+    if rows.shape[1] < max(H * (2 * dk + dv), i_off + H, f_off + H, g_off + H * dv) or min(i_off, f_off, g_off) < 0:
+        raise KernelError(f"rows of {rows.shape[1]} do not hold q, k, v and gates of {H} heads of {dk} / {dv}")
+    if dk > MLSTM_MAX_KEY_DIM:
+        raise KernelError(f"key size {dk} is above {MLSTM_MAX_KEY_DIM}")
+    if pool.dtype != F32 or not pool.is_contiguous() or tuple(pool.shape[1:]) != (H, dv + 1, dk):
+        raise KernelError(f"the state pool must be float32 [rows, {H}, {dv + 1}, {dk}], got {tuple(pool.shape)}")
+    if pool_m.dtype != F32 or not pool_m.is_contiguous() or tuple(pool_m.shape) != (pool.shape[0], H):
+        raise KernelError(f"the running maxima must be float32 [{pool.shape[0]}, {H}], got {tuple(pool_m.shape)}")
+    for t, nm in ((state_in, "state_in"), (state_out, "state_out"), (seg_offsets, "seg_offsets")):
+        _i32(t, nm)
+    if state_in.numel() < segments or state_out.numel() < segments or seg_offsets.numel() < segments + 1:
+        raise KernelError("state rows and offsets must cover every segment")
+    if norm_weight.shape != (H * dv,) or not norm_weight.is_contiguous():
+        raise KernelError(f"the norm's weight must be [{H * dv}]")
+    for t in (bias_i, bias_f):
+        if t.shape != (H,) or not t.is_contiguous() or t.dtype != bias_i.dtype:
+            raise KernelError(f"the gates' biases must be [{H}] of one dtype")
+    args = (rows.data_ptr(), rows.stride(0), _dt(rows), bias_i.data_ptr(), bias_f.data_ptr(), _dt(bias_i), int(i_off), int(f_off), int(g_off),
+            float(cap), float(dk) ** -0.5, pool.data_ptr(), pool_m.data_ptr(), state_in.data_ptr(), state_out.data_ptr(), seg_offsets.data_ptr(),
+            int(segments), H, int(dk), int(dv))
+    piece = MLSTM_PIECE or mlstm_piece(T, H, dv, _num_cus(rows.device))
+    slots = T // piece + int(segments)
+    chunked = MLSTM_CHUNK_FROM > 0 and max_len is not None and max_len >= MLSTM_CHUNK_FROM and dk <= MLSTM_CHUNK_MAX_KEY_DIM and slots <= 65535
+    stepped = not chunked or segments > 1
+    normed = (not chunked or dv <= MLSTM_CHUNK_COLS) and (not stepped or bool(_lib().ilm_mlstm_step_norm_ok(dk, dv)))
+    y = torch.empty((T, H * dv), dtype=out_dtype, device=rows.device) if normed else None
+    o = None if normed else torch.empty((T, H * dv), dtype=F32, device=rows.device)
+    norm = (norm_weight.data_ptr(), _dt(norm_weight), float(eps), H * dv, _DT[out_dtype])
+    if chunked:
+        ws = torch.empty((slots * H * _lib().ilm_mlstm_chunk_ws(dk, dv),), dtype=F32, device=rows.device)
+        _run("ilm_mlstm_chunks", _ptr(o), _ptr(y), *args, T, MLSTM_CHUNK_FROM, piece, *norm, ws.data_ptr(), _stream())
+    if stepped:
+        _run("ilm_mlstm_step", _ptr(o), _ptr(y), *args, MLSTM_CHUNK_FROM - 1 if chunked else 1 << 30, *norm, _stream())
+    if normed:
+        return y
+    return group_norm_gate(o, norm_weight, eps, H, gate=rows[:, g_off:g_off + H * dv], gate_act="sigmoid", out_dtype=out_dtype)

@@ -1,1 +1,1 @@
-from . import bebuzen, kekevik, minicpm4, moputar, patadra, pugavik  # noqa: F401
+from . import bebuzen, kekevik, lizezen, minicpm4, moputar, patadra, pugavik  # noqa: F401

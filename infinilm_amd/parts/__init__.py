@@ -1,4 +1,4 @@
-from . import (attention, block, conv_attention, delta_rule, differential_attention, ends, latent_attention, linear_attention, mlp, moe, norm, parallel, rotary, selective_scan, side_input, state_space,  # noqa: F401
+from . import (attention, block, conv_attention, delta_rule, differential_attention, ends, latent_attention, linear_attention, mlp, mlstm, moe, norm, parallel, rotary, selective_scan, side_input, state_space,  # noqa: F401
                temperature)   # (register the built-in kinds)
 from .base import (BuildContext, FeedForward, HyperStreams, Mixer, Norm, Param, Part, PositionEncoding, ResidualStream)
 from .block import build_block

@@ -35,6 +35,10 @@ class GQAttention(Mixer):
     `head_mix`: the scaled scores are mixed over the heads before the softmax, s_h = sum_g M[h, g] raw_g, with a tensor
     M [heads, heads]; `sink`: every head's softmax denominator holds one more term exp(sink_h), a tensor [heads] with no
     key and no value.  Both are float32 whatever the activations' dtype; `mix_names` are their tensor names.
+    `values_are_keys`: there is no value projection, the keys as projected are the values (the position encoding is made for it);
+    `head_gate`: every head's result is multiplied by sigmoid of one number a token, a projection named by it with a row a head;
+    `float_weights`: the softmax weights stay float32 up to the second product; `head_multiple`: heads are filled up to a multiple of
+    it also where the two sizes agree.
     `position_prefix`: the sub-name under which the position encoding's own tensors lie ("": directly under the mixer's)."""
 
     def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int, qkv_bias: bool,
@@ -43,21 +47,34 @@ class GQAttention(Mixer):
                  names: Sequence[str] = ("q_proj", "k_proj", "v_proj", "o_proj"), suffix: str = "weight",
                  whole_output: bool = False, head_mix: bool = False, sink: bool = False,
                  mix_names: Sequence[str] = ("head_mix", "sink"), position_prefix: str = "position", bias_suffix: str = "bias",
-                 keep_first: int = 0, fixed_sink: Optional[float] = None):
+                 keep_first: int = 0, fixed_sink: Optional[float] = None, values_are_keys: bool = False, head_gate: Optional[str] = None,
+                 float_weights: bool = False, head_multiple: int = 1):
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} query heads do not divide into {num_kv_heads} groups")
         self.nh, self.nkv = int(num_heads), int(num_kv_heads)
         self.dn = int(head_dim)                                       # entries of a query or key head that count
         self.dv = int(value_dim) if value_dim is not None else self.dn
         self.d = self.dn if self.dv == self.dn else -(-max(self.dn, self.dv) // 16) * 16   # the head size that runs
+        self.d = -(-self.d // int(head_multiple)) * int(head_multiple)
+        self.float_weights = bool(float_weights)
+        self.values_are_keys = bool(values_are_keys)
+        if self.values_are_keys and self.dv != self.dn:
+            raise ValueError(f"values of {self.dv} cannot be keys of {self.dn}")
         self.scale = float(scale)
         self.softcap = float(softcap)
         self.window = int(window)
         self.whole_output = bool(whole_output)
         qn, kn, vn, on = names
-        self.qkv = FusedLinear(hidden_size, [self.nh * self.d, self.nkv * self.d, self.nkv * self.d], [qn, kn, vn],
-                               qkv_bias, ctx, suffix=suffix, bias_suffix=bias_suffix,
-                               out_heads=[(self.nh, self.dn, self.d), (self.nkv, self.dn, self.d), (self.nkv, self.dv, self.d)])
+        kv = 1 if self.values_are_keys else 2
+        sizes, pieces = [self.nh * self.d] + [self.nkv * self.d] * kv, [qn, kn, vn][:1 + kv]
+        heads = [(self.nh, self.dn, self.d), (self.nkv, self.dn, self.d), (self.nkv, self.dv, self.d)][:1 + kv]
+        self.qkv_width = sum(sizes)
+        self.gated = head_gate is not None
+        if self.gated:       # (filled up, so that rows stay 16-byte aligned)
+            sizes.append(-(-self.nh // 8) * 8)
+            pieces.append(head_gate)
+            heads.append((1, self.nh, sizes[-1]))
+        self.qkv = FusedLinear(hidden_size, sizes, pieces, qkv_bias, ctx, suffix=suffix, bias_suffix=bias_suffix, out_heads=heads)
         self.o_proj = Linear(self.nh * self.d, hidden_size, on, out_bias, ctx, suffix=suffix, bias_suffix=bias_suffix,
                              in_heads=(self.nh, self.dv, self.d))
         self.position = build_position_encoding(position, ctx)
@@ -98,16 +115,17 @@ class GQAttention(Mixer):
 
     def takes_frag(self, rows: int) -> bool:
         fn = getattr(self.position, "takes_frag", None)
-        return bool(fn is not None and fn(rows, self.qkv, self.nh, self.nkv, self.d))
+        return bool(fn is not None and not self.gated and not self.values_are_keys and fn(rows, self.qkv, self.nh, self.nkv, self.d))
 
     def forward(self, x, batch, cache_view, tail=None):
         pe = self.position
         pe.check(batch)
         qkv = None
-        if batch.taps is None:   # (a dump of the rotated rows needs them in one piece)
+        if batch.taps is None and not self.gated and not self.values_are_keys:   # (a dump of the rotated rows needs them in one piece)
             qkv = pe.project_encode_store(x, self.qkv, batch, cache_view, self.nh, self.nkv, self.d)
         if qkv is None:
-            qkv = self.qkv.forward(x)
+            rows = self.qkv.forward(x)
+            qkv = rows[:, :self.qkv_width] if self.gated else rows
             pe.encode_and_store(qkv, batch, cache_view, self.nh, self.nkv, self.d)
             if batch.taps is not None:
                 batch.taps.setdefault("qkv_rotated", []).append(qkv.clone())
@@ -122,6 +140,8 @@ class GQAttention(Mixer):
                                           seg_offsets=batch.seg_offsets, keep_first=self.keep_first)
         else:
             o = self._plain_attention(qkv, batch, cache_view)
+        if self.gated:
+            kernels.head_gate_(o, rows[:, self.qkv_width:self.qkv_width + self.nh], self.nh, self.d)
         if tail is not None:   # the output projection adds into the residual stream itself, where its kernel can
             deferred = self.o_proj.forward_tail(o, tail)
             if deferred is not None:
@@ -131,5 +151,6 @@ class GQAttention(Mixer):
     def _plain_attention(self, qkv, batch, cache_view):
         o = kernels.paged_attention(qkv, cache_view.k, cache_view.v, cache_view.block_tables, batch.seg_of_token,
                                     batch.positions, self.nh, self.nkv, self.d, self.scale, self.window,
-                                    batch.max_total_len, batch.att_tiles, batch.att_single_rows, softcap=self.softcap)
+                                    batch.max_total_len, batch.att_tiles, batch.att_single_rows, softcap=self.softcap,
+                                    float_weights=self.float_weights)
         return o

@@ -156,6 +156,24 @@ class ResidualStream:
         self.push(branch, scale)
         self.pending_norm = norm
 
+    def take_addends(self) -> list:
+        """Everything that is due to the stream as (tensor, scale) pairs, for a kernel that sums them into it."""
+        if self.pending_gate is not None:
+            self.settle()
+        if self.pending_norm is not None:
+            norm, self.pending_norm = self.pending_norm, None
+            self.pending = norm.apply(self.pending)
+        addends = ([(self.pending, self.pending_scale)] if self.pending is not None else []) + self.more
+        self.pending, self.pending_scale, self.more = None, 1.0, []
+        return addends
+
+    def project_beside(self, other: torch.Tensor, proj, dtype: torch.dtype) -> None:
+        """The stream becomes proj([stream | other]) after everything that is due to it; the product's operands are `dtype`, its
+        result float32.  `other` float32 [T, hidden]."""
+        from .. import kernels
+        rows = kernels.add_beside(self.residual, self.take_addends(), other, dtype)
+        self.residual = proj.forward(rows, out_dtype=torch.float32)
+
     def settle(self) -> None:
         """Applies a norm that is still due to the pending branch, so that `pending` is what is added."""
         if self.pending_norm is not None:
@@ -285,6 +303,9 @@ class Mixer(Part):
 
 class FeedForward(Part):
     records_mixed_steps = False   # as for a mixer: nothing in forward depends on the host's view of the batch
+    # a bias [hidden] of the last projection that forward has left out: the arrangement adds it to the stream as one row for all
+    # tokens (a part only does so when it is asked to)
+    deferred_bias: Optional[torch.Tensor] = None
 
     def takes_deferred(self, rows: int) -> bool:
         """Whether forward accepts a DeferredNorm of `rows` rows as x."""

@@ -117,7 +117,8 @@ class SandwichNormBlock:
 @register_arrangement("parallel_residual")
 class ParallelResidualBlock:
     """x += s * (mixer(h) + ffn(h)) with h = norm1(x): one norm, and both sublayers read its output.  A layer may have no
-    feed-forward.  Both outputs are left with the stream and summed into it inside the next norm's kernel."""
+    feed-forward.  Both outputs (and a bias that the feed-forward leaves to the sum, `FeedForward.deferred_bias`) are left with the
+    stream and summed into it inside the next norm's kernel."""
 
     def __init__(self, spec: LayerSpec, ctx: BuildContext):
         self.spec = spec
@@ -149,6 +150,8 @@ class ParallelResidualBlock:
         stream.push(self.mixer.forward(h, batch, cache_view), self.residual_scale)
         if self.ffn is not None:
             stream.push_more(self.ffn.forward(h, batch), self.residual_scale)
+            if self.ffn.deferred_bias is not None:
+                stream.push_more(self.ffn.deferred_bias, self.residual_scale)
 
 
 @register_arrangement("gated_pre_norm")

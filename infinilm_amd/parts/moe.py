@@ -21,6 +21,7 @@ import torch
 from .. import kernels
 from .base import BuildContext, FeedForward, Param
 from .linear import FusedLinear, Linear
+from .mlp import SwiGLU
 from .registry import register_feed_forward
 
 
@@ -144,3 +145,72 @@ class RoutedActivationExperts(FeedForward):
         if self.shared_ff:
             shared = self.shared_down.forward(kernels.activation(self.shared_up.forward(x), self.activation))
         return kernels.moe_combine(pair_out, plan, shared, None, weighted=True)
+
+
+@register_feed_forward("routed_gated_experts")
+class RoutedGatedExperts(FeedForward):
+    """SwiGLU experts weighed on their way out, some of which may be the identity:
+
+      z = W_router h (float32)      s = softmax(z) over all experts, the last `identity` of which have no matrices and return h
+      the `top` experts with the largest s + correction are chosen; the experts form `groups` equal groups of neighbours, of which
+          only the `keep` whose largest s + correction is largest may be chosen from
+      y = sum over the chosen e of  weight_scale * s_e / (sum of the chosen s + 1e-20) * (h, or W_down,e (silu(W_gate,e h) * W_up,e h))
+        + sigmoid(w_sg . h) * (the same form of expert for every token)                                    (if `shared_ff`)
+
+    The experts' matrices lie stacked as for `routed_experts`.  Routing, ordering and the experts' products run on the device
+    alone; weights and sums over a token's experts are float32.  Pairs of identity experts take no part in the products."""
+    records_mixed_steps = True
+    trace: Optional[list] = None     # as `RoutedExperts.trace`
+
+    def __init__(self, hidden_size: int, experts: int, top: int, expert_ff: int, ctx: BuildContext, identity: int = 0,
+                 groups: int = 1, keep: int = 1, weight_scale: float = 1.0, shared_ff: int = 0,
+                 names=("router", "correction", "e{}", "gate", "up", "down", "shared", "sg")):
+        self.W, self.E, self.identity, self.top, self.ff = int(hidden_size), int(experts), int(identity), int(top), int(expert_ff)
+        self.groups, self.keep, self.weight_scale = int(groups), int(keep), float(weight_scale)
+        total = self.E + self.identity
+        if self.groups < 1 or total % self.groups or not 1 <= self.keep <= self.groups:
+            raise ValueError(f"{self.keep} of {self.groups} groups of {total} experts")
+        if not 1 <= self.top <= self.keep * (total // self.groups):
+            raise ValueError(f"{self.top} of the {self.keep * (total // self.groups)} experts of {self.keep} groups a token")
+        self.shared_ff = int(shared_ff or 0)
+        self.names = tuple(names)
+        rn, cn, en, gn, un, dn, sn, sgn = self.names
+        self.dtype = ctx.dtype
+        rows, rnames = [total], [rn]
+        if self.shared_ff:
+            rows.append(1)
+            rnames.append(f"{sn}.{sgn}")
+        self.router = FusedLinear(self.W, rows, rnames, False, ctx, suffix="")
+        self.correction = torch.empty((total,), dtype=torch.float32, device=ctx.device)
+        self.w_gate_up = torch.empty((self.E, 2 * self.ff, self.W), dtype=ctx.dtype, device=ctx.device)
+        self.w_down = torch.empty((self.E, self.W, self.ff), dtype=ctx.dtype, device=ctx.device)
+        self.shared = SwiGLU(self.W, self.shared_ff, False, ctx, names=(f"{sn}.{gn}", f"{sn}.{un}", f"{sn}.{dn}"), suffix="",
+                             whole_output=True) if self.shared_ff else None
+
+    def named_parameters(self) -> Dict[str, Param]:
+        rn, cn, en, gn, un, dn, sn, sgn = self.names
+        out = dict(self.router.named_parameters())
+        out[cn] = Param(self.correction)
+        for e in range(self.E):
+            pre = en.format(e)
+            out[f"{pre}.{gn}"] = Param(self.w_gate_up[e, :self.ff])
+            out[f"{pre}.{un}"] = Param(self.w_gate_up[e, self.ff:])
+            out[f"{pre}.{dn}"] = Param(self.w_down[e])
+        if self.shared is not None:
+            out.update(self.shared.named_parameters())
+        return out
+
+    def forward(self, x, batch) -> torch.Tensor:
+        logits = kernels.gemm(x, self.router.weight, None, 1.0, torch.float32)          # [T, experts + identity (+ 1)]
+        plan = kernels.moe_route(logits, self.E, self.top, softmax=True, weight_scale=self.weight_scale, identity=self.identity,
+                                 correction=self.correction, groups=self.groups, keep=self.keep, normalise=True,
+                                 big_tiles_ok=x.dtype == torch.bfloat16 and self.W % 8 == 0 and self.ff % 8 == 0 and x.stride(0) % 8 == 0)
+        if RoutedGatedExperts.trace is not None:
+            RoutedGatedExperts.trace.append(plan.ids.clone())
+        act = kernels.moe_gemm(x, self.w_gate_up, plan, True, act="silu", weighted=False)      # [pairs, ff], ordered by expert
+        pair_out = kernels.moe_gemm(act, self.w_down, plan, False)                             # [pairs, hidden]
+        shared = gate = None
+        if self.shared is not None:
+            shared = self.shared.forward(x, batch)
+            gate = logits[:, self.E + self.identity:]
+        return kernels.moe_combine(pair_out, plan, shared, gate, weighted=True, identity_rows=x if self.identity else None)

@@ -126,12 +126,27 @@ class LayerNorm(Norm):
         return out
 
     def forward(self, stream: ResidualStream, frag: bool = False):
-        if stream.pending_gate is not None:
-            stream.settle()
-        if stream.pending_norm is not None:
-            norm, stream.pending_norm = stream.pending_norm, None
-            stream.pending = norm.apply(stream.pending)
-        addends = ([(stream.pending, stream.pending_scale)] if stream.pending is not None else []) + stream.more
-        x = kernels.add_layernorm(stream.residual, addends, self.weight, self.bias, self.eps, self.dtype)
-        stream.pending, stream.pending_scale, stream.more = None, 1.0, []
-        return x
+        return kernels.add_layernorm(stream.residual, stream.take_addends(), self.weight, self.bias, self.eps, self.dtype)
+
+
+@register_norm("dynamic_tanh")
+class DynamicTanh(Norm):
+    """tanh(alpha x) * weight + bias, alpha one number for the whole row: no mean and no variance.  Fused with the sums that are due
+    to the residual stream, as `layernorm`.  Names as there; `alpha_name`: alpha's tensor, without dimensions, float32 here."""
+
+    def __init__(self, size: int, ctx: BuildContext, bias: bool = True, param_name: str = "weight", bias_name: str = "bias",
+                 alpha_name: str = "alpha"):
+        self.size, self.dtype = int(size), ctx.dtype
+        self.param_name, self.bias_name, self.alpha_name = param_name, bias_name, alpha_name
+        self.weight = torch.empty((self.size,), dtype=ctx.dtype, device=ctx.device)
+        self.bias = torch.empty((self.size,), dtype=ctx.dtype, device=ctx.device) if bias else None
+        self.alpha = torch.empty((), dtype=torch.float32, device=ctx.device)
+
+    def named_parameters(self) -> Dict[str, Param]:
+        out = {self.param_name: Param(self.weight, neutral=1.0), self.alpha_name: Param(self.alpha, neutral=0.5)}
+        if self.bias is not None:
+            out[self.bias_name] = Param(self.bias)
+        return out
+
+    def forward(self, stream: ResidualStream, frag: bool = False):
+        return kernels.add_dynamic_tanh(stream.residual, stream.take_addends(), self.alpha, self.weight, self.bias, self.dtype)

@@ -183,6 +183,20 @@ def pair_frequencies(dims: int, base: float, device) -> Optional[torch.Tensor]:
     return torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / dims).to(torch.float32).to(device)
 
 
+def stretched_frequencies(dims: int, base: float, factor: float, original: float, fast: float, slow: float, last: int) -> list:
+    """base^(-2i/dims), i < dims/2, with the slow ones stretched ("YaRN"): a pair that turns `fast` times or more within `original`
+    positions keeps its rate, one that turns `slow` times or less has it divided by `factor`, and between the two pairs' numbers
+    (rounded outwards, at least 0 and at most `last`) a ramp leads from one to the other.  In float64."""
+    pair = lambda turns: dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+    lo, hi = max(math.floor(pair(fast)), 0), min(math.ceil(pair(slow)), last)
+    out = []
+    for i in range(dims // 2):
+        f = base ** (-2.0 * i / dims)
+        ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+        out.append(f / factor * ramp + f * (1.0 - ramp))
+    return out
+
+
 @register_position_encoding("normed_pair_rotary")
 class NormedPairRotary(PositionEncoding):
     """Queries and keys normed per head, then turned in neighbouring pairs; values of unit size:
@@ -194,15 +208,19 @@ class NormedPairRotary(PositionEncoding):
       v <- v / sqrt(mean(v^2) + eps)                                       per head over its `value_dim` entries (`v_norm`)
 
     One kernel does all of it and writes k and v into the cache.  The angle is formed in float32 from the position in
-    the kernel (no table, so no bound on positions).  `names`: the two weights' tensor names."""
+    the kernel (no table, so no bound on positions).  `names`: the two weights' tensor names.  `half_pairs`: entry i is paired with
+    entry i + rotary_dim / 2 instead; `magnitude`: cosine and sine times it; `values_are_keys`: the rows hold no values, the keys
+    as projected are the values."""
     head_dim = 0    # any size the mixer runs: the entries beyond `dim` / `value_dim` are zeros
 
     def __init__(self, dim: int, value_dim: int, rotary_dim: int, theta: float, eps: float, ctx: BuildContext,
-                 qk_norm: bool = True, v_norm: bool = False, names=("q_norm", "k_norm"), frequencies=None):
+                 qk_norm: bool = True, v_norm: bool = False, names=("q_norm", "k_norm"), frequencies=None, half_pairs: bool = False,
+                 magnitude: float = 1.0, values_are_keys: bool = False):
         self.dim, self.value_dim, self.rotary_dim = int(dim), int(value_dim), int(rotary_dim)
         if self.rotary_dim % 2 or not 0 <= self.rotary_dim <= self.dim:
             raise ValueError(f"rotary_dim {rotary_dim} must be even and at most the head size {dim}")
         self.eps, self.v_norm, self.names = float(eps), bool(v_norm), tuple(names)
+        self.half_pairs, self.magnitude, self.values_are_keys = bool(half_pairs), float(magnitude), bool(values_are_keys)
         # `frequencies`: the rotary_dim / 2 turning rates themselves (a design that scales them), in place of theta^(-2i/dims)
         if frequencies is not None and self.rotary_dim:
             if len(frequencies) != self.rotary_dim // 2:
@@ -221,4 +239,5 @@ class NormedPairRotary(PositionEncoding):
 
     def encode_and_store(self, qkv, batch, view, nh, nkv, d):
         kernels.qkv_norm_rope_kvwrite(qkv, batch.positions, self.freq, self.q_weight, self.k_weight, view.k, view.v, view.slots,
-                                      nh, nkv, d, self.dim, self.value_dim, self.rotary_dim, self.v_norm, self.eps)
+                                      nh, nkv, d, self.dim, self.value_dim, self.rotary_dim, self.v_norm, self.eps, half=self.half_pairs,
+                                      magnitude=self.magnitude, values_are_keys=self.values_are_keys)
