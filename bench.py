@@ -54,8 +54,9 @@ def main() -> int:
                     help="instead of the default workload: prefill and decode throughput of another design (--design) beside MiniCPM4 "
                          "at equal layer sizes (random weights), with the time and the roofline share of every kernel")
     ap.add_argument("--design-shapes", default="1024,4096", help="widths to compare with --designs")
-    ap.add_argument("--design", default="kekevik", choices=["kekevik", "pugavik", "patadra", "bebuzen", "moputar"],
-                    help="the design that --designs puts beside MiniCPM4 (moputar: beside Kekevik too, whose recurrence is the closest to its)")
+    ap.add_argument("--design", default="kekevik", choices=["kekevik", "pugavik", "patadra", "bebuzen", "moputar", "lizezen"],
+                    help="the design that --designs puts beside MiniCPM4 (moputar: beside Kekevik too, whose recurrence is the closest to its; "
+                         "lizezen: beside Moputar and Patadra too, for its recurrence and its experts)")
     args = ap.parse_args()
     if args.gpus != 1 or int(os.environ.get("WORLD_SIZE", "1")) != 1:
         print("bench.py measures one GPU: this engine has no multi-GPU path (N>1 is not run)")
@@ -83,7 +84,7 @@ def main() -> int:
 
 
 def compare_designs(args) -> dict:
-    """`--design` (and with moputar Kekevik too) beside MiniCPM4 at equal width, layers, heads, head size and feed-forward parameters: prefill of
+    """`--design` (and with moputar Kekevik, with lizezen Moputar and Patadra too) beside MiniCPM4 at equal width, layers, heads, head size and feed-forward parameters: prefill of
     `--prefill-tokens` tokens in one step, decode at batch 8 and 64 over `--context` tokens (recorded steps), and for
     every kernel entry point its calls, its time a call in eager steps and, where one bound names it, the share of that
     bound it reaches: bytes it must move over the HBM peak, or floating-point work over the vector float32 peak."""
@@ -94,7 +95,7 @@ def compare_designs(args) -> dict:
     from infinilm_amd.sampling import Sampler, SamplingParams
     from infinilm_amd.weights import fill_random_
     sys.path.insert(0, os.path.join(ROOT, "examples"))
-    from shapes import bebuzen_shape, kekevik_shape, moputar_shape, patadra_shape, pugavik_shape
+    from shapes import bebuzen_shape, kekevik_shape, lizezen_shape, moputar_shape, patadra_shape, pugavik_shape
 
     layers = 8 if args.layers == 32 else args.layers
     T, ctx, ps = args.prefill_tokens, min(args.context, 2048), args.page_size
@@ -113,13 +114,20 @@ def compare_designs(args) -> dict:
             design: patadra_shape(width, heads, d, layers, V) if design == "patadra" else
             bebuzen_shape(width, heads, d, kv, layers, V) if design == "bebuzen" else
             moputar_shape(width, heads, d, kv, layers, V) if design == "moputar" else
+            lizezen_shape(width, heads, d, kv, layers, V) if design == "lizezen" else
             (kekevik_shape if design == "kekevik" else pugavik_shape)(width, heads, d, kv, layers, V, 6 * width)}
         if design == "moputar":
             cfgs["kekevik"] = kekevik_shape(width, heads, d, kv, layers, V, 6 * width)
+        if design == "lizezen":
+            cfgs["moputar"] = moputar_shape(width, heads, d, kv, layers, V)
+            cfgs["patadra"] = patadra_shape(width, heads, d, layers, V)
         rec = {}
         for name, cfg in cfgs.items():
             model = build_model(cfg, "bfloat16", "cuda:0")
             fill_random_(model, seed=0, std=0.02, norm_init="one_plus")
+            for pname, p in model.named_parameters().items():
+                if pname.endswith(".correction"):      # (random corrections would outweigh the scores: every token the same experts)
+                    p.tensor.zero_()
             Hs = model.spec.hidden_size
             params = sum(p.tensor.numel() for p in model.named_parameters().values())
             r = {"parameters": params}
@@ -253,17 +261,36 @@ def compare_designs(args) -> dict:
                             T * C * (2 + 4) / us(rep_p, "ilm_conv_delta_inputs") / HBM_PEAK, 4)
                         share["conv_norm_rope_kvwrite prefill (rows read and written, mean of both layer kinds / HBM peak)"] = round(
                             T * (Ca + heads * d) / 2 * (2 + 2) / us(rep_p, "ilm_conv_norm_rope_kvwrite") / HBM_PEAK, 4)
+                    if name == "lizezen":
+                        f = cfg["layers"][1]["mlp"]
+                        E, top, ff = f["router"]["experts"], f["router"]["top"], f["expert"]["ff"]
+                        real = top * E / (E + f["router"]["identity"])      # pairs a token that have matrices, on average
+                        share["attention decode, both kinds (cache read / HBM peak)"] = round(64 * ctx * kvb / us(rep_d, "ilm_attn_mfma") / HBM_PEAK, 4)
+                        share["attention prefill, both kinds (4 d flops a visible key and head / bf16 matrix peak)"] = round(
+                            4.0 * T * T / 2 * heads * d / us(rep_p, "ilm_attn_tile") / FLOP_PEAK["bf16"], 4)
+                        share["mlstm_step decode (state read + written / HBM peak)"] = round(64 * 2 * state / us(rep_d, "ilm_mlstm_step") / HBM_PEAK, 4)
+                        share["mlstm_chunks prefill (4 dk dv flops a token and head / float32 vector peak)"] = round(
+                            4.0 * T * heads * d * d / us(rep_p, "ilm_mlstm_chunks") / FLOP_PEAK["fp32"], 4)
+                        share["dynamic tanh prefill (stream read + written, two branches read, rows written / HBM peak)"] = round(
+                            T * Hs * (4 + 4 + 2 + 2 + 2) / us(rep_p, "ilm_add_rows (dynamic tanh)") / HBM_PEAK, 4)
+                        share["qkv_norm_rope_kvwrite prefill (query and key rows read and written / HBM peak)"] = round(
+                            T * (heads + 2 * kv) * d * (2 + 2) / us(rep_p, "ilm_qkv_norm_rope_kvwrite") / HBM_PEAK, 4)
+                        gu, dn = "ilm_moe_gemm (gate/up)", "ilm_moe_gemm (down)"
+                        share["experts' gate/up product prefill (flops / bf16 matrix peak)"] = round(2.0 * T * real * 2 * ff * Hs / us(rep_p, gu) / FLOP_PEAK["bf16"], 4)
+                        share["experts' down product prefill (flops / bf16 matrix peak)"] = round(2.0 * T * real * ff * Hs / us(rep_p, dn) / FLOP_PEAK["bf16"], 4)
+                        share["experts' gate/up product decode (all experts' weights read / HBM peak)"] = round(E * 2 * ff * Hs * 2 / us(rep_d, gu) / HBM_PEAK, 4)
+                        share["experts' down product decode (all experts' weights read / HBM peak)"] = round(E * ff * Hs * 2 / us(rep_d, dn) / HBM_PEAK, 4)
                     if name == "minicpm4" and us(rep_p, "library_gemm"):
                         flops = 2.0 * T * Hs * ((heads + 2 * kv) * d + heads * d + 3 * cfg["intermediate_size"]) * layers
                         share["library products prefill, all of a step (flops / bf16 matrix peak)"] = round(
                             flops / (rep_p["library_gemm"]["total_ms"] * 1e-3 / 2) / FLOP_PEAK["bf16"], 4)
-                    if name not in ("pugavik", "patadra", "bebuzen", "moputar") and us(rep_d, "ilm_decay_scan"):
+                    if name not in ("pugavik", "patadra", "bebuzen", "moputar", "lizezen") and us(rep_d, "ilm_decay_scan"):
                         share["decay_scan decode (state read + written / HBM peak)"] = round(64 * 2 * state / us(rep_d, "ilm_decay_scan") / HBM_PEAK, 4)
                         share["decay_scan prefill (4 dk dv flops a token and head / float32 vector peak)"] = round(
                             4.0 * T * heads * d * d / us(rep_p, "ilm_decay_scan") / FLOP_PEAK["fp32"], 4)
-                    if name not in ("pugavik", "patadra", "bebuzen", "moputar") and us(rep_d, "ilm_attn_mfma"):
+                    if name not in ("pugavik", "patadra", "bebuzen", "moputar", "lizezen") and us(rep_d, "ilm_attn_mfma"):
                         share["attention decode (cache read / HBM peak)"] = round(64 * ctx * kvb / us(rep_d, "ilm_attn_mfma") / HBM_PEAK, 4)
-                    if name not in ("pugavik", "patadra", "bebuzen", "moputar") and us(rep_p, "ilm_attn_tile"):
+                    if name not in ("pugavik", "patadra", "bebuzen", "moputar", "lizezen") and us(rep_p, "ilm_attn_tile"):
                         share["attention prefill (4 d flops a visible key and head / bf16 matrix peak)"] = round(
                             4.0 * T * T / 2 * heads * d / us(rep_p, "ilm_attn_tile") / FLOP_PEAK["bf16"], 4)
                     if name == "pugavik":

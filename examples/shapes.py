@@ -157,3 +157,29 @@ def moputar_shape(width: int, heads: int, head_dim: int, kv_heads: int, layers: 
         out.append({"type": kind, "mixer": dict(mixer), "mlp": dict(mlp)})
     return {"architecture": "Moputar", "vocab": vocab, "width": width, "streams": streams, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-5},
             "layers": out}
+
+
+def lizezen_shape(width: int, heads: int, head_dim: int, kv_heads: int, layers: int, vocab: int, experts: int = 14, identity: int = 2,
+                  top: int = 2, loop: dict = None) -> dict:
+    """A Lizezen configuration with the layer sizes of a transformer of this width: four layer kinds in turn (a matrix memory with a
+    dense feed-forward of 6 x width, as many weights as a gated one of 4 x width; an attention with experts; an attention whose values are its
+    keys, with stretched frequencies and capped scores, with the dense feed-forward; a matrix memory with experts), `experts` experts of
+    `width` inner units and `identity` identity experts in four groups of which two are kept, `top` a token, beside a shared expert of
+    the same size.  `loop` (default: the second and third layer, once): the stretch that begins with a product over the stream and
+    the embedding's output."""
+    mem = {"heads": heads, "dim": head_dim, "vdim": head_dim, "gate_cap": 12.0}
+    att = {"heads": heads, "kv_heads": kv_heads, "dim": head_dim, "vdim": head_dim, "scale": head_dim ** -0.5,
+           "rot": {"base": 10000.0, "dims": head_dim}}
+    att2 = dict(att, softcap=30.0, rot={"base": 1000000.0, "dims": head_dim,
+                                        "scaling": {"factor": 4.0, "original": 4096, "fast": 24.0, "slow": 2.0}})
+    dense = {"kind": "dense", "ff": 6 * width}
+    moe = {"kind": "moe", "expert": {"ff": width}, "shared": {"ff": width},
+           "router": {"experts": experts, "identity": identity, "groups": {"count": 4, "keep": 2}, "top": top, "scale": 2.5}}
+    kinds = [("mlstm", mem, dense), ("attention", att, moe), ("attention_2", att2, dense), ("mlstm", mem, moe)]
+    out = [{"type": t, "mixer": dict(m), "mlp": dict(f)} for t, m, f in (kinds[i % 4] for i in range(layers))]
+    cfg = {"architecture": "Lizezen", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": out}
+    if loop is None and layers >= 3:
+        loop = {"start": 1, "stop": 3, "times": 1}
+    if loop:
+        cfg["loop"] = dict(loop)
+    return cfg

@@ -86,6 +86,26 @@ __device__ __forceinline__ int first_key(int p, int reach) {
     return reach < 0 ? p - p % -reach : 0;
 }
 
+// Activations
+__device__ __forceinline__ float silu_f(float x) { return x / (1.0f + expf(-x)); }
+__device__ __forceinline__ float sigmoid_f(float x) { return 1.0f / (1.0f + expf(-x)); }
+
+#define ILM_ACT_NONE 0
+#define ILM_ACT_SILU 1
+#define ILM_ACT_SIGMOID 2
+#define ILM_ACT_RELU2 3
+#define ILM_ACT_GELU_TANH 4
+
+__device__ __forceinline__ float act_f(float x, int kind) {
+    switch (kind) {
+        case ILM_ACT_SILU: return silu_f(x);
+        case ILM_ACT_SIGMOID: return sigmoid_f(x);
+        case ILM_ACT_RELU2: { const float r = fmaxf(x, 0.f); return r * r; }
+        case ILM_ACT_GELU_TANH: return 0.5f * x * (1.0f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
+        default: return x;
+    }
+}
+
 // The gate's activation of a gated feed-forward
 #define ILM_GLU_SILU 0
 #define ILM_GLU_GELU_TANH 1

@@ -1,4 +1,4 @@
-// C[M,N] = alpha * (X[M,K] W[N,K]^T + bias) for few rows of X (M <= 64), bfloat16 in, float
+// C[M,N] = act(alpha * (X[M,K] W[N,K]^T + bias)) (act: none, or one of the activations of common.h) for few rows of X (M <= 64), bfloat16 in, float
 // accumulation: the decode-side projection, bound by reading W once from HBM.
 //
 // v_mfma_f32_16x16x32_bf16 with W rows on the A side and tokens on the B side: one accumulator is
@@ -27,7 +27,7 @@ template <int WAVES, int MG, int RT, int UNROLL, typename TC>
 __global__ void __launch_bounds__(WAVES * 64)
 gemm_skinny_stream_kernel(TC* __restrict__ C, const bf16* __restrict__ X, const bf16* __restrict__ W,
                           const bf16* __restrict__ bias, int M, int N, int K, int lda, int ldw, int ldc,
-                          float alpha) {
+                          float alpha, int act) {
     __shared__ float part[WAVES][RT][MG][64][4];
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int r = lane & 15, q = lane >> 4;
@@ -115,7 +115,7 @@ gemm_skinny_stream_kernel(TC* __restrict__ C, const bf16* __restrict__ X, const 
         const int m = g * 16 + (l & 15);
         if (n < N && m < M) {
             if (bias != nullptr) v += to_f32(bias[n]);
-            C[(size_t)m * ldc + n] = from_f32<TC>(alpha * v);
+            C[(size_t)m * ldc + n] = from_f32<TC>(act != ILM_ACT_NONE ? act_f(alpha * v, act) : alpha * v);
         }
     }
 }
@@ -126,7 +126,7 @@ template <int WAVES, int KSTEPS, int MG, typename TC>
 __global__ void __launch_bounds__(WAVES * 64)
 gemm_skinny_resident_kernel(TC* __restrict__ C, const bf16* __restrict__ X, const bf16* __restrict__ W,
                             const bf16* __restrict__ bias, int M, int N, int K, int lda, int ldw, int ldc,
-                            float alpha, int ntiles, int ks) {
+                            float alpha, int ntiles, int ks, int act) {
     // ks <= KSTEPS: k-steps a wave really takes (K spread evenly over the waves); its other slots load
     // its first address again (a cache hit, no branch around the loads) and multiply by zeros
     static_assert(WAVES * 64 >= 256 * MG, "one reducing thread an output");
@@ -196,7 +196,7 @@ gemm_skinny_resident_kernel(TC* __restrict__ C, const bf16* __restrict__ X, cons
             const int m = g * 16 + (l & 15);
             if (n < N && m < M) {
                 if (bias != nullptr) v += to_f32(bias[n]);
-                C[(size_t)m * ldc + n] = from_f32<TC>(alpha * v);
+                C[(size_t)m * ldc + n] = from_f32<TC>(act != ILM_ACT_NONE ? act_f(alpha * v, act) : alpha * v);
             }
         }
         buf ^= 1;  // the other buffer is free: its readers passed the barrier above one tile ago
@@ -452,7 +452,7 @@ gemm_gateup_swiglu_pair_kernel(bf16* __restrict__ C, const bf16* __restrict__ X,
 
 // variant: 0 = choose; 4 = resident; 1, 2, 3, 5, 6 = shapes of the stream kernel (see below)
 extern "C" int ilm_gemm_skinny(void* C, const void* X, const void* W, const void* bias, int M, int N,
-                               int K, int lda, int ldw, int ldc, float alpha, int out_dtype, int variant,
+                               int K, int lda, int ldw, int ldc, float alpha, int act, int out_dtype, int variant,
                                hipStream_t stream) {
     ILM_REQUIRE(M > 0 && M <= 64 && N > 0 && K > 0, "gemm_skinny: needs 1 <= M <= 64, got M=%d N=%d K=%d", M, N, K);
     ILM_REQUIRE(K % 8 == 0 && lda % 8 == 0 && ldw % 8 == 0, "gemm_skinny: K=%d lda=%d ldw=%d must be multiples of 8",
@@ -460,6 +460,7 @@ extern "C" int ilm_gemm_skinny(void* C, const void* X, const void* W, const void
     ILM_REQUIRE(((uintptr_t)X & 15) == 0 && ((uintptr_t)W & 15) == 0, "gemm_skinny: operands must be 16-byte aligned");
     ILM_REQUIRE(lda >= K && ldw >= K && ldc >= N, "gemm_skinny: strides too small");
     ILM_REQUIRE(out_dtype == ILM_DTYPE_BF16 || out_dtype == ILM_DTYPE_F32, "gemm_skinny: unknown output dtype %d", out_dtype);
+    ILM_REQUIRE(act >= ILM_ACT_NONE && act <= ILM_ACT_GELU_TANH, "gemm_skinny: unknown activation %d", act);
     const int mg = (M + 15) / 16;
     const int ksteps = (K + 31) / 32;
     // two groups of 16 rows take the 8-wave shapes (256 registers a wave): K up to 8 * 16 k-steps
@@ -475,7 +476,7 @@ extern "C" int ilm_gemm_skinny(void* C, const void* X, const void* W, const void
         const int grid = ntiles < ilm_num_cus() * PER_CU ? ntiles : ilm_num_cus() * PER_CU;                         \
         gemm_skinny_resident_kernel<WV, KS, MGR, TC><<<grid, WV * 64, 0, stream>>>(                         \
             (TC*)C, (const bf16*)X, (const bf16*)W, (const bf16*)bias, M, N, K, lda, ldw, ldc, alpha, ntiles, \
-            (ksteps + WV - 1) / WV);                                                                        \
+            (ksteps + WV - 1) / WV, act);                                                                        \
     }
         // measured on MI355X at K = 4096: 8 waves of 16 k-steps (more loads in flight a wave) win where the
         // tiles are at most one a compute unit (o projection, 9.1 against 10.2 us) or many (gate/up 47.8
@@ -515,7 +516,7 @@ extern "C" int ilm_gemm_skinny(void* C, const void* X, const void* W, const void
     const int grid = (N + 16 * rt - 1) / (16 * rt);
 #define SK_CASE(WV, MG, RT, U, TC)                                                                          \
     gemm_skinny_stream_kernel<WV, MG, RT, U, TC><<<grid, WV * 64, 0, stream>>>(                             \
-        (TC*)C, (const bf16*)X, (const bf16*)W, (const bf16*)bias, M, N, K, lda, ldw, ldc, alpha)
+        (TC*)C, (const bf16*)X, (const bf16*)W, (const bf16*)bias, M, N, K, lda, ldw, ldc, alpha, act)
 #define SK_MG(WV, RT, U, TC)                    \
     switch (mg) {                               \
         case 1: SK_CASE(WV, 1, RT, U, TC); break; \

@@ -17,6 +17,8 @@
 //            projections: few output tiles and a long K)
 //   swiglu   a tile is the 8 gate rows and the 8 up rows of the same outputs: act = silu(gate) * up in
 //            bfloat16 rows, gate and up rounded to bfloat16 first, as the unfused path stores them
+//   act      C = f(X W^T + bias) in bfloat16, f one of the activations of common.h (or none), all of K in one workgroup (a
+//            feed-forward's first product without a gate)
 #include "common.h"
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
@@ -26,21 +28,21 @@ typedef __attribute__((ext_vector_type(4))) float f32x4;
 #define GT_THREADS (GT_WAVES * 64)
 #define GT_NT (GT_WAVES * 16)   // W rows a workgroup
 
-enum { GT_PARTS = 0, GT_SWIGLU = 1 };
+enum { GT_PARTS = 0, GT_SWIGLU = 1, GT_ACT = 2 };
 
 struct GtArgs {
     const bf16* X;
     const bf16* W;
-    const bf16* bias;   // swiglu: [2 I] or null
+    const bf16* bias;   // swiglu: [2 I] or null; act: [N] or null
     int M, N, K;        // N: rows of W (parts), outputs I (swiglu: W has 2 I rows)
     int lda, ldw;
     int chunks, chunks_per_part;
     float* C;           // parts
     int ldc;
     size_t part_stride;
-    bf16* act;          // swiglu
+    bf16* act;          // swiglu, act
     int ld_act;
-    int glu;            // swiglu: the gate's activation (glu_act in common.h)
+    int glu;            // swiglu: the gate's activation (glu_act in common.h); act: the activation (act_f)
 };
 
 __device__ __forceinline__ f32x4 gt_mfma(uint4 a, uint4 b, f32x4 c) {
@@ -202,6 +204,29 @@ gemm_tall_kernel(const GtArgs A) {
                     if (n + e < A.N) dst[e] = acc[g][e];
             }
         }
+    } else if (EPI == GT_ACT) {
+        const int n = tile * 16 + q * 4;
+        float b[4] = {0.f, 0.f, 0.f, 0.f};
+        if (A.bias != nullptr) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) b[e] = to_f32(A.bias[n + e < A.N ? n + e : A.N - 1]);
+        }
+#pragma unroll
+        for (int g = 0; g < MG; ++g) {
+            const int m = g * 16 + r;
+            if (m >= M) continue;
+            bf16 o[4];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) o[e] = from_f32<bf16>(act_f(acc[g][e] + b[e], A.glu));
+            bf16* dst = A.act + (size_t)m * A.ld_act + n;
+            if (n + 3 < A.N && (A.ld_act & 3) == 0 && ((uintptr_t)A.act & 7) == 0) {
+                *reinterpret_cast<uint2*>(dst) = *reinterpret_cast<const uint2*>(o);
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (n + e < A.N) dst[e] = o[e];
+            }
+        }
     } else {
         // gate rows for q < 2, up rows for q >= 2: the lane 32 further on holds the up sums of this lane's outputs
         const int I = A.N;
@@ -308,5 +333,20 @@ extern "C" int ilm_gemm_tall_swiglu(void* act, int ld_act, const void* X, int ld
     a.act = (bf16*)act; a.ld_act = ld_act; a.glu = glu;
     gt_launch<GT_SWIGLU>(a, kc, dim3((I + GT_NT / 2 - 1) / (GT_NT / 2), 1), frag_w, stream);
     ILM_LAUNCH_CHECK("gemm_tall_swiglu");
+    return 0;
+}
+
+// C [M, ldc] = f(X W^T + bias), f the activation `act` (0: none); otherwise as ilm_gemm_tall with one part.
+extern "C" int ilm_gemm_tall_act(void* C, int ldc, const void* X, int lda, const void* W, int ldw, const void* bias, int M, int N, int K,
+                                 int kc, int frag_w, int act, hipStream_t stream) {
+    if (gt_check("gemm_tall_act", M, N, K, kc, X, lda, W, ldw, frag_w)) return -1;
+    ILM_REQUIRE(ldc >= N && act >= ILM_ACT_NONE && act <= ILM_ACT_GELU_TANH, "gemm_tall_act: ldc=%d act=%d", ldc, act);
+    GtArgs a = {};
+    a.X = (const bf16*)X; a.W = (const bf16*)W; a.bias = (const bf16*)bias; a.M = M; a.N = N; a.K = K; a.lda = lda; a.ldw = ldw;
+    a.chunks = (K + kc - 1) / kc;
+    a.chunks_per_part = a.chunks;
+    a.act = (bf16*)C; a.ld_act = ldc; a.glu = act;
+    gt_launch<GT_ACT>(a, kc, dim3((N + GT_NT - 1) / GT_NT, 1), frag_w, stream);
+    ILM_LAUNCH_CHECK("gemm_tall_act");
     return 0;
 }

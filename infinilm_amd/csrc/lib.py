@@ -44,7 +44,8 @@ _SIGNATURES = {
     "ilm_attn_f32": [_P, _P, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _F, _P],
     "ilm_gemm_basic": [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P],
     "ilm_attn_basic": [_P, _P, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _F, _P],
-    "ilm_gemm_skinny": [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P],
+    "ilm_gemm_skinny": [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P],
+    "ilm_gemm_tall_act": [_P, _I, _P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P],
     "ilm_attn_mfma": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _F, _I, _P],
     "ilm_attn_mfma_static": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P],
     "ilm_attn_tile": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _F, _I, _P],
@@ -135,9 +136,10 @@ def load(verbose: bool = True) -> ctypes.CDLL:
     lib.ilm_attn_maps_mfma_ok.argtypes = [c_int, c_int, c_int, c_int, c_int, c_int]
     lib.ilm_delta_step_norm_ok.restype = c_int
     lib.ilm_delta_step_norm_ok.argtypes = [c_int, c_int]
-    for name in ("ilm_mlstm_step_norm_ok", "ilm_mlstm_chunk_ws"):
-        getattr(lib, name).restype = c_int
-        getattr(lib, name).argtypes = [c_int, c_int]
+    lib.ilm_mlstm_step_norm_ok.restype = c_int
+    lib.ilm_mlstm_step_norm_ok.argtypes = [c_int, c_int]
+    lib.ilm_mlstm_chunk_ws.restype = c_int
+    lib.ilm_mlstm_chunk_ws.argtypes = [c_int, c_int, c_int]
     lib.ilm_delta_chunk_ws.restype = c_int
     lib.ilm_delta_chunk_ws.argtypes = [c_int, c_int]
     lib.ilm_attn_static_init.restype = c_int

@@ -15,25 +15,6 @@ __device__ __forceinline__ void stf(void* p, int dt, size_t i, float v) {
     if (dt == ILM_DTYPE_F32) ((float*)p)[i] = v;
     else ((uint16_t*)p)[i] = __builtin_bit_cast(uint16_t, (__bf16)v);
 }
-__device__ __forceinline__ float silu_f(float x) { return x / (1.0f + expf(-x)); }
-__device__ __forceinline__ float sigmoid_f(float x) { return 1.0f / (1.0f + expf(-x)); }
-
-#define RC_ACT_NONE 0
-#define RC_ACT_SILU 1
-#define RC_ACT_SIGMOID 2
-#define RC_ACT_RELU2 3
-#define RC_ACT_GELU_TANH 4
-
-__device__ __forceinline__ float act_f(float x, int kind) {
-    switch (kind) {
-        case RC_ACT_SILU: return silu_f(x);
-        case RC_ACT_SIGMOID: return sigmoid_f(x);
-        case RC_ACT_RELU2: { const float r = fmaxf(x, 0.f); return r * r; }
-        case RC_ACT_GELU_TANH: return 0.5f * x * (1.0f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
-        default: return x;
-    }
-}
-
 // eight consecutive elements as floats / from floats (16-byte accesses for bfloat16, two for float)
 __device__ __forceinline__ void ld8(const void* p, int dt, size_t i, float (&v)[8]) {
     if (dt == ILM_DTYPE_F32) {
@@ -86,7 +67,7 @@ unary_vec_kernel(uint16_t* __restrict__ out, const uint16_t* __restrict__ in, in
 extern "C" int ilm_unary(void* out, const void* in, int T_, int n, int out_stride, int in_stride, int kind, int out_dt,
                          int in_dt, hipStream_t stream) {
     ILM_REQUIRE(T_ > 0 && n > 0 && T_ <= 65535 * 32768, "unary: bad sizes T=%d n=%d", T_, n);
-    ILM_REQUIRE(kind >= 0 && kind <= RC_ACT_GELU_TANH, "unary: unknown activation %d", kind);
+    ILM_REQUIRE(kind >= 0 && kind <= ILM_ACT_GELU_TANH, "unary: unknown activation %d", kind);
     if (out_dt == ILM_DTYPE_BF16 && in_dt == ILM_DTYPE_BF16 && n % 8 == 0 && out_stride % 8 == 0 && in_stride % 8 == 0
         && ((uintptr_t)out & 15) == 0 && ((uintptr_t)in & 15) == 0) {
         for (int t0 = 0; t0 < T_; t0 += 65535) {

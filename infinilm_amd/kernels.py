@@ -381,9 +381,12 @@ def gemm(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None, 
             if alpha != 1.0:
                 _run("ilm_scale_rows", out.data_ptr(), M, N, out.stride(0), float(alpha), _stream())
             return out
-    if fast and aligned and M <= 64 and (few or not library_ok):
+    # (33 to 64 rows with a bias: the vendor library's product with the bias row as its addend, below; 64 rows, K 4096, 24,576 outputs:
+    # 106 us with the few-rows kernel, whose X no longer fits the registers)
+    biased_many = fast and bias is not None and alpha == 1.0 and out_dtype == BF16 and USE_LIBRARY_GEMM and not few and M > 32
+    if fast and aligned and M <= 64 and (few or not library_ok) and not biased_many:
         _run("ilm_gemm_skinny", out.data_ptr(), a.data_ptr(), w.data_ptr(), _ptr(bias), M, N, K, a.stride(0),
-             w.stride(0), out.stride(0), float(alpha), _DT[out_dtype], SKINNY_VARIANT, _stream())
+             w.stride(0), out.stride(0), float(alpha), 0, _DT[out_dtype], SKINNY_VARIANT, _stream())
         return out
     if M > 16 and fast and bias is not None and alpha == 1.0 and out_dtype == BF16 and USE_LIBRARY_GEMM:
         # many rows with a bias: the vendor library's product with the bias row as its addend
@@ -490,6 +493,29 @@ def gemm_tall_swiglu(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tens
     return act
 
 
+def linear_activation(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], kind: str, frag_w=None) -> torch.Tensor:
+    """act(x W^T + bias) for a feed-forward without a gate, `kind` one of ACTIVATIONS.  Few rows in bfloat16: bias and activation in
+    the product's epilogue (up to 32 rows with X in registers, 17 to 208 with chunks of X in LDS where the outputs fill the
+    chip); else the product and the activation's kernel."""
+    M, K = x.shape
+    N = w.shape[0]
+    code = activation_code(kind)
+    if x.dtype == BF16 and not FORCE_BASIC and _mfma_operands_ok(x, w, K) and (bias is None or bias.dtype == BF16):
+        _dev(x, w, bias)
+        out = torch.empty((M, N), dtype=BF16, device=x.device)
+        if USE_TALL and max(TALL_MIN_ROWS, 17) <= M <= TALL_GATEUP_MAX_ROWS and N >= TALL_ACT_MIN_OUTPUTS:
+            fw = _frag_of(frag_w) if USE_FRAG else None
+            _run("ilm_gemm_tall_act", out.data_ptr(), N, x.data_ptr(), x.stride(0), fw.data.data_ptr() if fw is not None else w.data_ptr(),
+                 0 if fw is not None else w.stride(0), _ptr(bias), M, N, K, 128, int(fw is not None), code, _stream())
+            return out
+        if _few_rows(M, K):
+            _run("ilm_gemm_skinny", out.data_ptr(), x.data_ptr(), w.data_ptr(), _ptr(bias), M, N, K, x.stride(0), w.stride(0), N, 1.0, code,
+                 _DT[BF16], SKINNY_VARIANT, _stream())
+            return out
+    return activation(gemm(x, w, bias), kind)
+
+
+TALL_ACT_MIN_OUTPUTS = int(os.environ.get("INFINILM_AMD_TALL_ACT_MIN", "8192"))   # outputs from which that product is used (a workgroup takes 128)
 USE_GATEUP_SWIGLU = os.environ.get("INFINILM_AMD_GATEUP_SWIGLU", "1") == "1"
 # outputs from which the gate/up kernel with X in LDS is used (-1: 48 a compute unit; 0: always, as its tests do)
 GATEUP_TALL_MIN_OUTPUTS = int(os.environ.get("INFINILM_AMD_GATEUP_TALL_MIN", "-1"))
@@ -2238,7 +2264,7 @@ MLSTM_MAX_PIECE = 1024
 
 
 def mlstm_piece(tokens: int, heads: int, dv: int, cus: int) -> int:
-    """Tokens a piece of a long segment: as long as the pieces of all heads still give every compute unit one."""
+    """Tokens a piece of a long segment: as long as the pieces of all heads still give each of `cus` places for a workgroup one."""
     blocks = heads * -(-dv // MLSTM_CHUNK_COLS)
     return MLSTM_CHUNK * max(1, min(MLSTM_MAX_PIECE // MLSTM_CHUNK, tokens * blocks // (MLSTM_CHUNK * cus)))
 
@@ -2278,7 +2304,9 @@ def mlstm(rows: torch.Tensor, bias_i: torch.Tensor, bias_f: torch.Tensor, i_off:
     args = (rows.data_ptr(), rows.stride(0), _dt(rows), bias_i.data_ptr(), bias_f.data_ptr(), _dt(bias_i), int(i_off), int(f_off), int(g_off),
             float(cap), float(dk) ** -0.5, pool.data_ptr(), pool_m.data_ptr(), state_in.data_ptr(), state_out.data_ptr(), seg_offsets.data_ptr(),
             int(segments), H, int(dk), int(dv))
-    piece = MLSTM_PIECE or mlstm_piece(T, H, dv, _num_cus(rows.device))
+    # (bfloat16 rows: two workgroups share a compute unit.  2,048 tokens, 32 heads of 128: 99, 80 and 85 us with pieces of 64, 128 and 256,
+    # 8 heads: 38, 46, 74; float rows, one workgroup a unit: 175, 160, 153 and 54, 77, 138)
+    piece = MLSTM_PIECE or mlstm_piece(T, H, dv, _num_cus(rows.device) * (2 if rows.dtype == BF16 else 1))
     slots = T // piece + int(segments)
     chunked = MLSTM_CHUNK_FROM > 0 and max_len is not None and max_len >= MLSTM_CHUNK_FROM and dk <= MLSTM_CHUNK_MAX_KEY_DIM and slots <= 65535
     stepped = not chunked or segments > 1
@@ -2287,7 +2315,7 @@ def mlstm(rows: torch.Tensor, bias_i: torch.Tensor, bias_f: torch.Tensor, i_off:
     o = None if normed else torch.empty((T, H * dv), dtype=F32, device=rows.device)
     norm = (norm_weight.data_ptr(), _dt(norm_weight), float(eps), H * dv, _DT[out_dtype])
     if chunked:
-        ws = torch.empty((slots * H * _lib().ilm_mlstm_chunk_ws(dk, dv),), dtype=F32, device=rows.device)
+        ws = torch.empty((slots * H * _lib().ilm_mlstm_chunk_ws(dk, dv, _dt(rows)) + 4 * T * H + 4,), dtype=F32, device=rows.device)
         _run("ilm_mlstm_chunks", _ptr(o), _ptr(y), *args, T, MLSTM_CHUNK_FROM, piece, *norm, ws.data_ptr(), _stream())
     if stepped:
         _run("ilm_mlstm_step", _ptr(o), _ptr(y), *args, MLSTM_CHUNK_FROM - 1 if chunked else 1 << 30, *norm, _stream())

@@ -89,4 +89,6 @@ class ActivationMLP(FeedForward):
         return out
 
     def forward(self, x, batch) -> torch.Tensor:
-        return self.down.forward(kernels.activation(self.up.forward(x), self.activation), allow_parts=not self.whole_output)
+        frag = self.up.frag_weight if kernels.frag_weight_ok(self.up.weight) and x.shape[0] <= kernels.TALL_MAX_ROWS else None
+        act = kernels.linear_activation(x, self.up.weight, self.up.bias, self.activation, frag_w=frag)
+        return self.down.forward(act, allow_parts=not self.whole_output)
