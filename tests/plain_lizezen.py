@@ -250,3 +250,144 @@ def forward(cfg: dict, w: Dict[str, torch.Tensor], tokens, dtype=torch.float64, 
         return rounded(dynamic_tanh(x, w, "final.norm")) @ w["head"].T
     finally:
         _ROUND[0] = _FORCED[0] = _CHOSEN[0] = None
+
+
+def greedy(cfg: dict, w: Dict[str, torch.Tensor], prompt, n: int) -> List[int]:
+    """The n tokens greedy decoding appends to `prompt` (the whole sequence is run again for every token)."""
+    toks = list(prompt)
+    for _ in range(n):
+        toks.append(int(torch.argmax(forward(cfg, w, toks)[-1])))
+    return toks[len(prompt):]
+
+
+# ---- configurations and weights for the tests --------------------------------------------------------------------------
+def tensor_shapes(cfg: dict) -> Dict[str, tuple]:
+    W = cfg["width"]
+    out = {"embed": (cfg["vocab"], W), "head": (cfg["vocab"], W)}
+    if cfg.get("loop"):
+        out["loop.in"] = (W, 2 * W)
+
+    def norm(name):
+        out.update({name: (W,), name + ".b": (W,), name + ".alpha": ()})
+
+    norm("final.norm")
+    for i, layer in enumerate(cfg["layers"]):
+        p, m = f"l{i}", layer["mixer"]
+        norm(p + ".norm1")
+        if layer["type"] == "mlstm":
+            H, dk, dv = m["heads"], m["dim"], m["vdim"]
+            out.update({p + ".mix.q": (H * dk, W), p + ".mix.k": (H * dk, W), p + ".mix.v": (H * dv, W), p + ".mix.g": (H * dv, W),
+                        p + ".mix.o": (W, H * dv), p + ".mix.norm": (H * dv,), p + ".mix.i": (H, W), p + ".mix.i.b": (H,),
+                        p + ".mix.f": (H, W), p + ".mix.f.b": (H,)})
+        else:
+            H, G, dk, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+            out.update({p + ".mix.q": (H * dk, W), p + ".mix.k": (G * dk, W), p + ".mix.o": (W, H * dv)})
+            if layer["type"] == "attention":
+                out[p + ".mix.v"] = (G * dv, W)
+            else:
+                out.update({p + ".mix.g": (H, W), p + ".mix.q.norm": (dk,), p + ".mix.k.norm": (dk,)})
+        f = layer.get("mlp")
+        if f and f["kind"] == "dense":
+            out.update({p + ".mlp.up": (f["ff"], W), p + ".mlp.up.b": (f["ff"],), p + ".mlp.down": (W, f["ff"]), p + ".mlp.down.b": (W,)})
+        elif f:
+            r = f["router"]
+            total = r["experts"] + r.get("identity", 0)
+            out.update({p + ".mlp.router": (total, W), p + ".mlp.correction": (total,)})
+            parts = [(f".e{e}", f["expert"]["ff"]) for e in range(r["experts"])]
+            if f.get("shared"):
+                parts.append((".shared", f["shared"]["ff"]))
+                out[p + ".mlp.shared.sg"] = (1, W)
+            for name, ff in parts:
+                out.update({p + ".mlp" + name + ".gate": (ff, W), p + ".mlp" + name + ".up": (ff, W), p + ".mlp" + name + ".down": (W, ff)})
+    return out
+
+
+def random_weights(cfg: dict, seed: int) -> Dict[str, torch.Tensor]:
+    """float32 tensors: matrices N(0, 1/in), norm weights near one, biases that spread the forget gates from fast to slow and the
+    input gates to both sides of zero, corrections of either sign that change many choices of experts."""
+    g = torch.Generator().manual_seed(seed)
+    out = {}
+    for name, shape in sorted(tensor_shapes(cfg).items()):
+        t = torch.randn(shape, generator=g)
+        if name.endswith(".alpha"):
+            t = 0.6 + 0.1 * t
+        elif name.endswith(".mix.f.b"):
+            t = 2.5 + 2.0 * t
+        elif name.endswith(".mix.i.b"):
+            t = -1.0 + 2.0 * t
+        elif name.endswith(".b"):
+            t = 0.1 * t
+        elif name.endswith(".correction"):
+            t = 0.15 * t - 0.1
+        elif name.endswith(".router"):
+            t = 2.0 * t / math.sqrt(shape[1])
+        elif len(shape) == 1:
+            t = 1.0 + 0.1 * t
+        elif name != "embed":
+            t = t / math.sqrt(shape[1])
+        out[name] = t
+    return out
+
+
+def mlstm_layer(heads, dim, vdim, cap, mlp):
+    return {"type": "mlstm", "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "gate_cap": cap}, "mlp": mlp}
+
+
+def attention_layer(kind, heads, kv_heads, dim, vdim, base, dims, mlp, scaling=None, softcap=None, scale=None):
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale if scale is not None else dim ** -0.5,
+         "rot": {"base": base, "dims": dims}}
+    if scaling:
+        m["rot"]["scaling"] = dict(zip(("factor", "original", "fast", "slow"), scaling))
+    if softcap:
+        m["softcap"] = softcap
+    return {"type": kind, "mixer": m, "mlp": mlp}
+
+
+def dense_mlp(ff):
+    return {"kind": "dense", "ff": ff}
+
+
+def moe_mlp(experts, identity, top, ff, shared_ff=0, groups=None, scale=1.0):
+    r = {"experts": experts, "top": top, "scale": scale}
+    if identity:
+        r["identity"] = identity
+    if groups:
+        r["groups"] = {"count": groups[0], "keep": groups[1]}
+    out = {"kind": "moe", "router": r, "expert": {"ff": ff}}
+    if shared_ff:
+        out["shared"] = {"ff": shared_ff}
+    return out
+
+
+def config_a():
+    """The first two layers run twice (the stream meets itself: x0 beside x0); heads of no multiple of 16 or 8; a part of each
+    head turned; more identity experts than others in a group; a layer without a feed-forward."""
+    return {"architecture": "Lizezen", "vocab": 61, "width": 40, "norm": {"eps": 1e-5}, "layers": [
+        attention_layer("attention", 4, 2, 12, 20, 500.0, 8, moe_mlp(4, 2, 2, 24, 20, (3, 2), 1.7)),
+        mlstm_layer(3, 10, 14, 9.0, dense_mlp(70)),
+        attention_layer("attention_2", 6, 3, 20, 20, 10000.0, 20, None, scaling=(4.0, 64, 6.0, 1.0), softcap=5.0)],
+        "loop": {"start": 0, "stop": 2, "times": 2}}
+
+
+def config_b():
+    """No loop; one group of experts, none of them the identity, no shared expert, one expert a token; scores without a cap where
+    the values are the keys and with one where they are not; one key/value head for all, one for each; no rotation in one layer."""
+    return {"architecture": "Lizezen", "vocab": 131, "width": 72, "norm": {"eps": 1e-6}, "layers": [
+        mlstm_layer(2, 20, 36, 15.0, moe_mlp(5, 0, 1, 40, scale=0.8)),
+        attention_layer("attention_2", 3, 1, 24, 24, 1000.0, 16, dense_mlp(96), scaling=(2.5, 100, 8.0, 2.0), scale=0.3),
+        attention_layer("attention", 5, 5, 16, 8, 10000.0, 0, None, softcap=8.0),
+        mlstm_layer(5, 7, 3, 4.0, None)]}
+
+
+def config_c():
+    """Sizes that take the matrix-core kernels; one layer in the middle runs three times; two groups of which one is kept; top as
+    large as a group; heads of 64 and 128 with values of another size."""
+    return {"architecture": "Lizezen", "vocab": 300, "width": 128, "norm": {"eps": 1e-5}, "layers": [
+        mlstm_layer(2, 64, 128, 12.0, dense_mlp(320)),
+        attention_layer("attention_2", 4, 2, 64, 64, 50000.0, 64, moe_mlp(6, 2, 4, 64, 48, (2, 1), 2.0), scaling=(8.0, 512, 16.0, 1.5), softcap=20.0),
+        attention_layer("attention", 4, 1, 128, 96, 10000.0, 64, moe_mlp(9, 3, 3, 32, 64, (4, 3), 1.0)),
+        mlstm_layer(4, 128, 32, 20.0, dense_mlp(256))],
+        "loop": {"start": 1, "stop": 2, "times": 3}}
+
+
+CONFIGS = {"A": config_a, "B": config_b, "C": config_c}
