@@ -13,8 +13,11 @@ def _factors(n: int, seed: int):
 
 
 def shape_config(name: str, layers: int = 0) -> dict:
-    """`name`: "8b", "0.5b", "2b" (MiniCPM4 family), "kekevik-<width>", "pugavik-<width>", "patadra-<width>", "bebuzen-<width>" or "moputar-<width>"
+    """`name`: "8b", "0.5b", "2b" (MiniCPM4 family), "kekevik-<width>", "pugavik-<width>", "patadra-<width>", "bebuzen-<width>", "moputar-<width>" or "lizezen-<width>"
     (those designs at that width, 8 layers unless told otherwise); `layers` > 0 overrides the number of layers."""
+    if name.startswith("lizezen-"):
+        width = int(name.split("-", 1)[1])
+        return lizezen_shape(width, width // 128, 128, 2, layers or 8, 32768)
     if name.startswith("moputar-"):
         width = int(name.split("-", 1)[1])
         return moputar_shape(width, width // 128, 128, 2, layers or 8, 32768)
