@@ -1,11 +1,12 @@
 """The matrix memory of an mLSTM (xLSTM): a linear attention whose state is written and forgotten through exponential gates.
 
-  q = W_q h / sqrt(dim), k = W_k h [heads, dim], v = W_v h [heads, vdim], without biases
-  per head a log input gate i = cap tanh((W_i h + b_i) / cap) and a log forget gate f = log sigmoid(cap tanh((W_f h + b_f) / cap))
-  a running maximum m (0 before a sequence's start), a matrix S [dim, vdim] and a vector n [dim] (zeros before it):
-        m_t = max(f + m_{t-1}, i),   S_t = exp(f + m_{t-1} - m_t) S_{t-1} + exp(i - m_t) k v^T,   n_t likewise with k alone
-        o_t = S_t^T q / (max(|n_t . q|, exp(-m_t)) + 1e-6)
-  o_t divided by its root mean square, times norm [heads vdim] and sigmoid(W_g h), per head; then the output product.
+  projections without bias: query and key heads of dim entries, value heads of vdim entries; queries by 1 / sqrt(dim)
+  two numbers a head and token, each squeezed to within +-cap by z -> cap tanh(z / cap) after its bias: i (the logarithm of how
+        strongly the token is written) and, through log sigmoid, f (the logarithm of what stays of the past)
+  a matrix S [dim, vdim], a vector n [dim] and a number m, all zero before a sequence's start; with vectors as rows
+        m' = max(f + m, i),   keep = e^(f + m - m'),   put = e^(i - m')
+        S' = keep S + put outer(k, v),   n' = keep n + put k,   y = q S' / (max(|q . n'|, e^-m') + 1e-6)
+  y of every head by its root mean square, times norm [heads vdim] and the sigmoid of a gate's projection; then the output product.
 
 Two states a request, float32 rows of the cache manager's pools: S with n as one row more, [heads, vdim + 1, dim], and m [heads].
 Everything between the projections is float32 whatever the activations' dtype.
